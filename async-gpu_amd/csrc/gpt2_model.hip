@@ -24,6 +24,7 @@
 #include "decode_step.h"
 #include "elementwise.h"
 #include "linear_common.h"
+#include "lm_runtime.h"
 
 
 namespace {
@@ -40,25 +41,32 @@ struct Block {
     Int4Lin lin[4];
 };
 
-struct DevBuf {
-    void *p = nullptr;
-    size_t bytes = 0;
-};
-
 }  // namespace
 
-struct agpu_gpt2 {
-    agpu_ctx *ctx = nullptr;
+struct agpu_gpt2 final : LmRuntime {
+    agpu_gpt2() : LmRuntime("gpt2") {}
+    int32_t check_ready() override;
+    int32_t ensure_buffers(int B, int new_len, bool all_rows_logits) override;
+    int logits_stride() const override;
+    int32_t launch_forward(const uint32_t *tokens, int B, int new_len, int max_kv, bool all_rows_logits, const ArgmaxAdvance *feed,
+                           bool *fed) override;
+    void mix_addresses(AddrHash &h, bool one_launch) const override;
+    void graphs_dropped() override;
+    int32_t prepare_steps(int B) override;
+    bool one_launch_ready() override;
+    bool one_launch_planned() const override { return pk.stages_dev != nullptr; }
+    int32_t launch_one_step() override;
+    int32_t check_waits() override;
+
     agpu_gpt2_config cfg{};
-    int d = 0, H = 0, ff = 0, V = 0, P = 0, Vpad = 0;
+    int d = 0, H = 0, ff = 0, Vpad = 0;
     float *wte = nullptr, *wpe = nullptr, *lnf_g = nullptr, *lnf_b = nullptr;
     float *wte_t = nullptr;  // [d, V], only for the f32 LM head
     std::vector<Block> blocks;
     Int4Lin lm_head;
     float *kcache = nullptr, *vcache = nullptr;  // [layer][max_batch][H][P][64]
-    int cache_len = 0;
     // activations (grown on demand, never inside a captured region)
-    DevBuf hid, qkv, att, ffn, lnb, last, logits, tok_in;
+    DevBuf hid, qkv, att, ffn, lnb, last;
     DevBuf kfrag, vfrag;  // K and V of one layer as bf16 operand fragments (prefill of one sequence from position 0)
     // batched decode (5 .. 16 sequences): the inputs of the Linears as bf16 pieces left by their producers (hidden rows
     // times the next LayerNorm's gains + their statistics, attention outputs, MLP activations), and per normalising
@@ -66,13 +74,6 @@ struct agpu_gpt2 {
     DevBuf px_h, px_att, px_ffn, px_stats, px_fold;
     bool px_fold_ready = false;
     bool px_off = false;  // AGPU_NO_PX in the environment: keep to the kernels that split their inputs themselves
-    uint32_t *cur_tok = nullptr, *next_tok = nullptr, *out_tok = nullptr;
-    int out_capacity = 0;  // steps recorded in out_tok
-    int *pos_dev = nullptr, *step_dev = nullptr;
-    std::map<long long, hipGraphExec_t> graphs;  // key: batch << 32 | kv bucket
-    std::map<long long, unsigned long long> graph_addr;  // per graph: fingerprint of the device addresses it was captured with
-    unsigned long long ws_epoch = 0;             // the context's scratch the graphs were captured with
-    hipEvent_t ev0 = nullptr, ev1 = nullptr, ev2 = nullptr;
     // early exit: per block one (confidence, arg-max) pair in host-visible memory and one event
     float *probe_conf_host = nullptr, *probe_conf_dev = nullptr;
     uint32_t *probe_tok_host = nullptr, *probe_tok_dev = nullptr;
@@ -83,9 +84,8 @@ struct agpu_gpt2 {
     bool pk_tried = false;
     bool pk_failed = false;   // a wait of the one-launch step gave up: per stage until the step is planned anew
     int pk_failed_looks = 0;  // looks at the decode path since then
-    long long n_one_launch = 0, n_per_stage = 0, n_wait_failures = 0;  // agpu_gpt2_decode_stats
+    long long n_wait_failures = 0;  // agpu_gpt2_decode_stats
     int pk_spin_limit = 0;    // test hook: poll rounds a wait may take (0 = default)
-    int decode_mode = AGPU_DECODE_AUTO;
 };
 
 namespace {
@@ -127,11 +127,6 @@ __global__ __launch_bounds__(256) void gather_last_rows_kernel(const float *__re
     dst[i] = src[((size_t)b * new_len + new_len - 1) * d + j];
 }
 
-__global__ void advance_counters_kernel(int *pos_dev, int *step_dev, int delta) {
-    *pos_dev += delta;
-    *step_dev += 1;
-}
-
 // The token chosen on the host becomes the current token; the position advances by one.
 __global__ void feed_token_kernel(uint32_t *cur_tok, uint32_t token, int *pos_dev) {
     cur_tok[0] = token;
@@ -150,16 +145,6 @@ __global__ __launch_bounds__(256) void kv_zero_rows_kernel(float *kcache, float 
     vcache[at] = 0.0f;
 }
 
-__global__ void set_counters_kernel(int *pos_dev, int pos, int *step_dev, int step) {
-    *pos_dev = pos;
-    if (step >= 0) *step_dev = step;
-}
-
-__global__ __launch_bounds__(256) void fill_u32_kernel(uint32_t *p, uint32_t v, size_t n) {
-    const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
-    if (i < n) p[i] = v;
-}
-
 // [rows, cols] -> [cols, rows]
 __global__ __launch_bounds__(256) void transpose_kernel(const float *__restrict__ in, float *out, int rows, int cols) {
     __shared__ float tile[32][33];
@@ -170,20 +155,6 @@ __global__ __launch_bounds__(256) void transpose_kernel(const float *__restrict_
     __syncthreads();
     for (int r = ty; r < 32; r += 8)
         if (bx + r < cols && by + tx < rows) out[(size_t)(bx + r) * rows + by + tx] = tile[tx][r];
-}
-
-int32_t dev_alloc(agpu_ctx *ctx, void **p, size_t bytes) {
-    hipError_t e = hipMalloc(p, bytes);
-    if (e != hipSuccess) return agpu_hip(ctx, e, "hipMalloc");
-    return AGPU_OK;
-}
-
-int32_t upload(agpu_ctx *ctx, void *dst, const void *src, size_t bytes, int on_device) {
-    hipError_t e = hipMemcpyAsync(dst, src, bytes, on_device ? hipMemcpyDeviceToDevice : hipMemcpyHostToDevice, ctx->stream);
-    if (e != hipSuccess) return agpu_hip(ctx, e, "hipMemcpyAsync");
-    // host sources may be freed by the caller right after the call returns
-    if (!on_device) return agpu_hip(ctx, hipStreamSynchronize(ctx->stream), "hipStreamSynchronize");
-    return AGPU_OK;
 }
 
 int32_t set_vec(agpu_ctx *ctx, float **dst, const float *src, size_t n, int on_device) {
@@ -202,62 +173,10 @@ void free_lin(Int4Lin &l) {
     l = Int4Lin{};
 }
 
-// Every device address a decode step refers to, folded into one word.  A captured graph holds these addresses; a
-// replay is only right while they are still the model's.  Every path that frees or moves one of them drops the graphs
-// (ensure, ensure_out_tokens, the weight setters, a new scratch); this is the check behind that rule.
-unsigned long long step_addresses(const agpu_gpt2 *m, bool one_launch) {
-    unsigned long long h = 1469598103934665603ull;
-    auto mix = [&](const void *p) { h = (h ^ (unsigned long long)(uintptr_t)p) * 1099511628211ull; };
-    for (const void *p : {(const void *)m->wte, (const void *)m->wpe, (const void *)m->lnf_g, (const void *)m->lnf_b, (const void *)m->wte_t,
-                          (const void *)m->kcache, (const void *)m->vcache, (const void *)m->cur_tok, (const void *)m->next_tok,
-                          (const void *)m->out_tok, (const void *)m->pos_dev, (const void *)m->step_dev, (const void *)m->lm_head.packed,
-                          (const void *)m->lm_head.scales, (const void *)m->ctx->workspace, (const void *)m->ctx->counters})
-        mix(p);
-    if (one_launch)  // the step's plan; a graph of per-stage launches does not refer to it
-        for (const void *p : {(const void *)m->pk.arena, (const void *)m->pk.xmem, (const void *)m->pk.stages_dev, (const void *)m->pk.state, (const void *)m->pk.ln_fold}) mix(p);
-    for (const DevBuf *b : {&m->hid, &m->qkv, &m->att, &m->ffn, &m->lnb, &m->last, &m->logits, &m->tok_in, &m->px_h, &m->px_att, &m->px_ffn,
-                            &m->px_stats, &m->px_fold})
-        mix(b->p);
-    for (const Block &b : m->blocks) {
-        for (const void *p : {(const void *)b.ln1_g, (const void *)b.ln1_b, (const void *)b.ln2_g, (const void *)b.ln2_b}) mix(p);
-        for (const Int4Lin &l : b.lin) {
-            mix(l.packed);
-            mix(l.scales);
-            mix(l.bias);
-        }
-    }
-    return h;
-}
-
-void drop_graphs(agpu_gpt2 *m) {
-    // a replay still on the stream must not lose its graph, nor the plan its arena
-    if (m->ctx && !m->graphs.empty()) (void)hipStreamSynchronize(m->ctx->stream);
-    for (auto &kv : m->graphs) (void)hipGraphExecDestroy(kv.second);
-    m->graphs.clear();
-    m->graph_addr.clear();
-    // the plan of the one-launch step holds the same addresses
-    agpu_step_plan_free(&m->pk);
-    m->pk_tried = false;
-}
-
 // A weight setter has replaced a tensor: nothing captured or folded from the old ones may be used again.
 void weights_changed(agpu_gpt2 *m) {
     drop_graphs(m);
     m->px_fold_ready = false;
-}
-
-// Grow a buffer; existing graphs hold the old address, so they are dropped.
-int32_t ensure(agpu_gpt2 *m, DevBuf &b, size_t bytes) {
-    if (b.bytes >= bytes) return AGPU_OK;
-    (void)hipStreamSynchronize(m->ctx->stream);
-    drop_graphs(m);
-    if (b.p) (void)hipFree(b.p);
-    b.p = nullptr;
-    b.bytes = 0;
-    int32_t rc = dev_alloc(m->ctx, &b.p, bytes);
-    if (rc != AGPU_OK) return rc;
-    b.bytes = bytes;
-    return AGPU_OK;
 }
 
 int32_t expected_dims(const agpu_gpt2 *m, int layer, int which, int &K, int &N) {
@@ -289,11 +208,8 @@ int32_t alloc_lin(agpu_gpt2 *m, Int4Lin &l, int K, int N, bool pad, bool with_bi
     if (rc != AGPU_OK) return rc;
     if (pad && l.Npad != N) {
         // pad columns: nibble 8 (= 0) and scale 0, so they produce exact zeros
-        hipLaunchKernelGGL(fill_u32_kernel, dim3((unsigned)((nw + 255) / 256)), dim3(256), 0, m->ctx->stream, l.packed,
-                           0x88888888u, nw);
-        hipLaunchKernelGGL(fill_u32_kernel, dim3((unsigned)((ns + 255) / 256)), dim3(256), 0, m->ctx->stream,
-                           reinterpret_cast<uint32_t *>(l.scales), 0u, ns);
-        rc = AGPU_LAUNCH_CHECK(m->ctx, "fill_u32_kernel");
+        rc = fill_u32(m->ctx, l.packed, 0x88888888u, nw);
+        if (rc == AGPU_OK) rc = fill_u32(m->ctx, l.scales, 0u, ns);
     }
     return rc;
 }
@@ -319,15 +235,6 @@ int32_t check_layer(agpu_gpt2 *m, int layer, int which, int K, int N) {
         return agpu_fail(m->ctx, AGPU_ERR_DIM_OUT_OF_RANGE, "gpt2: linear index %d out of range", which);
     if (K != eK || N != eN)
         return agpu_fail(m->ctx, AGPU_ERR_SHAPE_MISMATCH, "gpt2: expected [K=%d, N=%d], got [K=%d, N=%d]", eK, eN, K, N);
-    return AGPU_OK;
-}
-
-// Token ids the host can see are checked before anything is launched.
-int32_t check_token_ids(agpu_gpt2 *m, const uint32_t *ids_host, size_t n, const char *who) {
-    for (size_t i = 0; i < n; ++i)
-        if (ids_host[i] >= (uint32_t)m->V)
-            return agpu_fail(m->ctx, AGPU_ERR_DIM_OUT_OF_RANGE, "%s: token id %u at index %zu is outside the vocabulary of %d", who,
-                             ids_host[i], i, m->V);
     return AGPU_OK;
 }
 
@@ -575,11 +482,14 @@ int32_t launch_gather_last(agpu_gpt2 *m, int B, int new_len) {
     return AGPU_LAUNCH_CHECK(m->ctx, "gather_last_rows_kernel");
 }
 
+}  // namespace
+
 // One forward over `new_len` tokens per sequence.  Every kernel reads the number of cached
 // positions from pos_dev, so the same launch sequence serves eager calls and graph replays.
 // max_kv bounds cache_len + new_len for sizing the attention key split.
-int32_t launch_forward(agpu_gpt2 *m, const uint32_t *tokens, int B, int new_len, int max_kv, bool all_rows_logits,
-                       const ArgmaxAdvance *feed = nullptr, bool *fed = nullptr) {
+int32_t agpu_gpt2::launch_forward(const uint32_t *tokens, int B, int new_len, int max_kv, bool all_rows_logits, const ArgmaxAdvance *feed,
+                                  bool *fed) {
+    agpu_gpt2 *m = this;
     if (fed) *fed = false;
     int32_t rc = launch_embed(m, tokens, B, new_len);
     for (int L = 0; rc == AGPU_OK && L < m->cfg.n_layer; ++L) rc = launch_block(m, L, B, new_len, max_kv);
@@ -591,9 +501,10 @@ int32_t launch_forward(agpu_gpt2 *m, const uint32_t *tokens, int B, int new_len,
     return launch_head(m, (float *)m->last.p, B);
 }
 
-int logits_stride(const agpu_gpt2 *m) { return m->cfg.lm_head == AGPU_LM_HEAD_INT4 ? m->Vpad : m->V; }
+int agpu_gpt2::logits_stride() const { return cfg.lm_head == AGPU_LM_HEAD_INT4 ? Vpad : V; }
 
-int32_t ensure_buffers(agpu_gpt2 *m, int B, int new_len, bool all_rows_logits) {
+int32_t agpu_gpt2::ensure_buffers(int B, int new_len, bool all_rows_logits) {
+    agpu_gpt2 *m = this;
     const size_t R = (size_t)B * new_len, d = m->d;
     const size_t Rl = all_rows_logits ? R : (size_t)B;
     int32_t rc;
@@ -603,7 +514,7 @@ int32_t ensure_buffers(agpu_gpt2 *m, int B, int new_len, bool all_rows_logits) {
     if ((rc = ensure(m, m->ffn, R * m->ff * 4)) != AGPU_OK) return rc;
     if ((rc = ensure(m, m->lnb, (R > Rl ? R : Rl) * d * 4)) != AGPU_OK) return rc;
     if ((rc = ensure(m, m->last, (size_t)B * d * 4)) != AGPU_OK) return rc;
-    if ((rc = ensure(m, m->logits, Rl * logits_stride(m) * 4)) != AGPU_OK) return rc;
+    if ((rc = ensure(m, m->logits, Rl * m->logits_stride() * 4)) != AGPU_OK) return rc;
     if (fragments_possible(m, B, new_len)) {
         const size_t bytes = agpu_attention_fragment_bytes(B * m->H, new_len);
         if ((rc = ensure(m, m->kfrag, bytes)) != AGPU_OK) return rc;
@@ -614,7 +525,8 @@ int32_t ensure_buffers(agpu_gpt2 *m, int B, int new_len, bool all_rows_logits) {
     return AGPU_OK;
 }
 
-int32_t check_ready(agpu_gpt2 *m) {
+int32_t agpu_gpt2::check_ready() {
+    agpu_gpt2 *m = this;
     if (!m->wte || !m->wpe || !m->lnf_g || !m->lnf_b) return agpu_fail(m->ctx, AGPU_ERR_NULL_POINTER, "gpt2: embeddings not set");
     for (int L = 0; L < m->cfg.n_layer; ++L) {
         const Block &b = m->blocks[L];
@@ -627,33 +539,7 @@ int32_t check_ready(agpu_gpt2 *m) {
     return AGPU_OK;
 }
 
-int32_t set_counters(agpu_gpt2 *m, int pos, int step) {
-    hipLaunchKernelGGL(set_counters_kernel, dim3(1), dim3(1), 0, m->ctx->stream, m->pos_dev, pos, m->step_dev, step);
-    return AGPU_LAUNCH_CHECK(m->ctx, "set_counters_kernel");
-}
-
-ArgmaxAdvance token_feed(const agpu_gpt2 *m, int B, int delta) {
-    ArgmaxAdvance adv{};
-    adv.cur_tok = m->cur_tok; adv.out_tok = m->out_tok; adv.pos_dev = m->pos_dev; adv.step_dev = m->step_dev;
-    adv.delta = delta; adv.out_capacity = m->out_capacity; adv.bump_counters = (B == 1);
-    return adv;
-}
-
-int32_t launch_argmax_advance(agpu_gpt2 *m, int B, int delta) {
-    const ArgmaxAdvance adv = token_feed(m, B, delta);
-    int32_t rc = agpu_argmax_rows_strided(m->ctx, (float *)m->logits.p, m->next_tok, B, m->V, logits_stride(m),
-                                          m->cfg.argmax_last, &adv);
-    if (rc != AGPU_OK || B == 1) return rc;
-    // several rows: the counters advance once every row has read them
-    hipLaunchKernelGGL(advance_counters_kernel, dim3(1), dim3(1), 0, m->ctx->stream, m->pos_dev, m->step_dev, delta);
-    return AGPU_LAUNCH_CHECK(m->ctx, "advance_counters_kernel");
-}
-
-int kv_bucket(const agpu_gpt2 *m, int kv_len) {
-    int b = 128;
-    while (b < kv_len) b *= 2;
-    return b < m->P ? b : m->P;
-}
+namespace {
 
 // The model as the one-launch decode step sees it (sequence 0 of the cache).
 PkModel pk_view(agpu_gpt2 *m) {
@@ -683,8 +569,11 @@ PkModel pk_view(agpu_gpt2 *m) {
     return v;
 }
 
+}  // namespace
+
 // Whether single-sequence decode steps run as one launch; builds the plan on first use (never inside a capture).
-bool pk_ready(agpu_gpt2 *m) {
+bool agpu_gpt2::one_launch_ready() {
+    agpu_gpt2 *m = this;
     if (m->decode_mode != AGPU_DECODE_AUTO || m->cfg.lm_head != AGPU_LM_HEAD_INT4) return false;
     if (m->pk_failed) {
         // whatever kept the step's workgroups from running together may be gone: another try after a while
@@ -705,126 +594,9 @@ bool pk_ready(agpu_gpt2 *m) {
     return true;
 }
 
-// One decode step as one launch per stage; the LM head picks and feeds the next token itself where it can.
-int32_t launch_step_per_stage(agpu_gpt2 *m, int B, int bucket) {
-    const ArgmaxAdvance feed = token_feed(m, B, 1);
-    bool fed = false;
-    int32_t rc = launch_forward(m, m->cur_tok, B, 1, bucket, false, &feed, &fed);
-    if (rc == AGPU_OK && !fed) rc = launch_argmax_advance(m, B, 1);
-    return rc;
-}
-
-// The captured decode step for (batch, kv bucket); captured on first use.
-// The one-launch step reads the position on the device and does not depend on the bucket: `reps` > 1 captures that many
-// of its launches in a row (one graph launch then costs its overhead once for `reps` tokens).
-int32_t decode_graph(agpu_gpt2 *m, int B, int bucket, hipGraphExec_t *out, int reps = 1) {
-    const long long key = reps > 1 ? ((1ll << 62) | reps) : (((long long)B << 32) | (unsigned)bucket);
-    if (m->ws_epoch != m->ctx->ws_epoch) {  // the scratch moved: captured launches point at the old one
-        drop_graphs(m);
-        m->ws_epoch = m->ctx->ws_epoch;
-    }
-    auto it = m->graphs.find(key);
-    if (it != m->graphs.end()) {
-        if (m->graph_addr[key] == step_addresses(m, reps > 1 || (B == 1 && m->pk.stages_dev != nullptr))) {
-            *out = it->second;
-            return AGPU_OK;
-        }
-        // an address changed under a cached graph: never replay it; every graph goes and this one is captured anew
-        drop_graphs(m);
-    }
-    agpu_ctx *ctx = m->ctx;
-    if (ctx->stream == nullptr)
-        return agpu_fail(ctx, AGPU_ERR_UNSUPPORTED, "gpt2: graph capture needs a context with its own stream (agpu_ctx_create)");
-    const bool one_launch = B == 1 && pk_ready(m);  // builds the plan: before the capture begins
-    hipError_t e = hipStreamBeginCapture(ctx->stream, hipStreamCaptureModeThreadLocal);
-    if (e != hipSuccess) return agpu_hip(ctx, e, "hipStreamBeginCapture");
-    int32_t rc;
-    if (one_launch) {
-        // one sequence: the whole step, arg-max and token feed included, is one launch
-        const PkModel view = pk_view(m);
-        rc = AGPU_OK;
-        for (int r = 0; r < reps && rc == AGPU_OK; ++r) rc = agpu_step_launch(ctx, view, m->pk, 0);
-    } else if (reps > 1) {
-        rc = agpu_fail(ctx, AGPU_ERR_UNSUPPORTED, "gpt2: several steps per graph need the one-launch step");
-    } else {
-        rc = launch_step_per_stage(m, B, bucket);
-    }
-    hipGraph_t graph = nullptr;
-    e = hipStreamEndCapture(ctx->stream, &graph);
-    if (rc != AGPU_OK) {
-        if (graph) (void)hipGraphDestroy(graph);
-        return rc;
-    }
-    if (e != hipSuccess) return agpu_hip(ctx, e, "hipStreamEndCapture");
-    hipGraphExec_t exec = nullptr;
-    e = hipGraphInstantiate(&exec, graph, nullptr, nullptr, 0);
-    (void)hipGraphDestroy(graph);
-    if (e != hipSuccess) return agpu_hip(ctx, e, "hipGraphInstantiate");
-    m->graphs[key] = exec;
-    m->graph_addr[key] = step_addresses(m, one_launch);
-    *out = exec;
-    return AGPU_OK;
-}
-
-int32_t ensure_out_tokens(agpu_gpt2 *m, int steps, int B) {
-    if (m->out_capacity >= steps && m->out_tok) return AGPU_OK;
-    (void)hipStreamSynchronize(m->ctx->stream);
-    drop_graphs(m);
-    if (m->out_tok) (void)hipFree(m->out_tok);
-    m->out_tok = nullptr;
-    const int cap = steps > m->P ? steps : m->P;
-    int32_t rc = dev_alloc(m->ctx, (void **)&m->out_tok, (size_t)cap * m->cfg.max_batch * sizeof(uint32_t));
-    if (rc != AGPU_OK) return rc;
-    m->out_capacity = cap;
-    (void)B;
-    return AGPU_OK;
-}
-
-// Replays `steps` decode steps; the host only tracks the position to pick the graph.
-int32_t run_decode_steps(agpu_gpt2 *m, int B, int steps) {
-    constexpr int kStepsPerGraph = 16;  // agpu_gpt2_decode_steps captures the same number ahead of its timed region
-    // the batched decode on pieces wants its buffers and folded LayerNorm vectors before a step is launched or captured
-    if (px_shape_ok(m, B, 1)) {
-        const int32_t rc = px_prepare(m);
-        if (rc != AGPU_OK) return rc;
-    }
-    int s = 0;
-    if (B == 1 && steps >= 2 && pk_ready(m)) {
-        // graphs of sixteen launches, then one graph of what is left (a graph launch costs 5.5 us, a node inside one 1.5)
-        while (s < steps) {
-            const int n = std::min(kStepsPerGraph, steps - s);
-            if (n < 2) break;
-            hipGraphExec_t exec;
-            const int32_t rc = decode_graph(m, 1, 0, &exec, n);
-            if (rc != AGPU_OK) return rc;
-            const hipError_t e = hipGraphLaunch(exec, m->ctx->stream);
-            if (e != hipSuccess) return agpu_hip(m->ctx, e, "hipGraphLaunch");
-            m->cache_len += n;
-            m->n_one_launch += n;
-            s += n;
-        }
-    }
-    for (; s < steps; ++s) {
-        const int bucket = kv_bucket(m, m->cache_len + 1);
-        if (B == 1 && pk_ready(m)) ++m->n_one_launch;
-        else ++m->n_per_stage;
-        if (m->decode_mode == AGPU_DECODE_EAGER) {
-            const int32_t rc = launch_step_per_stage(m, B, bucket);
-            if (rc != AGPU_OK) return rc;
-        } else {
-            hipGraphExec_t exec;
-            const int32_t rc = decode_graph(m, B, bucket, &exec);
-            if (rc != AGPU_OK) return rc;
-            const hipError_t e = hipGraphLaunch(exec, m->ctx->stream);
-            if (e != hipSuccess) return agpu_hip(m->ctx, e, "hipGraphLaunch");
-        }
-        m->cache_len += 1;
-    }
-    return AGPU_OK;
-}
-
 // After a synchronisation: whether a wait inside a one-launch decode step gave up since the last check.
-int32_t pk_check(agpu_gpt2 *m) {
+int32_t agpu_gpt2::check_waits() {
+    agpu_gpt2 *m = this;
     if (!m->pk.stages_dev) return AGPU_OK;
     unsigned int err = 0u;
     int32_t rc = agpu_step_take_error(m->ctx, m->pk, &err);
@@ -845,6 +617,35 @@ int32_t pk_check(agpu_gpt2 *m) {
     return AGPU_OK;
 }
 
+int32_t agpu_gpt2::launch_one_step() { return agpu_step_launch(ctx, pk_view(this), pk, 0); }
+
+int32_t agpu_gpt2::prepare_steps(int B) { return px_shape_ok(this, B, 1) ? px_prepare(this) : AGPU_OK; }
+
+// The plan of the one-launch step holds the same addresses as the graphs.
+void agpu_gpt2::graphs_dropped() {
+    agpu_step_plan_free(&pk);
+    pk_tried = false;
+}
+
+void agpu_gpt2::mix_addresses(AddrHash &h, bool one_launch) const {
+    for (const void *p : {(const void *)wte, (const void *)wpe, (const void *)lnf_g, (const void *)lnf_b, (const void *)wte_t,
+                          (const void *)kcache, (const void *)vcache, (const void *)lm_head.packed, (const void *)lm_head.scales})
+        h.mix(p);
+    if (one_launch)  // the step's plan; a graph of per-stage launches does not refer to it
+        for (const void *p : {(const void *)pk.arena, (const void *)pk.xmem, (const void *)pk.stages_dev, (const void *)pk.state, (const void *)pk.ln_fold}) h.mix(p);
+    for (const DevBuf *b : {&hid, &qkv, &att, &ffn, &lnb, &last, &px_h, &px_att, &px_ffn, &px_stats, &px_fold}) h.mix(b->p);
+    for (const Block &b : blocks) {
+        for (const void *p : {(const void *)b.ln1_g, (const void *)b.ln1_b, (const void *)b.ln2_g, (const void *)b.ln2_b}) h.mix(p);
+        for (const Int4Lin &l : b.lin) {
+            h.mix(l.packed);
+            h.mix(l.scales);
+            h.mix(l.bias);
+        }
+    }
+}
+
+namespace {
+
 int32_t ensure_probes(agpu_gpt2 *m) {
     if (m->probe_conf_host) return AGPU_OK;
     agpu_ctx *ctx = m->ctx;
@@ -863,7 +664,7 @@ int32_t ensure_probes(agpu_gpt2 *m) {
 
 // Confidence and arg-max of logits row 0 into probe slot L, then the slot's event.
 int32_t launch_probe(agpu_gpt2 *m, int L) {
-    int32_t rc = agpu_argmax_rows_strided(m->ctx, (float *)m->logits.p, m->probe_tok_dev + L, 1, m->V, logits_stride(m),
+    int32_t rc = agpu_argmax_rows_strided(m->ctx, (float *)m->logits.p, m->probe_tok_dev + L, 1, m->V, m->logits_stride(),
                                           m->cfg.argmax_last, nullptr, m->probe_conf_dev + L);
     if (rc != AGPU_OK) return rc;
     return agpu_hip(m->ctx, hipEventRecord(m->probe_ev[L], m->ctx->stream), "hipEventRecord");
@@ -950,29 +751,16 @@ AGPU_EXPORT int32_t agpu_gpt2_create(agpu_ctx *ctx, const agpu_gpt2_config *cfg,
     agpu_gpt2 *m = new (std::nothrow) agpu_gpt2();
     if (m) m->px_off = getenv("AGPU_NO_PX") != nullptr;
     if (!m) return AGPU_ERR_NULL_POINTER;
-    m->ctx = ctx;
-    ctx->refs.fetch_add(1);
     m->cfg = *cfg;
     m->d = cfg->n_embd;
     m->H = cfg->n_head;
     m->ff = 4 * cfg->n_embd;  // Gpt2Config::ffn_dim, gpt2.rs:90-92
-    m->V = cfg->vocab_size;
-    m->P = cfg->n_positions;
-    m->Vpad = ceil_div(m->V, 256) * 256;
+    m->Vpad = ceil_div(cfg->vocab_size, 256) * 256;
     m->blocks.resize(cfg->n_layer);
+    int32_t rc = lm_init(m, ctx, cfg->vocab_size, cfg->n_positions, cfg->max_batch, cfg->argmax_last);
     const size_t cache_elems = (size_t)cfg->n_layer * cfg->max_batch * m->H * m->P * DH;
-    int32_t rc = dev_alloc(ctx, (void **)&m->kcache, cache_elems * 4);
+    if (rc == AGPU_OK) rc = dev_alloc(ctx, (void **)&m->kcache, cache_elems * 4);
     if (rc == AGPU_OK) rc = dev_alloc(ctx, (void **)&m->vcache, cache_elems * 4);
-    if (rc == AGPU_OK) rc = dev_alloc(ctx, (void **)&m->cur_tok, (size_t)cfg->max_batch * 4);
-    if (rc == AGPU_OK) rc = dev_alloc(ctx, (void **)&m->next_tok, (size_t)cfg->max_batch * 4);
-    if (rc == AGPU_OK) rc = dev_alloc(ctx, (void **)&m->pos_dev, 2 * sizeof(int));
-    if (rc == AGPU_OK) {
-        m->step_dev = m->pos_dev + 1;
-        rc = agpu_hip(ctx, hipMemset(m->pos_dev, 0, 2 * sizeof(int)), "hipMemset");
-    }
-    if (rc == AGPU_OK) rc = agpu_hip(ctx, hipEventCreate(&m->ev0), "hipEventCreate");
-    if (rc == AGPU_OK) rc = agpu_hip(ctx, hipEventCreate(&m->ev1), "hipEventCreate");
-    if (rc == AGPU_OK) rc = agpu_hip(ctx, hipEventCreate(&m->ev2), "hipEventCreate");
     if (rc != AGPU_OK) {
         agpu_gpt2_destroy(m);
         return rc;
@@ -992,17 +780,15 @@ AGPU_EXPORT int32_t agpu_gpt2_destroy(agpu_gpt2 *m) {
     }
     free_lin(m->lm_head);
     for (void *p : {(void *)m->wte, (void *)m->wpe, (void *)m->lnf_g, (void *)m->lnf_b, (void *)m->wte_t, (void *)m->kcache,
-                    (void *)m->vcache, (void *)m->cur_tok, (void *)m->next_tok, (void *)m->out_tok, (void *)m->pos_dev,
-                    m->hid.p, m->qkv.p, m->att.p, m->ffn.p, m->lnb.p, m->last.p, m->logits.p, m->tok_in.p, m->kfrag.p, m->vfrag.p,
+                    (void *)m->vcache,
+                    m->hid.p, m->qkv.p, m->att.p, m->ffn.p, m->lnb.p, m->last.p, m->kfrag.p, m->vfrag.p,
                     m->px_h.p, m->px_att.p, m->px_ffn.p, m->px_stats.p, m->px_fold.p})
         if (p) (void)hipFree(p);
-    for (hipEvent_t e : {m->ev0, m->ev1, m->ev2})
-        if (e) (void)hipEventDestroy(e);
     for (hipEvent_t e : m->probe_ev)
         if (e) (void)hipEventDestroy(e);
     if (m->probe_conf_host) (void)hipHostFree(m->probe_conf_host);
     if (m->probe_tok_host) (void)hipHostFree(m->probe_tok_host);
-    agpu_ctx_release(m->ctx);
+    lm_release(m);
     delete m;
     return AGPU_OK;
 }
@@ -1113,18 +899,12 @@ AGPU_EXPORT int64_t agpu_gpt2_quantized_memory_bytes(const agpu_gpt2 *m) {
 
 AGPU_EXPORT int32_t agpu_gpt2_set_decode_mode(agpu_gpt2 *m, int32_t mode) {
     if (!m) return AGPU_ERR_NULL_POINTER;
-    if (mode != AGPU_DECODE_AUTO && mode != AGPU_DECODE_PER_STAGE && mode != AGPU_DECODE_EAGER)
-        return agpu_fail(m->ctx, AGPU_ERR_DIM_OUT_OF_RANGE, "gpt2_set_decode_mode: unknown mode %d", mode);
-    if (mode != m->decode_mode) {
-        (void)hipStreamSynchronize(m->ctx->stream);
-        drop_graphs(m);
-        m->decode_mode = mode;
-    }
-    if (mode == AGPU_DECODE_AUTO) {  // asked for again: the one-launch step gets another try
+    const int32_t rc = lm_set_decode_mode(m, mode);
+    if (rc == AGPU_OK && mode == AGPU_DECODE_AUTO) {  // asked for again: the one-launch step gets another try
         m->pk_failed = false;
         m->pk_failed_looks = 0;
     }
-    return AGPU_OK;
+    return rc;
 }
 
 AGPU_EXPORT int32_t agpu_gpt2_decode_stats(agpu_gpt2 *m, int64_t *stats_out_host) {
@@ -1153,46 +933,10 @@ AGPU_EXPORT int32_t agpu_gpt2_set_decode_wait_limit(agpu_gpt2 *m, int32_t poll_r
 }
 
 AGPU_EXPORT int32_t agpu_gpt2_reset_cache(agpu_gpt2 *m) {
-    if (!m) return AGPU_ERR_NULL_POINTER;
-    m->cache_len = 0;
-    return set_counters(m, 0, 0);
+    return m ? lm_reset_cache(m) : AGPU_ERR_NULL_POINTER;
 }
 
 AGPU_EXPORT int32_t agpu_gpt2_cache_len(const agpu_gpt2 *m) { return m ? m->cache_len : 0; }
-
-AGPU_EXPORT int32_t agpu_gpt2_forward_cached(agpu_gpt2 *m, const uint32_t *tokens, int32_t batch, int32_t new_len,
-                                             float *logits, int32_t all_rows) {
-    if (!m) return AGPU_ERR_NULL_POINTER;
-    agpu_ctx *ctx = m->ctx;
-    AGPU_REQUIRE_CTX(ctx);
-    if (!tokens) return agpu_fail(ctx, AGPU_ERR_NULL_POINTER, "gpt2_forward_cached: null tokens");
-    if (batch <= 0 || batch > m->cfg.max_batch)
-        return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "gpt2_forward_cached: batch %d not in 1..%d", batch, m->cfg.max_batch);
-    if (new_len <= 0) return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "gpt2_forward_cached: new_len must be positive");
-    if (m->cache_len + new_len > m->P)
-        return agpu_fail(ctx, AGPU_ERR_DIM_OUT_OF_RANGE, "gpt2_forward_cached: %d cached + %d new positions exceed n_positions %d",
-                         m->cache_len, new_len, m->P);
-    int32_t rc = check_ready(m);
-    if (rc != AGPU_OK) return rc;
-    if ((rc = ensure_buffers(m, batch, new_len, all_rows != 0)) != AGPU_OK) return rc;
-    if ((rc = ensure_out_tokens(m, m->P, batch)) != AGPU_OK) return rc;
-    if ((rc = set_counters(m, m->cache_len, -1)) != AGPU_OK) return rc;
-    if ((rc = launch_forward(m, tokens, batch, new_len, m->cache_len + new_len, all_rows != 0)) != AGPU_OK) return rc;
-    // keep the device-side generation state usable: next token = arg-max of the last rows
-    if (!all_rows) {
-        if ((rc = launch_argmax_advance(m, batch, new_len)) != AGPU_OK) return rc;
-    } else {
-        if ((rc = set_counters(m, m->cache_len + new_len, -1)) != AGPU_OK) return rc;
-    }
-    m->cache_len += new_len;
-    if (logits) {
-        const size_t rows = all_rows ? (size_t)batch * new_len : (size_t)batch;
-        hipError_t e = hipMemcpy2DAsync(logits, (size_t)m->V * 4, m->logits.p, (size_t)logits_stride(m) * 4, (size_t)m->V * 4,
-                                        rows, hipMemcpyDeviceToDevice, ctx->stream);
-        if (e != hipSuccess) return agpu_hip(ctx, e, "hipMemcpy2DAsync(logits)");
-    }
-    return AGPU_OK;
-}
 
 namespace {
 
@@ -1205,10 +949,10 @@ int32_t forward_staged(agpu_gpt2 *m, const uint32_t *tokens, int seq_len, float 
     if (seq_len <= 0 || seq_len > m->P) return agpu_fail(ctx, AGPU_ERR_DIM_OUT_OF_RANGE, "%s: seq_len %d not in 1..%d", who, seq_len, m->P);
     const int n_rep = m->cfg.n_layer + 3;
     if (capacity < n_rep) return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "%s: %d reports do not fit %d entries", who, n_rep, capacity);
-    int32_t rc = check_ready(m);
+    int32_t rc = m->check_ready();
     if (rc != AGPU_OK) return rc;
-    if ((rc = ensure_buffers(m, 1, seq_len, false)) != AGPU_OK) return rc;
-    if ((rc = ensure_out_tokens(m, m->P, 1)) != AGPU_OK) return rc;
+    if ((rc = m->ensure_buffers(1, seq_len, false)) != AGPU_OK) return rc;
+    if ((rc = ensure_out_tokens(m, m->P)) != AGPU_OK) return rc;
     m->cache_len = 0;
     if ((rc = set_counters(m, 0, -1)) != AGPU_OK) return rc;
     const int d = m->d;
@@ -1307,34 +1051,6 @@ AGPU_EXPORT int32_t agpu_gpt2_forward_diagnostic(agpu_gpt2 *m, const uint32_t *t
                           top5_logits_out_host, "gpt2_forward_diagnostic");
 }
 
-AGPU_EXPORT int32_t agpu_gpt2_decode_steps(agpu_gpt2 *m, int32_t batch, int32_t steps, float *ms_total_out_host) {
-    if (!m) return AGPU_ERR_NULL_POINTER;
-    agpu_ctx *ctx = m->ctx;
-    AGPU_REQUIRE_CTX(ctx);
-    if (batch <= 0 || batch > m->cfg.max_batch || steps < 0)
-        return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "gpt2_decode_steps: bad batch/steps");
-    if (m->cache_len == 0) return agpu_fail(ctx, AGPU_ERR_UNSUPPORTED, "gpt2_decode_steps: run a prefill first");
-    if (m->cache_len + steps > m->P)
-        return agpu_fail(ctx, AGPU_ERR_DIM_OUT_OF_RANGE, "gpt2_decode_steps: %d cached + %d steps exceed n_positions %d",
-                         m->cache_len, steps, m->P);
-    int32_t rc = ensure_buffers(m, batch, 1, false);
-    if (rc != AGPU_OK) return rc;
-    // capture outside the timed region
-    hipGraphExec_t exec;
-    if (batch == 1 && steps >= 2 && pk_ready(m)) {
-        if (steps >= 16 && (rc = decode_graph(m, 1, 0, &exec, 16)) != AGPU_OK) return rc;
-        if (steps % 16 >= 2 && (rc = decode_graph(m, 1, 0, &exec, steps % 16)) != AGPU_OK) return rc;
-    }
-    for (int s = 0; s < steps && m->decode_mode != AGPU_DECODE_EAGER; ++s)
-        if ((rc = decode_graph(m, batch, kv_bucket(m, m->cache_len + 1 + s), &exec)) != AGPU_OK) return rc;
-    if ((rc = agpu_hip(ctx, hipEventRecord(m->ev0, ctx->stream), "hipEventRecord")) != AGPU_OK) return rc;
-    if ((rc = run_decode_steps(m, batch, steps)) != AGPU_OK) return rc;
-    if ((rc = agpu_hip(ctx, hipEventRecord(m->ev1, ctx->stream), "hipEventRecord")) != AGPU_OK) return rc;
-    if ((rc = agpu_hip(ctx, hipEventSynchronize(m->ev1), "hipEventSynchronize")) != AGPU_OK) return rc;
-    if (ms_total_out_host) (void)hipEventElapsedTime(ms_total_out_host, m->ev0, m->ev1);
-    return pk_check(m);
-}
-
 #ifdef AGPU_PK_TRACE
 // Debug builds only: the one-launch step's mirrors (device pointer, floats of one mirror) and the floats of one set of partial sums.
 AGPU_EXPORT int32_t agpu_gpt2_debug_arena(agpu_gpt2 *m, void **arena_out, unsigned long long *mirror_elems, unsigned long long *parts_elems) {
@@ -1346,7 +1062,7 @@ AGPU_EXPORT int32_t agpu_gpt2_debug_arena(agpu_gpt2 *m, void **arena_out, unsign
 }
 // Debug builds only: one step of the one-launch decode with time stamps, [grid][n_stages][4] ticks of 10 ns.
 AGPU_EXPORT int32_t agpu_gpt2_decode_trace(agpu_gpt2 *m, int32_t mode, unsigned long long *out_host, int32_t *grid_out, int32_t *stages_out) {
-    if (!pk_ready(m)) return AGPU_ERR_UNSUPPORTED;
+    if (!m->one_launch_ready()) return AGPU_ERR_UNSUPPORTED;
     const size_t n = (size_t)m->pk.grid * m->pk.n_stages * 8;
     unsigned long long *dev = nullptr;
     if (hipMalloc((void **)&dev, n * 8) != hipSuccess) return AGPU_ERR_WORKSPACE;
@@ -1362,29 +1078,15 @@ AGPU_EXPORT int32_t agpu_gpt2_decode_trace(agpu_gpt2 *m, int32_t mode, unsigned 
 }
 #endif
 
-AGPU_EXPORT int32_t agpu_gpt2_last_logits(agpu_gpt2 *m, int32_t batch, float *logits_out_host) {
-    if (!m) return AGPU_ERR_NULL_POINTER;
-    agpu_ctx *ctx = m->ctx;
-    if (!logits_out_host) return agpu_fail(ctx, AGPU_ERR_NULL_POINTER, "gpt2_last_logits: null pointer");
-    if (batch <= 0 || batch > m->cfg.max_batch) return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "gpt2_last_logits: bad batch");
-    const size_t stride = logits_stride(m);
-    if (!m->logits.p || m->logits.bytes < (size_t)batch * stride * 4)
-        return agpu_fail(ctx, AGPU_ERR_UNSUPPORTED, "gpt2_last_logits: no forward has run for this batch");
-    hipError_t e = hipMemcpy2DAsync(logits_out_host, (size_t)m->V * 4, m->logits.p, stride * 4, (size_t)m->V * 4, (size_t)batch,
-                                    hipMemcpyDeviceToHost, ctx->stream);
-    if (e == hipSuccess) e = hipStreamSynchronize(ctx->stream);
-    return agpu_hip(ctx, e, "gpt2_last_logits");
-}
-
 AGPU_EXPORT int32_t agpu_gpt2_decode_floor(agpu_gpt2 *m, int32_t steps, float *ms_total_out_host) {
     if (!m) return AGPU_ERR_NULL_POINTER;
     agpu_ctx *ctx = m->ctx;
     if (steps < 0) return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "gpt2_decode_floor: bad steps");
-    int32_t rc = check_ready(m);
+    int32_t rc = m->check_ready();
     if (rc != AGPU_OK) return rc;
-    if ((rc = ensure_buffers(m, 1, 1, false)) != AGPU_OK) return rc;
-    if ((rc = ensure_out_tokens(m, 1, 1)) != AGPU_OK) return rc;
-    if (!pk_ready(m)) return agpu_fail(ctx, AGPU_ERR_UNSUPPORTED, "gpt2_decode_floor: this model does not take the one-launch decode step");
+    if ((rc = m->ensure_buffers(1, 1, false)) != AGPU_OK) return rc;
+    if ((rc = ensure_out_tokens(m, 1)) != AGPU_OK) return rc;
+    if (!m->one_launch_ready()) return agpu_fail(ctx, AGPU_ERR_UNSUPPORTED, "gpt2_decode_floor: this model does not take the one-launch decode step");
     const PkModel v = pk_view(m);
     if ((rc = agpu_hip(ctx, hipEventRecord(m->ev0, ctx->stream), "hipEventRecord")) != AGPU_OK) return rc;
     for (int s = 0; s < steps; ++s)
@@ -1392,127 +1094,7 @@ AGPU_EXPORT int32_t agpu_gpt2_decode_floor(agpu_gpt2 *m, int32_t steps, float *m
     if ((rc = agpu_hip(ctx, hipEventRecord(m->ev1, ctx->stream), "hipEventRecord")) != AGPU_OK) return rc;
     if ((rc = agpu_hip(ctx, hipEventSynchronize(m->ev1), "hipEventSynchronize")) != AGPU_OK) return rc;
     if (ms_total_out_host) (void)hipEventElapsedTime(ms_total_out_host, m->ev0, m->ev1);
-    return pk_check(m);
-}
-
-AGPU_EXPORT int32_t agpu_gpt2_generate_cached(agpu_gpt2 *m, const uint32_t *prompt_host, int32_t batch, int32_t prompt_len,
-                                              int32_t max_new_tokens, int32_t eos, uint32_t *tokens_out_host,
-                                              int32_t *lengths_out_host, float *timing_ms_out_host) {
-    if (!m) return AGPU_ERR_NULL_POINTER;
-    agpu_ctx *ctx = m->ctx;
-    AGPU_REQUIRE_CTX(ctx);
-    if (!prompt_host || !tokens_out_host || !lengths_out_host)
-        return agpu_fail(ctx, AGPU_ERR_NULL_POINTER, "gpt2_generate_cached: null pointer");
-    if (batch <= 0 || batch > m->cfg.max_batch || prompt_len <= 0 || max_new_tokens < 0)
-        return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "gpt2_generate_cached: bad batch/prompt_len/max_new_tokens");
-    // the last generated token is never fed back, so prompt_len + max_new_tokens - 1 positions are cached
-    if (prompt_len + (max_new_tokens > 0 ? max_new_tokens - 1 : 0) > m->P)
-        return agpu_fail(ctx, AGPU_ERR_DIM_OUT_OF_RANGE, "gpt2_generate_cached: prompt %d + %d new tokens exceed n_positions %d",
-                         prompt_len, max_new_tokens, m->P);
-    int32_t rc = check_token_ids(m, prompt_host, (size_t)batch * prompt_len, "gpt2_generate_cached");
-    if (rc != AGPU_OK) return rc;
-    const int total = prompt_len + max_new_tokens;
-    for (int b = 0; b < batch; ++b) {
-        std::memcpy(tokens_out_host + (size_t)b * total, prompt_host + (size_t)b * prompt_len, (size_t)prompt_len * 4);
-        lengths_out_host[b] = prompt_len;
-    }
-    if (max_new_tokens == 0) return AGPU_OK;
-    if ((rc = check_ready(m)) != AGPU_OK) return rc;
-    if ((rc = ensure(m, m->tok_in, (size_t)batch * prompt_len * 4)) != AGPU_OK) return rc;
-    if ((rc = ensure_buffers(m, batch, prompt_len, false)) != AGPU_OK) return rc;
-    if ((rc = ensure_out_tokens(m, max_new_tokens, batch)) != AGPU_OK) return rc;
-    if ((rc = upload(ctx, m->tok_in.p, prompt_host, (size_t)batch * prompt_len * 4, 0)) != AGPU_OK) return rc;
-    if ((rc = agpu_gpt2_reset_cache(m)) != AGPU_OK) return rc;
-
-    (void)hipEventRecord(m->ev0, ctx->stream);
-    if ((rc = agpu_gpt2_forward_cached(m, (const uint32_t *)m->tok_in.p, batch, prompt_len, nullptr, 0)) != AGPU_OK) return rc;
-    (void)hipEventRecord(m->ev1, ctx->stream);
-    if ((rc = run_decode_steps(m, batch, max_new_tokens - 1)) != AGPU_OK) return rc;
-    (void)hipEventRecord(m->ev2, ctx->stream);
-
-    std::vector<uint32_t> gen((size_t)max_new_tokens * batch);
-    rc = agpu_memcpy_d2h(ctx, gen.data(), m->out_tok, gen.size() * 4);
-    if (rc != AGPU_OK) return rc;
-    if ((rc = pk_check(m)) != AGPU_OK) return rc;
-    if (timing_ms_out_host) {
-        (void)hipEventElapsedTime(&timing_ms_out_host[0], m->ev0, m->ev1);
-        (void)hipEventElapsedTime(&timing_ms_out_host[1], m->ev1, m->ev2);
-    }
-    for (int b = 0; b < batch; ++b) {
-        int len = prompt_len;
-        for (int s = 0; s < max_new_tokens; ++s) {
-            const uint32_t t = gen[(size_t)s * batch + b];
-            if (eos >= 0 && t == (uint32_t)eos) break;  // stop before appending (gpt2.rs:762,776)
-            tokens_out_host[(size_t)b * total + len++] = t;
-        }
-        lengths_out_host[b] = len;
-    }
-    return AGPU_OK;
-}
-
-// sampling.hip
-int32_t agpu_top_k_launch(agpu_ctx *ctx, const float *logits, int rows, int n, int stride, int k, float temperature,
-                          uint32_t *idx_out, float *val_out);
-extern "C" uint32_t agpu_top_k_draw_host(const float *ranked_vals, const uint32_t *ranked_idx, int32_t k, float r);
-extern "C" float agpu_simple_rng_next_f32(uint64_t *state);
-
-AGPU_EXPORT int32_t agpu_gpt2_generate_cached_sampling(agpu_gpt2 *m, const uint32_t *prompt_host, int32_t prompt_len,
-                                                       int32_t max_new_tokens, int32_t top_k, float temperature,
-                                                       uint64_t *rng_state, int32_t eos, uint32_t *tokens_out_host,
-                                                       int32_t *length_out_host) {
-    if (!m) return AGPU_ERR_NULL_POINTER;
-    agpu_ctx *ctx = m->ctx;
-    AGPU_REQUIRE_CTX(ctx);
-    if (!prompt_host || !tokens_out_host || !length_out_host || !rng_state)
-        return agpu_fail(ctx, AGPU_ERR_NULL_POINTER, "gpt2_generate_cached_sampling: null pointer");
-    if (prompt_len <= 0 || max_new_tokens < 0 || top_k <= 0)
-        return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "gpt2_generate_cached_sampling: bad prompt_len/max_new_tokens/top_k");
-    if (prompt_len + (max_new_tokens > 0 ? max_new_tokens - 1 : 0) > m->P)
-        return agpu_fail(ctx, AGPU_ERR_DIM_OUT_OF_RANGE,
-                         "gpt2_generate_cached_sampling: prompt %d + %d new tokens exceed n_positions %d", prompt_len,
-                         max_new_tokens, m->P);
-    int32_t rc = check_token_ids(m, prompt_host, (size_t)prompt_len, "gpt2_generate_cached_sampling");
-    if (rc != AGPU_OK) return rc;
-    std::memcpy(tokens_out_host, prompt_host, (size_t)prompt_len * 4);
-    int len = prompt_len;
-    *length_out_host = len;
-    if (max_new_tokens == 0) return AGPU_OK;
-    if ((rc = check_ready(m)) != AGPU_OK) return rc;
-    const int k = top_k < m->V ? top_k : m->V;
-    if (k > 1024) return agpu_fail(ctx, AGPU_ERR_UNSUPPORTED, "gpt2_generate_cached_sampling: top_k = %d exceeds 1024", top_k);
-    uint32_t *idx_dev = nullptr;
-    float *val_dev = nullptr;
-    if ((rc = dev_alloc(ctx, (void **)&idx_dev, (size_t)k * 4)) != AGPU_OK) return rc;
-    if ((rc = dev_alloc(ctx, (void **)&val_dev, (size_t)k * 4)) != AGPU_OK) {
-        (void)hipFree(idx_dev);
-        return rc;
-    }
-    std::vector<uint32_t> idx((size_t)k);
-    std::vector<float> val((size_t)k);
-    if ((rc = ensure(m, m->tok_in, (size_t)prompt_len * 4)) == AGPU_OK) rc = ensure_buffers(m, 1, prompt_len, false);
-    if (rc == AGPU_OK) rc = ensure_out_tokens(m, max_new_tokens, 1);
-    if (rc == AGPU_OK) rc = upload(ctx, m->tok_in.p, prompt_host, (size_t)prompt_len * 4, 0);
-    if (rc == AGPU_OK) rc = agpu_gpt2_reset_cache(m);
-    for (int step = 0; rc == AGPU_OK && step < max_new_tokens; ++step) {
-        // logits of the last position: the prefill first, then one replayed decode step per token.  The
-        // replayed graph also runs the arg-max feed; its token is overwritten by the sampled one below.
-        if (step == 0) rc = agpu_gpt2_forward_cached(m, (const uint32_t *)m->tok_in.p, 1, prompt_len, nullptr, 0);
-        else rc = run_decode_steps(m, 1, 1);
-        if (rc != AGPU_OK) break;
-        rc = agpu_top_k_launch(ctx, (const float *)m->logits.p, 1, m->V, logits_stride(m), k, temperature, idx_dev, val_dev);
-        if (rc == AGPU_OK) rc = agpu_memcpy_d2h(ctx, idx.data(), idx_dev, (size_t)k * 4);
-        if (rc == AGPU_OK) rc = agpu_memcpy_d2h(ctx, val.data(), val_dev, (size_t)k * 4);
-        if (rc != AGPU_OK) break;
-        const uint32_t next = agpu_top_k_draw_host(val.data(), idx.data(), k, agpu_simple_rng_next_f32(rng_state));
-        if (eos >= 0 && next == (uint32_t)eos) break;  // gpt2.rs:956-958, 970-972
-        tokens_out_host[len++] = next;
-        if (step + 1 < max_new_tokens) rc = upload(ctx, m->cur_tok, &next, 4, 0);
-    }
-    (void)hipFree(idx_dev);
-    (void)hipFree(val_dev);
-    *length_out_host = len;
-    if (rc == AGPU_OK) rc = pk_check(m);
-    return rc;
+    return m->check_waits();
 }
 
 AGPU_EXPORT int32_t agpu_gpt2_forward_early_exit(agpu_gpt2 *m, const uint32_t *tokens, int32_t seq_len, float threshold,
@@ -1524,9 +1106,9 @@ AGPU_EXPORT int32_t agpu_gpt2_forward_early_exit(agpu_gpt2 *m, const uint32_t *t
     if (seq_len <= 0) return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "gpt2_forward_early_exit: seq_len must be positive");
     if (seq_len > m->P)
         return agpu_fail(ctx, AGPU_ERR_DIM_OUT_OF_RANGE, "gpt2_forward_early_exit: %d tokens exceed n_positions %d", seq_len, m->P);
-    int32_t rc = check_ready(m);
+    int32_t rc = m->check_ready();
     if (rc == AGPU_OK) rc = ensure_probes(m);
-    if (rc == AGPU_OK) rc = ensure_buffers(m, 1, seq_len, true);
+    if (rc == AGPU_OK) rc = m->ensure_buffers(1, seq_len, true);
     if (rc == AGPU_OK) rc = agpu_gpt2_reset_cache(m);
     if (rc == AGPU_OK) rc = launch_embed(m, tokens, 1, seq_len);
     const int nl = m->cfg.n_layer;
@@ -1551,7 +1133,7 @@ AGPU_EXPORT int32_t agpu_gpt2_forward_early_exit(agpu_gpt2 *m, const uint32_t *t
     *layers_used_out_host = used;
     if (logits_out) {
         if ((rc = launch_head(m, (float *)m->hid.p, seq_len)) != AGPU_OK) return rc;
-        hipError_t e = hipMemcpy2DAsync(logits_out, (size_t)m->V * 4, m->logits.p, (size_t)logits_stride(m) * 4, (size_t)m->V * 4,
+        hipError_t e = hipMemcpy2DAsync(logits_out, (size_t)m->V * 4, m->logits.p, (size_t)m->logits_stride() * 4, (size_t)m->V * 4,
                                         (size_t)seq_len, hipMemcpyDeviceToDevice, ctx->stream);
         if (e != hipSuccess) return agpu_hip(ctx, e, "hipMemcpy2DAsync(logits)");
     }
@@ -1579,11 +1161,11 @@ AGPU_EXPORT int32_t agpu_gpt2_generate_cached_early_exit(agpu_gpt2 *m, const uin
     int len = prompt_len, steps = 0;
     *length_out_host = len;
     *steps_out_host = 0;
-    rc = check_ready(m);
+    rc = m->check_ready();
     if (rc == AGPU_OK) rc = ensure_probes(m);
     if (rc == AGPU_OK) rc = ensure(m, m->tok_in, (size_t)prompt_len * 4);
-    if (rc == AGPU_OK) rc = ensure_buffers(m, 1, prompt_len, false);
-    if (rc == AGPU_OK) rc = ensure_out_tokens(m, m->P, 1);
+    if (rc == AGPU_OK) rc = m->ensure_buffers(1, prompt_len, false);
+    if (rc == AGPU_OK) rc = ensure_out_tokens(m, m->P);
     if (rc == AGPU_OK) rc = upload(ctx, m->tok_in.p, prompt_host, (size_t)prompt_len * 4, 0);
     if (rc == AGPU_OK) rc = agpu_gpt2_reset_cache(m);
     // prefill: every layer (gpt2.rs:849-857); its arg-max is already the current token on the device
@@ -1607,34 +1189,37 @@ AGPU_EXPORT int32_t agpu_gpt2_generate_cached_early_exit(agpu_gpt2 *m, const uin
     return rc;
 }
 
-AGPU_EXPORT int32_t agpu_gpt2_generate(agpu_gpt2 *m, const uint32_t *prompt_host, int32_t prompt_len, int32_t max_new_tokens,
-                                       int32_t eos, uint32_t *tokens_out_host, int32_t *length_out_host) {
+// ---- the generation entry points: shared with the other models (lm_runtime.hip) ----
+
+AGPU_EXPORT int32_t agpu_gpt2_forward_cached(agpu_gpt2 *m, const uint32_t *tokens, int32_t batch, int32_t new_len, float *logits,
+                                             int32_t all_rows) {
+    return m ? lm_forward_cached(m, tokens, batch, new_len, logits, all_rows) : AGPU_ERR_NULL_POINTER;
+}
+
+AGPU_EXPORT int32_t agpu_gpt2_decode_steps(agpu_gpt2 *m, int32_t batch, int32_t steps, float *ms_total_out_host) {
+    return m ? lm_decode_steps(m, batch, steps, ms_total_out_host) : AGPU_ERR_NULL_POINTER;
+}
+
+AGPU_EXPORT int32_t agpu_gpt2_last_logits(agpu_gpt2 *m, int32_t batch, float *logits_out_host) {
+    return m ? lm_last_logits(m, batch, logits_out_host) : AGPU_ERR_NULL_POINTER;
+}
+
+AGPU_EXPORT int32_t agpu_gpt2_generate_cached(agpu_gpt2 *m, const uint32_t *prompt_host, int32_t batch, int32_t prompt_len,
+                                              int32_t max_new_tokens, int32_t eos, uint32_t *tokens_out_host, int32_t *lengths_out_host,
+                                              float *timing_ms_out_host) {
     if (!m) return AGPU_ERR_NULL_POINTER;
-    agpu_ctx *ctx = m->ctx;
-    AGPU_REQUIRE_CTX(ctx);
-    if (!prompt_host || !tokens_out_host || !length_out_host)
-        return agpu_fail(ctx, AGPU_ERR_NULL_POINTER, "gpt2_generate: null pointer");
-    if (prompt_len <= 0 || max_new_tokens < 0)
-        return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "gpt2_generate: bad prompt_len/max_new_tokens");
-    int32_t rc = check_token_ids(m, prompt_host, (size_t)prompt_len, "gpt2_generate");
-    if (rc != AGPU_OK) return rc;
-    std::memcpy(tokens_out_host, prompt_host, (size_t)prompt_len * 4);
-    int len = prompt_len;
-    if ((rc = check_ready(m)) != AGPU_OK) return rc;
-    for (int step = 0; step < max_new_tokens; ++step) {
-        if (len > m->P) {
-            rc = agpu_fail(ctx, AGPU_ERR_DIM_OUT_OF_RANGE, "gpt2_generate: sequence length %d exceeds n_positions %d", len, m->P);
-            break;
-        }
-        if ((rc = ensure(m, m->tok_in, (size_t)len * 4)) != AGPU_OK) break;
-        if ((rc = upload(ctx, m->tok_in.p, tokens_out_host, (size_t)len * 4, 0)) != AGPU_OK) break;
-        if ((rc = agpu_gpt2_reset_cache(m)) != AGPU_OK) break;
-        if ((rc = agpu_gpt2_forward_cached(m, (const uint32_t *)m->tok_in.p, 1, len, nullptr, 0)) != AGPU_OK) break;
-        uint32_t next = 0;
-        if ((rc = agpu_memcpy_d2h(ctx, &next, m->next_tok, 4)) != AGPU_OK) break;
-        if (eos >= 0 && next == (uint32_t)eos) break;
-        tokens_out_host[len++] = next;
-    }
-    *length_out_host = len;
-    return rc;
+    return lm_generate_cached(m, prompt_host, batch, prompt_len, max_new_tokens, eos, tokens_out_host, lengths_out_host, timing_ms_out_host);
+}
+
+AGPU_EXPORT int32_t agpu_gpt2_generate_cached_sampling(agpu_gpt2 *m, const uint32_t *prompt_host, int32_t prompt_len, int32_t max_new_tokens,
+                                                       int32_t top_k, float temperature, uint64_t *rng_state, int32_t eos,
+                                                       uint32_t *tokens_out_host, int32_t *length_out_host) {
+    if (!m) return AGPU_ERR_NULL_POINTER;
+    return lm_generate_cached_sampling(m, prompt_host, prompt_len, max_new_tokens, top_k, temperature, rng_state, eos, tokens_out_host,
+                                       length_out_host);
+}
+
+AGPU_EXPORT int32_t agpu_gpt2_generate(agpu_gpt2 *m, const uint32_t *prompt_host, int32_t prompt_len, int32_t max_new_tokens, int32_t eos,
+                                       uint32_t *tokens_out_host, int32_t *length_out_host) {
+    return m ? lm_generate(m, prompt_host, prompt_len, max_new_tokens, eos, tokens_out_host, length_out_host) : AGPU_ERR_NULL_POINTER;
 }
