@@ -13,6 +13,8 @@ ERR_NULL_POINTER, ERR_UNSUPPORTED, ERR_WORKSPACE, ERR_DEVICE_WAIT, ERR_BUSY = -4
 EPI_NONE, EPI_GELU_TANH, EPI_GELU_QUICK, EPI_FORCE_LITERAL, EPI_FORCE_FP32_GEMV = 0, 1, 2, 0x100, 0x200
 QUANT_RUST, QUANT_SCRIPT = 0, 1
 GELU_TANH, GELU_QUICK = 0, 1
+DTYPE_BF16, DTYPE_F32 = 0, 1
+MIXER_LATENT_ATTENTION, MIXER_CHANNEL_DELTA = 0, 1
 
 
 class AgpuError(RuntimeError):
@@ -117,6 +119,24 @@ SIGNATURES = {
     "agpu_gpt2_set_decode_wait_limit": (_i32, [_vp, _i32]),
     "agpu_gpt2_decode_floor": (_i32, [_vp, _i32, _vp]),
     "agpu_gpt2_last_logits": (_i32, [_vp, _i32, _vp]),
+    # include/agpu_ritevik.h
+    "agpu_ritevik_create": (_i32, [_vp, _vp, _vp, C.POINTER(_vp)]),
+    "agpu_ritevik_destroy": (_i32, [_vp]),
+    "agpu_ritevik_set_tensor": (_i32, [_vp, C.c_char_p, _vp, _i32, C.c_int64, C.c_int64]),
+    "agpu_ritevik_tensor_info": (_i32, [_vp, _i32, C.POINTER(C.c_char_p), _vp, _vp, _vp]),
+    "agpu_ritevik_weight_bytes": (C.c_int64, [_vp]),
+    "agpu_ritevik_cache_bytes": (C.c_int64, [_vp]),
+    "agpu_ritevik_layer_runs": (_i32, [_vp]),
+    "agpu_ritevik_reset_cache": (_i32, [_vp]),
+    "agpu_ritevik_cache_len": (_i32, [_vp]),
+    "agpu_ritevik_forward_cached": (_i32, [_vp, _vp, _i32, _i32, _vp, _i32]),
+    "agpu_ritevik_generate_cached": (_i32, [_vp, _vp, _i32, _i32, _i32, _i32, _vp, _vp, _vp]),
+    "agpu_ritevik_generate": (_i32, [_vp, _vp, _i32, _i32, _i32, _vp, _vp]),
+    "agpu_ritevik_generate_cached_sampling": (_i32, [_vp, _vp, _i32, _i32, _i32, _f, _vp, _i32, _vp, _vp]),
+    "agpu_ritevik_set_decode_mode": (_i32, [_vp, _i32]),
+    "agpu_ritevik_decode_steps": (_i32, [_vp, _i32, _i32, _vp]),
+    "agpu_ritevik_last_logits": (_i32, [_vp, _i32, _vp]),
+    "agpu_ritevik_layer_streams": (_i32, [_vp, _vp, _i32, _vp]),
 }
 
 
@@ -131,6 +151,20 @@ class Gpt2ConfigStruct(C.Structure):
     _fields_ = [("n_layer", _i32), ("n_embd", _i32), ("n_head", _i32), ("vocab_size", _i32), ("n_positions", _i32),
                 ("layer_norm_epsilon", _f), ("group_size", _i32), ("max_batch", _i32), ("lm_head", _i32),
                 ("gelu", _i32), ("argmax_last", _i32)]
+
+
+class RitevikConfigStruct(C.Structure):
+    """agpu_ritevik_config of include/agpu_ritevik.h."""
+    _fields_ = [("n_layer", _i32), ("width", _i32), ("vocab_size", _i32), ("n_positions", _i32), ("max_batch", _i32),
+                ("norm_eps", _f), ("loop_start", _i32), ("loop_stop", _i32), ("loop_times", _i32), ("side_dim", _i32),
+                ("dtype", _i32), ("argmax_last", _i32)]
+
+
+class RitevikLayerStruct(C.Structure):
+    """agpu_ritevik_layer of include/agpu_ritevik.h."""
+    _fields_ = [("mixer", _i32), ("heads", _i32), ("dim", _i32), ("vdim", _i32), ("ff", _i32), ("kv_rank", _i32),
+                ("rot_dim", _i32), ("rot_dims", _i32), ("scale", _f), ("rot_base", C.c_double), ("kv_heads", _i32),
+                ("conv", _i32), ("decay_rank", _i32), ("gate_rank", _i32)]
 
 
 def cdll():

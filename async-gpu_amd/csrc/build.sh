@@ -1,5 +1,6 @@
 #!/bin/bash
-# Compiles libagpu_hip.so for gfx950 in-tree (no GPU needed: hipcc cross-compiles).
+# Compiles libagpu_hip.so for gfx950 in-tree (no GPU needed: hipcc cross-compiles).  `build.sh library` stops there; without
+# an argument the tracing build of the library, the C++ host tests and the example program follow.
 set -euo pipefail
 cd "$(dirname "$0")"
 HIPCC=${HIPCC:-/opt/rocm/bin/hipcc}
@@ -16,8 +17,10 @@ done
 g++ -O2 -std=c++17 -fPIC -fopenmp -fvisibility=hidden -ffp-contract=off -c quantize_host.cpp -o build/quantize_host.o &
 pids+=($!)
 for p in "${pids[@]}"; do wait "$p"; done
-"$HIPCC" --offload-arch=gfx950 -shared -fPIC -o ../libagpu_hip.so build/*.o -fopenmp
+"$HIPCC" --offload-arch=gfx950 -shared -fPIC -o build/libagpu_hip.so build/*.o -fopenmp
+mv build/libagpu_hip.so ../libagpu_hip.so
 echo "built $(cd .. && pwd)/libagpu_hip.so"
+if [ "${1:-}" = library ]; then exit 0; fi
 # The same library with time stamps inside the one-launch decode step (bench_configs.py --stamps): the two sources that
 # know about them compiled again with -DAGPU_PK_TRACE, every other object shared.
 mkdir -p build/trace

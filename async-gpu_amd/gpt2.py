@@ -5,7 +5,7 @@ import ctypes as C
 import numpy as np
 
 from . import _lib
-from ._lib import AgpuError
+from .language_model import LanguageModel, _np
 
 LM_HEAD_INT4, LM_HEAD_F32 = 0, 1
 LINEAR_INDEX = {"qkv": 0, "proj": 1, "fc": 2, "fc_proj": 3}
@@ -40,13 +40,12 @@ class Gpt2Config:
                                      int(self.argmax_last))
 
 
-def _np(a, dtype):
-    return np.ascontiguousarray(a, dtype=dtype)
-
-
-class Int4Gpt2Model:
+class Int4Gpt2Model(LanguageModel):
     """Device-resident int4 GPT-2.  `ctx` must own its stream (Context(device) without a stream
     argument): the decode loop is captured into HIP graphs on it."""
+
+    prefix = "agpu_gpt2"
+    default_eos = 50256
 
     def __init__(self, config, ctx=None, device=0):
         self.config = config
@@ -57,26 +56,6 @@ class Int4Gpt2Model:
         rc = self._lib.agpu_gpt2_create(self.ctx.handle, C.byref(st), C.byref(h))
         self._check(rc)
         self.handle = h
-
-    def _check(self, rc):
-        if rc != 0:
-            raise AgpuError(rc, self._lib.agpu_last_error_string(self.ctx.handle).decode())
-
-    def _call(self, name, *args):
-        fn = getattr(self._lib, name)
-        conv = [_lib.ptr(a) if (t is C.c_void_p) else a for a, t in zip(args, fn.argtypes[1:])]
-        self._check(fn(self.handle, *conv))
-
-    def close(self):
-        if getattr(self, "handle", None):
-            self._lib.agpu_gpt2_destroy(self.handle)
-            self.handle = None
-
-    def __del__(self):
-        try:
-            self.close()
-        except Exception:
-            pass
 
     # ---- weights -------------------------------------------------------------------------
     def set_embeddings(self, wte, wpe, lnf_g, lnf_b):
@@ -150,37 +129,6 @@ class Int4Gpt2Model:
         return int(self._lib.agpu_gpt2_quantized_memory_bytes(self.handle))
 
     # ---- inference -----------------------------------------------------------------------
-    def reset_cache(self):
-        self._call("agpu_gpt2_reset_cache")
-
-    def cache_len(self):
-        return int(self._lib.agpu_gpt2_cache_len(self.handle))
-
-    def forward_cached(self, tokens, all_rows=True):
-        """tokens [batch, new_len] (numpy); returns logits as numpy, [batch, new_len, V] or [batch, V]."""
-        tokens = np.atleast_2d(_np(tokens, np.uint32))
-        B, n = tokens.shape
-        V = self.config.vocab_size
-        p = C.c_void_p()
-        self.ctx.call("agpu_malloc", tokens.nbytes, C.byref(p))
-        rows = B * n if all_rows else B
-        lg = C.c_void_p()
-        self.ctx.call("agpu_malloc", rows * V * 4, C.byref(lg))
-        try:
-            self.ctx.call("agpu_memcpy_h2d", p.value, tokens, tokens.nbytes)
-            self._call("agpu_gpt2_forward_cached", p.value, B, n, lg.value, int(all_rows))
-            out = np.empty((B, n, V) if all_rows else (B, V), np.float32)
-            self.ctx.call("agpu_memcpy_d2h", out, lg.value, out.nbytes)
-        finally:
-            self.ctx.call("agpu_free", p.value)
-            self.ctx.call("agpu_free", lg.value)
-        return out
-
-    def forward(self, tokens):
-        """Int4Gpt2Model::forward (gpt2.rs:1522-1533): uncached, logits [seq, V] of one sequence."""
-        self.reset_cache()
-        return self.forward_cached(np.asarray(tokens).reshape(1, -1), all_rows=True)[0]
-
     def _forward_staged(self, tokens, diagnostic):
         tokens = _np(tokens, np.uint32).reshape(-1)
         n_rep = self.config.n_layer + 3
@@ -238,34 +186,6 @@ class Int4Gpt2Model:
             print(f"  token {int(t)}: {float(s):.4f}", file=out)
         return logits, reports, top_tok, top_val
 
-    def generate_cached(self, prompt, max_new_tokens, eos=50256):
-        """Returns (list of token arrays per sequence, (prefill_ms, decode_ms))."""
-        prompt = np.atleast_2d(_np(prompt, np.uint32))
-        B, n = prompt.shape
-        out = np.zeros((B, n + max_new_tokens), np.uint32)
-        lens = np.zeros(B, np.int32)
-        ms = np.zeros(2, np.float32)
-        self._call("agpu_gpt2_generate_cached", prompt, B, n, max_new_tokens, eos, out, lens, ms)
-        return [out[b, :lens[b]].copy() for b in range(B)], (float(ms[0]), float(ms[1]))
-
-    def generate_text(self, tokenizer, prompt, max_new_tokens, eos=50256):
-        """Text in, text out, as the reference's callers do around the model (tokenizer.encode(prompt) -> tokens ->
-        generate -> tokenizer.decode, gpt2.rs:1619-1630, 1790-1836): greedy continuation of `prompt`, prompt included."""
-        tokens = tokenizer.encode(prompt)
-        if not tokens:
-            raise ValueError("empty prompt")
-        (out,), _ = self.generate_cached(np.asarray(tokens, np.uint32), max_new_tokens, eos=eos)
-        return tokenizer.decode(out.tolist())
-
-    def generate_cached_sampling(self, prompt, max_new_tokens, top_k, temperature, rng, eos=50256):
-        """Int4Gpt2Model::generate_cached_sampling (gpt2.rs:931-977); rng is an ops.SimpleRng and is advanced."""
-        prompt = _np(prompt, np.uint32).ravel()
-        out = np.zeros(prompt.size + max_new_tokens, np.uint32)
-        n = C.c_int32(0)
-        self._call("agpu_gpt2_generate_cached_sampling", prompt, prompt.size, max_new_tokens, top_k, float(temperature),
-                   C.addressof(rng._s), eos, out, C.addressof(n))
-        return out[: n.value].copy()
-
     def forward_early_exit(self, tokens, threshold):
         """Gpt2Model::forward_early_exit (gpt2.rs:797-830) -> (logits [seq, V] numpy, layers used)."""
         tokens = _np(tokens, np.uint32).ravel()
@@ -295,26 +215,6 @@ class Int4Gpt2Model:
                    C.addressof(n), layers, C.addressof(steps))
         return out[: n.value].copy(), layers[: steps.value].copy()
 
-    def generate(self, prompt, max_new_tokens, eos=50256):
-        prompt = _np(prompt, np.uint32).ravel()
-        out = np.zeros(prompt.size + max_new_tokens, np.uint32)
-        n = C.c_int32(0)
-        self._call("agpu_gpt2_generate", prompt, prompt.size, max_new_tokens, eos, out, C.addressof(n))
-        return out[: n.value].copy()
-
-    def decode_steps(self, batch, steps):
-        """Replays `steps` decode steps from the current state; returns the total milliseconds."""
-        ms = C.c_float(0)
-        self._call("agpu_gpt2_decode_steps", batch, steps, C.addressof(ms))
-        return float(ms.value)
-
-    DECODE_AUTO, DECODE_PER_STAGE, DECODE_EAGER = 0, 1, 2
-
-    def set_decode_mode(self, mode):
-        """DECODE_AUTO: single-sequence steps run as one launch where the shape allows; DECODE_PER_STAGE: one launch per stage,
-        replayed as a HIP graph; DECODE_EAGER: the same launches without a graph."""
-        self._call("agpu_gpt2_set_decode_mode", mode)
-
     def decode_is_one_launch(self):
         return bool(self._lib.agpu_gpt2_decode_is_one_launch(self.handle))
 
@@ -333,9 +233,3 @@ class Int4Gpt2Model:
         ms = C.c_float(0)
         self._call("agpu_gpt2_decode_floor", steps, C.addressof(ms))
         return float(ms.value)
-
-    def last_logits(self, batch=1):
-        """[batch, vocab] logits of the last position as the most recent forward or decode step left them."""
-        out = np.empty((batch, self.config.vocab_size), np.float32)
-        self._call("agpu_gpt2_last_logits", batch, out)
-        return out

@@ -179,6 +179,61 @@ def quantize_gpt2_file(src, dst, group=32, quantize_fn=None, lm_head_int4=True):
     return cfg, qz
 
 
+def read_safetensors(path):
+    """{name: (dtype, array)} of a safetensors file without copying it: the file is mapped, dtype is the file's own name
+    ("BF16", "F32", ...), bf16 values come as uint16 (numpy has no bfloat16).  A file is an 8-byte little-endian length,
+    that many bytes of JSON (name -> dtype, shape, data_offsets) and the data."""
+    if not os.path.exists(path):
+        raise FileNotFoundError(path)
+    types = {"BF16": np.uint16, "F16": np.float16, "F32": np.float32, "I32": np.int32, "U32": np.uint32, "I64": np.int64, "U8": np.uint8}
+    size = os.path.getsize(path)
+    if size < 8:
+        raise ModelFileError(f"{path}: not a safetensors file")
+    with open(path, "rb") as f:
+        n = int.from_bytes(f.read(8), "little")
+        if n > size - 8:
+            raise ModelFileError(f"{path}: header of {n} bytes in a file of {size}")
+        header = json.loads(f.read(n))
+    raw = np.memmap(path, np.uint8, "r", offset=8 + n) if size > 8 + n else np.empty(0, np.uint8)
+    out = {}
+    for name, e in header.items():
+        if name == "__metadata__":
+            continue
+        if e["dtype"] not in types:
+            raise ModelFileError(f"tensor '{name}': dtype {e['dtype']} is not known")
+        lo, hi = e["data_offsets"]
+        t = np.dtype(types[e["dtype"]])
+        count = int(np.prod(e["shape"], dtype=np.int64))
+        if lo < 0 or hi > raw.size or hi - lo != count * t.itemsize:
+            raise ModelFileError(f"tensor '{name}': bytes {lo} .. {hi} do not hold {e['shape']} of {e['dtype']}")
+        out[name] = (e["dtype"], np.frombuffer(raw[lo:hi].tobytes(), t).reshape(e["shape"]))
+    return out
+
+
+def write_safetensors(path, tensors):
+    """{name: (dtype, array)} as read_safetensors returns it -> a file."""
+    header, blobs, at = {}, [], 0
+    for name, (dtype, a) in tensors.items():
+        b = np.ascontiguousarray(a).tobytes()
+        header[name] = {"dtype": dtype, "shape": list(a.shape), "data_offsets": [at, at + len(b)]}
+        blobs.append(b)
+        at += len(b)
+    text = json.dumps(header).encode()
+    text += b" " * (-len(text) % 8)
+    with open(path, "wb") as f:
+        f.write(len(text).to_bytes(8, "little") + text + b"".join(blobs))
+
+
+def f32_to_bf16(a):
+    """float32 -> bf16 bits (uint16), round to nearest even."""
+    u = np.ascontiguousarray(a, np.float32).view(np.uint32)
+    return ((u + 0x7FFF + ((u >> 16) & 1)) >> 16).astype(np.uint16)
+
+
+def bf16_to_f32(a):
+    return (np.ascontiguousarray(a, np.uint16).astype(np.uint32) << 16).view(np.float32)
+
+
 def count_params(path):
     """(values, bytes) of every tensor in a safetensors file: what the reference's loader reports as total_params and
     memory_bytes (model.rs:380-396); packed int4 words count eight values each."""
