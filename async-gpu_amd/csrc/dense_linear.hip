@@ -199,7 +199,7 @@ __global__ __launch_bounds__(64 * NW) void dense_rows_kernel(DenseRows in, void 
     });
 }
 
-// ---- 5 .. 32 rows: 16 columns per workgroup, the waves split K, operands straight from memory ----
+// ---- few rows or few columns: 16 columns and up to 32 rows per workgroup, the waves split K, operands straight from memory ----
 constexpr int kSkinnyWaves = 8;
 
 template <int RT>  // row tiles of 16
@@ -207,11 +207,11 @@ __global__ __launch_bounds__(64 * kSkinnyWaves) void dense_skinny_kernel(const u
                                                                          int ldw, int M, int N, int K, DenseOut o) {
     __shared__ float red[kSkinnyWaves][RT][16][17];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, rc = lane & 15, kq = lane >> 4;
-    const int n0 = blockIdx.x * 16;
+    const int n0 = blockIdx.x * 16, m0 = blockIdx.y * 16 * RT;
     const uint16_t *wp = w + (size_t)min(n0 + rc, N - 1) * ldw + kq * 8;
     const uint16_t *ap[RT];
 #pragma unroll
-    for (int t = 0; t < RT; ++t) ap[t] = a + (size_t)min(t * 16 + rc, M - 1) * lda + kq * 8;
+    for (int t = 0; t < RT; ++t) ap[t] = a + (size_t)min(m0 + t * 16 + rc, M - 1) * lda + kq * 8;
     f32x4 acc[RT];
 #pragma unroll
     for (int t = 0; t < RT; ++t) acc[t] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
@@ -240,7 +240,7 @@ __global__ __launch_bounds__(64 * kSkinnyWaves) void dense_skinny_kernel(const u
         for (int r = 0; r < 4; ++r) red[wave][t][kq * 4 + r][rc] = acc[t][r];
     __syncthreads();
     for (int i = threadIdx.x; i < RT * 256; i += 64 * kSkinnyWaves) {
-        const int t = i >> 8, r = (i >> 4) & 15, c = i & 15, m = t * 16 + r, n = n0 + c;
+        const int t = i >> 8, r = (i >> 4) & 15, c = i & 15, m = m0 + t * 16 + r, n = n0 + c;
         if (m >= M || n >= N) continue;
         auto total = [&](int col) {
             float s = 0.0f;
@@ -459,13 +459,13 @@ int32_t dense_rows_launch(agpu_ctx *ctx, const DenseRows &in, int M, void *h, in
 int32_t dense_gemm_bf16_launch(agpu_ctx *ctx, const uint16_t *a, int lda, const uint16_t *w, int ldw, int M, int N, int K, const DenseOut &o) {
     if (M <= 0 || N <= 0 || K <= 0 || K % 32 != 0 || lda % 8 != 0 || ldw % 8 != 0 || (o.n_plain < N && (o.n_plain % 2 != 0 || N % 2 != 0)))
         return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "dense_gemm: M %d, N %d, K %d, lda %d, ldw %d not supported", M, N, K, lda, ldw);
-    if (M <= kDenseSkinnyRows) {
-        const dim3 grid((unsigned)ceil_div(N, 16)), block(64 * kSkinnyWaves);
+    auto tiles = [&](int bm, int bn) { return ceil_div(M, bm) * ceil_div(N, bn); };
+    if (M <= kDenseSkinnyRows || 2 * tiles(32, 64) < ctx->num_cus) {
+        const dim3 grid((unsigned)ceil_div(N, 16), (unsigned)ceil_div(M, 32)), block(64 * kSkinnyWaves);
         if (M <= 16) hipLaunchKernelGGL(dense_skinny_kernel<1>, grid, block, 0, ctx->stream, a, lda, w, ldw, M, N, K, o);
         else hipLaunchKernelGGL(dense_skinny_kernel<2>, grid, block, 0, ctx->stream, a, lda, w, ldw, M, N, K, o);
         return AGPU_LAUNCH_CHECK(ctx, "dense_skinny_kernel");
     }
-    auto tiles = [&](int bm, int bn) { return ceil_div(M, bm) * ceil_div(N, bn); };
     if (tiles(128, 128) >= ctx->num_cus) {
         hipLaunchKernelGGL((dense_gemm_bf16_kernel<128, 128, 2, 2>), dim3((unsigned)tiles(128, 128)), dim3(256), 0, ctx->stream, a, lda, w, ldw, M, N, K,
                            ceil_div(N, 128), o);

@@ -19,7 +19,7 @@ struct DeltaWeights {
     const float *conv = nullptr;    // [channels][taps], last tap is the current token's
     const float *a_log = nullptr;   // [heads]
     const float *dt_bias = nullptr; // [heads * dim]
-    const uint16_t *a2 = nullptr;   // [heads * dim][rank_ap]
+    const uint16_t *a2 = nullptr;   // [heads * state_row][rank_ap], zero padded per head
     const uint16_t *g2 = nullptr;   // [heads * vdim][rank_gp]
     const float *norm = nullptr;    // [vdim], plain
 };
@@ -36,9 +36,9 @@ struct DeltaArgs {
     void *out = nullptr;  // rows, stride ldo: heads x vdim, bf16 or fp32
     int ldo = 0, out_bf16 = 0;
     // scratch of the many-token form, fp32 rows
-    float *qk = nullptr;    // [rows][2 * kv_heads * dim]: q | k, unit vectors
+    float *qk = nullptr;    // [rows][2 * kv_heads * state_row]: q | k, unit vectors
     float *v = nullptr;     // [rows][heads * vdim]
-    float *g = nullptr;     // [rows][heads * dim]: in: W_a2 a1, out: decay
+    float *g = nullptr;     // [rows][heads * state_row]: in: W_a2 a1, out: decay
     float *bkq = nullptr;   // [rows][heads + kv_heads]: beta | k . q
     float *gate = nullptr;  // [rows][heads * vdim]: W_g2 g1
     float *o = nullptr;     // [rows][heads * vdim]

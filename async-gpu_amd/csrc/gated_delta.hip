@@ -15,65 +15,89 @@ constexpr int kRecWaves = 4;
 __device__ __forceinline__ float softplus_dev(float v) { return fmaxf(v, 0.0f) + log1pf(expf(-fabsf(v))); }
 __device__ __forceinline__ float decay_dev(float a_log, float step) { return expf(-expf(a_log) * softplus_dev(step)); }
 
-// The convolution input of channel c (source column `col` of the projection) at token `s` of the portion; before the
-// portion the ring, before the sequence zero.
-__device__ __forceinline__ float conv_input(const DeltaArgs &a, int channels, int b, int pos, int s, int c, int col) {
-    if (s >= 0) return a.proj[(size_t)(b * a.new_len + s) * a.ld + col];
-    const int p = pos + s;
-    return p >= 0 ? a.ring[((size_t)b * a.s.taps + p % a.s.taps) * channels + c] : 0.0f;
-}
-
-__device__ __forceinline__ float conv_silu(const DeltaArgs &a, int channels, int b, int pos, int s, int c, int col) {
+// Convolution and silu of channel c (source column `col` of the projection) at token `t` of the portion.  Inputs before the
+// portion come from the ring, before the sequence they are zero.  pos_slot = pos % taps.  Loads go four taps at a time and
+// without branches.
+__device__ __forceinline__ float conv_silu(const DeltaArgs &a, int channels, int b, int pos, int pos_slot, int t, int c, int col) {
     const int n = a.s.taps;
-    const float *w = a.w.conv + (size_t)c * n;
-    float v = 0.0f;
-    for (int j = 0; j < n; ++j) v = fmaf(w[j], conv_input(a, channels, b, pos, s - (n - 1) + j, c, col), v);
+    const float *cur = a.proj + (size_t)(b * a.new_len + t) * a.ld + col;
+    const float *ring = a.ring + (size_t)b * n * channels + c, *w = a.w.conv + (size_t)c * n;
+    float v = w[n - 1] * cur[0];
+#pragma unroll 1
+    for (int k0 = 1; k0 < n; k0 += 4) {
+        float x[4], f[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int k = k0 + e;
+            const bool on = k < n && pos + t >= k;
+            int slot = pos_slot + t - k;
+            slot = slot < 0 ? slot + n : slot;
+            const float *p = t >= k ? cur - (size_t)k * a.ld : ring + (size_t)slot * channels;
+            x[e] = *(on ? p : cur);
+            f[e] = on ? w[n - 1 - min(k, n - 1)] : 0.0f;
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v = fmaf(f[e], x[e], v);
+    }
     return silu_dev(v);
 }
 
-// One workgroup per token row: convolution, unit vectors, decays, step sizes.
-__global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaArgs a, int channels) {
+constexpr int kPrepareWidth = 1024;  // channels of v or g per workgroup
+
+// grid (rows, parts): the first parts take four heads of q and k each (convolution, unit vectors; one wave per head), then
+// come parts of v (convolution), then parts of g (decays; the first of them also the step sizes).  q, k and g leave with one
+// padded row per head.
+__global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaArgs a, int channels, int head_row, int qk_parts, int v_parts) {
+    __shared__ float sx[2][4][kMaxDim];
     const DeltaShape &s = a.s;
-    const int row = blockIdx.x, b = row / a.new_len, t = row % a.new_len, pos = *a.pos_dev;
+    const int row = blockIdx.x, b = row / a.new_len, t = row % a.new_len, pos = *a.pos_dev, pos_slot = pos % s.taps;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int nk = s.kv_heads * s.dim, nv = s.heads * s.vdim;
-    float *qk = a.qk + (size_t)row * 2 * nk;
     float *bkq = a.bkq + (size_t)row * (s.heads + s.kv_heads);
-    for (int h = wave; h < s.kv_heads; h += 4) {
-        float q[kMaxDim / 64], k[kMaxDim / 64];
-        float qq = 0.0f, kk = 0.0f;
-#pragma unroll
-        for (int i = 0; i < kMaxDim / 64; ++i) {
-            const int d = lane + 64 * i, c = h * s.dim + d;
-            q[i] = k[i] = 0.0f;
-            if (d < s.dim) {
-                q[i] = conv_silu(a, channels, b, pos, t, c, a.col_q + c);
-                k[i] = conv_silu(a, channels, b, pos, t, nk + c, a.col_k + c);
-            }
-            qq += q[i] * q[i];
-            kk += k[i] * k[i];
+    int part = blockIdx.y;
+    if (part < qk_parts) {
+        const int h = part * 4 + wave;
+        if (h >= s.kv_heads) return;
+        float *q_out = a.qk + ((size_t)row * 2 * s.kv_heads + h) * head_row, *k_out = q_out + (size_t)s.kv_heads * head_row;
+#pragma unroll 1
+        for (int i = lane; i < 2 * head_row; i += 64) {
+            const int k = i >= head_row, d = i - k * head_row, c = h * s.dim + min(d, s.dim - 1);
+            const float v = conv_silu(a, channels, b, pos, pos_slot, t, k * nk + c, (k ? a.col_k : a.col_q) + c);
+            sx[k][wave][d] = d < s.dim ? v : 0.0f;
+        }
+        __builtin_amdgcn_wave_barrier();  // a wave reads what it wrote itself
+        float qq = 0.0f, kk = 0.0f, dot = 0.0f;
+        for (int d = lane; d < head_row; d += 64) {
+            const float q = sx[0][wave][d], k = sx[1][wave][d];
+            qq = fmaf(q, q, qq);
+            kk = fmaf(k, k, kk);
+            dot = fmaf(q, k, dot);
         }
         const float rq = 1.0f / sqrtf(wave_sum(qq) + 1e-6f) / sqrtf((float)s.dim), rk = 1.0f / sqrtf(wave_sum(kk) + 1e-6f);
-        float dot = 0.0f;
-#pragma unroll
-        for (int i = 0; i < kMaxDim / 64; ++i) {
-            const int d = lane + 64 * i;
-            q[i] *= rq;
-            k[i] *= rk;
-            dot += q[i] * k[i];
-            if (d < s.dim) {
-                qk[h * s.dim + d] = q[i];
-                qk[nk + h * s.dim + d] = k[i];
-            }
-        }
         dot = wave_sum(dot);
-        if (lane == 0) bkq[s.heads + h] = dot;
+        for (int d = lane; d < head_row; d += 64) {
+            q_out[d] = sx[0][wave][d] * rq;
+            k_out[d] = sx[1][wave][d] * rk;
+        }
+        if (lane == 0) bkq[s.heads + h] = dot * rq * rk;
+        return;
     }
-    for (int c = threadIdx.x; c < nv; c += 256) a.v[(size_t)row * nv + c] = conv_silu(a, channels, b, pos, t, 2 * nk + c, a.col_v + c);
-    const float *p = a.proj + (size_t)row * a.ld;
-    for (int h = threadIdx.x; h < s.heads; h += 256) bkq[h] = sigmoid_dev(p[a.col_b + h]);
-    float *g = a.g + (size_t)row * s.heads * s.dim;
-    for (int c = threadIdx.x; c < s.heads * s.dim; c += 256) g[c] = decay_dev(a.w.a_log[c / s.dim], g[c] + a.w.dt_bias[c]);
+    part -= qk_parts;
+    if (part < v_parts) {
+#pragma unroll 1
+        for (int c = part * kPrepareWidth + threadIdx.x; c < min((part + 1) * kPrepareWidth, nv); c += 256)
+            a.v[(size_t)row * nv + c] = conv_silu(a, channels, b, pos, pos_slot, t, 2 * nk + c, a.col_v + c);
+        return;
+    }
+    part -= v_parts;
+    if (part == 0)
+        for (int h = threadIdx.x; h < s.heads; h += 256) bkq[h] = sigmoid_dev(a.proj[(size_t)row * a.ld + a.col_b + h]);
+    float *g = a.g + (size_t)row * s.heads * head_row;
+#pragma unroll 2
+    for (int c = part * kPrepareWidth + threadIdx.x; c < min((part + 1) * kPrepareWidth, s.heads * head_row); c += 256) {
+        const int h = c / head_row, d = c % head_row;
+        g[c] = d < s.dim ? decay_dev(a.w.a_log[h], g[c] + a.w.dt_bias[h * s.dim + d]) : 1.0f;
+    }
 }
 
 // The convolution inputs of the last `taps` tokens of the portion into the ring (after every read of the old ones).
@@ -102,36 +126,53 @@ __global__ __launch_bounds__(64 * kRecWaves) void delta_recurrence_kernel(DeltaA
     const DeltaShape &s = a.s;
     const int t = threadIdx.x, lane = t & 63, wave = t >> 6, l32 = lane & 31, half = lane >> 5;
     const int h = blockIdx.y, b = blockIdx.z, j0 = blockIdx.x * COLS, j = j0 + wave * 2 + half;
-    const int hk = h / (s.heads / s.kv_heads), nk = s.kv_heads * s.dim, nv = s.heads * s.vdim, T = a.new_len;
+    const int hk = h / (s.heads / s.kv_heads), nv = s.heads * s.vdim, T = a.new_len;
     const size_t row0 = (size_t)b * T;
     float *st = a.state + (((size_t)b * s.heads + h) * s.vdim + min(j, s.vdim - 1)) * DP + l32 * DR;
     float S[DR];
 #pragma unroll
     for (int r = 0; r < DR; ++r) S[r] = st[r];
-    auto stage = [&](int buf, int t0) {
-        for (int i = t; i < kChunk * 3 * DP; i += NT) {
-            const int d = i % DP, w = (i / DP) % 3, tok = t0 + i / (3 * DP);
-            const size_t row = row0 + min(tok, T - 1);
-            const int dd = min(d, s.dim - 1);
-            const float *src = w == 2 ? a.g + row * s.heads * s.dim + h * s.dim : a.qk + row * 2 * nk + w * nk + hk * s.dim;
-            const float v = d < s.dim ? src[dd] : 0.0f;
-            sv[buf][i / (3 * DP)][w][d] = tok < T ? v : (w == 2 ? 1.0f : 0.0f);  // behind the last token nothing moves
+    // The vectors of a chunk: requested into registers before the chunk in front of it is worked on, put into LDS after.
+    constexpr int QUADS = kChunk * 3 * DP / 4, QN = (QUADS + NT - 1) / NT;
+    static_assert(kChunk * (COLS + 2) <= NT, "one scalar per thread");
+    const float *qk = a.qk + (row0 * 2 * s.kv_heads + hk) * DP, *gp = a.g + (row0 * s.heads + h) * DP;
+    float4 rq[QN];
+    float rs = 0.0f;
+    auto request = [&](int t0) {
+#pragma unroll
+        for (int n = 0; n < QN; ++n) {
+            const int i = min(t + n * NT, QUADS - 1), d4 = i % (DP / 4), w = (i / (DP / 4)) % 3, tok = min(t0 + i / (3 * DP / 4), T - 1);
+            const float *src = w == 2 ? gp + (size_t)tok * s.heads * DP : qk + (size_t)tok * 2 * s.kv_heads * DP + w * s.kv_heads * DP;
+            rq[n] = *(const float4 *)(src + 4 * d4);
         }
-        for (int i = t; i < kChunk * (COLS + 2); i += NT) {
-            const int c = i % (COLS + 2);
-            const size_t row = row0 + min(t0 + i / (COLS + 2), T - 1);
+        if (t < kChunk * (COLS + 2)) {
+            const int c = t % (COLS + 2);
+            const size_t row = row0 + min(t0 + t / (COLS + 2), T - 1);
             const float *bkq = a.bkq + row * (s.heads + s.kv_heads);
-            float v;
-            if (c < COLS) v = a.v[row * nv + h * s.vdim + min(j0 + c, s.vdim - 1)];
-            else v = c == COLS ? bkq[h] : bkq[s.heads + hk];
-            sc[buf][i / (COLS + 2)][c] = v;
+            rs = c < COLS ? a.v[row * nv + h * s.vdim + min(j0 + c, s.vdim - 1)] : bkq[c == COLS ? h : s.heads + hk];
         }
     };
+    auto stage = [&](int buf, int t0) {
+#pragma unroll
+        for (int n = 0; n < QN; ++n) {
+            const int i = t + n * NT, d4 = i % (DP / 4), w = (i / (DP / 4)) % 3, tok = i / (3 * DP / 4);
+            if (i >= QUADS) continue;
+            float4 v = rq[n];
+            if (t0 + tok >= T) {  // behind the last token nothing moves
+                const float f = w == 2 ? 1.0f : 0.0f;
+                v = make_float4(f, f, f, f);
+            }
+            *(float4 *)&sv[buf][tok][w][4 * d4] = v;
+        }
+        if (t < kChunk * (COLS + 2)) sc[buf][t / (COLS + 2)][t % (COLS + 2)] = rs;
+    };
+    request(0);
     stage(0, 0);
+    __syncthreads();
     int buf = 0;
     for (int t0 = 0; t0 < T; t0 += kChunk, buf ^= 1) {
-        __syncthreads();
-        if (t0 + kChunk < T) stage(buf ^ 1, t0 + kChunk);
+        const bool more = t0 + kChunk < T;
+        if (more) request(t0 + kChunk);
         // the vectors of the next token are on their way while this one is worked on
         float q[DR], k[DR], g[DR], v, beta, kq;
         auto fetch = [&](int i) {
@@ -166,6 +207,8 @@ __global__ __launch_bounds__(64 * kRecWaves) void delta_recurrence_kernel(DeltaA
             for (int r = 0; r < DR; ++r) S[r] = fmaf(kc[r], u, S[r]);
             if (l32 == 0 && j < s.vdim && t0 + i < T) a.o[(row0 + t0 + i) * nv + h * s.vdim + j] = fmaf(kqc, u, qs);
         }
+        if (more) stage(buf ^ 1, t0 + kChunk);
+        __syncthreads();
     }
     if (j < s.vdim) {
 #pragma unroll
@@ -191,124 +234,167 @@ __global__ __launch_bounds__(256) void delta_gate_kernel(DeltaArgs a) {
     }
 }
 
-// Low-rank product: out[r] = sum_k w[row0 + r][k] x[k] for r < n, rank a multiple of 32; 16 lanes per row.
-__device__ __forceinline__ void low_rank(const uint16_t *w, int rank, const float *x, float *out, int n, int threads) {
-    const int lane = threadIdx.x & 63, kl = lane & 15, group = threadIdx.x >> 4;
-    for (int r = group; r < n; r += threads / 16) {
-        float acc = 0.0f;
-        for (int k = kl * 8; k < rank; k += 128) {
-            const uint4 v = *(const uint4 *)(w + (size_t)r * rank + k);
-            const uint32_t u[4] = {v.x, v.y, v.z, v.w};
+constexpr int kStepThreads = 512, kStepGroups = kStepThreads / 16;
+
+// Eight values of a bf16 row against eight floats.
+__device__ __forceinline__ float dot8(const uint4 &v, const float *x, float acc) {
+    const uint32_t u[4] = {v.x, v.y, v.z, v.w};
 #pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                acc = fmaf(__uint_as_float(u[e] << 16), x[k + 2 * e], acc);
-                acc = fmaf(__uint_as_float(u[e] & 0xffff0000u), x[k + 2 * e + 1], acc);
-            }
-        }
-        acc = row16_sum(acc);
-        if (kl == 0) out[r] = acc;
+    for (int e = 0; e < 4; ++e) {
+        acc = fmaf(__uint_as_float(u[e] << 16), x[2 * e], acc);
+        acc = fmaf(__uint_as_float(u[e] & 0xffff0000u), x[2 * e + 1], acc);
     }
+    return acc;
 }
 
-constexpr int kStepThreads = 512;
-
-// One token of one sequence and head: grid (heads, batch).  NF float4 of a state column per lane of 16.
-template <int NF>
+// One token of one sequence and head: grid (heads, batch).  NF float4 of a state column per lane of 16, CI columns per group.
+// The state and the first rows of the low-rank factors are requested before anything else.  The code is kept short: at
+// this size a launch waits for its instructions as much as for its data.
+template <int NF, int CI>
 __global__ __launch_bounds__(kStepThreads) void delta_step_kernel(DeltaArgs a, int channels, int rank_ap, int rank_gp, int state_row) {
     extern __shared__ float low[];  // a1 [rank_ap], g1 [rank_gp]
-    __shared__ __align__(16) float sq[kMaxDim], sk[kMaxDim], sg[kMaxDim];
-    __shared__ float svv[kMaxDim], sgate[kMaxDim], so[kMaxDim];
+    __shared__ __align__(16) float sx[4][kMaxDim];  // q, k, g, v
+    __shared__ float sgate[kMaxDim], so[kMaxDim];
     __shared__ float red[4];
     const DeltaShape &s = a.s;
     const int t = threadIdx.x, lane = t & 63, wave = t >> 6;
-    const int h = blockIdx.x, b = blockIdx.y, group = s.heads / s.kv_heads, hk = h / group, pos = *a.pos_dev;
+    const int h = blockIdx.x, b = blockIdx.y, group = s.heads / s.kv_heads, hk = h / group, pos = *a.pos_dev, pos_slot = pos % s.taps;
     const int nk = s.kv_heads * s.dim;
     const float *p = a.proj + (size_t)b * a.ld;
     float *state = a.state + ((size_t)b * s.heads + h) * s.vdim * state_row;
-    const int kl = lane & 15, col0 = t >> 4;  // 32 columns at a time
-    constexpr int COLS = kStepThreads / 16;
-    // the first columns of the state are requested before anything else
-    float4 first[NF];
+    const int kl = lane & 15, col0 = t >> 4;
+    float4 S[CI][NF];
 #pragma unroll
-    for (int f = 0; f < NF; ++f) {
-        const int d = kl * 4 + 64 * f;
-        first[f] = (d < state_row && col0 < s.vdim) ? *(const float4 *)(state + (size_t)col0 * state_row + d) : make_float4(0, 0, 0, 0);
-    }
-    for (int k = t; k < rank_ap; k += kStepThreads) low[k] = p[a.col_a1 + k];
-    for (int k = t; k < rank_gp; k += kStepThreads) low[rank_ap + k] = p[a.col_g1 + k];
-    for (int d = t; d < kMaxDim; d += kStepThreads) {
-        const int c = hk * s.dim + d;
-        sq[d] = d < s.dim ? conv_silu(a, channels, b, pos, 0, c, a.col_q + c) : 0.0f;
-        sk[d] = d < s.dim ? conv_silu(a, channels, b, pos, 0, nk + c, a.col_k + c) : 0.0f;
-        sg[d] = 0.0f;
-        const int cv = h * s.vdim + d;
-        if (d < s.vdim) svv[d] = conv_silu(a, channels, b, pos, 0, 2 * nk + cv, a.col_v + cv);
-    }
-    // the new inputs into the ring: a slot that no tap of this token reads.  q and k by the first head of a group.
-    float *slot = a.ring + ((size_t)b * s.taps + pos % s.taps) * channels;
-    if (h % group == 0)
-        for (int d = t; d < s.dim; d += kStepThreads) {
-            const int c = hk * s.dim + d;
-            slot[c] = p[a.col_q + c];
-            slot[nk + c] = p[a.col_k + c];
+    for (int i = 0; i < CI; ++i)
+#pragma unroll
+        for (int f = 0; f < NF; ++f)  // clamped addresses; what lies outside is never used
+            S[i][f] = *(const float4 *)(state + (size_t)min(col0 + i * kStepGroups, s.vdim - 1) * state_row + min(kl * 4 + 64 * f, state_row - 4));
+    // rows of W_a2 and W_g2 of this head, 4 lanes per row: r = t / 4, + 128, ...
+    const uint16_t *wa = a.w.a2 + (size_t)h * state_row * rank_ap, *wg = a.w.g2 + (size_t)h * s.vdim * rank_gp;
+    const int rows = s.dim + s.vdim, part = t & 3;
+    uint4 wp[2][4];
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int r = min((t >> 2) + 128 * i, rows - 1), rank = r < s.dim ? rank_ap : rank_gp;
+            wp[i][j] = *(const uint4 *)((r < s.dim ? wa + (size_t)r * rank_ap : wg + (size_t)(r - s.dim) * rank_gp) + min(part * 8 + 32 * j, rank - 8));
         }
-    for (int d = t; d < s.vdim; d += kStepThreads) slot[2 * nk + h * s.vdim + d] = p[a.col_v + h * s.vdim + d];
+    for (int k = t; k < rank_ap + rank_gp; k += kStepThreads) low[k] = p[k < rank_ap ? a.col_a1 + k : a.col_g1 + k - rank_ap];
+    // convolution of the head's q, k and v; the new inputs go into a ring slot that no tap of this token reads (q and k by
+    // the first head of a group)
+    float *slot = a.ring + ((size_t)b * s.taps + pos_slot) * channels;
+#pragma unroll 1
+    for (int i = t; i < 2 * state_row + s.vdim; i += kStepThreads) {
+        const int w = i < state_row ? 0 : (i < 2 * state_row ? 1 : 3), d = i - min(w, 2) * state_row;
+        const bool on = w == 3 || d < s.dim;
+        const int c = w == 3 ? h * s.vdim + d : hk * s.dim + min(d, s.dim - 1);
+        const int ch = min(w, 2) * nk + c, col = (w == 0 ? a.col_q : (w == 1 ? a.col_k : a.col_v)) + c;
+        const float v = conv_silu(a, channels, b, pos, pos_slot, 0, ch, col);
+        sx[w][d] = on ? v : 0.0f;
+        if (on && (w == 3 || h % group == 0)) slot[ch] = p[col];
+    }
     __syncthreads();
-    low_rank(a.w.a2 + (size_t)h * s.dim * rank_ap, rank_ap, low, sg, s.dim, kStepThreads);
-    low_rank(a.w.g2 + (size_t)h * s.vdim * rank_gp, rank_gp, low + rank_ap, sgate, s.vdim, kStepThreads);
+    // raw low-rank products to sx[2] and sgate
+    auto put = [&](int r, float acc) {
+        acc += dpp_move<0xb1, 0xf>(0.0f, acc);
+        acc += dpp_move<0x4e, 0xf>(0.0f, acc);
+        if (part == 0 && r < rows) (r < s.dim ? sx[2][r] : sgate[r - s.dim]) = acc;
+    };
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+        const int r = (t >> 2) + 128 * i, rank = r < s.dim ? rank_ap : rank_gp;
+        const float *x = low + (r < s.dim ? 0 : rank_ap);
+        float acc = 0.0f;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int k = part * 8 + 32 * j;
+            const float v = dot8(wp[i][j], x + min(k, rank - 8), acc);
+            acc = k < rank ? v : acc;
+        }
+#pragma unroll 1
+        for (int k = part * 8 + 128; k < rank; k += 32)
+            acc = dot8(*(const uint4 *)((r < s.dim ? wa + (size_t)r * rank_ap : wg + (size_t)min(r - s.dim, s.vdim - 1) * rank_gp) + k), x + k, acc);
+        put(r, acc);
+    }
+#pragma unroll 1
+    for (int r = (t >> 2) + 256; r < (rows + 127) / 128 * 128; r += 128) {
+        const int rr = min(r, rows - 1), rank = rr < s.dim ? rank_ap : rank_gp;
+        const uint16_t *w = rr < s.dim ? wa + (size_t)rr * rank_ap : wg + (size_t)(rr - s.dim) * rank_gp;
+        const float *x = low + (rr < s.dim ? 0 : rank_ap);
+        float acc = 0.0f;
+#pragma unroll 1
+        for (int k = part * 8; k < rank; k += 32) acc = dot8(*(const uint4 *)(w + k), x + k, acc);
+        put(r, acc);
+    }
     if (wave < 3) {  // |q|^2, |k|^2, q . k
         float v = 0.0f;
-        for (int d = lane; d < kMaxDim; d += 64) v += (wave == 1 ? sk[d] : sq[d]) * (wave == 0 ? sq[d] : sk[d]);
+        for (int d = lane; d < state_row; d += 64) v += sx[wave == 1][d] * sx[wave != 0][d];
         v = wave_sum(v);
         if (lane == 0) red[wave] = v;
     }
     __syncthreads();
     const float rq = 1.0f / sqrtf(red[0] + 1e-6f) / sqrtf((float)s.dim), rk = 1.0f / sqrtf(red[1] + 1e-6f);
     const float kq = red[2] * rq * rk, beta = sigmoid_dev(p[a.col_b + h]);
-    for (int d = t; d < s.dim; d += kStepThreads) sg[d] = decay_dev(a.w.a_log[h], sg[d] + a.w.dt_bias[h * s.dim + d]);
+    if (t < state_row) sx[2][t] = t < s.dim ? decay_dev(a.w.a_log[h], sx[2][t] + a.w.dt_bias[h * s.dim + t]) : 0.0f;
     __syncthreads();
-    for (int j = col0; j < s.vdim; j += COLS) {
-        float4 S[NF], k4[NF];
+#pragma unroll
+    for (int i = 0; i < CI; ++i) {
+        const int j = col0 + i * kStepGroups;
         float ks = 0.0f, qs = 0.0f;
 #pragma unroll
         for (int f = 0; f < NF; ++f) {
             const int d = kl * 4 + 64 * f;
-            S[f] = first[f];
-            if (j != col0) S[f] = d < state_row ? *(const float4 *)(state + (size_t)j * state_row + d) : make_float4(0, 0, 0, 0);
-            const float4 g4 = *(const float4 *)&sg[d], q4 = *(const float4 *)&sq[d];
-            k4[f] = *(const float4 *)&sk[d];
-            S[f].x *= g4.x; S[f].y *= g4.y; S[f].z *= g4.z; S[f].w *= g4.w;
-            ks += S[f].x * k4[f].x + S[f].y * k4[f].y + S[f].z * k4[f].z + S[f].w * k4[f].w;
-            qs += S[f].x * q4.x + S[f].y * q4.y + S[f].z * q4.z + S[f].w * q4.w;
+            if (d >= state_row) continue;
+            const float4 g4 = *(const float4 *)&sx[2][d], q4 = *(const float4 *)&sx[0][d], k4 = *(const float4 *)&sx[1][d];
+            float4 &v = S[i][f];
+            v.x *= g4.x; v.y *= g4.y; v.z *= g4.z; v.w *= g4.w;
+            ks += v.x * k4.x + v.y * k4.y + v.z * k4.z + v.w * k4.w;
+            qs += v.x * q4.x + v.y * q4.y + v.z * q4.z + v.w * q4.w;
         }
         ks = row16_sum(ks) * rk;
         qs = row16_sum(qs) * rq;
-        const float u = beta * (svv[j] - ks), uk = u * rk;
+        if (j >= s.vdim) continue;
+        const float u = beta * (sx[3][j] - ks), uk = u * rk;
 #pragma unroll
         for (int f = 0; f < NF; ++f) {
             const int d = kl * 4 + 64 * f;
-            S[f].x = fmaf(k4[f].x, uk, S[f].x);
-            S[f].y = fmaf(k4[f].y, uk, S[f].y);
-            S[f].z = fmaf(k4[f].z, uk, S[f].z);
-            S[f].w = fmaf(k4[f].w, uk, S[f].w);
-            if (d < state_row) *(float4 *)(state + (size_t)j * state_row + d) = S[f];
+            if (d >= state_row) continue;
+            const float4 k4 = *(const float4 *)&sx[1][d];
+            float4 &v = S[i][f];
+            v.x = fmaf(k4.x, uk, v.x);
+            v.y = fmaf(k4.y, uk, v.y);
+            v.z = fmaf(k4.z, uk, v.z);
+            v.w = fmaf(k4.w, uk, v.w);
+            *(float4 *)(state + (size_t)j * state_row + d) = v;
         }
         if (kl == 0) so[j] = fmaf(kq, u, qs);
     }
     __syncthreads();
-    if (wave == 0) {
-        float sum = 0.0f;
-        for (int d = lane; d < s.vdim; d += 64) sum += so[d] * so[d];
-        sum = wave_sum(sum);
-        if (lane == 0) red[3] = 1.0f / sqrtf(sum / (float)s.vdim + s.eps);
-    }
-    __syncthreads();
-    for (int d = t; d < s.vdim; d += kStepThreads) {
-        const float v = so[d] * red[3] * a.w.norm[d] * sigmoid_dev(sgate[d]);
-        const size_t at = (size_t)b * a.ldo + h * s.vdim + d;
+    float sum = 0.0f;  // every wave for itself
+    for (int d = lane; d < s.vdim; d += 64) sum = fmaf(so[d], so[d], sum);
+    const float rs = 1.0f / sqrtf(wave_sum(sum) / (float)s.vdim + s.eps);
+    if (t < s.vdim) {
+        const float v = so[t] * rs * a.w.norm[t] * sigmoid_dev(sgate[t]);
+        const size_t at = (size_t)b * a.ldo + h * s.vdim + t;
         if (a.out_bf16) ((uint16_t *)a.out)[at] = f32_to_bf16(v);
         else ((float *)a.out)[at] = v;
     }
+}
+
+template <int NF>
+void step_run(agpu_ctx *ctx, const DeltaArgs &a) {
+    const DeltaShape &s = a.s;
+    const dim3 grid((unsigned)s.heads, (unsigned)a.batch), block(kStepThreads);
+    const size_t lds = (size_t)(s.rank_ap() + s.rank_gp()) * sizeof(float);
+    const int ci = ceil_div(s.vdim, kStepGroups);
+#define AGPU_DELTA_STEP(CI) \
+    hipLaunchKernelGGL((delta_step_kernel<NF, CI>), grid, block, lds, ctx->stream, a, s.channels(), s.rank_ap(), s.rank_gp(), s.state_row())
+    if (ci <= 1) AGPU_DELTA_STEP(1);
+    else if (ci <= 2) AGPU_DELTA_STEP(2);
+    else if (ci <= 4) AGPU_DELTA_STEP(4);
+    else AGPU_DELTA_STEP(8);
+#undef AGPU_DELTA_STEP
 }
 
 int32_t check(agpu_ctx *ctx, const DeltaArgs &a) {
@@ -329,16 +415,10 @@ int32_t delta_step_launch(agpu_ctx *ctx, const DeltaArgs &a) {
     int32_t rc = check(ctx, a);
     if (rc != AGPU_OK) return rc;
     if (a.new_len != 1) return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "gated_delta: the step takes one token per sequence");
-    const DeltaShape &s = a.s;
-    const dim3 grid((unsigned)s.heads, (unsigned)a.batch), block(kStepThreads);
-    const size_t lds = (size_t)(s.rank_ap() + s.rank_gp()) * sizeof(float);
-    const int nf = ceil_div(s.state_row(), 64);
-#define AGPU_DELTA_STEP(NF) \
-    hipLaunchKernelGGL(delta_step_kernel<NF>, grid, block, lds, ctx->stream, a, s.channels(), s.rank_ap(), s.rank_gp(), s.state_row())
-    if (nf <= 1) AGPU_DELTA_STEP(1);
-    else if (nf <= 2) AGPU_DELTA_STEP(2);
-    else AGPU_DELTA_STEP(4);
-#undef AGPU_DELTA_STEP
+    const int nf = ceil_div(a.s.state_row(), 64);
+    if (nf <= 1) step_run<1>(ctx, a);
+    else if (nf <= 2) step_run<2>(ctx, a);
+    else step_run<4>(ctx, a);
     return AGPU_LAUNCH_CHECK(ctx, "delta_step_kernel");
 }
 
@@ -347,7 +427,9 @@ int32_t delta_prefill_launch(agpu_ctx *ctx, const DeltaArgs &a) {
     if (rc != AGPU_OK) return rc;
     const DeltaShape &s = a.s;
     const unsigned rows = (unsigned)(a.batch * a.new_len);
-    hipLaunchKernelGGL(delta_prepare_kernel, dim3(rows), dim3(256), 0, ctx->stream, a, s.channels());
+    const int qk_parts = ceil_div(s.kv_heads, 4), v_parts = ceil_div(s.heads * s.vdim, kPrepareWidth), g_parts = ceil_div(s.heads * s.state_row(), kPrepareWidth);
+    hipLaunchKernelGGL(delta_prepare_kernel, dim3(rows, (unsigned)(qk_parts + v_parts + g_parts)), dim3(256), 0, ctx->stream, a, s.channels(), s.state_row(),
+                       qk_parts, v_parts);
     if ((rc = AGPU_LAUNCH_CHECK(ctx, "delta_prepare_kernel")) != AGPU_OK) return rc;
     hipLaunchKernelGGL(delta_ring_kernel, dim3((unsigned)ceil_div(s.channels(), 256), (unsigned)s.taps, (unsigned)a.batch), dim3(256), 0, ctx->stream, a,
                        s.channels());

@@ -13,7 +13,7 @@ struct LatentShape {
     int rotp() const { return (rot + 7) / 8 * 8; }
     int vdimp() const { return (vdim + 31) / 32 * 32; }
     int rankp() const { return (rank + 31) / 32 * 32; }
-    int cache_row() const { return rankp() + rotp(); }              // [latent | rotated key part], zero padded
+    int cache_row() const { return rankp() + (rot + 31) / 32 * 32; }  // [latent | rotated key part], zero padded
     int query_row() const { return (dimp() + rotp() + 15) / 16 * 16; }  // one head's bf16 query in the tiled kernel
 };
 
@@ -40,7 +40,7 @@ struct LatentArgs {
     void *out = nullptr;          // [rows], stride ldo: heads x vdim, bf16 or fp32
     int ldo = 0, out_bf16 = 0;
     // scratch
-    float *qlat = nullptr;      // absorbed: rows * heads * cache_row
+    void *qlat = nullptr;       // absorbed: rows * heads * cache_row floats
     float *partial = nullptr;   // absorbed: latent_partial_floats
     uint16_t *qb = nullptr;     // tiled: rows * heads * query_row
     uint16_t *kx = nullptr;     // tiled: [batch][kv_max][heads * dimp]

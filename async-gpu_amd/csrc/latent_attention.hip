@@ -1,8 +1,10 @@
 // Latent attention (latent_attention.h).  Two forms of the same mathematics:
 //
 // absorbed (decode, short portions, fp32 models): the query of a head goes through W_uk^T once and then meets the cached
-//   latents directly, so the cache is read as it is, once per four heads.  Launches: prepare (cache row, absorbed and
-//   rotated queries) -> attend (keys split over workgroups) -> merge with the sink, then W_uv.
+//   latents directly, so the cache is read as it is.  Launches: absorb (cache row, absorbed and rotated queries) -> attend
+//   (keys split over workgroups) -> merge with the sink, then W_uv.  With a bf16 cache 16 heads meet the cache on the bf16
+//   matrix cores, queries and probabilities as two bf16 pieces each (16 bits of mantissa); with an fp32 cache, or a latent
+//   too wide for the LDS, four heads at a time on fp32 FMAs.
 // tiled (prompts of a bf16 model): keys and transposed values of every head are expanded by two GEMMs, then S^T = K Q^T and
 //   O^T = V^T P^T on v_mfma_f32_32x32x16_bf16 with an online softmax.  The key rows of a tile are dealt to the rows of
 //   the first product so that the probabilities come out as the second product's operand: row i of a 32-key tile is key
@@ -14,11 +16,13 @@
 namespace {
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef float f32x4 __attribute__((ext_vector_type(4)));
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 
 constexpr int kHeadTile = 4;    // heads per workgroup of the absorbed kernel (one softmax per wave)
 constexpr int kKeyChunk = 64;   // keys per step: one per lane
 constexpr int kMaxSplits = 64;
+constexpr int kMatrixHeads = 16;  // heads per workgroup of the matrix-core kernel
 constexpr float kMinusInf = -3.0e38f;
 
 __global__ void rope_table_kernel(float2 *table, int positions, int half, double base) {
@@ -46,10 +50,10 @@ __device__ __forceinline__ uint16_t to_cache<uint16_t>(float v) { return f32_to_
 
 // The cache row of one token: normed latent and rotated key part.  256 threads.
 template <typename CT>
-__device__ __forceinline__ void write_cache_row(const LatentArgs &a, const LatentShape &s, int rankp, int rotp, int row, int pos, float *red) {
+__device__ __forceinline__ void write_cache_row(const LatentArgs &a, const LatentShape &s, int rankp, int row_len, int row, int pos, float *red) {
     const int t = threadIdx.x, b = row / a.new_len;
     const float *src = a.down + (size_t)row * a.ld;
-    CT *dst = (CT *)a.cache + ((size_t)b * a.positions + pos) * (rankp + rotp);
+    CT *dst = (CT *)a.cache + ((size_t)b * a.positions + pos) * row_len;
     float sum = 0.0f;
     for (int k = t; k < s.rank; k += 256) sum += src[k] * src[k];
     sum = wave_sum(sum);
@@ -58,56 +62,74 @@ __device__ __forceinline__ void write_cache_row(const LatentArgs &a, const Laten
     const float rs = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)s.rank + s.eps);
     for (int k = t; k < rankp; k += 256) dst[k] = to_cache<CT>(k < s.rank ? src[k] * rs * a.w.norm[k] : 0.0f);
     const float2 *cs = a.w.rope + (size_t)pos * (s.rot_dims >> 1);
-    for (int i = t; i < rotp; i += 256) dst[rankp + i] = to_cache<CT>(i < s.rot ? rotated(src + s.rank, i, s.rot_dims, cs) : 0.0f);
+    for (int i = t; i < row_len - rankp; i += 256) dst[rankp + i] = to_cache<CT>(i < s.rot ? rotated(src + s.rank, i, s.rot_dims, cs) : 0.0f);
 }
 
-// grid (1 + heads, rows): block 0 writes the cache row, block 1 + h the absorbed query of head h.
+// A query value for the attend kernel: fp32, or two bf16 pieces whose sum carries 16 bits of its mantissa.
 template <typename CT>
-__global__ __launch_bounds__(256) void latent_absorb_kernel(LatentArgs a, int rankp, int rotp, int dimp) {
-    __shared__ float sq[1024];       // the head's unrotated query
-    __shared__ float part[256 * 8];  // partial sums [group of d][rankp]
+__device__ __forceinline__ void put_query(void *qlat, size_t at, size_t pieces, float v);
+template <>
+__device__ __forceinline__ void put_query<float>(void *qlat, size_t at, size_t, float v) { ((float *)qlat)[at] = v; }
+template <>
+__device__ __forceinline__ void put_query<uint16_t>(void *qlat, size_t at, size_t pieces, float v) {
+    const uint16_t hi = f32_to_bf16(v);
+    ((uint16_t *)qlat)[at] = hi;
+    ((uint16_t *)qlat)[pieces + at] = f32_to_bf16(v - bf16_to_f32(hi));
+}
+
+// grid (1 + heads * ceil(rankp / 128), rows): block 0 writes the cache row, the others 128 columns of a head's absorbed query.
+// QT: how the attend kernel reads queries (uint16_t: bf16 pieces).
+template <typename CT, typename QT>
+__global__ __launch_bounds__(256) void latent_absorb_kernel(LatentArgs a, int rankp, int row_len, int dimp, int col_blocks) {
+    __shared__ float part[16][128];
     __shared__ float red[4];
     const LatentShape &s = a.s;
     const int t = threadIdx.x, row = blockIdx.y;
     const int pos = *a.pos_dev + row % a.new_len;
     if (blockIdx.x == 0) {
-        write_cache_row<CT>(a, s, rankp, rotp, row, pos, red);
+        write_cache_row<CT>(a, s, rankp, row_len, row, pos, red);
         return;
     }
-    const int h = blockIdx.x - 1;
+    const int h = (blockIdx.x - 1) / col_blocks, cb = (blockIdx.x - 1) % col_blocks;
     const float *q = a.q + (size_t)row * a.ld + (size_t)h * (s.dim + s.rot);
-    float *dst = a.qlat + ((size_t)row * s.heads + h) * (rankp + rotp);
-    const float2 *cs = a.w.rope + (size_t)pos * (s.rot_dims >> 1);
-    for (int i = t; i < s.dim; i += 256) sq[i] = q[i];
-    for (int i = t; i < rotp; i += 256) dst[rankp + i] = i < s.rot ? rotated(q + s.dim, i, s.rot_dims, cs) : 0.0f;
-    __syncthreads();
-    for (int base = 0; base < rankp; base += 2048) {  // 8 columns per thread, 256 threads at most side by side
-        const int width = min(rankp - base, 2048), lanes = width >> 3, groups = 256 / lanes;
-        const int g = t / lanes, c8 = (t % lanes) * 8;
-        float acc[8] = {0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f};
-        if (g < groups) {
-            const uint16_t *w = a.w.uk + (size_t)h * dimp * rankp + base + c8;
-#pragma unroll 4
-            for (int d = g; d < s.dim; d += groups) {
-                const uint4 v = *(const uint4 *)(w + (size_t)d * rankp);
-                const float x = sq[d];
-                const uint32_t u[4] = {v.x, v.y, v.z, v.w};
+    const size_t at = ((size_t)row * s.heads + h) * row_len, pieces = (size_t)gridDim.y * s.heads * row_len;
+    // 16 lanes take the columns, 16 groups the query's dimensions; loads are clamped, not skipped
+    const int c = cb * 128 + (t & 15) * 8, g = t >> 4;
+    const uint16_t *w = a.w.uk + (size_t)h * dimp * rankp + min(c, rankp - 8);
+    float acc[8] = {0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll 1
+    for (int d0 = g; d0 < s.dim; d0 += 16 * 8) {
+        uint4 v[8];
+        float x[8];
 #pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    acc[2 * e] = fmaf(__uint_as_float(u[e] << 16), x, acc[2 * e]);
-                    acc[2 * e + 1] = fmaf(__uint_as_float(u[e] & 0xffff0000u), x, acc[2 * e + 1]);
-                }
+        for (int u = 0; u < 8; ++u) {
+            const int d = min(d0 + 16 * u, s.dim - 1);
+            v[u] = *(const uint4 *)(w + (size_t)d * rankp);
+            x[u] = d0 + 16 * u < s.dim ? q[d] : 0.0f;
+        }
+#pragma unroll
+        for (int u = 0; u < 8; ++u) {
+            const uint32_t p[4] = {v[u].x, v[u].y, v[u].z, v[u].w};
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                acc[2 * e] = fmaf(__uint_as_float(p[e] << 16), x[u], acc[2 * e]);
+                acc[2 * e + 1] = fmaf(__uint_as_float(p[e] & 0xffff0000u), x[u], acc[2 * e + 1]);
             }
+        }
+    }
+    *(float4 *)&part[g][(t & 15) * 8] = make_float4(acc[0], acc[1], acc[2], acc[3]);
+    *(float4 *)&part[g][(t & 15) * 8 + 4] = make_float4(acc[4], acc[5], acc[6], acc[7]);
+    if (cb == 0) {
+        const float2 *cs = a.w.rope + (size_t)pos * (s.rot_dims >> 1);
+        for (int i = t; i < row_len - rankp; i += 256)
+            put_query<QT>(a.qlat, at + rankp + i, pieces, i < s.rot ? rotated(q + s.dim, i, s.rot_dims, cs) : 0.0f);
+    }
+    __syncthreads();
+    if (t < 128 && cb * 128 + t < rankp) {
+        float v = 0.0f;
 #pragma unroll
-            for (int e = 0; e < 8; ++e) part[(size_t)g * width + c8 + e] = acc[e];
-        }
-        __syncthreads();
-        for (int c = t; c < width; c += 256) {
-            float v = 0.0f;
-            for (int i = 0; i < groups; ++i) v += part[(size_t)i * width + c];
-            dst[base + c] = v;
-        }
-        __syncthreads();
+        for (int i = 0; i < 16; ++i) v += part[i][t];
+        put_query<QT>(a.qlat, at + cb * 128 + t, pieces, v);
     }
 }
 
@@ -161,13 +183,27 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(LatentArgs a, const 
         const int k0 = ck * kKeyChunk;
         const CT *mine = cache + (size_t)min(k0 + lane, kv - 1) * row_len;
         float part[kHeadTile] = {0.0f, 0.0f, 0.0f, 0.0f};
-        for (int c = wave * 8; c < row_len; c += 32) {
-            float v[8];
-            load8(mine + c, v);
+        constexpr int U = 3;  // requests in flight; row_len is a multiple of 32, so every wave has row_len / 32 of them
+        int c = wave * 8;
+        auto add = [&](int at, const float (&v)[8]) {
 #pragma unroll
             for (int i = 0; i < kHeadTile; ++i)
 #pragma unroll
-                for (int e = 0; e < 8; ++e) part[i] = fmaf(q[i][c + e], v[e], part[i]);
+                for (int e = 0; e < 8; ++e) part[i] = fmaf(q[i][at + e], v[e], part[i]);
+        };
+#pragma unroll 1
+        for (; c + 32 * (U - 1) < row_len; c += 32 * U) {
+            float v[U][8];
+#pragma unroll
+            for (int u = 0; u < U; ++u) load8(mine + c + 32 * u, v[u]);
+#pragma unroll
+            for (int u = 0; u < U; ++u) add(c + 32 * u, v[u]);
+        }
+#pragma unroll 1
+        for (; c < row_len; c += 32) {
+            float v[8];
+            load8(mine + c, v);
+            add(c, v);
         }
 #pragma unroll
         for (int i = 0; i < kHeadTile; ++i) sc[wave][i][lane] = part[i];
@@ -194,7 +230,8 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(LatentArgs a, const 
                 acc[i][j][1] *= cr;
             }
         }
-#pragma unroll 4
+        constexpr int KU = NI <= 4 ? 16 / NI : 2;  // rows requested at a time
+#pragma unroll KU
         for (int kk = 0; kk < 16; ++kk) {
             const int key = wave * 16 + kk;
             const CT *vr = cache + (size_t)min(k0 + key, kv - 1) * row_len;
@@ -203,7 +240,7 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(LatentArgs a, const 
 #pragma unroll
             for (int j = 0; j < NI; ++j) {
                 const int c = 2 * lane + 128 * j;
-                const float2 v = c < rankp ? load2(vr + c) : make_float2(0.0f, 0.0f);
+                const float2 v = load2(vr + min(c, rankp - 2));  // columns beyond the latent are dropped below
 #pragma unroll
                 for (int i = 0; i < kHeadTile; ++i) {
                     acc[i][j][0] = fmaf(pv[i], v.x, acc[i][j][0]);
@@ -232,45 +269,212 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(LatentArgs a, const 
         *(float2 *)(part_ml + (((size_t)row * s.heads + h0 + wave) * splits + blockIdx.x) * 2) = make_float2(m, l);
 }
 
+// grid (splits, ceil(heads / 16), rows), four waves; bf16 cache.  A chunk of 64 cache rows goes to LDS; wave w scores keys
+// 16 w .. + 15 for 16 heads (v_mfma_f32_16x16x32_bf16, queries as two pieces), 16 threads per head do the softmax, and the
+// waves share the latent's columns of the second product (probabilities as two pieces).  CT column tiles of 16 per wave.
+template <int CT>
+__global__ __launch_bounds__(256) void latent_attend_matrix_kernel(LatentArgs a, int rankp, int row_len, int splits) {
+    extern __shared__ __align__(16) uint16_t tile[];  // [64][ld], then the queries [2][16][ld]
+    __shared__ float sc[kMatrixHeads][kKeyChunk + 4];
+    __shared__ __align__(16) uint16_t pr[2][kMatrixHeads][kKeyChunk + 8];
+    __shared__ float corr[kMatrixHeads];
+    const LatentShape &s = a.s;
+    const int t = threadIdx.x, lane = t & 63, wave = t >> 6, lr = lane & 15, lq = lane >> 4;
+    const int row = blockIdx.z, h0 = blockIdx.y * kMatrixHeads, b = row / a.new_len, ld = row_len + 8, n32 = row_len >> 5;
+    const int kv = *a.pos_dev + row % a.new_len + 1;
+    const int chunks = (kv + kKeyChunk - 1) / kKeyChunk;
+    const int per = (chunks + splits - 1) / splits;
+    const int c_lo = min((int)blockIdx.x * per, chunks), c_hi = min(c_lo + per, chunks);
+    const uint16_t *cache = (const uint16_t *)a.cache + (size_t)b * a.positions * row_len;
+    uint16_t *sq = tile + kKeyChunk * ld;
+    const size_t pieces = (size_t)gridDim.z * s.heads * row_len;
+    if (c_lo < c_hi) {  // 16 threads per head
+        const int h = t >> 4;
+        const uint16_t *q = (const uint16_t *)a.qlat + ((size_t)row * s.heads + min(h0 + h, s.heads - 1)) * row_len;
+#pragma unroll 4
+        for (int c = (t & 15) * 8; c < row_len; c += 128) {
+            const uint4 hi = *(const uint4 *)(q + c), lo = *(const uint4 *)(q + pieces + c);
+            *(uint4 *)(sq + h * ld + c) = hi;
+            *(uint4 *)(sq + (kMatrixHeads + h) * ld + c) = lo;
+        }
+    }
+    f32x4 acc[CT];
+#pragma unroll
+    for (int i = 0; i < CT; ++i) acc[i] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+    float m = kMinusInf, l = 0.0f;  // of head h0 + t / 16
+    for (int ck = c_lo; ck < c_hi; ++ck) {
+        const int k0 = ck * kKeyChunk;
+        {  // four threads per key
+            const uint16_t *src = cache + (size_t)min(k0 + (t >> 2), kv - 1) * row_len + (t & 3) * 8;
+            uint16_t *dst = tile + (t >> 2) * ld + (t & 3) * 8;
+            constexpr int U = 9;
+#pragma unroll 1
+            for (int n = 0; n < n32; n += U) {
+                uint4 v[U];
+#pragma unroll
+                for (int u = 0; u < U; ++u) v[u] = *(const uint4 *)(src + min(n + u, n32 - 1) * 32);
+#pragma unroll
+                for (int u = 0; u < U; ++u) *(uint4 *)(dst + min(n + u, n32 - 1) * 32) = v[u];
+            }
+        }
+        __syncthreads();
+        f32x4 sv = {0.0f, 0.0f, 0.0f, 0.0f};
+        {
+            const uint16_t *kp = tile + (wave * 16 + lr) * ld + lq * 8, *qh = sq + lr * ld + lq * 8, *ql = qh + kMatrixHeads * ld;
+            f32x4 s2 = sv;
+            auto fma_step = [&](int n, f32x4 &c) {
+                const bf16x8 kf = *(const bf16x8 *)(kp + n * 32), qlo = *(const bf16x8 *)(ql + n * 32), qhi = *(const bf16x8 *)(qh + n * 32);
+                c = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qlo, kf, c, 0, 0, 0);
+                c = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qhi, kf, c, 0, 0, 0);
+            };
+            int n = 0;
+            for (; n + 1 < n32; n += 2) {
+                fma_step(n, sv);
+                fma_step(n + 1, s2);
+            }
+            if (n < n32) fma_step(n, sv);
+            sv += s2;
+        }
+        // result register r of lane l: head 4 (l / 16) + r, key l % 16
+#pragma unroll
+        for (int r = 0; r < 4; ++r) sc[lq * 4 + r][wave * 16 + lr] = sv[r] * s.scale;
+        __syncthreads();
+        {
+            const int h = t >> 4;
+            float v[4], top = kMinusInf;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                v[e] = k0 + lr + 16 * e < kv ? sc[h][lr + 16 * e] : kMinusInf;
+                top = fmaxf(top, v[e]);
+            }
+            const float m_new = fmaxf(m, row16_max(top));
+            float sum = 0.0f;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const float p = v[e] > kMinusInf ? expf(v[e] - m_new) : 0.0f;
+                sum += p;
+                const uint16_t hi = f32_to_bf16(p);
+                pr[0][h][lr + 16 * e] = hi;
+                pr[1][h][lr + 16 * e] = f32_to_bf16(p - bf16_to_f32(hi));
+            }
+            const float cr = expf(m - m_new);
+            l = l * cr + row16_sum(sum);
+            m = m_new;
+            if (lr == 0) corr[h] = cr;
+        }
+        __syncthreads();
+        float cr[4];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) cr[r] = corr[lq * 4 + r];
+        bf16x8 pf[2][2];
+#pragma unroll
+        for (int st = 0; st < 2; ++st)
+#pragma unroll
+            for (int pc = 0; pc < 2; ++pc) pf[st][pc] = *(const bf16x8 *)&pr[pc][lr][32 * st + 8 * lq];
+#pragma unroll
+        for (int i = 0; i < CT; ++i) {
+            const int c = (wave + 4 * i) * 16;
+            if (c >= rankp) continue;
+#pragma unroll
+            for (int r = 0; r < 4; ++r) acc[i][r] *= cr[r];
+#pragma unroll
+            for (int st = 0; st < 2; ++st) {
+                const uint16_t *vp = tile + (32 * st + 8 * lq) * ld + c + lr;
+                uint32_t w[4];
+#pragma unroll
+                for (int e = 0; e < 4; ++e) w[e] = (uint32_t)vp[2 * e * ld] | ((uint32_t)vp[(2 * e + 1) * ld] << 16);
+                const bf16x8 vf = __builtin_bit_cast(bf16x8, make_uint4(w[0], w[1], w[2], w[3]));
+                acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf[st][1], vf, acc[i], 0, 0, 0);
+                acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf[st][0], vf, acc[i], 0, 0, 0);
+            }
+        }
+        __syncthreads();  // the next chunk overwrites the tile
+    }
+    float *part_o = a.partial;
+    float *part_ml = a.partial + (size_t)gridDim.z * s.heads * splits * rankp;
+#pragma unroll
+    for (int i = 0; i < CT; ++i) {
+        const int c = (wave + 4 * i) * 16 + lr;
+        if (c >= rankp) continue;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int h = h0 + lq * 4 + r;
+            if (h < s.heads) part_o[(((size_t)row * s.heads + h) * splits + blockIdx.x) * rankp + c] = acc[i][r];
+        }
+    }
+    if (lr == 0 && h0 + (t >> 4) < s.heads)
+        *(float2 *)(part_ml + (((size_t)row * s.heads + h0 + (t >> 4)) * splits + blockIdx.x) * 2) = make_float2(m, l);
+}
+
+size_t matrix_lds_bytes(const LatentShape &s) { return (size_t)(kKeyChunk + 2 * kMatrixHeads) * (s.cache_row() + 8) * 2; }
+// 12 KiB of the 160 KiB are the kernel's static arrays.
+bool matrix_supported(const LatentShape &s) { return matrix_lds_bytes(s) <= 148 * 1024; }
+
 // grid (ceil(vdim / 32), heads, rows): merges the key splits of a head, adds the sink to the denominator, applies W_uv.
 __global__ __launch_bounds__(256) void latent_merge_kernel(LatentArgs a, int rankp, int vdimp, int splits) {
-    extern __shared__ float olat[];  // [rankp]
+    extern __shared__ float olat[];  // [4][rankp]: one quarter of the splits each, then their sum
     __shared__ float wt[kMaxSplits];
-    __shared__ float inv;
     const LatentShape &s = a.s;
     const int t = threadIdx.x, h = blockIdx.y, row = blockIdx.z;
-    const int lane = t & 63, wave = t >> 6;
+    const int lane = t & 63, wave = t >> 6, sub = lane >> 4, kl = lane & 15;
     const size_t at = ((size_t)row * s.heads + h) * splits;
     const float *part_o = a.partial + at * rankp;
     const float *part_ml = a.partial + (size_t)gridDim.z * s.heads * splits * rankp + at * 2;
-    if (wave == 0) {
-        const float2 ml = lane < splits ? *(const float2 *)(part_ml + 2 * lane) : make_float2(kMinusInf, 0.0f);
-        const float sink = a.w.sink ? a.w.sink[h] : kMinusInf;
-        const float top = fmaxf(wave_max(ml.x), sink);
-        const float w = expf(ml.x - top);
-        if (lane < kMaxSplits) wt[lane] = w;
-        const float sum = wave_sum(w * ml.y) + expf(sink - top);
-        if (lane == 0) inv = 1.0f / sum;
+    // this thread's rows of W_uv, the first 512 columns: two rows of 16 lanes
+    const uint16_t *wv = a.w.uv + ((size_t)h * vdimp + blockIdx.x * 32 + wave * 4 + sub) * rankp;
+    uint4 first[2][4];
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) first[i][j] = *(const uint4 *)(wv + (size_t)i * 16 * rankp + min(kl * 8 + 128 * j, rankp - 8));
+    // every wave for itself: the weights of the splits
+    const float2 ml = lane < splits ? *(const float2 *)(part_ml + 2 * lane) : make_float2(kMinusInf, 0.0f);
+    const float sink = a.w.sink ? a.w.sink[h] : kMinusInf;
+    const float top = fmaxf(wave_max(ml.x), sink);
+    const float w = expf(ml.x - top);
+    const float inv = 1.0f / (wave_sum(w * ml.y) + expf(sink - top));
+    if (wave == 0) wt[lane] = w * inv;
+    __syncthreads();
+    for (int c = lane * 4; c < rankp; c += 256) {
+        float4 v = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+#pragma unroll 4
+        for (int i = wave; i < splits; i += 4) {
+            const float4 o = *(const float4 *)(part_o + (size_t)i * rankp + c);
+            const float f = wt[i];
+            v.x = fmaf(f, o.x, v.x);
+            v.y = fmaf(f, o.y, v.y);
+            v.z = fmaf(f, o.z, v.z);
+            v.w = fmaf(f, o.w, v.w);
+        }
+        *(float4 *)(olat + wave * rankp + c) = v;
     }
     __syncthreads();
-    for (int c = t; c < rankp; c += 256) {
-        float v = 0.0f;
-        for (int i = 0; i < splits; ++i) v = fmaf(wt[i], part_o[(size_t)i * rankp + c], v);
-        olat[c] = v * inv;
-    }
+    for (int c = t; c < rankp; c += 256) olat[c] += olat[rankp + c] + olat[2 * rankp + c] + olat[3 * rankp + c];
     __syncthreads();
-    const int sub = lane >> 4, kl = lane & 15;
-    for (int r = wave * 4 + sub; r < 32; r += 16) {
-        const int dv = blockIdx.x * 32 + r;  // < vdimp
-        const uint16_t *w = a.w.uv + ((size_t)h * vdimp + dv) * rankp;
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
         float acc = 0.0f;
-        for (int c = kl * 8; c < rankp; c += 128) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int c = kl * 8 + 128 * j;
+            const uint32_t u[4] = {first[i][j].x, first[i][j].y, first[i][j].z, first[i][j].w};
+            float part = 0.0f;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                part = fmaf(__uint_as_float(u[e] << 16), olat[min(c, rankp - 8) + 2 * e], part);
+                part = fmaf(__uint_as_float(u[e] & 0xffff0000u), olat[min(c, rankp - 8) + 2 * e + 1], part);
+            }
+            acc += c < rankp ? part : 0.0f;
+        }
+#pragma unroll 1
+        for (int c = kl * 8 + 512; c < rankp; c += 128) {
             float v[8];
-            load8(w + c, v);
+            load8(wv + (size_t)i * 16 * rankp + c, v);
 #pragma unroll
             for (int e = 0; e < 8; ++e) acc = fmaf(v[e], olat[c + e], acc);
         }
         acc = row16_sum(acc);
+        const int dv = blockIdx.x * 32 + i * 16 + wave * 4 + sub;
         if (kl == 0 && dv < s.vdim) {
             const size_t o = (size_t)row * a.ldo + (size_t)h * s.vdim + dv;
             if (a.out_bf16) ((uint16_t *)a.out)[o] = f32_to_bf16(acc);
@@ -280,11 +484,11 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(LatentArgs a, int ran
 }
 
 // One workgroup per row: the cache row and the bf16 queries of every head.
-__global__ __launch_bounds__(256) void latent_tiled_prepare_kernel(LatentArgs a, int rankp, int rotp, int dimp, int query_row) {
+__global__ __launch_bounds__(256) void latent_tiled_prepare_kernel(LatentArgs a, int rankp, int row_len, int dimp, int query_row) {
     __shared__ float red[4];
     const LatentShape &s = a.s;
     const int row = blockIdx.x, pos = *a.pos_dev + row % a.new_len;
-    write_cache_row<uint16_t>(a, s, rankp, rotp, row, pos, red);
+    write_cache_row<uint16_t>(a, s, rankp, row_len, row, pos, red);
     const float2 *cs = a.w.rope + (size_t)pos * (s.rot_dims >> 1);
     const float *q = a.q + (size_t)row * a.ld;
     uint16_t *dst = a.qb + (size_t)row * s.heads * query_row;
@@ -301,8 +505,8 @@ __global__ __launch_bounds__(256) void latent_tiled_prepare_kernel(LatentArgs a,
 // One wave = 32 queries of a head; SPLIT: the four waves of a workgroup share one query block's key tiles (and merge),
 // else each wave has its own query block.  DQ steps of 16 query dimensions, DV tiles of 32 value dimensions.
 template <int DQ, int DV, bool SPLIT>
-__global__ __launch_bounds__(256, 1) void latent_tiled_kernel(LatentArgs a, int rankp, int rotp, int dimp, int vdimp, int query_row, int kv_stride,
-                                                              int blocks) {
+__global__ __launch_bounds__(256, 1) void latent_tiled_kernel(LatentArgs a, int rankp, int row_len, int rotp, int dimp, int vdimp, int query_row,
+                                                              int kv_stride, int blocks) {
     extern __shared__ float shm[];
     const LatentShape &s = a.s;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, li = lane & 31, lh = lane >> 5;
@@ -315,7 +519,7 @@ __global__ __launch_bounds__(256, 1) void latent_tiled_kernel(LatentArgs a, int 
     const int qi = q0 + li;
     const int last_key = pos + min(q0 + 31, T - 1);
     const int tiles = active ? last_key / 32 + 1 : 0;
-    const int row_len = rankp + rotp, ldk = s.heads * dimp;
+    const int ldk = s.heads * dimp;
     const uint16_t *qp = a.qb + ((size_t)(b * T + min(qi, T - 1)) * s.heads + h) * query_row;
     bf16x8 qf[DQ];
 #pragma unroll
@@ -456,12 +660,23 @@ int32_t attend_run(agpu_ctx *ctx, const LatentArgs &a, int rows, int splits) {
     const LatentShape &s = a.s;
     const dim3 grid((unsigned)splits, (unsigned)ceil_div(s.heads, kHeadTile), (unsigned)rows), block(256);
     const int ni = ceil_div(s.rankp(), 128);
-    if (ni <= 1) hipLaunchKernelGGL((latent_attend_kernel<CT, 1>), grid, block, 0, ctx->stream, a, a.qlat, s.rankp(), s.cache_row(), splits);
-    else if (ni <= 2) hipLaunchKernelGGL((latent_attend_kernel<CT, 2>), grid, block, 0, ctx->stream, a, a.qlat, s.rankp(), s.cache_row(), splits);
-    else if (ni <= 4) hipLaunchKernelGGL((latent_attend_kernel<CT, 4>), grid, block, 0, ctx->stream, a, a.qlat, s.rankp(), s.cache_row(), splits);
-    else if (ni <= 8) hipLaunchKernelGGL((latent_attend_kernel<CT, 8>), grid, block, 0, ctx->stream, a, a.qlat, s.rankp(), s.cache_row(), splits);
+    if (ni <= 1) hipLaunchKernelGGL((latent_attend_kernel<CT, 1>), grid, block, 0, ctx->stream, a, (const float *)a.qlat, s.rankp(), s.cache_row(), splits);
+    else if (ni <= 2) hipLaunchKernelGGL((latent_attend_kernel<CT, 2>), grid, block, 0, ctx->stream, a, (const float *)a.qlat, s.rankp(), s.cache_row(), splits);
+    else if (ni <= 4) hipLaunchKernelGGL((latent_attend_kernel<CT, 4>), grid, block, 0, ctx->stream, a, (const float *)a.qlat, s.rankp(), s.cache_row(), splits);
+    else if (ni <= 8) hipLaunchKernelGGL((latent_attend_kernel<CT, 8>), grid, block, 0, ctx->stream, a, (const float *)a.qlat, s.rankp(), s.cache_row(), splits);
     else return agpu_fail(ctx, AGPU_ERR_UNSUPPORTED, "latent_attention: latent size %d exceeds 1024", s.rank);
     return AGPU_LAUNCH_CHECK(ctx, "latent_attend_kernel");
+}
+
+template <int CT>
+int32_t attend_matrix_run(agpu_ctx *ctx, const LatentArgs &a, int rows, int splits) {
+    const LatentShape &s = a.s;
+    const size_t lds = matrix_lds_bytes(s);
+    if (lds > 48 * 1024)
+        (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&latent_attend_matrix_kernel<CT>), hipFuncAttributeMaxDynamicSharedMemorySize, 148 * 1024);
+    hipLaunchKernelGGL(latent_attend_matrix_kernel<CT>, dim3((unsigned)splits, (unsigned)ceil_div(s.heads, kMatrixHeads), (unsigned)rows), dim3(256), lds,
+                       ctx->stream, a, s.rankp(), s.cache_row(), splits);
+    return AGPU_LAUNCH_CHECK(ctx, "latent_attend_matrix_kernel");
 }
 
 template <int DQ, int DV>
@@ -475,10 +690,10 @@ int32_t tiled_run(agpu_ctx *ctx, const LatentArgs &a) {
             (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&latent_tiled_kernel<DQ, DV, true>), hipFuncAttributeMaxDynamicSharedMemorySize,
                                       160 * 1024);
         hipLaunchKernelGGL((latent_tiled_kernel<DQ, DV, true>), dim3((unsigned)blocks, (unsigned)s.heads, (unsigned)a.batch), dim3(256), lds, ctx->stream,
-                           a, s.rankp(), s.rotp(), s.dimp(), s.vdimp(), s.query_row(), kvs, blocks);
+                           a, s.rankp(), s.cache_row(), s.rotp(), s.dimp(), s.vdimp(), s.query_row(), kvs, blocks);
     } else {
         hipLaunchKernelGGL((latent_tiled_kernel<DQ, DV, false>), dim3((unsigned)ceil_div(blocks, 4), (unsigned)s.heads, (unsigned)a.batch), dim3(256), 0,
-                           ctx->stream, a, s.rankp(), s.rotp(), s.dimp(), s.vdimp(), s.query_row(), kvs, blocks);
+                           ctx->stream, a, s.rankp(), s.cache_row(), s.rotp(), s.dimp(), s.vdimp(), s.query_row(), kvs, blocks);
     }
     return AGPU_LAUNCH_CHECK(ctx, "latent_tiled_kernel");
 }
@@ -503,8 +718,8 @@ int32_t check_shape(agpu_ctx *ctx, const LatentArgs &a) {
 }  // namespace
 
 int latent_splits(const agpu_ctx *ctx, const LatentShape &s, int rows, int kv_max) {
-    const int chunks = ceil_div(kv_max, kKeyChunk), others = ceil_div(s.heads, kHeadTile) * rows;
-    return std::max(1, std::min({chunks, kMaxSplits, ceil_div(2 * ctx->num_cus, others)}));
+    const int chunks = ceil_div(kv_max, kKeyChunk), others = ceil_div(s.heads, kMatrixHeads) * rows;
+    return std::max(1, std::min({chunks, kMaxSplits, ceil_div(ctx->num_cus, others)}));
 }
 
 size_t latent_partial_floats(const LatentShape &s, int rows, int splits) { return (size_t)rows * s.heads * splits * (s.rankp() + 2); }
@@ -521,14 +736,29 @@ int32_t latent_absorbed_launch(agpu_ctx *ctx, const LatentArgs &a) {
     if (rc != AGPU_OK) return rc;
     const LatentShape &s = a.s;
     const int rows = a.batch * a.new_len, splits = latent_splits(ctx, s, rows, a.kv_max);
-    const dim3 grid((unsigned)(1 + s.heads), (unsigned)rows), block(256);
-    if (a.cache_bf16) hipLaunchKernelGGL(latent_absorb_kernel<uint16_t>, grid, block, 0, ctx->stream, a, s.rankp(), s.rotp(), s.dimp());
-    else hipLaunchKernelGGL(latent_absorb_kernel<float>, grid, block, 0, ctx->stream, a, s.rankp(), s.rotp(), s.dimp());
+    const bool matrix = a.cache_bf16 && matrix_supported(s);
+    const int col_blocks = ceil_div(s.rankp(), 128);
+    const dim3 grid((unsigned)(1 + s.heads * col_blocks), (unsigned)rows), block(256);
+#define AGPU_ABSORB(CT, QT) \
+    hipLaunchKernelGGL((latent_absorb_kernel<CT, QT>), grid, block, 0, ctx->stream, a, s.rankp(), s.cache_row(), s.dimp(), col_blocks)
+    if (matrix) AGPU_ABSORB(uint16_t, uint16_t);
+    else if (a.cache_bf16) AGPU_ABSORB(uint16_t, float);
+    else AGPU_ABSORB(float, float);
+#undef AGPU_ABSORB
     if ((rc = AGPU_LAUNCH_CHECK(ctx, "latent_absorb_kernel")) != AGPU_OK) return rc;
-    rc = a.cache_bf16 ? attend_run<uint16_t>(ctx, a, rows, splits) : attend_run<float>(ctx, a, rows, splits);
+    if (matrix) {
+        const int ct = ceil_div(s.rankp(), 64);
+        if (ct <= 2) rc = attend_matrix_run<2>(ctx, a, rows, splits);
+        else if (ct <= 4) rc = attend_matrix_run<4>(ctx, a, rows, splits);
+        else if (ct <= 8) rc = attend_matrix_run<8>(ctx, a, rows, splits);
+        else rc = attend_matrix_run<12>(ctx, a, rows, splits);
+        if (ct > 12) return agpu_fail(ctx, AGPU_ERR_UNSUPPORTED, "latent_attention: latent size %d", s.rank);
+    } else {
+        rc = a.cache_bf16 ? attend_run<uint16_t>(ctx, a, rows, splits) : attend_run<float>(ctx, a, rows, splits);
+    }
     if (rc != AGPU_OK) return rc;
     hipLaunchKernelGGL(latent_merge_kernel, dim3((unsigned)(s.vdimp() / 32), (unsigned)s.heads, (unsigned)rows), dim3(256),
-                       (size_t)s.rankp() * sizeof(float), ctx->stream, a, s.rankp(), s.vdimp(), splits);
+                       (size_t)4 * s.rankp() * sizeof(float), ctx->stream, a, s.rankp(), s.vdimp(), splits);
     return AGPU_LAUNCH_CHECK(ctx, "latent_merge_kernel");
 }
 
@@ -539,7 +769,7 @@ int32_t latent_tiled_launch(agpu_ctx *ctx, const LatentArgs &a) {
     if (rc != AGPU_OK) return rc;
     const LatentShape &s = a.s;
     if (!a.cache_bf16 || !latent_tiled_supported(s)) return agpu_fail(ctx, AGPU_ERR_UNSUPPORTED, "latent_attention: no tiled kernel for this shape");
-    hipLaunchKernelGGL(latent_tiled_prepare_kernel, dim3((unsigned)(a.batch * a.new_len)), dim3(256), 0, ctx->stream, a, s.rankp(), s.rotp(), s.dimp(),
+    hipLaunchKernelGGL(latent_tiled_prepare_kernel, dim3((unsigned)(a.batch * a.new_len)), dim3(256), 0, ctx->stream, a, s.rankp(), s.cache_row(), s.dimp(),
                        s.query_row());
     if ((rc = AGPU_LAUNCH_CHECK(ctx, "latent_tiled_prepare_kernel")) != AGPU_OK) return rc;
     const int kvs = latent_kv_stride(a.kv_max);

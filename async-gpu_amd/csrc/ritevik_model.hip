@@ -265,8 +265,8 @@ int32_t build_layer(agpu_ritevik *m, int i) {
         AGPU_TRY(add_vec(m, p + "mix.A_log", &L.a_log, 1, c.heads));
         AGPU_TRY(add_vec(m, p + "mix.dt_bias", &L.dt_bias, 1, (int64_t)c.heads * c.dim));
         AGPU_TRY(add_vec(m, p + "mix.norm", &L.mix_norm, 1, c.vdim));
-        AGPU_TRY(new_mat(m, L.a2, c.heads * c.dim, s.rank_ap()));
-        add_rows(m, p + "mix.a2", L.a2, 0, 0, (int64_t)c.heads * c.dim, c.decay_rank);
+        AGPU_TRY(new_mat(m, L.a2, c.heads * s.state_row(), s.rank_ap()));
+        add_head_rows(m, p + "mix.a2", L.a2, c.heads, c.dim, s.state_row(), c.decay_rank);
         AGPU_TRY(new_mat(m, L.g2, nv, s.rank_gp()));
         add_rows(m, p + "mix.g2", L.g2, 0, 0, nv, c.gate_rank);
         L.dw.conv = L.conv; L.dw.a_log = L.a_log; L.dw.dt_bias = L.dt_bias; L.dw.a2 = L.a2.w; L.dw.g2 = L.g2.w; L.dw.norm = L.mix_norm;
@@ -386,7 +386,7 @@ int32_t mixer(agpu_ritevik *m, const Run &r, int B, int new_len, int max_kv, voi
         a.out = cat;
         a.ldo = L.cat_k();
         a.out_bf16 = cat_bf16;
-        a.qlat = (float *)m->qlat.p;
+        a.qlat = m->qlat.p;
         a.partial = (float *)m->partial.p;
         a.qb = (uint16_t *)m->qb.p;
         a.kx = (uint16_t *)m->kx.p;
@@ -419,10 +419,10 @@ int32_t mixer(agpu_ritevik *m, const Run &r, int B, int new_len, int max_kv, voi
             a.o = (float *)m->dout.p;
             // the low-rank products in fp32: they feed decays and gates
             DenseOut og, oo;
-            og.n_plain = og.ldo = L.ds.heads * L.ds.dim;
+            og.n_plain = og.ldo = L.a2.N;
             og.out = a.g;
             AGPU_TRY(dense_gemm_f32_launch(m->ctx, proj + L.col_a1, L.n_plain, L.a2.w, L.a2.K, R, L.a2.N, L.a2.K, og));
-            oo.n_plain = oo.ldo = L.ds.heads * L.ds.vdim;
+            oo.n_plain = oo.ldo = L.g2.N;
             oo.out = a.gate;
             AGPU_TRY(dense_gemm_f32_launch(m->ctx, proj + L.col_g1, L.n_plain, L.g2.w, L.g2.K, R, L.g2.N, L.g2.K, oo));
             AGPU_TRY(delta_prefill_launch(m->ctx, a));
@@ -593,9 +593,9 @@ int32_t agpu_ritevik::ensure_buffers(int B, int new_len, bool all_rows_logits) {
             }
         } else if (new_len > 1) {
             const DeltaShape &s = L.ds;
-            AGPU_TRY(ensure(this, dqk, R * 2 * s.kv_heads * s.dim * f));
+            AGPU_TRY(ensure(this, dqk, R * 2 * s.kv_heads * s.state_row() * f));
             AGPU_TRY(ensure(this, dv, R * s.heads * s.vdim * f));
-            AGPU_TRY(ensure(this, dg, R * s.heads * s.dim * f));
+            AGPU_TRY(ensure(this, dg, R * s.heads * s.state_row() * f));
             AGPU_TRY(ensure(this, dbkq, R * (s.heads + s.kv_heads) * f));
             AGPU_TRY(ensure(this, dgate, R * s.heads * s.vdim * f));
             AGPU_TRY(ensure(this, dout, R * s.heads * s.vdim * f));

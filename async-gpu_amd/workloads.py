@@ -129,3 +129,84 @@ def random_prompt(cfg, seed, length, batch=None):
     rng = np.random.default_rng(seed + 1000)
     shape = (length,) if batch is None else (batch, length)
     return rng.integers(0, cfg["vocab"], size=shape).astype(np.uint32)
+
+
+# Ritevik shapes of the size of a real model's layers, beside the GPT-2 of the same width and number of layer runs.
+# Three delta layers per attention layer; the middle third of the small one runs twice.
+def ritevik_spec(width, heads, head_dim, rot_dim, kv_rank, ff, n_layer, vocab, side_dim, loop=None):
+    latent = dict(type="latent_attention", mlp=dict(kind="dense", ff=ff),
+                  mixer=dict(heads=heads, dim=head_dim, rot_dim=rot_dim, vdim=head_dim, kv_rank=kv_rank, scale=(head_dim + rot_dim) ** -0.5,
+                             rot=dict(base=10000.0, dims=rot_dim)))
+    delta = dict(type="channel_delta", mlp=dict(kind="dense", ff=ff),
+                 mixer=dict(heads=heads, kv_heads=heads, dim=head_dim, vdim=head_dim, conv=4))
+    return dict(architecture="Ritevik", width=width, vocab=vocab, norm=dict(eps=1e-6), token_side=dict(dim=side_dim) if side_dim else None, loop=loop,
+                layers=[latent if i % 4 == 3 else delta for i in range(n_layer)])
+
+
+RITEVIK_SMALL = ritevik_spec(768, 12, 64, 32, 256, 3072, 8, 50257, 64, loop=dict(start=2, stop=6, times=2))  # 12 layer runs
+RITEVIK_LARGE = ritevik_spec(2048, 16, 128, 64, 512, 8192, 24, 50257, 128)
+
+
+def ritevik_tensors(spec, seed, rank=None):
+    """{name: (dtype, array)} of random bf16 weights.  Matrices are cut from one pool of N(0, 1) values scaled to 1 / sqrt(K), so
+    a model of billions of weights takes seconds; `rank` is the low-rank size of the delta layers (default: head dim)."""
+    from .weights import f32_to_bf16
+    rng = np.random.default_rng(seed)
+    pool = rng.standard_normal(1 << 22, dtype=np.float32)
+    out = {}
+
+    def mat(name, rows, cols, gain=1.0):
+        n, lo = rows * cols, int(rng.integers(0, pool.size))
+        base = f32_to_bf16(np.roll(pool, -lo)[: min(n, pool.size)] * np.float32(gain / np.sqrt(cols)))
+        out[name] = ("BF16", np.resize(base, (rows, cols)))
+
+    def vec(name, shape, centre=0.0, spread=0.1):
+        out[name] = ("BF16", f32_to_bf16((centre + spread * rng.standard_normal(shape)).astype(np.float32)))
+
+    d, V, n_layer = spec["width"], spec["vocab"], len(spec["layers"])
+    mat("embed", V, d, np.sqrt(d))
+    vec("embed.norm", d)
+    if spec.get("loop"):
+        mat("loop.in", d, 2 * d)
+        vec("loop.step", (spec["loop"]["times"], d))
+    side = (spec.get("token_side") or {}).get("dim", 0)
+    if side:
+        mat("side.embed", V, n_layer * side, np.sqrt(n_layer * side))
+    for i, e in enumerate(spec["layers"]):
+        p, m = f"l{i}.", e["mixer"]
+        H, D, DV = m["heads"], m["dim"], m["vdim"]
+        vec(p + "norm1", d)
+        if e["type"] == "latent_attention":
+            R, Ck = m["rot_dim"], m["kv_rank"]
+            mat(p + "mix.q", H * (D + R), d)
+            mat(p + "mix.dkv", Ck + R, d)
+            vec(p + "mix.dkv.norm", Ck, 1.0)
+            mat(p + "mix.uk", H * D, Ck)
+            mat(p + "mix.uv", H * DV, Ck)
+            vec(p + "mix.sink", H, 0.0, 1.0)
+        else:
+            r = rank or D
+            for t, ch in (("q", m["kv_heads"] * D), ("k", m["kv_heads"] * D), ("v", H * DV)):
+                mat(p + "mix." + t, ch, d)
+                vec(p + f"mix.{t}.conv", (ch, m["conv"]), 0.0, 0.6)
+            mat(p + "mix.b", H, d)
+            vec(p + "mix.A_log", H, 0.0, 0.5)
+            vec(p + "mix.norm", DV, 1.0)
+            mat(p + "mix.a1", r, d)
+            mat(p + "mix.a2", H * D, r)
+            vec(p + "mix.dt_bias", H * D, -2.0, 1.0)
+            mat(p + "mix.g1", r, d)
+            mat(p + "mix.g2", H * DV, r)
+        mat(p + "mix.o", d, H * DV, 0.3)
+        if e.get("mlp"):
+            ff = e["mlp"]["ff"]
+            mat(p + "mlp.gate", ff, d)
+            mat(p + "mlp.up", ff, d)
+            mat(p + "mlp.down", d, ff, 0.5)
+        if side:
+            mat(p + "side.gate", side, d)
+            mat(p + "side.proj", d, side)
+            vec(p + "side.norm", d, 0.2)
+    vec("final.norm", d)
+    mat("head", V, d)
+    return out
