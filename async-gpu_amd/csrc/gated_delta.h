@@ -36,9 +36,9 @@ struct DeltaArgs {
     void *out = nullptr;  // rows, stride ldo: heads x vdim, bf16 or fp32
     int ldo = 0, out_bf16 = 0;
     // scratch of the many-token form, fp32 rows
-    float *qk = nullptr;    // [rows][2 * kv_heads * state_row]: q | k, unit vectors
+    float *qkg = nullptr;   // [rows][heads][3][state_row]: unit vectors q and k, decays g
     float *v = nullptr;     // [rows][heads * vdim]
-    float *g = nullptr;     // [rows][heads * state_row]: in: W_a2 a1, out: decay
+    float *step = nullptr;  // [rows][heads * state_row]: W_a2 a1
     float *bkq = nullptr;   // [rows][heads + kv_heads]: beta | k . q
     float *gate = nullptr;  // [rows][heads * vdim]: W_g2 g1
     float *o = nullptr;     // [rows][heads * vdim]
@@ -47,5 +47,5 @@ struct DeltaArgs {
 bool delta_supported(const DeltaShape &s);
 // One new token per sequence, everything after the projections in one launch.
 int32_t delta_step_launch(agpu_ctx *ctx, const DeltaArgs &a);
-// Any number of tokens; `g` and `gate` hold the low-rank products already.
+// Any number of tokens; `step` and `gate` hold the low-rank products already.
 int32_t delta_prefill_launch(agpu_ctx *ctx, const DeltaArgs &a);

@@ -45,8 +45,8 @@ __device__ __forceinline__ float conv_silu(const DeltaArgs &a, int channels, int
 constexpr int kPrepareWidth = 1024;  // channels of v or g per workgroup
 
 // grid (rows, parts): the first parts take four heads of q and k each (convolution, unit vectors; one wave per head), then
-// come parts of v (convolution), then parts of g (decays; the first of them also the step sizes).  q, k and g leave with one
-// padded row per head.
+// come parts of v (convolution), then parts of g (decays; the first of them also the step sizes).  q, k and g of a head leave
+// side by side, in padded rows.
 __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaArgs a, int channels, int head_row, int qk_parts, int v_parts) {
     __shared__ float sx[2][4][kMaxDim];
     const DeltaShape &s = a.s;
@@ -58,7 +58,8 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaArgs a, int cha
     if (part < qk_parts) {
         const int h = part * 4 + wave;
         if (h >= s.kv_heads) return;
-        float *q_out = a.qk + ((size_t)row * 2 * s.kv_heads + h) * head_row, *k_out = q_out + (size_t)s.kv_heads * head_row;
+        const int group = s.heads / s.kv_heads;
+        float *out = a.qkg + ((size_t)row * s.heads + h * group) * 3 * head_row;
 #pragma unroll 1
         for (int i = lane; i < 2 * head_row; i += 64) {
             const int k = i >= head_row, d = i - k * head_row, c = h * s.dim + min(d, s.dim - 1);
@@ -75,10 +76,11 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaArgs a, int cha
         }
         const float rq = 1.0f / sqrtf(wave_sum(qq) + 1e-6f) / sqrtf((float)s.dim), rk = 1.0f / sqrtf(wave_sum(kk) + 1e-6f);
         dot = wave_sum(dot);
-        for (int d = lane; d < head_row; d += 64) {
-            q_out[d] = sx[0][wave][d] * rq;
-            k_out[d] = sx[1][wave][d] * rk;
-        }
+        for (int i = 0; i < group; ++i)
+            for (int d = lane; d < head_row; d += 64) {
+                out[i * 3 * head_row + d] = sx[0][wave][d] * rq;
+                out[(i * 3 + 1) * head_row + d] = sx[1][wave][d] * rk;
+            }
         if (lane == 0) bkq[s.heads + h] = dot * rq * rk;
         return;
     }
@@ -92,11 +94,12 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaArgs a, int cha
     part -= v_parts;
     if (part == 0)
         for (int h = threadIdx.x; h < s.heads; h += 256) bkq[h] = sigmoid_dev(a.proj[(size_t)row * a.ld + a.col_b + h]);
-    float *g = a.g + (size_t)row * s.heads * head_row;
+    const float *step = a.step + (size_t)row * s.heads * head_row;
+    float *g = a.qkg + (size_t)row * s.heads * 3 * head_row + 2 * head_row;
 #pragma unroll 2
     for (int c = part * kPrepareWidth + threadIdx.x; c < min((part + 1) * kPrepareWidth, s.heads * head_row); c += 256) {
         const int h = c / head_row, d = c % head_row;
-        g[c] = d < s.dim ? decay_dev(a.w.a_log[h], g[c] + a.w.dt_bias[h * s.dim + d]) : 1.0f;
+        g[h * 3 * head_row + d] = d < s.dim ? decay_dev(a.w.a_log[h], step[c] + a.w.dt_bias[h * s.dim + d]) : 1.0f;
     }
 }
 
@@ -126,7 +129,7 @@ __global__ __launch_bounds__(64 * kRecWaves) void delta_recurrence_kernel(DeltaA
     const DeltaShape &s = a.s;
     const int t = threadIdx.x, lane = t & 63, wave = t >> 6, l32 = lane & 31, half = lane >> 5;
     const int h = blockIdx.y, b = blockIdx.z, j0 = blockIdx.x * COLS, j = j0 + wave * 2 + half;
-    const int hk = h / (s.heads / s.kv_heads), nv = s.heads * s.vdim, T = a.new_len;
+    const int nv = s.heads * s.vdim, T = a.new_len;
     const size_t row0 = (size_t)b * T;
     float *st = a.state + (((size_t)b * s.heads + h) * s.vdim + min(j, s.vdim - 1)) * DP + l32 * DR;
     float S[DR];
@@ -135,36 +138,37 @@ __global__ __launch_bounds__(64 * kRecWaves) void delta_recurrence_kernel(DeltaA
     // The vectors of a chunk: requested into registers before the chunk in front of it is worked on, put into LDS after.
     constexpr int QUADS = kChunk * 3 * DP / 4, QN = (QUADS + NT - 1) / NT;
     static_assert(kChunk * (COLS + 2) <= NT, "one scalar per thread");
-    const float *qk = a.qk + (row0 * 2 * s.kv_heads + hk) * DP, *gp = a.g + (row0 * s.heads + h) * DP;
+    const float *vec = a.qkg + (row0 * s.heads + h) * 3 * DP;
+    const int token = s.heads * 3 * DP;  // floats from a token to the next
+    // this thread's scalar: a value of v, beta or k . q of token t / (COLS + 2)
+    const int sct = t / (COLS + 2), scc = t % (COLS + 2), nb = s.heads + s.kv_heads;
+    const float *scp = scc < COLS ? a.v + row0 * nv + h * s.vdim + min(j0 + scc, s.vdim - 1)
+                                  : a.bkq + row0 * nb + (scc == COLS ? h : s.heads + h / (s.heads / s.kv_heads));
+    const int scs = scc < COLS ? nv : nb;
     float4 rq[QN];
     float rs = 0.0f;
     auto request = [&](int t0) {
 #pragma unroll
         for (int n = 0; n < QN; ++n) {
-            const int i = min(t + n * NT, QUADS - 1), d4 = i % (DP / 4), w = (i / (DP / 4)) % 3, tok = min(t0 + i / (3 * DP / 4), T - 1);
-            const float *src = w == 2 ? gp + (size_t)tok * s.heads * DP : qk + (size_t)tok * 2 * s.kv_heads * DP + w * s.kv_heads * DP;
-            rq[n] = *(const float4 *)(src + 4 * d4);
+            const int i = t + n * NT, tok = min(t0 + i / (3 * DP / 4), T - 1);
+            rq[n] = *(const float4 *)(vec + (size_t)tok * token + 4 * (i % (3 * DP / 4)));
         }
-        if (t < kChunk * (COLS + 2)) {
-            const int c = t % (COLS + 2);
-            const size_t row = row0 + min(t0 + t / (COLS + 2), T - 1);
-            const float *bkq = a.bkq + row * (s.heads + s.kv_heads);
-            rs = c < COLS ? a.v[row * nv + h * s.vdim + min(j0 + c, s.vdim - 1)] : bkq[c == COLS ? h : s.heads + hk];
-        }
+        rs = scp[(size_t)min(t0 + min(sct, kChunk - 1), T - 1) * scs];
     };
     auto stage = [&](int buf, int t0) {
+        if (t0 + kChunk > T) {  // behind the last token nothing moves
 #pragma unroll
-        for (int n = 0; n < QN; ++n) {
-            const int i = t + n * NT, d4 = i % (DP / 4), w = (i / (DP / 4)) % 3, tok = i / (3 * DP / 4);
-            if (i >= QUADS) continue;
-            float4 v = rq[n];
-            if (t0 + tok >= T) {  // behind the last token nothing moves
-                const float f = w == 2 ? 1.0f : 0.0f;
-                v = make_float4(f, f, f, f);
+            for (int n = 0; n < QN; ++n) {
+                const int i = t + n * NT;
+                if (t0 + i / (3 * DP / 4) < T) continue;
+                const float f = i % (3 * DP / 4) >= 2 * DP / 4 ? 1.0f : 0.0f;
+                rq[n] = make_float4(f, f, f, f);
             }
-            *(float4 *)&sv[buf][tok][w][4 * d4] = v;
         }
-        if (t < kChunk * (COLS + 2)) sc[buf][t / (COLS + 2)][t % (COLS + 2)] = rs;
+#pragma unroll
+        for (int n = 0; n < QN; ++n)
+            if (t + n * NT < QUADS) *(float4 *)(&sv[buf][0][0][0] + 4 * (t + n * NT)) = rq[n];
+        if (t < kChunk * (COLS + 2)) sc[buf][sct][scc] = rs;
     };
     request(0);
     stage(0, 0);
@@ -187,6 +191,7 @@ __global__ __launch_bounds__(64 * kRecWaves) void delta_recurrence_kernel(DeltaA
             kq = sc[buf][i][COLS + 1];
         };
         fetch(0);
+        float out = 0.0f;
 #pragma unroll 4
         for (int i = 0; i < kChunk; ++i) {
             float kc[DR];
@@ -205,8 +210,9 @@ __global__ __launch_bounds__(64 * kRecWaves) void delta_recurrence_kernel(DeltaA
             const float u = bc * (vc - ks);
 #pragma unroll
             for (int r = 0; r < DR; ++r) S[r] = fmaf(kc[r], u, S[r]);
-            if (l32 == 0 && j < s.vdim && t0 + i < T) a.o[(row0 + t0 + i) * nv + h * s.vdim + j] = fmaf(kqc, u, qs);
+            out = l32 == i ? fmaf(kqc, u, qs) : out;  // lane i keeps the output of token i
         }
+        if (l32 < kChunk && j < s.vdim && t0 + l32 < T) a.o[(row0 + t0 + l32) * nv + h * s.vdim + j] = out;
         if (more) stage(buf ^ 1, t0 + kChunk);
         __syncthreads();
     }

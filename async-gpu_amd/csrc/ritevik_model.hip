@@ -122,7 +122,7 @@ struct agpu_ritevik final : LmRuntime {
     float *state = nullptr;  // delta states and convolution rings of every run
     size_t latent_elems = 0, state_floats = 0;
     int max_cat = 0, max_in = 0;
-    DevBuf xa, xb, x0, y, h, proj, cat, side, qlat, partial, qb, kx, vx, dqk, dv, dg, dbkq, dgate, dout;
+    DevBuf xa, xb, x0, y, h, proj, cat, side, qlat, partial, qb, kx, vx, dqkg, dv, dstep, dbkq, dgate, dout;
     float *tap = nullptr;  // residual stream after every layer run, [runs][rows][dp] (agpu_ritevik_layer_streams)
 
     bool small(int rows) const { return dense_gemv_supported(rows, std::max(max_cat, loop_in.K)); }
@@ -411,16 +411,16 @@ int32_t mixer(agpu_ritevik *m, const Run &r, int B, int new_len, int max_kv, voi
         if (new_len == 1) {
             AGPU_TRY(delta_step_launch(m->ctx, a));
         } else {
-            a.qk = (float *)m->dqk.p;
+            a.qkg = (float *)m->dqkg.p;
             a.v = (float *)m->dv.p;
-            a.g = (float *)m->dg.p;
+            a.step = (float *)m->dstep.p;
             a.bkq = (float *)m->dbkq.p;
             a.gate = (float *)m->dgate.p;
             a.o = (float *)m->dout.p;
             // the low-rank products in fp32: they feed decays and gates
             DenseOut og, oo;
             og.n_plain = og.ldo = L.a2.N;
-            og.out = a.g;
+            og.out = a.step;
             AGPU_TRY(dense_gemm_f32_launch(m->ctx, proj + L.col_a1, L.n_plain, L.a2.w, L.a2.K, R, L.a2.N, L.a2.K, og));
             oo.n_plain = oo.ldo = L.g2.N;
             oo.out = a.gate;
@@ -593,9 +593,9 @@ int32_t agpu_ritevik::ensure_buffers(int B, int new_len, bool all_rows_logits) {
             }
         } else if (new_len > 1) {
             const DeltaShape &s = L.ds;
-            AGPU_TRY(ensure(this, dqk, R * 2 * s.kv_heads * s.state_row() * f));
+            AGPU_TRY(ensure(this, dqkg, R * s.heads * 3 * s.state_row() * f));
             AGPU_TRY(ensure(this, dv, R * s.heads * s.vdim * f));
-            AGPU_TRY(ensure(this, dg, R * s.heads * s.state_row() * f));
+            AGPU_TRY(ensure(this, dstep, R * s.heads * s.state_row() * f));
             AGPU_TRY(ensure(this, dbkq, R * (s.heads + s.kv_heads) * f));
             AGPU_TRY(ensure(this, dgate, R * s.heads * s.vdim * f));
             AGPU_TRY(ensure(this, dout, R * s.heads * s.vdim * f));
@@ -650,8 +650,8 @@ AGPU_EXPORT int32_t agpu_ritevik_destroy(agpu_ritevik *m) {
     if (!m) return AGPU_OK;
     if (m->ctx) (void)hipStreamSynchronize(m->ctx->stream);
     for (void *p : m->owned) (void)hipFree(p);
-    for (DevBuf *b : {&m->xa, &m->xb, &m->x0, &m->y, &m->h, &m->proj, &m->cat, &m->side, &m->qlat, &m->partial, &m->qb, &m->kx, &m->vx, &m->dqk, &m->dv,
-                      &m->dg, &m->dbkq, &m->dgate, &m->dout})
+    for (DevBuf *b : {&m->xa, &m->xb, &m->x0, &m->y, &m->h, &m->proj, &m->cat, &m->side, &m->qlat, &m->partial, &m->qb, &m->kx, &m->vx, &m->dqkg, &m->dv,
+                      &m->dstep, &m->dbkq, &m->dgate, &m->dout})
         if (b->p) (void)hipFree(b->p);
     lm_release(m);
     delete m;
