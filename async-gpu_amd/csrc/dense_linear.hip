@@ -43,42 +43,59 @@ __device__ __forceinline__ float block_sum(float v, float *red) {
     return s;
 }
 
-// One row of DenseRows: h (and x2 behind it) goes through `put(k, value)`, k = 0 .. K - 1.
+// One row of DenseRows: h (and x2 behind it) goes through `put(k, value)`, k = 0 .. K - 1.  The first kRowRegs * NT columns
+// of x and y are read once and stay in registers; a wider row reads the rest again in every pass.
+constexpr int kRowRegs = 4;
 template <int NW, typename Put>
 __device__ __forceinline__ void run_row(const DenseRows &in, int m, bool write_x, float *red, Put put) {
-    const int t = threadIdx.x, nt = NW * 64;
+    constexpr int NT = NW * 64;
+    const int t = threadIdx.x;
     const size_t row = (size_t)(in.map_stride > 0 ? in.map_stride * (m + 1) - 1 : m) * in.ldx;
-    const float *x = in.x + row;
+    const float *x = in.x + row, *y = in.y ? in.y + row : nullptr;
+    float v[kRowRegs], yv[kRowRegs], yw[kRowRegs], nw[kRowRegs], v2[kRowRegs];
+#pragma unroll
+    for (int i = 0; i < kRowRegs; ++i) {  // clamped addresses; columns beyond d count as zero
+        const int k = t + i * NT, kc = min(k, in.d - 1);
+        v[i] = x[kc];
+        yv[i] = y ? y[kc] : 0.0f;
+        yw[i] = y ? in.y_w[kc] : 0.0f;
+        nw[i] = in.norm_w ? in.norm_w[kc] : 0.0f;
+        v2[i] = in.x2 ? in.x2[row + min(k, in.dp - 1)] : 0.0f;
+    }
     float rs_y = 0.0f;
-    if (in.y) {
-        const float *y = in.y + row;
+    if (y) {
         float s = 0.0f;
-        for (int k = t; k < in.d; k += nt) s += y[k] * y[k];
+#pragma unroll
+        for (int i = 0; i < kRowRegs; ++i) s += t + i * NT < in.d ? yv[i] * yv[i] : 0.0f;
+#pragma unroll 1
+        for (int k = t + kRowRegs * NT; k < in.d; k += NT) s += y[k] * y[k];
         s = block_sum<NW>(s, red);
         rs_y = 1.0f / sqrtf(s / (float)in.d + in.eps);
     }
-    auto value = [&](int k) -> float {
-        float v = x[k];
-        if (in.y) v += in.y[row + k] * rs_y * in.y_w[k];
-        return v;
-    };
-    float rs_x = 0.0f;
+#pragma unroll
+    for (int i = 0; i < kRowRegs; ++i) v[i] = t + i * NT < in.d ? v[i] + yv[i] * rs_y * yw[i] : 0.0f;
+    auto value = [&](int k) -> float { return y ? x[k] + y[k] * rs_y * in.y_w[k] : x[k]; };
+    float rs_x = 1.0f;
     if (in.norm_w) {
         float s = 0.0f;
-        for (int k = t; k < in.d; k += nt) {
-            const float v = value(k);
-            s += v * v;
-        }
+#pragma unroll
+        for (int i = 0; i < kRowRegs; ++i) s += v[i] * v[i];
+#pragma unroll 1
+        for (int k = t + kRowRegs * NT; k < in.d; k += NT) s += value(k) * value(k);
         s = block_sum<NW>(s, red);
         rs_x = 1.0f / sqrtf(s / (float)in.d + in.eps);
     }
-    for (int k = t; k < in.dp; k += nt) {
-        float v = k < in.d ? value(k) : 0.0f;
-        if (write_x) in.x_out[row + k] = v;
-        if (in.norm_w && k < in.d) v = v * rs_x * (in.norm_off + in.norm_w[k]);
-        put(k, v);
-        if (in.x2) put(in.dp + k, in.x2[row + k]);
-    }
+    auto finish = [&](int k, float a, float w, float b) {
+        if (write_x) in.x_out[row + k] = a;
+        put(k, in.norm_w ? a * rs_x * (in.norm_off + w) : a);
+        if (in.x2) put(in.dp + k, b);
+    };
+#pragma unroll
+    for (int i = 0; i < kRowRegs; ++i)
+        if (t + i * NT < in.dp) finish(t + i * NT, v[i], nw[i], v2[i]);
+#pragma unroll 1
+    for (int k = t + kRowRegs * NT; k < in.dp; k += NT)
+        finish(k, k < in.d ? value(k) : 0.0f, in.norm_w && k < in.d ? in.norm_w[k] : 0.0f, in.x2 ? in.x2[row + k] : 0.0f);
 }
 
 // ---- decode GEMV: a wave takes 4 * RPL weight rows, 16 lanes x 8 values along K per row and chunk of 128; the waves of a
@@ -111,7 +128,7 @@ __global__ __launch_bounds__(64 * kGemvWaves) void dense_gemv_kernel(DenseRows i
         }
     };
     request(wk);
-#pragma unroll
+#pragma unroll 1
     for (int m = 0; m < MT; ++m) {
         float *xm = xs + (size_t)m * K;
         if (m < M) {
@@ -200,18 +217,16 @@ __global__ __launch_bounds__(64 * NW) void dense_rows_kernel(DenseRows in, void 
 }
 
 // ---- few rows or few columns: 16 columns and up to 32 rows per workgroup, the waves split K, operands straight from memory ----
-constexpr int kSkinnyWaves = 8;
-
-template <int RT>  // row tiles of 16
+template <int RT, int kSkinnyWaves>  // row tiles of 16, waves
 __global__ __launch_bounds__(64 * kSkinnyWaves) void dense_skinny_kernel(const uint16_t *__restrict__ a, int lda, const uint16_t *__restrict__ w,
                                                                          int ldw, int M, int N, int K, DenseOut o) {
     __shared__ float red[kSkinnyWaves][RT][16][17];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, rc = lane & 15, kq = lane >> 4;
     const int n0 = blockIdx.x * 16, m0 = blockIdx.y * 16 * RT;
-    const uint16_t *wp = w + (size_t)min(n0 + rc, N - 1) * ldw + kq * 8;
+    const uint16_t *wp = w + (size_t)min(n0 + rc, N - 1) * ldw;
     const uint16_t *ap[RT];
 #pragma unroll
-    for (int t = 0; t < RT; ++t) ap[t] = a + (size_t)min(m0 + t * 16 + rc, M - 1) * lda + kq * 8;
+    for (int t = 0; t < RT; ++t) ap[t] = a + (size_t)min(m0 + t * 16 + rc, M - 1) * lda;
     f32x4 acc[RT];
 #pragma unroll
     for (int t = 0; t < RT; ++t) acc[t] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
@@ -221,11 +236,11 @@ __global__ __launch_bounds__(64 * kSkinnyWaves) void dense_skinny_kernel(const u
         uint4 bw[U], aw[U][RT];
 #pragma unroll
         for (int u = 0; u < U; ++u) {
-            const int s = s0 + u * kSkinnyWaves;
+            const int s = s0 + u * kSkinnyWaves, k = s * 32 + kq * 8;
             const bool on = s < steps;
-            bw[u] = on ? *(const uint4 *)(wp + (size_t)s * 32) : make_uint4(0, 0, 0, 0);
+            bw[u] = on ? *(const uint4 *)(wp + k) : make_uint4(0, 0, 0, 0);
 #pragma unroll
-            for (int t = 0; t < RT; ++t) aw[u][t] = on ? *(const uint4 *)(ap[t] + (size_t)s * 32) : make_uint4(0, 0, 0, 0);
+            for (int t = 0; t < RT; ++t) aw[u][t] = on ? *(const uint4 *)(ap[t] + k) : make_uint4(0, 0, 0, 0);
         }
 #pragma unroll
         for (int u = 0; u < U; ++u)
@@ -284,15 +299,19 @@ __device__ __forceinline__ void store_tile(const DenseOut &o, const f32x16 &c, f
 }
 
 // ---- tiled bf16 GEMM: BM x BN per workgroup of WM x WN waves, 64 k per step, two LDS buffers, 16-byte chunks of a row
-// rotated by row % 8 against bank conflicts ----
-template <int BM, int BN, int WM, int WN>
-__global__ __launch_bounds__(64 * WM *WN) void dense_gemm_bf16_kernel(const uint16_t *__restrict__ a, int lda, const uint16_t *__restrict__ w,
+// rotated by row % 8 against bank conflicts.  With KG > 1 there are KG such groups of waves, which take the K steps in turn
+// (each with its own buffers) and add their results up in LDS at the end ----
+template <int BM, int BN, int WM, int WN, int KG>
+__global__ __launch_bounds__(64 * WM * WN * KG) void dense_gemm_bf16_kernel(const uint16_t *__restrict__ a, int lda, const uint16_t *__restrict__ w,
                                                                       int ldw, int M, int N, int K, int tiles_n, DenseOut o) {
     constexpr int NT = 64 * WM * WN, TM = BM / WM / 32, TN = BN / WN / 32;
     constexpr int CA = BM * 8 / NT, CB = BN * 8 / NT;  // 16-byte chunks per thread and step
-    __shared__ uint4 sab[2 * (BM + BN) * 8];  // both operands twice, then the waves' result tiles
-    static_assert(sizeof(sab) >= sizeof(float) * WM * WN * 32 * kTileLd, "the result tiles fit the operand buffers");
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, wm = wave / WN, wn = wave % WN;
+    extern __shared__ uint4 shm[];  // per group both operands twice; then the groups' results and the waves' result tiles
+    constexpr int GROUP = 2 * (BM + BN) * 8;
+    static_assert(GROUP * 16 >= 4 * WM * WN * 32 * kTileLd && GROUP * 16 >= 4 * BM * BN, "the results fit the operand buffers");
+    const int lane = threadIdx.x & 63, wave = (threadIdx.x % NT) >> 6, wm = wave / WN, wn = wave % WN;
+    const int tid = threadIdx.x % NT, group = threadIdx.x / NT;
+    uint4 *sab = shm + group * GROUP;
     // workgroups b, b + 8, ... share an XCD: give each XCD a contiguous run of row tiles so that W tiles stay in its L2
     const int nb = gridDim.x;
     int b = blockIdx.x;
@@ -305,24 +324,24 @@ __global__ __launch_bounds__(64 * WM *WN) void dense_gemm_bf16_kernel(const uint
     auto request = [&](int k0) {
 #pragma unroll
         for (int i = 0; i < CA; ++i) {
-            const int c = threadIdx.x + i * NT, r = c >> 3, k = k0 + (c & 7) * 8;
+            const int c = tid + i * NT, r = c >> 3, k = k0 + (c & 7) * 8;
             ra[i] = k < K ? *(const uint4 *)(a + (size_t)min(m0 + r, M - 1) * lda + k) : make_uint4(0, 0, 0, 0);
         }
 #pragma unroll
         for (int i = 0; i < CB; ++i) {
-            const int c = threadIdx.x + i * NT, r = c >> 3, k = k0 + (c & 7) * 8;
+            const int c = tid + i * NT, r = c >> 3, k = k0 + (c & 7) * 8;
             rb[i] = k < K ? *(const uint4 *)(w + (size_t)min(n0 + r, N - 1) * ldw + k) : make_uint4(0, 0, 0, 0);
         }
     };
     auto stage = [&](int buf) {
 #pragma unroll
         for (int i = 0; i < CA; ++i) {
-            const int c = threadIdx.x + i * NT, r = c >> 3;
+            const int c = tid + i * NT, r = c >> 3;
             sab[buf * BM * 8 + r * 8 + ((c & 7) ^ (r & 7))] = ra[i];
         }
 #pragma unroll
         for (int i = 0; i < CB; ++i) {
-            const int c = threadIdx.x + i * NT, r = c >> 3;
+            const int c = tid + i * NT, r = c >> 3;
             sab[2 * BM * 8 + buf * BN * 8 + r * 8 + ((c & 7) ^ (r & 7))] = rb[i];
         }
     };
@@ -333,14 +352,14 @@ __global__ __launch_bounds__(64 * WM *WN) void dense_gemm_bf16_kernel(const uint
         for (int j = 0; j < TN; ++j)
 #pragma unroll
             for (int r = 0; r < 16; ++r) acc[i][j][r] = 0.0f;
-    request(0);
+    request(group * 64);
     stage(0);
     __syncthreads();
     const int lr = lane & 31, lh = lane >> 5;
     int buf = 0;
-    for (int k0 = 0; k0 < K; k0 += 64, buf ^= 1) {
-        const bool more = k0 + 64 < K;
-        if (more) request(k0 + 64);
+    for (int k0 = 0; k0 < K; k0 += 64 * KG, buf ^= 1) {  // a group past K works on zeros
+        const bool more = k0 + 64 * KG < K;
+        if (more) request(k0 + (KG + group) * 64);
 #pragma unroll
         for (int s = 0; s < 4; ++s) {
             bf16x8 av[TM], bv[TN];
@@ -361,6 +380,28 @@ __global__ __launch_bounds__(64 * WM *WN) void dense_gemm_bf16_kernel(const uint
         }
         if (more) stage(buf ^ 1);
         __syncthreads();
+    }
+    if (KG > 1) {
+        float *mine = (float *)sab + wave * TM * TN * 1024 + lane;
+        if (group > 0) {
+#pragma unroll
+            for (int i = 0; i < TM; ++i)
+#pragma unroll
+                for (int j = 0; j < TN; ++j)
+#pragma unroll
+                    for (int r = 0; r < 16; ++r) mine[((i * TN + j) * 16 + r) * 64] = acc[i][j][r];
+        }
+        __syncthreads();
+        if (group > 0) return;
+        for (int g = 1; g < KG; ++g) {
+            const float *other = mine + (size_t)g * GROUP * 4;
+#pragma unroll
+            for (int i = 0; i < TM; ++i)
+#pragma unroll
+                for (int j = 0; j < TN; ++j)
+#pragma unroll
+                    for (int r = 0; r < 16; ++r) acc[i][j][r] += other[((i * TN + j) * 16 + r) * 64];
+        }
     }
 #pragma unroll
     for (int i = 0; i < TM; ++i)
@@ -429,6 +470,17 @@ int32_t gemv_run(agpu_ctx *ctx, const DenseRows &in, const uint16_t *w, int M, i
     return AGPU_LAUNCH_CHECK(ctx, "dense_gemv_kernel");
 }
 
+template <int BM, int BN, int WM, int WN, int KG>
+void gemm_run(agpu_ctx *ctx, const uint16_t *a, int lda, const uint16_t *w, int ldw, int M, int N, int K, const DenseOut &o) {
+    constexpr size_t lds = (size_t)KG * 2 * (BM + BN) * 8 * 16;
+    if (lds > 64 * 1024)
+        (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&dense_gemm_bf16_kernel<BM, BN, WM, WN, KG>), hipFuncAttributeMaxDynamicSharedMemorySize,
+                                  (int)lds);
+    const int tn = ceil_div(N, BN);
+    hipLaunchKernelGGL((dense_gemm_bf16_kernel<BM, BN, WM, WN, KG>), dim3((unsigned)(ceil_div(M, BM) * tn)), dim3(64 * WM * WN * KG), lds, ctx->stream, a,
+                       lda, w, ldw, M, N, K, tn, o);
+}
+
 }  // namespace
 
 bool dense_gemv_supported(int M, int K) {
@@ -451,8 +503,9 @@ int32_t dense_gemv_launch(agpu_ctx *ctx, const DenseRows &in, const uint16_t *w,
 }
 
 int32_t dense_rows_launch(agpu_ctx *ctx, const DenseRows &in, int M, void *h, int ldh, int h_bf16) {
-    if (in.dp <= 512) hipLaunchKernelGGL(dense_rows_kernel<1>, dim3((unsigned)M), dim3(64), 0, ctx->stream, in, h, ldh, h_bf16);
-    else hipLaunchKernelGGL(dense_rows_kernel<4>, dim3((unsigned)M), dim3(256), 0, ctx->stream, in, h, ldh, h_bf16);
+    if (in.dp <= 256) hipLaunchKernelGGL(dense_rows_kernel<1>, dim3((unsigned)M), dim3(64), 0, ctx->stream, in, h, ldh, h_bf16);
+    else if (in.dp <= 1024) hipLaunchKernelGGL(dense_rows_kernel<4>, dim3((unsigned)M), dim3(256), 0, ctx->stream, in, h, ldh, h_bf16);
+    else hipLaunchKernelGGL(dense_rows_kernel<8>, dim3((unsigned)M), dim3(512), 0, ctx->stream, in, h, ldh, h_bf16);
     return AGPU_LAUNCH_CHECK(ctx, "dense_rows_kernel");
 }
 
@@ -461,21 +514,24 @@ int32_t dense_gemm_bf16_launch(agpu_ctx *ctx, const uint16_t *a, int lda, const 
         return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "dense_gemm: M %d, N %d, K %d, lda %d, ldw %d not supported", M, N, K, lda, ldw);
     auto tiles = [&](int bm, int bn) { return ceil_div(M, bm) * ceil_div(N, bn); };
     if (M <= kDenseSkinnyRows || 2 * tiles(32, 64) < ctx->num_cus) {
-        const dim3 grid((unsigned)ceil_div(N, 16), (unsigned)ceil_div(M, 32)), block(64 * kSkinnyWaves);
-        if (M <= 16) hipLaunchKernelGGL(dense_skinny_kernel<1>, grid, block, 0, ctx->stream, a, lda, w, ldw, M, N, K, o);
-        else hipLaunchKernelGGL(dense_skinny_kernel<2>, grid, block, 0, ctx->stream, a, lda, w, ldw, M, N, K, o);
+        const dim3 grid((unsigned)ceil_div(N, 16), (unsigned)ceil_div(M, 32));
+        // fewer workgroups than CUs and a long K: more waves each, for more requests in flight per CU
+        const bool deep = (int)(grid.x * grid.y) <= ctx->num_cus && K >= 2048;
+#define AGPU_SKINNY(RT, NW) hipLaunchKernelGGL((dense_skinny_kernel<RT, NW>), grid, dim3(64 * NW), 0, ctx->stream, a, lda, w, ldw, M, N, K, o)
+        if (M <= 16) {
+            if (deep) AGPU_SKINNY(1, 16);
+            else AGPU_SKINNY(1, 8);
+        } else {
+            if (deep) AGPU_SKINNY(2, 16);
+            else AGPU_SKINNY(2, 8);
+        }
+#undef AGPU_SKINNY
         return AGPU_LAUNCH_CHECK(ctx, "dense_skinny_kernel");
     }
-    if (tiles(128, 128) >= ctx->num_cus) {
-        hipLaunchKernelGGL((dense_gemm_bf16_kernel<128, 128, 2, 2>), dim3((unsigned)tiles(128, 128)), dim3(256), 0, ctx->stream, a, lda, w, ldw, M, N, K,
-                           ceil_div(N, 128), o);
-    } else if (tiles(64, 64) >= ctx->num_cus) {
-        hipLaunchKernelGGL((dense_gemm_bf16_kernel<64, 64, 2, 2>), dim3((unsigned)tiles(64, 64)), dim3(256), 0, ctx->stream, a, lda, w, ldw, M, N, K,
-                           ceil_div(N, 64), o);
-    } else {
-        hipLaunchKernelGGL((dense_gemm_bf16_kernel<32, 64, 1, 2>), dim3((unsigned)tiles(32, 64)), dim3(128), 0, ctx->stream, a, lda, w, ldw, M, N, K,
-                           ceil_div(N, 64), o);
-    }
+    if (tiles(128, 128) >= ctx->num_cus) gemm_run<128, 128, 2, 2, 1>(ctx, a, lda, w, ldw, M, N, K, o);
+    else if (M > 256 && tiles(128, 64) >= ctx->num_cus) gemm_run<128, 64, 2, 2, 2>(ctx, a, lda, w, ldw, M, N, K, o);
+    else if (tiles(64, 64) >= ctx->num_cus) gemm_run<64, 64, 2, 2, 2>(ctx, a, lda, w, ldw, M, N, K, o);
+    else gemm_run<32, 64, 1, 2, 4>(ctx, a, lda, w, ldw, M, N, K, o);
     return AGPU_LAUNCH_CHECK(ctx, "dense_gemm_bf16_kernel");
 }
 

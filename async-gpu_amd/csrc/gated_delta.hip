@@ -42,64 +42,118 @@ __device__ __forceinline__ float conv_silu(const DeltaArgs &a, int channels, int
     return silu_dev(v);
 }
 
-constexpr int kPrepareWidth = 1024;  // channels of v or g per workgroup
+// The same for up to kTokens tokens from t0 on, each input loaded once; put(i, value of token t0 + i).
+constexpr int kTokens = 8, kWindow = 4;
+template <typename Put>
+__device__ __forceinline__ void conv_silu_run(const DeltaArgs &a, int channels, int b, int pos, int pos_slot, int t0, int c, int col, Put put) {
+    const int n = a.s.taps, T = a.new_len;
+    if (n > kWindow) {
+#pragma unroll 1
+        for (int i = 0; i < kTokens && t0 + i < T; ++i) put(i, conv_silu(a, channels, b, pos, pos_slot, t0 + i, c, col));
+        return;
+    }
+    const float *base = a.proj + (size_t)b * T * a.ld + col, *ring = a.ring + (size_t)b * n * channels + c, *w = a.w.conv + (size_t)c * n;
+    float f[kWindow], x[kTokens + kWindow - 1];
+#pragma unroll
+    for (int e = 0; e < kWindow; ++e) f[e] = e >= kWindow - n ? w[max(e - (kWindow - n), 0)] : 0.0f;
+#pragma unroll
+    for (int e = 0; e < kWindow - 1; ++e) {  // the tokens in front of t0
+        const int k = kWindow - 1 - e, t = t0 - k;
+        int slot = pos_slot + t;
+        slot = slot < 0 ? slot + n : slot;
+        const bool on = k < n && pos + t >= 0;
+        const float *p = t >= 0 ? base + (size_t)t * a.ld : ring + (size_t)slot * channels;
+        const float v = *(on ? p : base);
+        x[e] = on ? v : 0.0f;
+    }
+#pragma unroll
+    for (int i = 0; i < kTokens; ++i) x[kWindow - 1 + i] = base[(size_t)min(t0 + i, T - 1) * a.ld];
+#pragma unroll
+    for (int i = 0; i < kTokens; ++i) {
+        float v = 0.0f;
+#pragma unroll
+        for (int e = 0; e < kWindow; ++e) v = fmaf(f[e], x[i + e], v);
+        put(i, silu_dev(v));
+    }
+}
 
-// grid (rows, parts): the first parts take four heads of q and k each (convolution, unit vectors; one wave per head), then
+constexpr int kPrepareWidth = 256;  // channels of v or g per workgroup
+
+// grid (groups of kTokens tokens, parts, batch): the first parts take two heads of q and k each (convolution, unit vectors), then
 // come parts of v (convolution), then parts of g (decays; the first of them also the step sizes).  q, k and g of a head leave
 // side by side, in padded rows.
 __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaArgs a, int channels, int head_row, int qk_parts, int v_parts) {
-    __shared__ float sx[2][4][kMaxDim];
+    extern __shared__ float sx[];  // [2 heads][q, k][kTokens][head_row]
     const DeltaShape &s = a.s;
-    const int row = blockIdx.x, b = row / a.new_len, t = row % a.new_len, pos = *a.pos_dev, pos_slot = pos % s.taps;
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-    const int nk = s.kv_heads * s.dim, nv = s.heads * s.vdim;
-    float *bkq = a.bkq + (size_t)row * (s.heads + s.kv_heads);
+    const int b = blockIdx.z, T = a.new_len, t0 = blockIdx.x * kTokens, nt = min(kTokens, T - t0), pos = *a.pos_dev, pos_slot = pos % s.taps;
+    const int t = threadIdx.x, lane = t & 63, wave = t >> 6;
+    const int nk = s.kv_heads * s.dim, nv = s.heads * s.vdim, nb = s.heads + s.kv_heads;
+    const size_t row0 = (size_t)b * T + t0;
     int part = blockIdx.y;
     if (part < qk_parts) {
-        const int h = part * 4 + wave;
-        if (h >= s.kv_heads) return;
-        const int group = s.heads / s.kv_heads;
-        float *out = a.qkg + ((size_t)row * s.heads + h * group) * 3 * head_row;
+        const int per = kTokens * head_row;
 #pragma unroll 1
-        for (int i = lane; i < 2 * head_row; i += 64) {
-            const int k = i >= head_row, d = i - k * head_row, c = h * s.dim + min(d, s.dim - 1);
-            const float v = conv_silu(a, channels, b, pos, pos_slot, t, k * nk + c, (k ? a.col_k : a.col_q) + c);
-            sx[k][wave][d] = d < s.dim ? v : 0.0f;
+        for (int i = t; i < 4 * head_row; i += 256) {
+            const int w = i / head_row, d = i % head_row, h = min(part * 2 + (w >> 1), s.kv_heads - 1), c = h * s.dim + min(d, s.dim - 1);
+            conv_silu_run(a, channels, b, pos, pos_slot, t0, (w & 1) * nk + c, ((w & 1) ? a.col_k : a.col_q) + c,
+                          [&](int e, float v) { sx[w * per + e * head_row + d] = d < s.dim ? v : 0.0f; });
         }
-        __builtin_amdgcn_wave_barrier();  // a wave reads what it wrote itself
-        float qq = 0.0f, kk = 0.0f, dot = 0.0f;
-        for (int d = lane; d < head_row; d += 64) {
-            const float q = sx[0][wave][d], k = sx[1][wave][d];
-            qq = fmaf(q, q, qq);
-            kk = fmaf(k, k, kk);
-            dot = fmaf(q, k, dot);
-        }
-        const float rq = 1.0f / sqrtf(wave_sum(qq) + 1e-6f) / sqrtf((float)s.dim), rk = 1.0f / sqrtf(wave_sum(kk) + 1e-6f);
-        dot = wave_sum(dot);
-        for (int i = 0; i < group; ++i)
+        __syncthreads();
+        const int group = s.heads / s.kv_heads;
+#pragma unroll 1
+        for (int i = wave; i < 2 * nt; i += 4) {  // one (head, token) per wave
+            const int h = part * 2 + (i & 1), e = i >> 1;
+            if (h >= s.kv_heads) continue;
+            const float *sq = sx + (size_t)(i & 1) * 2 * per + e * head_row, *sk = sq + per;
+            float qq = 0.0f, kk = 0.0f, dot = 0.0f;
             for (int d = lane; d < head_row; d += 64) {
-                out[i * 3 * head_row + d] = sx[0][wave][d] * rq;
-                out[(i * 3 + 1) * head_row + d] = sx[1][wave][d] * rk;
+                const float q = sq[d], k = sk[d];
+                qq = fmaf(q, q, qq);
+                kk = fmaf(k, k, kk);
+                dot = fmaf(q, k, dot);
             }
-        if (lane == 0) bkq[s.heads + h] = dot * rq * rk;
+            const float rq = 1.0f / sqrtf(wave_sum(qq) + 1e-6f) / sqrtf((float)s.dim), rk = 1.0f / sqrtf(wave_sum(kk) + 1e-6f);
+            dot = wave_sum(dot);
+            float *out = a.qkg + ((row0 + e) * s.heads + h * group) * 3 * head_row;
+            for (int g = 0; g < group; ++g)
+                for (int d = lane; d < head_row; d += 64) {
+                    out[g * 3 * head_row + d] = sq[d] * rq;
+                    out[(g * 3 + 1) * head_row + d] = sk[d] * rk;
+                }
+            if (lane == 0) a.bkq[(row0 + e) * nb + s.heads + h] = dot * rq * rk;
+        }
         return;
     }
     part -= qk_parts;
     if (part < v_parts) {
-#pragma unroll 1
-        for (int c = part * kPrepareWidth + threadIdx.x; c < min((part + 1) * kPrepareWidth, nv); c += 256)
-            a.v[(size_t)row * nv + c] = conv_silu(a, channels, b, pos, pos_slot, t, 2 * nk + c, a.col_v + c);
+        const int c = part * kPrepareWidth + t;
+        if (c < nv)
+            conv_silu_run(a, channels, b, pos, pos_slot, t0, 2 * nk + c, a.col_v + c, [&](int e, float v) {
+                if (e < nt) a.v[(row0 + e) * nv + c] = v;
+            });
         return;
     }
     part -= v_parts;
     if (part == 0)
-        for (int h = threadIdx.x; h < s.heads; h += 256) bkq[h] = sigmoid_dev(a.proj[(size_t)row * a.ld + a.col_b + h]);
-    const float *step = a.step + (size_t)row * s.heads * head_row;
-    float *g = a.qkg + (size_t)row * s.heads * 3 * head_row + 2 * head_row;
-#pragma unroll 2
-    for (int c = part * kPrepareWidth + threadIdx.x; c < min((part + 1) * kPrepareWidth, s.heads * head_row); c += 256) {
-        const int h = c / head_row, d = c % head_row;
-        g[h * 3 * head_row + d] = d < s.dim ? decay_dev(a.w.a_log[h], step[c] + a.w.dt_bias[h * s.dim + d]) : 1.0f;
+        for (int i = t; i < s.heads * nt; i += 256) {
+            const int e = i / s.heads, h = i % s.heads;
+            a.bkq[(row0 + e) * nb + h] = sigmoid_dev(a.proj[(row0 + e) * a.ld + a.col_b + h]);
+        }
+    const int c = part * kPrepareWidth + t;
+    if (c >= s.heads * head_row) return;
+    const int h = c / head_row, d = c % head_row;
+    const float a_log = a.w.a_log[h], bias = d < s.dim ? a.w.dt_bias[h * s.dim + d] : 0.0f;
+    const float *step = a.step + row0 * s.heads * head_row + c;
+    float *g = a.qkg + (row0 * s.heads + h) * 3 * head_row + 2 * head_row + d;
+    float x[kTokens];
+#pragma unroll
+    for (int e = 0; e < kTokens; ++e) x[e] = step[(size_t)min(e, nt - 1) * s.heads * head_row];
+#pragma unroll 1
+    for (int e = 0; e < nt; ++e) {
+        float v = x[0];
+#pragma unroll
+        for (int i = 1; i < kTokens; ++i) v = e == i ? x[i] : v;
+        g[(size_t)e * s.heads * 3 * head_row] = d < s.dim ? decay_dev(a_log, v + bias) : 1.0f;
     }
 }
 
@@ -433,9 +487,9 @@ int32_t delta_prefill_launch(agpu_ctx *ctx, const DeltaArgs &a) {
     if (rc != AGPU_OK) return rc;
     const DeltaShape &s = a.s;
     const unsigned rows = (unsigned)(a.batch * a.new_len);
-    const int qk_parts = ceil_div(s.kv_heads, 4), v_parts = ceil_div(s.heads * s.vdim, kPrepareWidth), g_parts = ceil_div(s.heads * s.state_row(), kPrepareWidth);
-    hipLaunchKernelGGL(delta_prepare_kernel, dim3(rows, (unsigned)(qk_parts + v_parts + g_parts)), dim3(256), 0, ctx->stream, a, s.channels(), s.state_row(),
-                       qk_parts, v_parts);
+    const int qk_parts = ceil_div(s.kv_heads, 2), v_parts = ceil_div(s.heads * s.vdim, kPrepareWidth), g_parts = ceil_div(s.heads * s.state_row(), kPrepareWidth);
+    hipLaunchKernelGGL(delta_prepare_kernel, dim3((unsigned)ceil_div(a.new_len, kTokens), (unsigned)(qk_parts + v_parts + g_parts), (unsigned)a.batch),
+                       dim3(256), (size_t)4 * kTokens * s.state_row() * sizeof(float), ctx->stream, a, s.channels(), s.state_row(), qk_parts, v_parts);
     if ((rc = AGPU_LAUNCH_CHECK(ctx, "delta_prepare_kernel")) != AGPU_OK) return rc;
     hipLaunchKernelGGL(delta_ring_kernel, dim3((unsigned)ceil_div(s.channels(), 256), (unsigned)s.taps, (unsigned)a.batch), dim3(256), 0, ctx->stream, a,
                        s.channels());
