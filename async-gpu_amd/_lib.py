@@ -14,6 +14,7 @@ EPI_NONE, EPI_GELU_TANH, EPI_GELU_QUICK, EPI_FORCE_LITERAL, EPI_FORCE_FP32_GEMV 
 QUANT_RUST, QUANT_SCRIPT = 0, 1
 GELU_TANH, GELU_QUICK = 0, 1
 DTYPE_BF16, DTYPE_F32 = 0, 1
+DENSE_GATED = 1
 MIXER_LATENT_ATTENTION, MIXER_CHANNEL_DELTA = 0, 1
 
 
@@ -92,6 +93,14 @@ SIGNATURES = {
     "agpu_bench_attention": (_i32, [_vp, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _vp]),
     "agpu_kv_append": (_i32, [_vp, _vp, _vp, _i32, _i32, _i32, _i32, _i32]),
     "agpu_gemm_f32": (_i32, [_vp, _vp, _vp, _vp, _i32, _i32, _i32]),
+    "agpu_rms_norm": (_i32, [_vp, _vp, _vp, _f, _vp, _i32, _i32, _f]),
+    "agpu_dense_linear": (_i32, [_vp, _vp, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _i32, _u32]),
+    "agpu_rope_table": (_i32, [_vp, _vp, _i32, _i32, C.c_double]),
+    "agpu_latent_cache_row": (_i32, [_i32, _i32]),
+    "agpu_latent_attention_workspace_bytes": (_sz, [_vp, _vp]),
+    "agpu_latent_attention": (_i32, [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp]),
+    "agpu_channel_delta_workspace_bytes": (_sz, [_vp, _vp]),
+    "agpu_channel_delta": (_i32, [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp]),
     # include/agpu_gpt2.h (first argument is the model handle, or the config / context)
     "agpu_gpt2_config_small": (_i32, [_vp]),
     "agpu_gpt2_config_xl": (_i32, [_vp]),
@@ -151,6 +160,18 @@ class Gpt2ConfigStruct(C.Structure):
     _fields_ = [("n_layer", _i32), ("n_embd", _i32), ("n_head", _i32), ("vocab_size", _i32), ("n_positions", _i32),
                 ("layer_norm_epsilon", _f), ("group_size", _i32), ("max_batch", _i32), ("lm_head", _i32),
                 ("gelu", _i32), ("argmax_last", _i32)]
+
+
+class LatentAttentionDesc(C.Structure):
+    """agpu_latent_attention_desc of include/agpu.h."""
+    _fields_ = [(n, _i32) for n in ("heads", "dim", "rot_dim", "rot_dims", "vdim", "rank")] + [("scale", _f), ("eps", _f)] + \
+               [(n, _i32) for n in ("positions", "batch", "new_len", "cached", "ld", "ldo", "cache_dtype", "tiled")]
+
+
+class ChannelDeltaDesc(C.Structure):
+    """agpu_channel_delta_desc of include/agpu.h."""
+    _fields_ = [(n, _i32) for n in ("heads", "kv_heads", "dim", "vdim", "taps", "decay_rank", "gate_rank")] + [("eps", _f)] + \
+               [(n, _i32) for n in ("batch", "new_len", "cached", "ld", "ldo", "col_q", "col_k", "col_v", "col_b", "col_a1", "col_g1")]
 
 
 class RitevikConfigStruct(C.Structure):

@@ -47,5 +47,5 @@ struct DeltaArgs {
 bool delta_supported(const DeltaShape &s);
 // One new token per sequence, everything after the projections in one launch.
 int32_t delta_step_launch(agpu_ctx *ctx, const DeltaArgs &a);
-// Any number of tokens; `step` and `gate` hold the low-rank products already.
+// Any number of tokens.
 int32_t delta_prefill_launch(agpu_ctx *ctx, const DeltaArgs &a);

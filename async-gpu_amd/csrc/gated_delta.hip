@@ -487,6 +487,16 @@ int32_t delta_prefill_launch(agpu_ctx *ctx, const DeltaArgs &a) {
     if (rc != AGPU_OK) return rc;
     const DeltaShape &s = a.s;
     const unsigned rows = (unsigned)(a.batch * a.new_len);
+    // the low-rank products in fp32: they feed decays and gates
+    DenseOut step, gate;
+    step.n_plain = step.ldo = s.heads * s.state_row();
+    step.out = a.step;
+    rc = dense_gemm_f32_launch(ctx, a.proj + a.col_a1, a.ld, a.w.a2, s.rank_ap(), (int)rows, step.n_plain, s.rank_ap(), step);
+    if (rc != AGPU_OK) return rc;
+    gate.n_plain = gate.ldo = s.heads * s.vdim;
+    gate.out = a.gate;
+    rc = dense_gemm_f32_launch(ctx, a.proj + a.col_g1, a.ld, a.w.g2, s.rank_gp(), (int)rows, gate.n_plain, s.rank_gp(), gate);
+    if (rc != AGPU_OK) return rc;
     const int qk_parts = ceil_div(s.kv_heads, 2), v_parts = ceil_div(s.heads * s.vdim, kPrepareWidth), g_parts = ceil_div(s.heads * s.state_row(), kPrepareWidth);
     hipLaunchKernelGGL(delta_prepare_kernel, dim3((unsigned)ceil_div(a.new_len, kTokens), (unsigned)(qk_parts + v_parts + g_parts), (unsigned)a.batch),
                        dim3(256), (size_t)4 * kTokens * s.state_row() * sizeof(float), ctx->stream, a, s.channels(), s.state_row(), qk_parts, v_parts);

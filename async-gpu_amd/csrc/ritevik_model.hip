@@ -417,14 +417,6 @@ int32_t mixer(agpu_ritevik *m, const Run &r, int B, int new_len, int max_kv, voi
             a.bkq = (float *)m->dbkq.p;
             a.gate = (float *)m->dgate.p;
             a.o = (float *)m->dout.p;
-            // the low-rank products in fp32: they feed decays and gates
-            DenseOut og, oo;
-            og.n_plain = og.ldo = L.a2.N;
-            og.out = a.step;
-            AGPU_TRY(dense_gemm_f32_launch(m->ctx, proj + L.col_a1, L.n_plain, L.a2.w, L.a2.K, R, L.a2.N, L.a2.K, og));
-            oo.n_plain = oo.ldo = L.g2.N;
-            oo.out = a.gate;
-            AGPU_TRY(dense_gemm_f32_launch(m->ctx, proj + L.col_g1, L.n_plain, L.g2.w, L.g2.K, R, L.g2.N, L.g2.K, oo));
             AGPU_TRY(delta_prefill_launch(m->ctx, a));
         }
     }

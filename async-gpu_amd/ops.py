@@ -300,3 +300,61 @@ def top_k_sample(logits, k, temperature, rng):
     context(lg.device.index or 0).call("agpu_top_k_sample", lg, lg.numel(), int(k), float(temperature), C.addressof(rng._s),
                                        C.addressof(tok))
     return int(tok.value)
+
+
+# ---- layers with bf16 weights (include/agpu.h); weights are int16 / uint16 bit patterns on the device ----
+
+def rms_norm(x, weight, eps, weight_offset=0.0):
+    """x / rms(x) * (weight_offset + weight) over the last dimension."""
+    d = x.shape[-1]
+    if weight.numel() != d:
+        _shape_err(f"weight of {d}", f"weight of {weight.numel()}")
+    y = torch.empty_like(_f32(x))
+    context(x.device.index or 0).call("agpu_rms_norm", x, weight, float(weight_offset), y, x.numel() // d, d, float(eps))
+    return y
+
+
+def dense_linear(x, w, bias=None, residual=None, dtype=_lib.DTYPE_BF16, gated=False):
+    """x [M, K] w [N, K]^T (+ bias) (+ residual); gated: silu(rows 0, 2, ..) * rows 1, 3, .. of w -> [M, N / 2]."""
+    (M, K), (N, K2) = x.shape, w.shape
+    if K != K2:
+        _shape_err(f"last dim = {K2}", f"last dim = {K}")
+    y = torch.empty((M, N // 2 if gated else N), dtype=torch.float32, device=x.device)
+    context(x.device.index or 0).call("agpu_dense_linear", _f32(x), w, bias, residual, y, M, N, K, dtype, _lib.DENSE_GATED if gated else 0)
+    return y
+
+
+def rope_table(positions, dims, base, device=0):
+    t = torch.empty((positions, dims // 2, 2), dtype=torch.float32, device=f"cuda:{device}")
+    context(device).call("agpu_rope_table", t, positions, dims, float(base))
+    return t
+
+
+def _workspace(c, name, desc, device):
+    import ctypes as C
+    n = getattr(_lib.cdll(), name)(c.handle, C.addressof(desc))
+    if n == 0:
+        raise AgpuError(_lib.ERR_SHAPE_MISMATCH, f"{name[:-len('_workspace_bytes')]}: sizes not supported")
+    return torch.empty(n, dtype=torch.uint8, device=device)
+
+
+def latent_attention(desc, q, down, norm, uk, uv, sink, rope, cache):
+    """agpu_latent_attention on a filled _lib.LatentAttentionDesc; appends to `cache`, returns [batch * new_len, heads * vdim]."""
+    import ctypes as C
+    c = context(q.device.index or 0)
+    desc.ldo = desc.heads * desc.vdim
+    out = torch.empty((desc.batch * desc.new_len, desc.ldo), dtype=torch.float32, device=q.device)
+    ws = _workspace(c, "agpu_latent_attention_workspace_bytes", desc, q.device)
+    c.call("agpu_latent_attention", C.addressof(desc), q, down, norm, uk, uv, sink, rope, cache, out, ws)
+    return out
+
+
+def channel_delta(desc, proj, conv, a_log, dt_bias, a2, g2, norm, state, ring):
+    """agpu_channel_delta on a filled _lib.ChannelDeltaDesc; advances `state` and `ring`, returns [batch * new_len, heads * vdim]."""
+    import ctypes as C
+    c = context(proj.device.index or 0)
+    desc.ldo = desc.heads * desc.vdim
+    out = torch.empty((desc.batch * desc.new_len, desc.ldo), dtype=torch.float32, device=proj.device)
+    ws = _workspace(c, "agpu_channel_delta_workspace_bytes", desc, proj.device)
+    c.call("agpu_channel_delta", C.addressof(desc), proj, conv, a_log, dt_bias, a2, g2, norm, state, ring, out, ws)
+    return out

@@ -349,6 +349,76 @@ int32_t agpu_kv_append(agpu_ctx *ctx, const float *src, float *cache, int32_t n_
 int32_t agpu_gemm_f32(agpu_ctx *ctx, const float *a, const float *b, float *c, int32_t M, int32_t N,
                       int32_t K);
 
+/* ---- layers with bf16 weights (no counterpart in the reference) ---------------------------
+ *
+ * Mechanisms of the models whose weights stay in bf16 (agpu_ritevik.h), one operator each with its constants as
+ * parameters.  Weights are bf16 bits, rows along the input axis ([out, in]); everything else is fp32. */
+
+#define AGPU_DTYPE_BF16 0
+#define AGPU_DTYPE_F32 1
+
+/* y = x / sqrt(mean(x^2) + eps) * (weight_offset + weight) over rows of d.  weight_offset 1: a weight stored around zero. */
+int32_t agpu_rms_norm(agpu_ctx *ctx, const float *x, const float *weight, float weight_offset, float *y, int32_t rows, int32_t d, float eps);
+
+#define AGPU_DENSE_GATED 1u /* rows 2 j and 2 j + 1 of w are a gate and its up: y [M, N / 2] = silu(gate) * up */
+/* y [M, N] = x [M, K] w [N, K]^T (+ bias) (+ residual, may alias y; neither with AGPU_DENSE_GATED).  K % 32 == 0.  Up to 4 rows
+ * run on fp32 FMAs; more rows on the matrix cores, with x rounded to bf16 (dtype AGPU_DTYPE_BF16) or in fp32
+ * (AGPU_DTYPE_F32).  The rounded rows live in the context's scratch. */
+int32_t agpu_dense_linear(agpu_ctx *ctx, const float *x, const uint16_t *w, const float *bias, const float *residual, float *y, int32_t M,
+                          int32_t N, int32_t K, int32_t dtype, uint32_t flags);
+
+/* cos and sin of p * base^(-2 i / dims), computed in double precision: table [positions][dims / 2] pairs of floats. */
+int32_t agpu_rope_table(agpu_ctx *ctx, float *table, int32_t positions, int32_t dims, double base);
+
+/*
+ * Latent attention over a cache of latents, causal, `new_len` new tokens of each of `batch` sequences behind `cached` ones:
+ *   q rows [batch * new_len, ld]: per head [dim | rot_dim], the rot_dim part not yet rotated; down rows [.., ld]: [rank | rot_dim]
+ *   c = RMS norm of the first rank columns of down (weight norm); k_rot = its last rot_dim, rotated; both appended to
+ *   cache [batch][positions][row] (row: agpu_latent_cache_row; bf16 or fp32 by cache_dtype; zeros beyond the columns used)
+ *   score = (q . W_uk c + q_rot . k_rot) * scale; softmax with exp(sink) of the head in the denominator (sink may be NULL);
+ *   out rows [.., ldo]: per head W_uv of the attended latent.
+ * The first rot_dims of the rot_dim dimensions turn, i with i + rot_dims / 2 (rope: agpu_rope_table).  uk
+ * [heads * dim][rank], uv [heads * vdim][rank].  Sizes: rank % 32 == 0, dim % 8 == 0, vdim % 32 == 0, rot_dim % 8 == 0 (the model
+ * driver pads; this operator does not), rank and dim <= 1024.  tiled != 0: the matrix-core form for prompts (bf16 cache,
+ * dim + rot_dim <= 192, vdim <= 128); else the form that reads the latents directly.  workspace: device memory of
+ * agpu_latent_attention_workspace_bytes.
+ */
+typedef struct agpu_latent_attention_desc {
+    int32_t heads, dim, rot_dim, rot_dims, vdim, rank;
+    float scale, eps;
+    int32_t positions, batch, new_len, cached, ld, ldo, cache_dtype, tiled;
+} agpu_latent_attention_desc;
+int32_t agpu_latent_cache_row(int32_t rank, int32_t rot_dim);
+size_t agpu_latent_attention_workspace_bytes(const agpu_ctx *ctx, const agpu_latent_attention_desc *desc);
+int32_t agpu_latent_attention(agpu_ctx *ctx, const agpu_latent_attention_desc *desc, const float *q, const float *down, const float *norm,
+                              const uint16_t *uk, const uint16_t *uv, const float *sink, const float *rope, void *cache, float *out,
+                              void *workspace);
+
+/*
+ * Gated delta rule with one decay per head and key channel, `new_len` tokens of each of `batch` sequences behind `cached` ones.
+ *   proj rows [batch * new_len, ld] hold the projections of the layer's input at columns col_*: q, k (kv_heads x dim), v (heads x
+ *   vdim), b (heads), a1 (decay_rank), g1 (gate_rank)
+ *   q, k, v pass a causal convolution of `taps` taps per channel (conv [q | k | v channels][taps], last column the current
+ *   token) and silu; q and k become x / sqrt(sum x^2 + 1e-6) per head, q also times dim^-1/2; head h uses q and k of head
+ *   h / (heads / kv_heads)
+ *   g = exp(-exp(a_log) * softplus(a2 a1 + dt_bias)), beta = sigmoid(b); per head S <- diag(g) S, u = beta (v - S^T k),
+ *   S <- S + k u^T, o = S^T q
+ *   out rows [.., ldo] = o / rms(o) * norm * sigmoid(g2 g1)
+ * a2 [heads * dim][decay_rank], g2 [heads * vdim][gate_rank].  state: fp32 [batch][heads][vdim][dim], ring [batch][taps][channels]:
+ * the convolution inputs of the last tokens (slot: position % taps); both start as zeros.  Sizes: dim % 32 == 0, ranks % 32 == 0,
+ * columns and ld % 4 == 0 (the model driver pads; this operator does not), dim and vdim <= 256.
+ */
+typedef struct agpu_channel_delta_desc {
+    int32_t heads, kv_heads, dim, vdim, taps, decay_rank, gate_rank;
+    float eps;
+    int32_t batch, new_len, cached, ld, ldo;
+    int32_t col_q, col_k, col_v, col_b, col_a1, col_g1;
+} agpu_channel_delta_desc;
+size_t agpu_channel_delta_workspace_bytes(const agpu_ctx *ctx, const agpu_channel_delta_desc *desc);
+int32_t agpu_channel_delta(agpu_ctx *ctx, const agpu_channel_delta_desc *desc, const float *proj, const float *conv, const float *a_log,
+                           const float *dt_bias, const uint16_t *a2, const uint16_t *g2, const float *norm, float *state, float *ring,
+                           float *out, void *workspace);
+
 #ifdef __cplusplus
 }
 #endif

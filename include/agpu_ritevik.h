@@ -29,9 +29,6 @@ extern "C" {
 
 typedef struct agpu_ritevik agpu_ritevik;
 
-#define AGPU_DTYPE_BF16 0
-#define AGPU_DTYPE_F32 1
-
 #define AGPU_MIXER_LATENT_ATTENTION 0
 #define AGPU_MIXER_CHANNEL_DELTA 1
 

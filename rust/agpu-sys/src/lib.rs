@@ -1,5 +1,5 @@
 //! agpu-sys: the raw `extern "C"` surface of libagpu_hip.so, the MI355X (gfx950) implementation of async_gpu's
-//! quantized GPT-2 inference path.  One declaration per function of `include/agpu.h` and `include/agpu_gpt2.h`,
+//! quantized GPT-2 inference path.  One declaration per function of `include/agpu.h`, `agpu_gpt2.h` and `agpu_ritevik.h`,
 //! in header order; `build.rs` compiles the HIP sources with hipcc and links the shared library.
 //!
 //! What each function replaces in the reference is stated next to its C declaration.  The safe layer over these
@@ -49,6 +49,97 @@ pub struct agpu_gpt2_config {
     pub argmax_last: i32,
 }
 
+/// `agpu_latent_attention_desc` of include/agpu.h.
+#[repr(C)]
+#[derive(Clone, Copy, Debug, Default)]
+pub struct agpu_latent_attention_desc {
+    pub heads: i32,
+    pub dim: i32,
+    pub rot_dim: i32,
+    pub rot_dims: i32,
+    pub vdim: i32,
+    pub rank: i32,
+    pub scale: f32,
+    pub eps: f32,
+    pub positions: i32,
+    pub batch: i32,
+    pub new_len: i32,
+    pub cached: i32,
+    pub ld: i32,
+    pub ldo: i32,
+    pub cache_dtype: i32,
+    pub tiled: i32,
+}
+
+/// `agpu_channel_delta_desc` of include/agpu.h.
+#[repr(C)]
+#[derive(Clone, Copy, Debug, Default)]
+pub struct agpu_channel_delta_desc {
+    pub heads: i32,
+    pub kv_heads: i32,
+    pub dim: i32,
+    pub vdim: i32,
+    pub taps: i32,
+    pub decay_rank: i32,
+    pub gate_rank: i32,
+    pub eps: f32,
+    pub batch: i32,
+    pub new_len: i32,
+    pub cached: i32,
+    pub ld: i32,
+    pub ldo: i32,
+    pub col_q: i32,
+    pub col_k: i32,
+    pub col_v: i32,
+    pub col_b: i32,
+    pub col_a1: i32,
+    pub col_g1: i32,
+}
+
+/// Opaque Ritevik model.
+#[repr(C)]
+pub struct agpu_ritevik {
+    _private: [u8; 0],
+}
+
+/// `agpu_ritevik_config` of include/agpu_ritevik.h.
+#[repr(C)]
+#[derive(Clone, Copy, Debug, Default)]
+pub struct agpu_ritevik_config {
+    pub n_layer: i32,
+    pub width: i32,
+    pub vocab_size: i32,
+    pub n_positions: i32,
+    pub max_batch: i32,
+    pub norm_eps: f32,
+    pub loop_start: i32,
+    pub loop_stop: i32,
+    pub loop_times: i32,
+    pub side_dim: i32,
+    pub dtype: i32,
+    pub argmax_last: i32,
+}
+
+/// `agpu_ritevik_layer` of include/agpu_ritevik.h.
+#[repr(C)]
+#[derive(Clone, Copy, Debug, Default)]
+pub struct agpu_ritevik_layer {
+    pub mixer: i32,
+    pub heads: i32,
+    pub dim: i32,
+    pub vdim: i32,
+    pub ff: i32,
+    pub kv_rank: i32,
+    pub rot_dim: i32,
+    pub rot_dims: i32,
+    pub scale: f32,
+    pub rot_base: f64,
+    pub kv_heads: i32,
+    pub conv: i32,
+    pub decay_rank: i32,
+    pub gate_rank: i32,
+}
+
 pub const AGPU_OK: i32 = 0;
 pub const AGPU_ERR_SHAPE_MISMATCH: i32 = -1;
 pub const AGPU_ERR_DIM_OUT_OF_RANGE: i32 = -2;
@@ -77,6 +168,11 @@ pub const AGPU_LINEAR_FC_PROJ: i32 = 3;
 pub const AGPU_DECODE_AUTO: i32 = 0;
 pub const AGPU_DECODE_PER_STAGE: i32 = 1;
 pub const AGPU_DECODE_EAGER: i32 = 2;
+pub const AGPU_DTYPE_BF16: i32 = 0;
+pub const AGPU_DTYPE_F32: i32 = 1;
+pub const AGPU_DENSE_GATED: u32 = 1;
+pub const AGPU_MIXER_LATENT_ATTENTION: i32 = 0;
+pub const AGPU_MIXER_CHANNEL_DELTA: i32 = 1;
 
 extern "C" {
     // ---- include/agpu.h ----
@@ -131,6 +227,14 @@ extern "C" {
     pub fn agpu_bench_attention(ctx: *mut agpu_ctx, q: *const f32, k: *const f32, v: *const f32, o: *mut f32, n_heads: i32, q_len: i32, kv_len: i32, q_offset: i32, kv_stride: i32, d_head: i32, causal: i32, reps: i32, us_per_launch_out_host: *mut f32) -> i32;
     pub fn agpu_kv_append(ctx: *mut agpu_ctx, src: *const f32, cache: *mut f32, n_heads: i32, src_stride: i32, max_seq: i32, write_pos: i32, d_head: i32) -> i32;
     pub fn agpu_gemm_f32(ctx: *mut agpu_ctx, a: *const f32, b: *const f32, c: *mut f32, M: i32, N: i32, K: i32) -> i32;
+    pub fn agpu_rms_norm(ctx: *mut agpu_ctx, x: *const f32, weight: *const f32, weight_offset: f32, y: *mut f32, rows: i32, d: i32, eps: f32) -> i32;
+    pub fn agpu_dense_linear(ctx: *mut agpu_ctx, x: *const f32, w: *const u16, bias: *const f32, residual: *const f32, y: *mut f32, M: i32, N: i32, K: i32, dtype: i32, flags: u32) -> i32;
+    pub fn agpu_rope_table(ctx: *mut agpu_ctx, table: *mut f32, positions: i32, dims: i32, base: f64) -> i32;
+    pub fn agpu_latent_cache_row(rank: i32, rot_dim: i32) -> i32;
+    pub fn agpu_latent_attention_workspace_bytes(ctx: *const agpu_ctx, desc: *const agpu_latent_attention_desc) -> usize;
+    pub fn agpu_latent_attention(ctx: *mut agpu_ctx, desc: *const agpu_latent_attention_desc, q: *const f32, down: *const f32, norm: *const f32, uk: *const u16, uv: *const u16, sink: *const f32, rope: *const f32, cache: *mut c_void, out: *mut f32, workspace: *mut c_void) -> i32;
+    pub fn agpu_channel_delta_workspace_bytes(ctx: *const agpu_ctx, desc: *const agpu_channel_delta_desc) -> usize;
+    pub fn agpu_channel_delta(ctx: *mut agpu_ctx, desc: *const agpu_channel_delta_desc, proj: *const f32, conv: *const f32, a_log: *const f32, dt_bias: *const f32, a2: *const u16, g2: *const u16, norm: *const f32, state: *mut f32, ring: *mut f32, out: *mut f32, workspace: *mut c_void) -> i32;
     // ---- include/agpu_gpt2.h ----
     pub fn agpu_gpt2_config_small(out: *mut agpu_gpt2_config) -> i32;
     pub fn agpu_gpt2_config_xl(out: *mut agpu_gpt2_config) -> i32;
@@ -158,4 +262,22 @@ extern "C" {
     pub fn agpu_gpt2_decode_floor(m: *mut agpu_gpt2, steps: i32, ms_total_out_host: *mut f32) -> i32;
     pub fn agpu_gpt2_last_logits(m: *mut agpu_gpt2, batch: i32, logits_out_host: *mut f32) -> i32;
     pub fn agpu_gpt2_decode_steps(m: *mut agpu_gpt2, batch: i32, steps: i32, ms_total_out_host: *mut f32) -> i32;
+    // ---- include/agpu_ritevik.h ----
+    pub fn agpu_ritevik_create(ctx: *mut agpu_ctx, cfg: *const agpu_ritevik_config, layers: *const agpu_ritevik_layer, out: *mut *mut agpu_ritevik) -> i32;
+    pub fn agpu_ritevik_destroy(m: *mut agpu_ritevik) -> i32;
+    pub fn agpu_ritevik_set_tensor(m: *mut agpu_ritevik, name: *const c_char, data_host: *const c_void, dtype: i32, rows: i64, cols: i64) -> i32;
+    pub fn agpu_ritevik_tensor_info(m: *const agpu_ritevik, i: i32, name_out: *mut *const c_char, rows_out: *mut i64, cols_out: *mut i64, is_set_out: *mut i32) -> i32;
+    pub fn agpu_ritevik_weight_bytes(m: *const agpu_ritevik) -> i64;
+    pub fn agpu_ritevik_cache_bytes(m: *const agpu_ritevik) -> i64;
+    pub fn agpu_ritevik_layer_runs(m: *const agpu_ritevik) -> i32;
+    pub fn agpu_ritevik_reset_cache(m: *mut agpu_ritevik) -> i32;
+    pub fn agpu_ritevik_cache_len(m: *const agpu_ritevik) -> i32;
+    pub fn agpu_ritevik_forward_cached(m: *mut agpu_ritevik, tokens: *const u32, batch: i32, new_len: i32, logits: *mut f32, all_rows: i32) -> i32;
+    pub fn agpu_ritevik_generate_cached(m: *mut agpu_ritevik, prompt_host: *const u32, batch: i32, prompt_len: i32, max_new_tokens: i32, eos: i32, tokens_out_host: *mut u32, lengths_out_host: *mut i32, timing_ms_out_host: *mut f32) -> i32;
+    pub fn agpu_ritevik_generate(m: *mut agpu_ritevik, prompt_host: *const u32, prompt_len: i32, max_new_tokens: i32, eos: i32, tokens_out_host: *mut u32, length_out_host: *mut i32) -> i32;
+    pub fn agpu_ritevik_generate_cached_sampling(m: *mut agpu_ritevik, prompt_host: *const u32, prompt_len: i32, max_new_tokens: i32, top_k: i32, temperature: f32, rng_state: *mut u64, eos: i32, tokens_out_host: *mut u32, length_out_host: *mut i32) -> i32;
+    pub fn agpu_ritevik_set_decode_mode(m: *mut agpu_ritevik, mode: i32) -> i32;
+    pub fn agpu_ritevik_decode_steps(m: *mut agpu_ritevik, batch: i32, steps: i32, ms_total_out_host: *mut f32) -> i32;
+    pub fn agpu_ritevik_last_logits(m: *mut agpu_ritevik, batch: i32, logits_out_host: *mut f32) -> i32;
+    pub fn agpu_ritevik_layer_streams(m: *mut agpu_ritevik, tokens: *const u32, new_len: i32, streams_out_host: *mut f32) -> i32;
 }

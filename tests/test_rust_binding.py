@@ -5,10 +5,12 @@ bound number of arguments."""
 import os
 import re
 
+import pytest
+
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
 SCALARS = {"int32_t": "i32", "uint32_t": "u32", "int64_t": "i64", "uint64_t": "u64", "size_t": "usize", "float": "f32",
-           "char": "c_char", "void": "c_void"}
+           "double": "f64", "uint16_t": "u16", "char": "c_char", "void": "c_void"}
 
 
 def c_type_to_rust(t):
@@ -67,9 +69,12 @@ def test_every_header_function_is_bound_with_the_same_signature():
         assert c[name] == r[name], f"{name}: header {c[name]} != binding {r[name]}"
 
 
-def test_config_struct_fields_match():
-    header = open(os.path.join(ROOT, "include", "agpu_gpt2.h")).read()
-    body = re.search(r"typedef struct agpu_gpt2_config \{(.*?)\} agpu_gpt2_config;", header, flags=re.S).group(1)
+@pytest.mark.parametrize("header_name, struct", [("agpu_gpt2.h", "agpu_gpt2_config"), ("agpu.h", "agpu_latent_attention_desc"),
+                                                 ("agpu.h", "agpu_channel_delta_desc"), ("agpu_ritevik.h", "agpu_ritevik_config"),
+                                                 ("agpu_ritevik.h", "agpu_ritevik_layer")])
+def test_config_struct_fields_match(header_name, struct):
+    header = open(os.path.join(ROOT, "include", header_name)).read()
+    body = re.search(r"typedef struct %s \{(.*?)\} %s;" % (struct, struct), header, flags=re.S).group(1)
     body = re.sub(r"/\*.*?\*/", "", body, flags=re.S)
     c_fields = []
     for decl in body.split(";"):
@@ -79,7 +84,7 @@ def test_config_struct_fields_match():
         ty, names = decl.split(" ", 1)
         c_fields += [(n.strip(), SCALARS[ty]) for n in names.split(",")]
     rust = open(os.path.join(ROOT, "rust", "agpu-sys", "src", "lib.rs")).read()
-    rbody = re.search(r"pub struct agpu_gpt2_config \{(.*?)\}", rust, flags=re.S).group(1)
+    rbody = re.search(r"pub struct %s \{(.*?)\}" % struct, rust, flags=re.S).group(1)
     r_fields = [(m.group(1), m.group(2)) for m in re.finditer(r"pub (\w+): (\w+),", rbody)]
     assert c_fields == r_fields
 
@@ -88,11 +93,11 @@ def test_constants_match_the_headers():
     rust = open(os.path.join(ROOT, "rust", "agpu-sys", "src", "lib.rs")).read()
     consts = {m.group(1): int(m.group(2), 0) for m in re.finditer(r"pub const (AGPU_\w+): \w+ = (-?(?:0x)?[0-9a-fA-F]+);", rust)}
     assert len(consts) >= 25
-    for fn in ("agpu.h", "agpu_gpt2.h"):
+    for fn in ("agpu.h", "agpu_gpt2.h", "agpu_ritevik.h"):
         text = open(os.path.join(ROOT, "include", fn)).read()
         for m in re.finditer(r"#define (AGPU_\w+) \(?(-?(?:0x)?[0-9a-fA-F]+)u?\)?", text):
             name, value = m.group(1), int(m.group(2), 0)
-            if name in ("AGPU_H", "AGPU_GPT2_H"):
+            if name in ("AGPU_H", "AGPU_GPT2_H", "AGPU_RITEVIK_H"):
                 continue
             assert name in consts, f"{name} of {fn} has no Rust constant"
             assert consts[name] == value, name
