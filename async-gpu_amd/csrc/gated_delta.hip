@@ -231,40 +231,46 @@ __global__ __launch_bounds__(64 * kRecWaves) void delta_recurrence_kernel(DeltaA
     for (int t0 = 0; t0 < T; t0 += kChunk, buf ^= 1) {
         const bool more = t0 + kChunk < T;
         if (more) request(t0 + kChunk);
-        // the vectors of the next token are on their way while this one is worked on
-        float q[DR], k[DR], g[DR], v, beta, kq;
-        auto fetch = [&](int i) {
-#pragma unroll
-            for (int r = 0; r < DR; ++r) {
-                q[r] = sv[buf][i][0][l32 * DR + r];
-                k[r] = sv[buf][i][1][l32 * DR + r];
-                g[r] = sv[buf][i][2][l32 * DR + r];
-            }
-            v = sc[buf][i][wave * 2 + half];
-            beta = sc[buf][i][COLS];
-            kq = sc[buf][i][COLS + 1];
+        // two sets of registers: the vectors of the next token are on their way while this one is worked on
+        struct Token {
+            float q[DR], k[DR], g[DR], v, beta, kq;
+        } even, odd;
+        constexpr int AL = DR % 4 == 0 ? 16 : (DR % 2 == 0 ? 8 : 4);
+        auto fetch = [&](Token &x, int i) {
+            __builtin_memcpy(x.q, __builtin_assume_aligned(&sv[buf][i][0][l32 * DR], AL), 4 * DR);
+            __builtin_memcpy(x.k, __builtin_assume_aligned(&sv[buf][i][1][l32 * DR], AL), 4 * DR);
+            __builtin_memcpy(x.g, __builtin_assume_aligned(&sv[buf][i][2][l32 * DR], AL), 4 * DR);
+            x.v = sc[buf][i][wave * 2 + half];
+            x.beta = sc[buf][i][COLS];
+            x.kq = sc[buf][i][COLS + 1];
         };
-        fetch(0);
         float out = 0.0f;
-#pragma unroll 4
-        for (int i = 0; i < kChunk; ++i) {
-            float kc[DR];
+        auto work = [&](const Token &x, int i) {
             float ks = 0.0f, qs = 0.0f;
-            const float vc = v, bc = beta, kqc = kq;
 #pragma unroll
             for (int r = 0; r < DR; ++r) {
-                kc[r] = k[r];
-                S[r] *= g[r];
-                ks = fmaf(S[r], kc[r], ks);
-                qs = fmaf(S[r], q[r], qs);
+                S[r] *= x.g[r];
+                ks = fmaf(S[r], x.k[r], ks);
+                qs = fmaf(S[r], x.q[r], qs);
             }
-            fetch(min(i + 1, kChunk - 1));
             ks = half_sum(ks);
             qs = half_sum(qs);
-            const float u = bc * (vc - ks);
+            const float u = x.beta * (x.v - ks);
 #pragma unroll
-            for (int r = 0; r < DR; ++r) S[r] = fmaf(kc[r], u, S[r]);
-            out = l32 == i ? fmaf(kqc, u, qs) : out;  // lane i keeps the output of token i
+            for (int r = 0; r < DR; ++r) S[r] = fmaf(x.k[r], u, S[r]);
+            out = l32 == i ? fmaf(x.kq, u, qs) : out;  // lane i keeps the output of token i
+        };
+        fetch(even, 0);
+#pragma unroll 1
+        for (int i = 0; i < kChunk; i += 2) {
+            fetch(odd, i + 1);
+            __builtin_amdgcn_sched_barrier(0);
+            work(even, i);
+            __builtin_amdgcn_sched_barrier(0);
+            fetch(even, min(i + 2, kChunk - 1));
+            __builtin_amdgcn_sched_barrier(0);
+            work(odd, i + 1);
+            __builtin_amdgcn_sched_barrier(0);
         }
         if (l32 < kChunk && j < s.vdim && t0 + l32 < T) a.o[(row0 + t0 + l32) * nv + h * s.vdim + j] = out;
         if (more) stage(buf ^ 1, t0 + kChunk);

@@ -23,6 +23,7 @@ constexpr int kHeadTile = 4;    // heads per workgroup of the absorbed kernel (o
 constexpr int kKeyChunk = 64;   // keys per step: one per lane
 constexpr int kMaxSplits = 64;
 constexpr int kMatrixHeads = 16;  // heads per workgroup of the matrix-core kernel
+constexpr int kMatrixChunk = 32;  // keys per step of the matrix-core kernel
 constexpr float kMinusInf = -3.0e38f;
 
 __global__ void rope_table_kernel(float2 *table, int positions, int half, double base) {
@@ -269,88 +270,82 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(LatentArgs a, const 
         *(float2 *)(part_ml + (((size_t)row * s.heads + h0 + wave) * splits + blockIdx.x) * 2) = make_float2(m, l);
 }
 
-// grid (splits, ceil(heads / 16), rows), four waves; bf16 cache.  A chunk of 64 cache rows goes to LDS; wave w scores keys
-// 16 w .. + 15 for 16 heads (v_mfma_f32_16x16x32_bf16, queries as two pieces), 16 threads per head do the softmax, and the
-// waves share the latent's columns of the second product (probabilities as two pieces).  CT column tiles of 16 per wave.
-template <int CT>
-__global__ __launch_bounds__(256) void latent_attend_matrix_kernel(LatentArgs a, int rankp, int row_len, int splits) {
-    extern __shared__ __align__(16) uint16_t tile[];  // [64][ld], then the queries [2][16][ld]
-    __shared__ float sc[kMatrixHeads][kKeyChunk + 4];
-    __shared__ __align__(16) uint16_t pr[2][kMatrixHeads][kKeyChunk + 8];
+// grid (splits, ceil(heads / 16), rows), four waves; bf16 cache.  A chunk of 32 cache rows goes to LDS.  Scores
+// (v_mfma_f32_16x16x32_bf16, queries as two pieces, in registers): the waves share the cache row's columns, 32 at a time, and
+// add up in LDS; 16 threads per head do the softmax; the waves share the latent's columns of the second product
+// (probabilities as two pieces).  CT column tiles of 16 per wave, NK steps of 32 cache columns per wave.
+template <int CT, int NK>
+__global__ __launch_bounds__(256, 2) void latent_attend_matrix_kernel(LatentArgs a, int rankp, int row_len, int splits) {
+    extern __shared__ __align__(16) uint16_t tile[];  // [32][ld]
+    __shared__ float sc[4][kMatrixHeads][kMatrixChunk + 4];
+    __shared__ __align__(16) uint16_t pr[2][kMatrixHeads][kMatrixChunk + 8];
     __shared__ float corr[kMatrixHeads];
     const LatentShape &s = a.s;
     const int t = threadIdx.x, lane = t & 63, wave = t >> 6, lr = lane & 15, lq = lane >> 4;
     const int row = blockIdx.z, h0 = blockIdx.y * kMatrixHeads, b = row / a.new_len, ld = row_len + 8, n32 = row_len >> 5;
     const int kv = *a.pos_dev + row % a.new_len + 1;
-    const int chunks = (kv + kKeyChunk - 1) / kKeyChunk;
+    const int chunks = (kv + kMatrixChunk - 1) / kMatrixChunk;
     const int per = (chunks + splits - 1) / splits;
     const int c_lo = min((int)blockIdx.x * per, chunks), c_hi = min(c_lo + per, chunks);
     const uint16_t *cache = (const uint16_t *)a.cache + (size_t)b * a.positions * row_len;
-    uint16_t *sq = tile + kKeyChunk * ld;
     const size_t pieces = (size_t)gridDim.z * s.heads * row_len;
-    if (c_lo < c_hi) {  // 16 threads per head
-        const int h = t >> 4;
-        const uint16_t *q = (const uint16_t *)a.qlat + ((size_t)row * s.heads + min(h0 + h, s.heads - 1)) * row_len;
-#pragma unroll 4
-        for (int c = (t & 15) * 8; c < row_len; c += 128) {
-            const uint4 hi = *(const uint4 *)(q + c), lo = *(const uint4 *)(q + pieces + c);
-            *(uint4 *)(sq + h * ld + c) = hi;
-            *(uint4 *)(sq + (kMatrixHeads + h) * ld + c) = lo;
-        }
+    bf16x8 qf[NK][2];  // of column step wave + 4 n; zero beyond the row
+    {
+        const uint16_t *q = (const uint16_t *)a.qlat + ((size_t)row * s.heads + min(h0 + lr, s.heads - 1)) * row_len + lq * 8;
+#pragma unroll
+        for (int n = 0; n < NK; ++n)
+#pragma unroll
+            for (int pc = 0; pc < 2; ++pc) {
+                const int step = wave + 4 * n;
+                const uint4 v = *(const uint4 *)(q + pc * pieces + min(step, n32 - 1) * 32);
+                qf[n][pc] = __builtin_bit_cast(bf16x8, step < n32 ? v : make_uint4(0, 0, 0, 0));
+            }
     }
     f32x4 acc[CT];
 #pragma unroll
     for (int i = 0; i < CT; ++i) acc[i] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
     float m = kMinusInf, l = 0.0f;  // of head h0 + t / 16
     for (int ck = c_lo; ck < c_hi; ++ck) {
-        const int k0 = ck * kKeyChunk;
-        {  // four threads per key
-            const uint16_t *src = cache + (size_t)min(k0 + (t >> 2), kv - 1) * row_len + (t & 3) * 8;
-            uint16_t *dst = tile + (t >> 2) * ld + (t & 3) * 8;
-            constexpr int U = 9;
-#pragma unroll 1
-            for (int n = 0; n < n32; n += U) {
-                uint4 v[U];
+        const int k0 = ck * kMatrixChunk;
+        {  // eight threads per key
+            const uint16_t *src = cache + (size_t)min(k0 + (t >> 3), kv - 1) * row_len;
+            uint16_t *dst = tile + (t >> 3) * ld;
+            constexpr int U = 2 * NK;  // row_len / 8 pieces of 16 bytes over 8 threads
+            uint4 v[U];
 #pragma unroll
-                for (int u = 0; u < U; ++u) v[u] = *(const uint4 *)(src + min(n + u, n32 - 1) * 32);
+            for (int u = 0; u < U; ++u) v[u] = *(const uint4 *)(src + min(((t & 7) + 8 * u) * 8, row_len - 8));
 #pragma unroll
-                for (int u = 0; u < U; ++u) *(uint4 *)(dst + min(n + u, n32 - 1) * 32) = v[u];
-            }
+            for (int u = 0; u < U; ++u) *(uint4 *)(dst + min(((t & 7) + 8 * u) * 8, row_len - 8)) = v[u];
         }
         __syncthreads();
-        f32x4 sv = {0.0f, 0.0f, 0.0f, 0.0f};
-        {
-            const uint16_t *kp = tile + (wave * 16 + lr) * ld + lq * 8, *qh = sq + lr * ld + lq * 8, *ql = qh + kMatrixHeads * ld;
-            f32x4 s2 = sv;
-            auto fma_step = [&](int n, f32x4 &c) {
-                const bf16x8 kf = *(const bf16x8 *)(kp + n * 32), qlo = *(const bf16x8 *)(ql + n * 32), qhi = *(const bf16x8 *)(qh + n * 32);
-                c = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qlo, kf, c, 0, 0, 0);
-                c = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qhi, kf, c, 0, 0, 0);
-            };
-            int n = 0;
-            for (; n + 1 < n32; n += 2) {
-                fma_step(n, sv);
-                fma_step(n + 1, s2);
-            }
-            if (n < n32) fma_step(n, sv);
-            sv += s2;
-        }
-        // result register r of lane l: head 4 (l / 16) + r, key l % 16
 #pragma unroll
-        for (int r = 0; r < 4; ++r) sc[lq * 4 + r][wave * 16 + lr] = sv[r] * s.scale;
+        for (int kt = 0; kt < 2; ++kt) {
+            f32x4 hi = {0.0f, 0.0f, 0.0f, 0.0f}, lo = hi;
+            const uint16_t *kp = tile + (kt * 16 + lr) * ld + lq * 8;
+#pragma unroll
+            for (int n = 0; n < NK; ++n) {
+                const bf16x8 kf = *(const bf16x8 *)(kp + min(wave + 4 * n, n32 - 1) * 32);
+                lo = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[n][1], kf, lo, 0, 0, 0);
+                hi = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[n][0], kf, hi, 0, 0, 0);
+            }
+            // result register r of lane l: head 4 (l / 16) + r, key l % 16
+#pragma unroll
+            for (int r = 0; r < 4; ++r) sc[wave][lq * 4 + r][kt * 16 + lr] = hi[r] + lo[r];
+        }
         __syncthreads();
         {
             const int h = t >> 4;
-            float v[4], top = kMinusInf;
+            float v[2];
 #pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                v[e] = k0 + lr + 16 * e < kv ? sc[h][lr + 16 * e] : kMinusInf;
-                top = fmaxf(top, v[e]);
+            for (int e = 0; e < 2; ++e) {
+                const int k = lr + 16 * e;
+                const float x = (sc[0][h][k] + sc[1][h][k] + sc[2][h][k] + sc[3][h][k]) * s.scale;
+                v[e] = k0 + k < kv ? x : kMinusInf;
             }
-            const float m_new = fmaxf(m, row16_max(top));
+            const float m_new = fmaxf(m, row16_max(fmaxf(v[0], v[1])));
             float sum = 0.0f;
 #pragma unroll
-            for (int e = 0; e < 4; ++e) {
+            for (int e = 0; e < 2; ++e) {
                 const float p = v[e] > kMinusInf ? expf(v[e] - m_new) : 0.0f;
                 sum += p;
                 const uint16_t hi = f32_to_bf16(p);
@@ -366,27 +361,19 @@ __global__ __launch_bounds__(256) void latent_attend_matrix_kernel(LatentArgs a,
         float cr[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) cr[r] = corr[lq * 4 + r];
-        bf16x8 pf[2][2];
+        const bf16x8 phi = *(const bf16x8 *)&pr[0][lr][8 * lq], plo = *(const bf16x8 *)&pr[1][lr][8 * lq];
 #pragma unroll
-        for (int st = 0; st < 2; ++st)
+        for (int i = 0; i < CT; ++i) {  // columns beyond the latent repeat its last ones and are dropped
+            const int c = min((wave + 4 * i) * 16, rankp - 16);
+            const uint16_t *vp = tile + 8 * lq * ld + c + lr;
+            uint32_t w[4];
 #pragma unroll
-            for (int pc = 0; pc < 2; ++pc) pf[st][pc] = *(const bf16x8 *)&pr[pc][lr][32 * st + 8 * lq];
-#pragma unroll
-        for (int i = 0; i < CT; ++i) {
-            const int c = (wave + 4 * i) * 16;
-            if (c >= rankp) continue;
+            for (int e = 0; e < 4; ++e) w[e] = (uint32_t)vp[2 * e * ld] | ((uint32_t)vp[(2 * e + 1) * ld] << 16);
+            const bf16x8 vf = __builtin_bit_cast(bf16x8, make_uint4(w[0], w[1], w[2], w[3]));
 #pragma unroll
             for (int r = 0; r < 4; ++r) acc[i][r] *= cr[r];
-#pragma unroll
-            for (int st = 0; st < 2; ++st) {
-                const uint16_t *vp = tile + (32 * st + 8 * lq) * ld + c + lr;
-                uint32_t w[4];
-#pragma unroll
-                for (int e = 0; e < 4; ++e) w[e] = (uint32_t)vp[2 * e * ld] | ((uint32_t)vp[(2 * e + 1) * ld] << 16);
-                const bf16x8 vf = __builtin_bit_cast(bf16x8, make_uint4(w[0], w[1], w[2], w[3]));
-                acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf[st][1], vf, acc[i], 0, 0, 0);
-                acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf[st][0], vf, acc[i], 0, 0, 0);
-            }
+            acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(plo, vf, acc[i], 0, 0, 0);
+            acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(phi, vf, acc[i], 0, 0, 0);
         }
         __syncthreads();  // the next chunk overwrites the tile
     }
@@ -406,12 +393,11 @@ __global__ __launch_bounds__(256) void latent_attend_matrix_kernel(LatentArgs a,
         *(float2 *)(part_ml + (((size_t)row * s.heads + h0 + (t >> 4)) * splits + blockIdx.x) * 2) = make_float2(m, l);
 }
 
-size_t matrix_lds_bytes(const LatentShape &s) { return (size_t)(kKeyChunk + 2 * kMatrixHeads) * (s.cache_row() + 8) * 2; }
-// 12 KiB of the 160 KiB are the kernel's static arrays.
-bool matrix_supported(const LatentShape &s) { return matrix_lds_bytes(s) <= 148 * 1024; }
+size_t matrix_lds_bytes(const LatentShape &s) { return (size_t)kMatrixChunk * (s.cache_row() + 8) * 2; }
+bool matrix_supported(const LatentShape &s) { return s.cache_row() <= 24 * 32; }
 
 // grid (ceil(vdim / 32), heads, rows): merges the key splits of a head, adds the sink to the denominator, applies W_uv.
-__global__ __launch_bounds__(256) void latent_merge_kernel(LatentArgs a, int rankp, int vdimp, int splits) {
+__global__ __launch_bounds__(256) void latent_merge_kernel(LatentArgs a, int rankp, int vdimp, int splits, int chunk) {
     extern __shared__ float olat[];  // [4][rankp]: one quarter of the splits each, then their sum
     __shared__ float wt[kMaxSplits];
     const LatentShape &s = a.s;
@@ -428,7 +414,9 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(LatentArgs a, int ran
 #pragma unroll
         for (int j = 0; j < 4; ++j) first[i][j] = *(const uint4 *)(wv + (size_t)i * 16 * rankp + min(kl * 8 + 128 * j, rankp - 8));
     // every wave for itself: the weights of the splits
-    const float2 ml = lane < splits ? *(const float2 *)(part_ml + 2 * lane) : make_float2(kMinusInf, 0.0f);
+    // the splits that had keys
+    const int chunks = (*a.pos_dev + row % a.new_len + chunk) / chunk, per = (chunks + splits - 1) / splits, used = (chunks + per - 1) / per;
+    const float2 ml = lane < used ? *(const float2 *)(part_ml + 2 * lane) : make_float2(kMinusInf, 0.0f);
     const float sink = a.w.sink ? a.w.sink[h] : kMinusInf;
     const float top = fmaxf(wave_max(ml.x), sink);
     const float w = expf(ml.x - top);
@@ -438,7 +426,7 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(LatentArgs a, int ran
     for (int c = lane * 4; c < rankp; c += 256) {
         float4 v = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
 #pragma unroll 4
-        for (int i = wave; i < splits; i += 4) {
+        for (int i = wave; i < used; i += 4) {
             const float4 o = *(const float4 *)(part_o + (size_t)i * rankp + c);
             const float f = wt[i];
             v.x = fmaf(f, o.x, v.x);
@@ -668,13 +656,13 @@ int32_t attend_run(agpu_ctx *ctx, const LatentArgs &a, int rows, int splits) {
     return AGPU_LAUNCH_CHECK(ctx, "latent_attend_kernel");
 }
 
-template <int CT>
+template <int CT, int NK>
 int32_t attend_matrix_run(agpu_ctx *ctx, const LatentArgs &a, int rows, int splits) {
     const LatentShape &s = a.s;
     const size_t lds = matrix_lds_bytes(s);
     if (lds > 48 * 1024)
-        (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&latent_attend_matrix_kernel<CT>), hipFuncAttributeMaxDynamicSharedMemorySize, 148 * 1024);
-    hipLaunchKernelGGL(latent_attend_matrix_kernel<CT>, dim3((unsigned)splits, (unsigned)ceil_div(s.heads, kMatrixHeads), (unsigned)rows), dim3(256), lds,
+        (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&latent_attend_matrix_kernel<CT, NK>), hipFuncAttributeMaxDynamicSharedMemorySize, 148 * 1024);
+    hipLaunchKernelGGL((latent_attend_matrix_kernel<CT, NK>), dim3((unsigned)splits, (unsigned)ceil_div(s.heads, kMatrixHeads), (unsigned)rows), dim3(256), lds,
                        ctx->stream, a, s.rankp(), s.cache_row(), splits);
     return AGPU_LAUNCH_CHECK(ctx, "latent_attend_matrix_kernel");
 }
@@ -718,8 +706,8 @@ int32_t check_shape(agpu_ctx *ctx, const LatentArgs &a) {
 }  // namespace
 
 int latent_splits(const agpu_ctx *ctx, const LatentShape &s, int rows, int kv_max) {
-    const int chunks = ceil_div(kv_max, kKeyChunk), others = ceil_div(s.heads, kMatrixHeads) * rows;
-    return std::max(1, std::min({chunks, kMaxSplits, ceil_div(ctx->num_cus, others)}));
+    const int chunks = ceil_div(kv_max, kMatrixChunk), others = ceil_div(s.heads, kMatrixHeads) * rows;
+    return std::max(1, std::min({chunks, kMaxSplits, ceil_div(2 * ctx->num_cus, others)}));
 }
 
 size_t latent_partial_floats(const LatentShape &s, int rows, int splits) { return (size_t)rows * s.heads * splits * (s.rankp() + 2); }
@@ -747,18 +735,18 @@ int32_t latent_absorbed_launch(agpu_ctx *ctx, const LatentArgs &a) {
 #undef AGPU_ABSORB
     if ((rc = AGPU_LAUNCH_CHECK(ctx, "latent_absorb_kernel")) != AGPU_OK) return rc;
     if (matrix) {
-        const int ct = ceil_div(s.rankp(), 64);
-        if (ct <= 2) rc = attend_matrix_run<2>(ctx, a, rows, splits);
-        else if (ct <= 4) rc = attend_matrix_run<4>(ctx, a, rows, splits);
-        else if (ct <= 8) rc = attend_matrix_run<8>(ctx, a, rows, splits);
-        else rc = attend_matrix_run<12>(ctx, a, rows, splits);
-        if (ct > 12) return agpu_fail(ctx, AGPU_ERR_UNSUPPORTED, "latent_attention: latent size %d", s.rank);
+        const int ct = ceil_div(s.rankp(), 64), nk = ceil_div(s.cache_row(), 128);
+        if (ct <= 2 && nk <= 2) rc = attend_matrix_run<2, 2>(ctx, a, rows, splits);
+        else if (ct <= 4 && nk <= 3) rc = attend_matrix_run<4, 3>(ctx, a, rows, splits);
+        else if (ct <= 8 && nk <= 5) rc = attend_matrix_run<8, 5>(ctx, a, rows, splits);
+        else rc = attend_matrix_run<12, 6>(ctx, a, rows, splits);
     } else {
         rc = a.cache_bf16 ? attend_run<uint16_t>(ctx, a, rows, splits) : attend_run<float>(ctx, a, rows, splits);
     }
     if (rc != AGPU_OK) return rc;
     hipLaunchKernelGGL(latent_merge_kernel, dim3((unsigned)(s.vdimp() / 32), (unsigned)s.heads, (unsigned)rows), dim3(256),
-                       (size_t)4 * s.rankp() * sizeof(float), ctx->stream, a, s.rankp(), s.vdimp(), splits);
+                       (size_t)4 * s.rankp() * sizeof(float), ctx->stream, a, s.rankp(), s.vdimp(), splits,
+                       matrix ? kMatrixChunk : kKeyChunk);
     return AGPU_LAUNCH_CHECK(ctx, "latent_merge_kernel");
 }
 

@@ -107,6 +107,9 @@ def main():
     ap.add_argument("--per-stage", action="store_true", help="time the one-launch-per-stage decode path (HIP graph of 62 launches)")
     ap.add_argument("--roofline-only", action="store_true",
                     help="only the dominant-kernel loop plus a 64 MiB device copy (calibration for rocprofv3 --pmc runs)")
+    ap.add_argument("--ritevik", nargs="*", choices=("small", "large"), metavar="SIZE",
+                    help="instead of the default workload: prefill and decode of Ritevik beside the int4 GPT-2 of the same size (small, large; "
+                         "default both), one JSON line")
     args = ap.parse_args()
     if args.gpus != 1:
         sys.exit("bench.py: this build measures one GPU only (every GPU box here has one MI355X); run with --gpus 1")
@@ -116,6 +119,10 @@ def main():
     if not torch.cuda.is_available():
         sys.exit("bench.py: no GPU visible; the HIP path has no CPU fallback")
     pkg = entry.load_package()
+    if args.ritevik is not None:
+        import bench_ritevik
+        bench_ritevik.run(args.ritevik or ("small", "large"))
+        return
     from async_gpu_amd import _lib, gpt2, ops, workloads
 
     cfg = workloads.GPT2_SMALL
