@@ -110,6 +110,8 @@ def main():
     ap.add_argument("--ritevik", nargs="*", choices=("small", "large"), metavar="SIZE",
                     help="instead of the default workload: prefill and decode of Ritevik beside the int4 GPT-2 of the same size (small, large; "
                          "default both), one JSON line")
+    ap.add_argument("--ritevik-trace", choices=("ritevik", "gpt2"), help="with --ritevik: a short run of that model alone, for kernel traces")
+    ap.add_argument("--ritevik-context", type=int, default=1024, help="with --ritevik-trace: prompt length")
     args = ap.parse_args()
     if args.gpus != 1:
         sys.exit("bench.py: this build measures one GPU only (every GPU box here has one MI355X); run with --gpus 1")
@@ -121,7 +123,7 @@ def main():
     pkg = entry.load_package()
     if args.ritevik is not None:
         import bench_ritevik
-        bench_ritevik.run(args.ritevik or ("small", "large"))
+        bench_ritevik.run(args.ritevik or ("small", "large"), args.ritevik_trace, args.ritevik_context)
         return
     from async_gpu_amd import _lib, gpt2, ops, workloads
 

@@ -73,14 +73,37 @@ def measure(model, vocab, prompts, seed=0):
     return out
 
 
-def run(sizes, emit=lambda d: print(json.dumps(d), flush=True)):
+def trace(model, vocab, context=1024, batch=16):
+    """A short run for kernel traces: three prefills, then decode steps launched one by one, of one sequence and of a batch."""
+    rng = np.random.default_rng(0)
+    model.set_decode_mode(model.DECODE_EAGER)
+    for _ in range(3):
+        model.reset_cache()
+        model.forward_cached(rng.integers(0, vocab, (1, context)), all_rows=False)
+    model.decode_steps(1, 32)
+    model.reset_cache()
+    model.forward_cached(rng.integers(0, vocab, (batch, context)), all_rows=False)
+    model.decode_steps(batch, 16)
+
+
+def run(sizes, trace_model=None, context=1024, emit=lambda d: print(json.dumps(d), flush=True)):
     from async_gpu_amd import gpt2, ritevik, workloads
     rows = []
     for size in sizes:
         c = SIZES[size]
         spec = workloads.RITEVIK_SMALL if size == "small" else workloads.RITEVIK_LARGE
         g = c["gpt2"]
+        if trace_model == "gpt2":
+            gm = gpt2.Int4Gpt2Model.from_quantized(gpt2.Gpt2Config(g["n_layer"], g["n_embd"], g["n_head"], vocab_size=g["vocab"], n_positions=c["positions"],
+                                                                   group_size=32, max_batch=16), gpt2_random_int4(g, c["positions"], 32, 1))
+            trace(gm, g["vocab"], context)
+            gm.close()
+            continue
         rm = ritevik.RitevikModel.from_tensors(spec, workloads.ritevik_tensors(spec, 1), n_positions=c["positions"], max_batch=16)
+        if trace_model == "ritevik":
+            trace(rm, spec["vocab"], context)
+            rm.close()
+            continue
         gm = gpt2.Int4Gpt2Model.from_quantized(gpt2.Gpt2Config(g["n_layer"], g["n_embd"], g["n_head"], vocab_size=g["vocab"], n_positions=c["positions"],
                                                                group_size=32, max_batch=16), gpt2_random_int4(g, c["positions"], 32, 1))
         both = {"ritevik": measure(rm, spec["vocab"], c["prompts"]), "gpt2_int4": measure(gm, g["vocab"], c["prompts"])}
@@ -96,6 +119,8 @@ def run(sizes, emit=lambda d: print(json.dumps(d), flush=True)):
                 rows.append(dict(size=size, model=name, what="prefill", batch=1, tokens=n, ms=round(ms, 3), tok_s=round(n * 1e3 / ms, 1)))
         rm.close()
         gm.close()
+    if trace_model:
+        return
     head = [r for r in rows if r["model"] == "ritevik" and r["what"] == "decode" and r["batch"] == 1][0]
     emit({"metric": f"Ritevik decode tok/s (B=1, {head['size']} layers, bf16 weights)", "value": head["tok_s"], "unit": "tok/s", "n_gpus": 1,
           "higher_is_better": True, "vs_baseline": None, "dtype": "bf16 weights, f32 residual, scores and state", "data": "synthetic", "rows": rows})
