@@ -16,6 +16,7 @@ GELU_TANH, GELU_QUICK = 0, 1
 DTYPE_BF16, DTYPE_F32 = 0, 1
 DENSE_GATED = 1
 MIXER_LATENT_ATTENTION, MIXER_CHANNEL_DELTA = 0, 1
+MIXER_MATRIX_MEMORY, MIXER_GROUPED_ATTENTION, MIXER_GATED_LRU = 2, 3, 4
 
 
 class AgpuError(RuntimeError):
@@ -146,6 +147,24 @@ SIGNATURES = {
     "agpu_ritevik_decode_steps": (_i32, [_vp, _i32, _i32, _vp]),
     "agpu_ritevik_last_logits": (_i32, [_vp, _i32, _vp]),
     "agpu_ritevik_layer_streams": (_i32, [_vp, _vp, _i32, _vp]),
+    # include/agpu_piralix.h
+    "agpu_piralix_create": (_i32, [_vp, _vp, _vp, C.POINTER(_vp)]),
+    "agpu_piralix_destroy": (_i32, [_vp]),
+    "agpu_piralix_set_tensor": (_i32, [_vp, C.c_char_p, _vp, _i32, C.c_int64, C.c_int64]),
+    "agpu_piralix_tensor_info": (_i32, [_vp, _i32, C.POINTER(C.c_char_p), _vp, _vp, _vp]),
+    "agpu_piralix_weight_bytes": (C.c_int64, [_vp]),
+    "agpu_piralix_cache_bytes": (C.c_int64, [_vp]),
+    "agpu_piralix_layer_runs": (_i32, [_vp]),
+    "agpu_piralix_reset_cache": (_i32, [_vp]),
+    "agpu_piralix_cache_len": (_i32, [_vp]),
+    "agpu_piralix_forward_cached": (_i32, [_vp, _vp, _i32, _i32, _vp, _i32]),
+    "agpu_piralix_generate_cached": (_i32, [_vp, _vp, _i32, _i32, _i32, _i32, _vp, _vp, _vp]),
+    "agpu_piralix_generate": (_i32, [_vp, _vp, _i32, _i32, _i32, _vp, _vp]),
+    "agpu_piralix_generate_cached_sampling": (_i32, [_vp, _vp, _i32, _i32, _i32, _f, _vp, _i32, _vp, _vp]),
+    "agpu_piralix_set_decode_mode": (_i32, [_vp, _i32]),
+    "agpu_piralix_decode_steps": (_i32, [_vp, _i32, _i32, _vp]),
+    "agpu_piralix_last_logits": (_i32, [_vp, _i32, _vp]),
+    "agpu_piralix_layer_streams": (_i32, [_vp, _vp, _i32, _vp]),
 }
 
 
@@ -186,6 +205,20 @@ class RitevikLayerStruct(C.Structure):
     _fields_ = [("mixer", _i32), ("heads", _i32), ("dim", _i32), ("vdim", _i32), ("ff", _i32), ("kv_rank", _i32),
                 ("rot_dim", _i32), ("rot_dims", _i32), ("scale", _f), ("rot_base", C.c_double), ("kv_heads", _i32),
                 ("conv", _i32), ("decay_rank", _i32), ("gate_rank", _i32)]
+
+
+class PiralixConfigStruct(C.Structure):
+    """agpu_piralix_config of include/agpu_piralix.h."""
+    _fields_ = [("n_layer", _i32), ("width", _i32), ("vocab_size", _i32), ("n_positions", _i32), ("max_batch", _i32),
+                ("norm_eps", _f), ("loop_start", _i32), ("loop_stop", _i32), ("loop_times", _i32), ("dtype", _i32), ("argmax_last", _i32)]
+
+
+class PiralixLayerStruct(C.Structure):
+    """agpu_piralix_layer of include/agpu_piralix.h."""
+    _fields_ = [("mixer", _i32), ("heads", _i32), ("dim", _i32), ("vdim", _i32), ("ff", _i32), ("ff_limit", _f), ("gate_cap", _f),
+                ("scale", _f), ("softcap", _f), ("kv_heads", _i32), ("rot_dims", _i32)] + \
+               [(n, C.c_double) for n in ("rot_base", "rot_factor", "rot_original", "rot_fast", "rot_slow")] + \
+               [("lru_width", _i32), ("blocks", _i32), ("conv", _i32)]
 
 
 def cdll():

@@ -18,7 +18,8 @@ __device__ __forceinline__ float silu_dev(float v) { return v / (1.0f + expf(-v)
 __device__ __forceinline__ float sigmoid_dev(float v) { return 1.0f / (1.0f + expf(-v)); }
 
 // Where the outputs of a dense Linear go.  Columns [0, n_plain) are plain; the columns behind them are pairs (gate, up)
-// of a gated feed-forward, column n_plain + 2 j and n_plain + 2 j + 1, and leave as act[m][j] = silu(gate) * up.
+// of a gated feed-forward, column n_plain + 2 j and n_plain + 2 j + 1, and leave as act[m][j] = silu(gate) * up, or with
+// act_limit > 0 as g sigmoid(1.702 g) (u + 1) with g = min(gate, act_limit), u = up clamped to +- act_limit.
 struct DenseOut {
     int n_plain = 0;
     float *out = nullptr;         // fp32, row stride ldo
@@ -33,12 +34,16 @@ struct DenseOut {
     int tab_ld = 0, tab_off = 0, tab_n = 0, vocab = 0;
     void *act = nullptr;  // bf16 or fp32, row stride ld_act
     int ld_act = 0, act_bf16 = 0;
+    float act_limit = 0.0f;
 };
 
 // What happens to the fp32 input rows in front of a Linear (and, in dense_rows_launch, on their own):
 //   x <- x + y / rms(y) * y_w                 (y != null: an RMS-normed addend with a plain weight)
+//   x <- x + add + add_vec                    (add, add_vec: each if not null; a row per row, one vector for all)
 //   h  = x / rms(x) * (norm_off + norm_w)     (norm_w != null)
 //   the Linear's input is [h | x2]            (x2 != null)
+// or, with gate: h = x / rms(x) * norm_w * sigmoid(gate), where the row is `groups` groups of group_p columns, of which the
+// first group_d count for the group's own rms (the rest is zero); nothing else applies then.
 // rms(z) = sqrt(mean(z^2) + eps) over the first d columns; columns d .. dp - 1 are zero everywhere.
 struct DenseRows {
     const float *x = nullptr;
@@ -49,6 +54,9 @@ struct DenseRows {
     const float *norm_w = nullptr;
     float norm_off = 0.0f, eps = 0.0f;
     const float *x2 = nullptr;                 // row stride ldx, dp columns
+    const float *add = nullptr, *add_vec = nullptr;  // row stride ldx; [d]
+    const float *gate = nullptr;               // row stride ld_gate, same columns as x
+    int ld_gate = 0, groups = 0, group_d = 0, group_p = 0;
     // Row m of the input is row map_stride * (m + 1) - 1 of x and y when map_stride > 0 (the last token of each sequence).
     int map_stride = 0;
 };
@@ -61,5 +69,6 @@ int32_t dense_rows_launch(agpu_ctx *ctx, const DenseRows &in, int M, void *h, in
 // y = A W^T on the matrix cores, A [M, K] with row stride lda, W with row stride ldw.  K % 32 == 0, lda % 8 == 0,
 // ldw % 8 == 0, 16-byte aligned.  bf16 A:
 int32_t dense_gemm_bf16_launch(agpu_ctx *ctx, const uint16_t *a, int lda, const uint16_t *w, int ldw, int M, int N, int K, const DenseOut &o);
-// fp32 A:
-int32_t dense_gemm_f32_launch(agpu_ctx *ctx, const float *a, int lda, const uint16_t *w, int ldw, int M, int N, int K, const DenseOut &o);
+// fp32 A; with `blocks` > 1 a block-diagonal Linear: block b reads columns b K .. of A and rows b N .. of W, and its outputs
+// (plain only) are columns b N ...
+int32_t dense_gemm_f32_launch(agpu_ctx *ctx, const float *a, int lda, const uint16_t *w, int ldw, int M, int N, int K, const DenseOut &o, int blocks = 1);

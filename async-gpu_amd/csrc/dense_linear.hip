@@ -24,7 +24,9 @@ __device__ __forceinline__ void store_plain(const DenseOut &o, int m, int n, flo
 }
 
 __device__ __forceinline__ void store_pair(const DenseOut &o, int m, int j, float gate, float up) {
-    const float a = silu_dev(gate) * up;
+    float a;
+    if (o.act_limit > 0.0f) a = gelu_quick_dev(fminf(gate, o.act_limit)) * (fminf(fmaxf(up, -o.act_limit), o.act_limit) + 1.0f);
+    else a = silu_dev(gate) * up;
     if (o.act_bf16) ((uint16_t *)o.act)[(size_t)m * o.ld_act + j] = f32_to_bf16(a);
     else ((float *)o.act)[(size_t)m * o.ld_act + j] = a;
 }
@@ -46,13 +48,16 @@ __device__ __forceinline__ float block_sum(float v, float *red) {
 // One row of DenseRows: h (and x2 behind it) goes through `put(k, value)`, k = 0 .. K - 1.  The first kRowRegs * NT columns
 // of x and y are read once and stay in registers; a wider row reads the rest again in every pass.
 constexpr int kRowRegs = 4;
-template <int NW, typename Put>
+enum RowKind { kRowPlain, kRowAdds, kRowGated };  // which parts of DenseRows a kernel has code for
+template <int NW, int KIND, typename Put>
 __device__ __forceinline__ void run_row(const DenseRows &in, int m, bool write_x, float *red, Put put) {
     constexpr int NT = NW * 64;
     const int t = threadIdx.x;
     const size_t row = (size_t)(in.map_stride > 0 ? in.map_stride * (m + 1) - 1 : m) * in.ldx;
     const float *x = in.x + row, *y = in.y ? in.y + row : nullptr;
-    float v[kRowRegs], yv[kRowRegs], yw[kRowRegs], nw[kRowRegs], v2[kRowRegs];
+    const float *add = KIND == kRowAdds && in.add ? in.add + row : nullptr, *add_vec = KIND == kRowAdds ? in.add_vec : nullptr;
+    auto added = [&](int k) -> float { return (add ? add[k] : 0.0f) + (add_vec ? add_vec[k] : 0.0f); };
+    float v[kRowRegs], yv[kRowRegs], yw[kRowRegs], nw[kRowRegs], v2[kRowRegs], av[kRowRegs];
 #pragma unroll
     for (int i = 0; i < kRowRegs; ++i) {  // clamped addresses; columns beyond d count as zero
         const int k = t + i * NT, kc = min(k, in.d - 1);
@@ -61,6 +66,7 @@ __device__ __forceinline__ void run_row(const DenseRows &in, int m, bool write_x
         yw[i] = y ? in.y_w[kc] : 0.0f;
         nw[i] = in.norm_w ? in.norm_w[kc] : 0.0f;
         v2[i] = in.x2 ? in.x2[row + min(k, in.dp - 1)] : 0.0f;
+        av[i] = KIND == kRowAdds ? added(kc) : 0.0f;
     }
     float rs_y = 0.0f;
     if (y) {
@@ -73,8 +79,8 @@ __device__ __forceinline__ void run_row(const DenseRows &in, int m, bool write_x
         rs_y = 1.0f / sqrtf(s / (float)in.d + in.eps);
     }
 #pragma unroll
-    for (int i = 0; i < kRowRegs; ++i) v[i] = t + i * NT < in.d ? v[i] + yv[i] * rs_y * yw[i] : 0.0f;
-    auto value = [&](int k) -> float { return y ? x[k] + y[k] * rs_y * in.y_w[k] : x[k]; };
+    for (int i = 0; i < kRowRegs; ++i) v[i] = t + i * NT < in.d ? v[i] + yv[i] * rs_y * yw[i] + av[i] : 0.0f;
+    auto value = [&](int k) -> float { return (y ? x[k] + y[k] * rs_y * in.y_w[k] : x[k]) + (KIND == kRowAdds ? added(k) : 0.0f); };
     float rs_x = 1.0f;
     if (in.norm_w) {
         float s = 0.0f;
@@ -98,11 +104,39 @@ __device__ __forceinline__ void run_row(const DenseRows &in, int m, bool write_x
         finish(k, k < in.d ? value(k) : 0.0f, in.norm_w && k < in.d ? in.norm_w[k] : 0.0f, in.x2 ? in.x2[row + k] : 0.0f);
 }
 
+// One gated row of DenseRows, a wave per group.
+template <int NW, typename Put>
+__device__ __forceinline__ void run_gated_row(const DenseRows &in, int m, Put put) {
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const size_t r = (size_t)(in.map_stride > 0 ? in.map_stride * (m + 1) - 1 : m);
+#pragma unroll 1
+    for (int g = wave; g < in.groups; g += NW) {
+        const float *x = in.x + r * in.ldx + g * in.group_p, *gate = in.gate + r * in.ld_gate + g * in.group_p, *w = in.norm_w + g * in.group_p;
+        float v[kRowRegs], gv[kRowRegs], wv[kRowRegs], s = 0.0f;
+#pragma unroll
+        for (int i = 0; i < kRowRegs; ++i) {
+            const int k = lane + 64 * i, kc = min(k, in.group_p - 1);
+            v[i] = k < in.group_p ? x[kc] : 0.0f;
+            gv[i] = gate[kc];
+            wv[i] = w[kc];
+            s = fmaf(v[i], v[i], s);
+        }
+#pragma unroll 1
+        for (int k = lane + 64 * kRowRegs; k < in.group_p; k += 64) s = fmaf(x[k], x[k], s);
+        const float rs = 1.0f / sqrtf(wave_sum(s) / (float)in.group_d + in.eps);
+#pragma unroll
+        for (int i = 0; i < kRowRegs; ++i)
+            if (lane + 64 * i < in.group_p) put(g * in.group_p + lane + 64 * i, v[i] * rs * wv[i] * sigmoid_dev(gv[i]));
+#pragma unroll 1
+        for (int k = lane + 64 * kRowRegs; k < in.group_p; k += 64) put(g * in.group_p + k, x[k] * rs * w[k] * sigmoid_dev(gate[k]));
+    }
+}
+
 // ---- decode GEMV: a wave takes 4 * RPL weight rows, 16 lanes x 8 values along K per row and chunk of 128; the waves of a
 // workgroup split K KS ways.  The first weights are requested before the rows are touched.
 constexpr int kGemvWaves = 8;
 
-template <int MT, int RPL>
+template <int MT, int RPL, int KIND>
 __global__ __launch_bounds__(64 * kGemvWaves) void dense_gemv_kernel(DenseRows in, const uint16_t *__restrict__ w, int M, int N, int K, int KS,
                                                                      DenseOut o) {
     extern __shared__ float lds[];
@@ -132,8 +166,10 @@ __global__ __launch_bounds__(64 * kGemvWaves) void dense_gemv_kernel(DenseRows i
     for (int m = 0; m < MT; ++m) {
         float *xm = xs + (size_t)m * K;
         if (m < M) {
-            if (in.y || in.norm_w) {
-                run_row<kGemvWaves>(in, m, in.x_out != nullptr && blockIdx.x == 0, wred, [&](int k, float v) { xm[k] = v; });
+            if (KIND == kRowGated) {
+                run_gated_row<kGemvWaves>(in, m, [&](int k, float v) { xm[k] = v; });
+            } else if (KIND == kRowAdds || in.y || in.norm_w) {
+                run_row<kGemvWaves, KIND>(in, m, in.x_out != nullptr && blockIdx.x == 0, wred, [&](int k, float v) { xm[k] = v; });
             } else {
                 const size_t row = (size_t)(in.map_stride > 0 ? in.map_stride * (m + 1) - 1 : m) * in.ldx;
                 for (int k = threadIdx.x * 4; k < in.dp; k += 256 * kGemvWaves) {
@@ -205,15 +241,17 @@ __global__ __launch_bounds__(64 * kGemvWaves) void dense_gemv_kernel(DenseRows i
     }
 }
 
-template <int NW>
+template <int NW, int KIND>
 __global__ __launch_bounds__(64 * NW) void dense_rows_kernel(DenseRows in, void *h, int ldh, int h_bf16) {
     __shared__ float red[NW];
     const int m = blockIdx.x;
-    run_row<NW>(in, m, in.x_out != nullptr, red, [&](int k, float v) {
+    auto put = [&](int k, float v) {
         if (!h) return;
         if (h_bf16) ((uint16_t *)h)[(size_t)m * ldh + k] = f32_to_bf16(v);
         else ((float *)h)[(size_t)m * ldh + k] = v;
-    });
+    };
+    if (KIND == kRowGated) run_gated_row<NW>(in, m, put);
+    else run_row<NW, KIND>(in, m, in.x_out != nullptr, red, put);
 }
 
 // ---- few rows or few columns: 16 columns and up to 32 rows per workgroup, the waves split K, operands straight from memory ----
@@ -419,6 +457,14 @@ __global__ __launch_bounds__(256) void dense_gemm_f32_kernel(const float *__rest
     static_assert(2 * 64 * LD >= 4 * 32 * kTileLd, "the result tiles fit the operand buffers");
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, wm = wave >> 1, wn = wave & 1;
     const int m0 = (blockIdx.x / tiles_n) * 64, n0 = (blockIdx.x % tiles_n) * 64;
+    if (blockIdx.y > 0) {  // block of a block-diagonal Linear: plain outputs only
+        a += (size_t)blockIdx.y * K;
+        w += (size_t)blockIdx.y * N * ldw;
+        if (o.out) o.out += (size_t)blockIdx.y * N;
+        if (o.out_bf16) o.out_bf16 += (size_t)blockIdx.y * N;
+        if (o.bias) o.bias += (size_t)blockIdx.y * N;
+        if (o.residual) o.residual += (size_t)blockIdx.y * N;
+    }
     f32x16 acc;
 #pragma unroll
     for (int r = 0; r < 16; ++r) acc[r] = 0.0f;
@@ -455,19 +501,39 @@ __global__ __launch_bounds__(256) void dense_gemm_f32_kernel(const float *__rest
 
 size_t gemv_lds_bytes(int MT, int RPL, int K) { return ((size_t)MT * K + (size_t)kGemvWaves * 4 * RPL * MT + kGemvWaves) * sizeof(float); }
 
-template <int MT, int RPL>
+template <int MT, int RPL, int KIND>
 int32_t gemv_run(agpu_ctx *ctx, const DenseRows &in, const uint16_t *w, int M, int N, int K, int KS, const DenseOut &o) {
     const int rows = 4 * RPL * (kGemvWaves / KS);
     const size_t lds = gemv_lds_bytes(MT, RPL, K);
     if (lds > 64 * 1024) {
         static bool raised = false;  // per instantiation; setting it twice is harmless
         if (!raised) {
-            (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&dense_gemv_kernel<MT, RPL>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute(reinterpret_cast<const void *>(&dense_gemv_kernel<MT, RPL, KIND>), hipFuncAttributeMaxDynamicSharedMemorySize,
+                                      160 * 1024);
             raised = true;
         }
     }
-    hipLaunchKernelGGL((dense_gemv_kernel<MT, RPL>), dim3((unsigned)ceil_div(N, rows)), dim3(64 * kGemvWaves), lds, ctx->stream, in, w, M, N, K, KS, o);
+    hipLaunchKernelGGL((dense_gemv_kernel<MT, RPL, KIND>), dim3((unsigned)ceil_div(N, rows)), dim3(64 * kGemvWaves), lds, ctx->stream, in, w, M, N, K, KS, o);
     return AGPU_LAUNCH_CHECK(ctx, "dense_gemv_kernel");
+}
+
+RowKind row_kind(const DenseRows &in) { return in.gate ? kRowGated : (in.add || in.add_vec ? kRowAdds : kRowPlain); }
+
+template <int MT, int RPL>
+int32_t gemv_run_kind(agpu_ctx *ctx, const DenseRows &in, const uint16_t *w, int M, int N, int K, int KS, const DenseOut &o) {
+    switch (row_kind(in)) {
+        case kRowGated: return gemv_run<MT, RPL, kRowGated>(ctx, in, w, M, N, K, KS, o);
+        case kRowAdds: return gemv_run<MT, RPL, kRowAdds>(ctx, in, w, M, N, K, KS, o);
+        default: return gemv_run<MT, RPL, kRowPlain>(ctx, in, w, M, N, K, KS, o);
+    }
+}
+
+template <int KIND>
+void rows_run(agpu_ctx *ctx, const DenseRows &in, int M, void *h, int ldh, int h_bf16) {
+    const dim3 grid((unsigned)M);
+    if (in.dp <= 256) hipLaunchKernelGGL((dense_rows_kernel<1, KIND>), grid, dim3(64), 0, ctx->stream, in, h, ldh, h_bf16);
+    else if (in.dp <= 1024) hipLaunchKernelGGL((dense_rows_kernel<4, KIND>), grid, dim3(256), 0, ctx->stream, in, h, ldh, h_bf16);
+    else hipLaunchKernelGGL((dense_rows_kernel<8, KIND>), grid, dim3(512), 0, ctx->stream, in, h, ldh, h_bf16);
 }
 
 template <int BM, int BN, int WM, int WN, int KG>
@@ -489,7 +555,8 @@ bool dense_gemv_supported(int M, int K) {
 }
 
 int32_t dense_gemv_launch(agpu_ctx *ctx, const DenseRows &in, const uint16_t *w, int M, int N, int K, const DenseOut &o) {
-    if (!dense_gemv_supported(M, K) || K % 32 != 0 || in.dp % 32 != 0 || K != in.dp * (in.x2 ? 2 : 1) || (in.x_out && in.x_out == in.x))
+    if (!dense_gemv_supported(M, K) || K % 32 != 0 || in.dp % 32 != 0 || K != in.dp * (in.x2 ? 2 : 1) || (in.x_out && in.x_out == in.x) ||
+        (in.gate && (in.groups * in.group_p != K || !in.norm_w)))
         return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "dense_gemv: M %d, N %d, K %d, dp %d not supported", M, N, K, in.dp);
     // K is split over the waves until the workgroups roughly fill the chip twice or a wave's share is one request
     const int nchunks = (K + 127) / 128;
@@ -497,15 +564,18 @@ int32_t dense_gemv_launch(agpu_ctx *ctx, const DenseRows &in, const uint16_t *w,
     const int rpl = wide ? 2 : 1;
     int KS = 8;
     while (KS > 1 && (ceil_div(N, 4 * rpl * (kGemvWaves / KS)) > 1024 || nchunks < KS)) KS /= 2;
-    if (M == 1) return wide ? gemv_run<1, 2>(ctx, in, w, M, N, K, KS, o) : gemv_run<1, 1>(ctx, in, w, M, N, K, KS, o);
-    if (M == 2) return wide ? gemv_run<2, 2>(ctx, in, w, M, N, K, KS, o) : gemv_run<2, 1>(ctx, in, w, M, N, K, KS, o);
-    return wide ? gemv_run<4, 2>(ctx, in, w, M, N, K, KS, o) : gemv_run<4, 1>(ctx, in, w, M, N, K, KS, o);
+    if (M == 1) return wide ? gemv_run_kind<1, 2>(ctx, in, w, M, N, K, KS, o) : gemv_run_kind<1, 1>(ctx, in, w, M, N, K, KS, o);
+    if (M == 2) return wide ? gemv_run_kind<2, 2>(ctx, in, w, M, N, K, KS, o) : gemv_run_kind<2, 1>(ctx, in, w, M, N, K, KS, o);
+    return wide ? gemv_run_kind<4, 2>(ctx, in, w, M, N, K, KS, o) : gemv_run_kind<4, 1>(ctx, in, w, M, N, K, KS, o);
 }
 
 int32_t dense_rows_launch(agpu_ctx *ctx, const DenseRows &in, int M, void *h, int ldh, int h_bf16) {
-    if (in.dp <= 256) hipLaunchKernelGGL(dense_rows_kernel<1>, dim3((unsigned)M), dim3(64), 0, ctx->stream, in, h, ldh, h_bf16);
-    else if (in.dp <= 1024) hipLaunchKernelGGL(dense_rows_kernel<4>, dim3((unsigned)M), dim3(256), 0, ctx->stream, in, h, ldh, h_bf16);
-    else hipLaunchKernelGGL(dense_rows_kernel<8>, dim3((unsigned)M), dim3(512), 0, ctx->stream, in, h, ldh, h_bf16);
+    if (in.gate && (in.groups * in.group_p != in.dp || !in.norm_w)) return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "dense_rows: bad groups");
+    switch (row_kind(in)) {
+        case kRowGated: rows_run<kRowGated>(ctx, in, M, h, ldh, h_bf16); break;
+        case kRowAdds: rows_run<kRowAdds>(ctx, in, M, h, ldh, h_bf16); break;
+        default: rows_run<kRowPlain>(ctx, in, M, h, ldh, h_bf16);
+    }
     return AGPU_LAUNCH_CHECK(ctx, "dense_rows_kernel");
 }
 
@@ -535,10 +605,11 @@ int32_t dense_gemm_bf16_launch(agpu_ctx *ctx, const uint16_t *a, int lda, const 
     return AGPU_LAUNCH_CHECK(ctx, "dense_gemm_bf16_kernel");
 }
 
-int32_t dense_gemm_f32_launch(agpu_ctx *ctx, const float *a, int lda, const uint16_t *w, int ldw, int M, int N, int K, const DenseOut &o) {
-    if (M <= 0 || N <= 0 || K <= 0 || K % 32 != 0 || lda % 4 != 0 || ldw % 8 != 0 || (o.n_plain < N && (o.n_plain % 2 != 0 || N % 2 != 0)))
+int32_t dense_gemm_f32_launch(agpu_ctx *ctx, const float *a, int lda, const uint16_t *w, int ldw, int M, int N, int K, const DenseOut &o, int blocks) {
+    if (blocks < 1 || (blocks > 1 && (o.n_plain < N || o.tab)) || M <= 0 || N <= 0 || K <= 0 || K % 32 != 0 || lda % 4 != 0 || ldw % 8 != 0 || (o.n_plain < N && (o.n_plain % 2 != 0 || N % 2 != 0)))
         return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "dense_gemm_f32: M %d, N %d, K %d, lda %d, ldw %d not supported", M, N, K, lda, ldw);
     const int tn = ceil_div(N, 64);
-    hipLaunchKernelGGL(dense_gemm_f32_kernel, dim3((unsigned)(ceil_div(M, 64) * tn)), dim3(256), 0, ctx->stream, a, lda, w, ldw, M, N, K, tn, o);
+    hipLaunchKernelGGL(dense_gemm_f32_kernel, dim3((unsigned)(ceil_div(M, 64) * tn), (unsigned)blocks), dim3(256), 0, ctx->stream, a, lda, w, ldw, M, N,
+                       K, tn, o);
     return AGPU_LAUNCH_CHECK(ctx, "dense_gemm_f32_kernel");
 }

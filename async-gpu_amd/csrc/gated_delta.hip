@@ -5,6 +5,7 @@
 //   o = S^T diag(g) q + (k . q) u      (the read-out of the updated state), S <- diag(g) S + k u^T,
 // so only one reduction over lanes sits between a token and the next.
 #include "gated_delta.h"
+#include "short_conv.h"
 
 namespace {
 
@@ -15,88 +16,31 @@ constexpr int kRecWaves = 4;
 __device__ __forceinline__ float softplus_dev(float v) { return fmaxf(v, 0.0f) + log1pf(expf(-fabsf(v))); }
 __device__ __forceinline__ float decay_dev(float a_log, float step) { return expf(-expf(a_log) * softplus_dev(step)); }
 
-// Convolution and silu of channel c (source column `col` of the projection) at token `t` of the portion.  Inputs before the
-// portion come from the ring, before the sequence they are zero.  pos_slot = pos % taps.  Loads go four taps at a time and
-// without branches.
-__device__ __forceinline__ float conv_silu(const DeltaArgs &a, int channels, int b, int pos, int pos_slot, int t, int c, int col) {
-    const int n = a.s.taps;
-    const float *cur = a.proj + (size_t)(b * a.new_len + t) * a.ld + col;
-    const float *ring = a.ring + (size_t)b * n * channels + c, *w = a.w.conv + (size_t)c * n;
-    float v = w[n - 1] * cur[0];
-#pragma unroll 1
-    for (int k0 = 1; k0 < n; k0 += 4) {
-        float x[4], f[4];
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const int k = k0 + e;
-            const bool on = k < n && pos + t >= k;
-            int slot = pos_slot + t - k;
-            slot = slot < 0 ? slot + n : slot;
-            const float *p = t >= k ? cur - (size_t)k * a.ld : ring + (size_t)slot * channels;
-            x[e] = *(on ? p : cur);
-            f[e] = on ? w[n - 1 - min(k, n - 1)] : 0.0f;
-        }
-#pragma unroll
-        for (int e = 0; e < 4; ++e) v = fmaf(f[e], x[e], v);
-    }
-    return silu_dev(v);
-}
-
-// The same for up to kTokens tokens from t0 on, each input loaded once; put(i, value of token t0 + i).
-constexpr int kTokens = 8, kWindow = 4;
-template <typename Put>
-__device__ __forceinline__ void conv_silu_run(const DeltaArgs &a, int channels, int b, int pos, int pos_slot, int t0, int c, int col, Put put) {
-    const int n = a.s.taps, T = a.new_len;
-    if (n > kWindow) {
-#pragma unroll 1
-        for (int i = 0; i < kTokens && t0 + i < T; ++i) put(i, conv_silu(a, channels, b, pos, pos_slot, t0 + i, c, col));
-        return;
-    }
-    const float *base = a.proj + (size_t)b * T * a.ld + col, *ring = a.ring + (size_t)b * n * channels + c, *w = a.w.conv + (size_t)c * n;
-    float f[kWindow], x[kTokens + kWindow - 1];
-#pragma unroll
-    for (int e = 0; e < kWindow; ++e) f[e] = e >= kWindow - n ? w[max(e - (kWindow - n), 0)] : 0.0f;
-#pragma unroll
-    for (int e = 0; e < kWindow - 1; ++e) {  // the tokens in front of t0
-        const int k = kWindow - 1 - e, t = t0 - k;
-        int slot = pos_slot + t;
-        slot = slot < 0 ? slot + n : slot;
-        const bool on = k < n && pos + t >= 0;
-        const float *p = t >= 0 ? base + (size_t)t * a.ld : ring + (size_t)slot * channels;
-        const float v = *(on ? p : base);
-        x[e] = on ? v : 0.0f;
-    }
-#pragma unroll
-    for (int i = 0; i < kTokens; ++i) x[kWindow - 1 + i] = base[(size_t)min(t0 + i, T - 1) * a.ld];
-#pragma unroll
-    for (int i = 0; i < kTokens; ++i) {
-        float v = 0.0f;
-#pragma unroll
-        for (int e = 0; e < kWindow; ++e) v = fmaf(f[e], x[i + e], v);
-        put(i, silu_dev(v));
-    }
+__device__ __forceinline__ ShortConv conv_of(const DeltaArgs &a, int channels) {
+    return ShortConv{a.proj, a.ld, a.ring, a.w.conv, channels, a.s.taps, a.new_len};
 }
 
 constexpr int kPrepareWidth = 256;  // channels of v or g per workgroup
 
-// grid (groups of kTokens tokens, parts, batch): the first parts take two heads of q and k each (convolution, unit vectors), then
+// grid (groups of kConvTokens tokens, parts, batch): the first parts take two heads of q and k each (convolution, unit vectors), then
 // come parts of v (convolution), then parts of g (decays; the first of them also the step sizes).  q, k and g of a head leave
 // side by side, in padded rows.
 __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaArgs a, int channels, int head_row, int qk_parts, int v_parts) {
-    extern __shared__ float sx[];  // [2 heads][q, k][kTokens][head_row]
+    extern __shared__ float sx[];  // [2 heads][q, k][kConvTokens][head_row]
     const DeltaShape &s = a.s;
-    const int b = blockIdx.z, T = a.new_len, t0 = blockIdx.x * kTokens, nt = min(kTokens, T - t0), pos = *a.pos_dev, pos_slot = pos % s.taps;
+    const int b = blockIdx.z, T = a.new_len, t0 = blockIdx.x * kConvTokens, nt = min(kConvTokens, T - t0), pos = *a.pos_dev, pos_slot = pos % s.taps;
     const int t = threadIdx.x, lane = t & 63, wave = t >> 6;
     const int nk = s.kv_heads * s.dim, nv = s.heads * s.vdim, nb = s.heads + s.kv_heads;
     const size_t row0 = (size_t)b * T + t0;
+    const ShortConv conv = conv_of(a, channels);
     int part = blockIdx.y;
     if (part < qk_parts) {
-        const int per = kTokens * head_row;
+        const int per = kConvTokens * head_row;
 #pragma unroll 1
         for (int i = t; i < 4 * head_row; i += 256) {
             const int w = i / head_row, d = i % head_row, h = min(part * 2 + (w >> 1), s.kv_heads - 1), c = h * s.dim + min(d, s.dim - 1);
-            conv_silu_run(a, channels, b, pos, pos_slot, t0, (w & 1) * nk + c, ((w & 1) ? a.col_k : a.col_q) + c,
-                          [&](int e, float v) { sx[w * per + e * head_row + d] = d < s.dim ? v : 0.0f; });
+            short_conv_run(conv, b, pos, pos_slot, t0, (w & 1) * nk + c, ((w & 1) ? a.col_k : a.col_q) + c,
+                          [&](int e, float v) { sx[w * per + e * head_row + d] = d < s.dim ? silu_dev(v) : 0.0f; });
         }
         __syncthreads();
         const int group = s.heads / s.kv_heads;
@@ -128,8 +72,8 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaArgs a, int cha
     if (part < v_parts) {
         const int c = part * kPrepareWidth + t;
         if (c < nv)
-            conv_silu_run(a, channels, b, pos, pos_slot, t0, 2 * nk + c, a.col_v + c, [&](int e, float v) {
-                if (e < nt) a.v[(row0 + e) * nv + c] = v;
+            short_conv_run(conv, b, pos, pos_slot, t0, 2 * nk + c, a.col_v + c, [&](int e, float v) {
+                if (e < nt) a.v[(row0 + e) * nv + c] = silu_dev(v);
             });
         return;
     }
@@ -145,14 +89,14 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(DeltaArgs a, int cha
     const float a_log = a.w.a_log[h], bias = d < s.dim ? a.w.dt_bias[h * s.dim + d] : 0.0f;
     const float *step = a.step + row0 * s.heads * head_row + c;
     float *g = a.qkg + (row0 * s.heads + h) * 3 * head_row + 2 * head_row + d;
-    float x[kTokens];
+    float x[kConvTokens];
 #pragma unroll
-    for (int e = 0; e < kTokens; ++e) x[e] = step[(size_t)min(e, nt - 1) * s.heads * head_row];
+    for (int e = 0; e < kConvTokens; ++e) x[e] = step[(size_t)min(e, nt - 1) * s.heads * head_row];
 #pragma unroll 1
     for (int e = 0; e < nt; ++e) {
         float v = x[0];
 #pragma unroll
-        for (int i = 1; i < kTokens; ++i) v = e == i ? x[i] : v;
+        for (int i = 1; i < kConvTokens; ++i) v = e == i ? x[i] : v;
         g[(size_t)e * s.heads * 3 * head_row] = d < s.dim ? decay_dev(a_log, v + bias) : 1.0f;
     }
 }
@@ -350,13 +294,14 @@ __global__ __launch_bounds__(kStepThreads) void delta_step_kernel(DeltaArgs a, i
     // convolution of the head's q, k and v; the new inputs go into a ring slot that no tap of this token reads (q and k by
     // the first head of a group)
     float *slot = a.ring + ((size_t)b * s.taps + pos_slot) * channels;
+    const ShortConv conv = conv_of(a, channels);
 #pragma unroll 1
     for (int i = t; i < 2 * state_row + s.vdim; i += kStepThreads) {
         const int w = i < state_row ? 0 : (i < 2 * state_row ? 1 : 3), d = i - min(w, 2) * state_row;
         const bool on = w == 3 || d < s.dim;
         const int c = w == 3 ? h * s.vdim + d : hk * s.dim + min(d, s.dim - 1);
         const int ch = min(w, 2) * nk + c, col = (w == 0 ? a.col_q : (w == 1 ? a.col_k : a.col_v)) + c;
-        const float v = conv_silu(a, channels, b, pos, pos_slot, 0, ch, col);
+        const float v = silu_dev(short_conv(conv, b, pos, pos_slot, 0, ch, col));
         sx[w][d] = on ? v : 0.0f;
         if (on && (w == 3 || h % group == 0)) slot[ch] = p[col];
     }
@@ -504,8 +449,8 @@ int32_t delta_prefill_launch(agpu_ctx *ctx, const DeltaArgs &a) {
     rc = dense_gemm_f32_launch(ctx, a.proj + a.col_g1, a.ld, a.w.g2, s.rank_gp(), (int)rows, gate.n_plain, s.rank_gp(), gate);
     if (rc != AGPU_OK) return rc;
     const int qk_parts = ceil_div(s.kv_heads, 2), v_parts = ceil_div(s.heads * s.vdim, kPrepareWidth), g_parts = ceil_div(s.heads * s.state_row(), kPrepareWidth);
-    hipLaunchKernelGGL(delta_prepare_kernel, dim3((unsigned)ceil_div(a.new_len, kTokens), (unsigned)(qk_parts + v_parts + g_parts), (unsigned)a.batch),
-                       dim3(256), (size_t)4 * kTokens * s.state_row() * sizeof(float), ctx->stream, a, s.channels(), s.state_row(), qk_parts, v_parts);
+    hipLaunchKernelGGL(delta_prepare_kernel, dim3((unsigned)ceil_div(a.new_len, kConvTokens), (unsigned)(qk_parts + v_parts + g_parts), (unsigned)a.batch),
+                       dim3(256), (size_t)4 * kConvTokens * s.state_row() * sizeof(float), ctx->stream, a, s.channels(), s.state_row(), qk_parts, v_parts);
     if ((rc = AGPU_LAUNCH_CHECK(ctx, "delta_prepare_kernel")) != AGPU_OK) return rc;
     hipLaunchKernelGGL(delta_ring_kernel, dim3((unsigned)ceil_div(s.channels(), 256), (unsigned)s.taps, (unsigned)a.batch), dim3(256), 0, ctx->stream, a,
                        s.channels());

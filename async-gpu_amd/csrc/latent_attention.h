@@ -4,6 +4,7 @@
 #pragma once
 #include "agpu_internal.h"
 #include "dense_linear.h"
+#include "rope.h"
 
 struct LatentShape {
     int heads = 0, dim = 0, rot = 0, rot_dims = 0, vdim = 0, rank = 0;  // rot_dims of the rot dimensions turn
@@ -57,5 +58,3 @@ int32_t latent_absorbed_launch(agpu_ctx *ctx, const LatentArgs &a);
 // on the bf16 matrix cores (fp32 scores and softmax).  bf16 cache only.
 bool latent_tiled_supported(const LatentShape &s);
 int32_t latent_tiled_launch(agpu_ctx *ctx, const LatentArgs &a);
-// cos and sin of p * base^(-2 i / dims) for p < positions, in double precision before rounding: [positions][dims / 2]
-int32_t rope_table_launch(agpu_ctx *ctx, float2 *table, int positions, int dims, double base);

@@ -26,14 +26,6 @@ constexpr int kMatrixHeads = 16;  // heads per workgroup of the matrix-core kern
 constexpr int kMatrixChunk = 32;  // keys per step of the matrix-core kernel
 constexpr float kMinusInf = -3.0e38f;
 
-__global__ void rope_table_kernel(float2 *table, int positions, int half, double base) {
-    const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
-    if (i >= (size_t)positions * half) return;
-    const int p = (int)(i / half), j = (int)(i % half);
-    const double a = (double)p * pow(base, -(double)j / (double)half);
-    table[i] = make_float2((float)cos(a), (float)sin(a));
-}
-
 // Element i of a rotated part v[0 .. rot): dimension i < dims / 2 turns with i + dims / 2.
 __device__ __forceinline__ float rotated(const float *v, int i, int dims, const float2 *cs) {
     const int half = dims >> 1;
@@ -711,13 +703,6 @@ int latent_splits(const agpu_ctx *ctx, const LatentShape &s, int rows, int kv_ma
 }
 
 size_t latent_partial_floats(const LatentShape &s, int rows, int splits) { return (size_t)rows * s.heads * splits * (s.rankp() + 2); }
-
-int32_t rope_table_launch(agpu_ctx *ctx, float2 *table, int positions, int dims, double base) {
-    const int half = dims / 2;
-    if (half == 0) return AGPU_OK;
-    hipLaunchKernelGGL(rope_table_kernel, dim3((unsigned)(((size_t)positions * half + 255) / 256)), dim3(256), 0, ctx->stream, table, positions, half, base);
-    return AGPU_LAUNCH_CHECK(ctx, "rope_table_kernel");
-}
 
 int32_t latent_absorbed_launch(agpu_ctx *ctx, const LatentArgs &a) {
     int32_t rc = check_shape(ctx, a);

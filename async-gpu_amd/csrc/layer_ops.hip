@@ -135,7 +135,10 @@ AGPU_EXPORT int32_t agpu_rope_table(agpu_ctx *ctx, float *table, int32_t positio
     AGPU_REQUIRE_CTX(ctx);
     AGPU_REQUIRE_PTR(ctx, table);
     if (positions <= 0 || dims <= 0 || dims % 2 != 0 || !(base > 0.0)) return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "rope_table: positions %d, dims %d", positions, dims);
-    return rope_table_launch(ctx, (float2 *)table, positions, dims, base);
+    RopeSpec spec;
+    spec.dims = dims;
+    spec.base = base;
+    return rope_table_launch(ctx, (float2 *)table, positions, spec);
 }
 
 AGPU_EXPORT int32_t agpu_latent_cache_row(int32_t rank, int32_t rot_dim) {

@@ -8,12 +8,7 @@
 // The side input's own norm and addition are left to whatever reads x next (DenseRows::y): the next layer's norm, the
 // loop's input or the head.  Up to four rows run as GEMVs that do this in their prologue; more rows go through
 // dense_rows_launch and the matrix cores.
-//
-// Storage: matrices are bf16 [N, K] with N and K padded to multiples of 32 by zeros; activation rows have padded strides
-// whose padding is zero, so no kernel needs to know the true sizes except the norms.
 #include <algorithm>
-#include <cstring>
-#include <functional>
 #include <new>
 #include <string>
 #include <vector>
@@ -22,18 +17,11 @@
 #include "dense_linear.h"
 #include "gated_delta.h"
 #include "latent_attention.h"
-#include "lm_runtime.h"
+#include "layered_model.h"
 
 namespace {
 
 constexpr int kTiledFrom = 16;  // new tokens per sequence from which latent attention takes the tiled form
-
-int pad32(int n) { return (n + 31) / 32 * 32; }
-
-struct Mat {
-    uint16_t *w = nullptr;
-    int N = 0, K = 0;
-};
 
 struct Layer {
     agpu_ritevik_layer c{};
@@ -57,37 +45,6 @@ struct Run {
     size_t state = 0, ring = 0;  // delta state of this run, floats
 };
 
-// A named weight: its shape in the file and how its rows reach the device.
-struct Slot {
-    std::string name;
-    int64_t rows = 0, cols = 0;
-    bool vec = false, set = false;
-    float **vec_dst = nullptr;      // vectors: fp32
-    size_t vec_off = 0;             // ... at this offset of the destination
-    std::function<int32_t(const uint16_t *)> place;  // matrices: bf16 rows
-};
-
-__global__ __launch_bounds__(256) void ritevik_embed_kernel(const uint32_t *__restrict__ tokens, const uint16_t *__restrict__ table,
-                                                            const float *__restrict__ weight, float *x, float *x0, int vocab, int d, int dp, float eps) {
-    __shared__ float red[4];
-    const int row = blockIdx.x, t = threadIdx.x;
-    const uint16_t *e = table + (size_t)min(tokens[row], (uint32_t)(vocab - 1)) * d;
-    float s = 0.0f;
-    for (int k = t; k < d; k += 256) {
-        const float v = bf16_to_f32(e[k]);
-        s += v * v;
-    }
-    s = wave_sum(s);
-    if ((t & 63) == 0) red[t >> 6] = s;
-    __syncthreads();
-    const float rs = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)d + eps);
-    for (int k = t; k < dp; k += 256) {
-        const float v = k < d ? bf16_to_f32(e[k]) * rs * (1.0f + weight[k]) : 0.0f;
-        x[(size_t)row * dp + k] = v;
-        if (x0) x0[(size_t)row * dp + k] = v;
-    }
-}
-
 // Columns [lo, hi) of rows [0, rows) to zero.
 template <typename T>
 __global__ __launch_bounds__(256) void zero_columns_kernel(T *p, int ld, int lo, int hi, int rows) {
@@ -97,24 +54,19 @@ __global__ __launch_bounds__(256) void zero_columns_kernel(T *p, int ld, int lo,
 
 }  // namespace
 
-struct agpu_ritevik final : LmRuntime {
-    agpu_ritevik() : LmRuntime("ritevik") {}
-    int32_t check_ready() override;
+struct agpu_ritevik final : LayeredModel {
+    agpu_ritevik() : LayeredModel("ritevik") {}
     int32_t ensure_buffers(int B, int new_len, bool all_rows_logits) override;
-    int logits_stride() const override { return pad32(V); }
+    int layer_runs() const override { return (int)runs.size(); }
     int32_t launch_forward(const uint32_t *tokens, int B, int new_len, int max_kv, bool all_rows_logits, const ArgmaxAdvance *feed,
                            bool *fed) override;
     void mix_addresses(AddrHash &h, bool one_launch) const override;
     int32_t reset_state() override;
 
     agpu_ritevik_config cfg{};
-    int d = 0, dp = 0, side_p = 0;
-    bool f32 = false;
+    int side_p = 0;
     std::vector<Layer> layers;
     std::vector<Run> runs;
-    std::vector<Slot> slots;
-    std::vector<void *> owned;  // weights, cache, state, tables
-    int64_t weight_bytes = 0, cache_bytes = 0;
     uint16_t *embed = nullptr, *side_embed = nullptr;
     float *embed_norm = nullptr, *final_norm = nullptr, *loop_step = nullptr;
     Mat loop_in, head;
@@ -123,80 +75,11 @@ struct agpu_ritevik final : LmRuntime {
     size_t latent_elems = 0, state_floats = 0;
     int max_cat = 0, max_in = 0;
     DevBuf xa, xb, x0, y, h, proj, cat, side, qlat, partial, qb, kx, vx, dqkg, dv, dstep, dbkq, dgate, dout;
-    float *tap = nullptr;  // residual stream after every layer run, [runs][rows][dp] (agpu_ritevik_layer_streams)
 
     bool small(int rows) const { return dense_gemv_supported(rows, std::max(max_cat, loop_in.K)); }
 };
 
 namespace {
-
-int32_t own(agpu_ritevik *m, void **p, size_t bytes, int64_t *count) {
-    bytes = (bytes + 15) / 16 * 16;
-    int32_t rc = dev_alloc(m->ctx, p, bytes);
-    if (rc != AGPU_OK) return rc;
-    m->owned.push_back(*p);
-    if (count) *count += (int64_t)bytes;
-    return fill_u32(m->ctx, *p, 0u, bytes / 4);
-}
-
-int32_t new_mat(agpu_ritevik *m, Mat &t, int N, int K) {
-    t.N = N;
-    t.K = K;
-    return own(m, (void **)&t.w, (size_t)N * K * 2, &m->weight_bytes);
-}
-
-// `rows` rows of `cols` values to rows row0, row0 + row_step, ... of t, from column col0 on.
-int32_t place_rows(agpu_ritevik *m, const Mat &t, int row0, int row_step, int col0, const uint16_t *src, int64_t rows, int64_t cols, int64_t src_ld) {
-    hipError_t e = hipMemcpy2DAsync(t.w + (size_t)row0 * t.K + col0, (size_t)row_step * t.K * 2, src, (size_t)src_ld * 2, (size_t)cols * 2, (size_t)rows,
-                                    hipMemcpyHostToDevice, m->ctx->stream);
-    if (e == hipSuccess) e = hipStreamSynchronize(m->ctx->stream);
-    return agpu_hip(m->ctx, e, "hipMemcpy2DAsync(weights)");
-}
-
-void add_mat(agpu_ritevik *m, const std::string &name, int64_t rows, int64_t cols, std::function<int32_t(const uint16_t *)> place) {
-    Slot s;
-    s.name = name;
-    s.rows = rows;
-    s.cols = cols;
-    s.place = std::move(place);
-    m->slots.push_back(std::move(s));
-}
-
-// A matrix that fills rows row0 .. of t from column col0 on.
-void add_rows(agpu_ritevik *m, const std::string &name, Mat t, int row0, int col0, int64_t rows, int64_t cols, int row_step = 1) {
-    add_mat(m, name, rows, cols, [=](const uint16_t *src) { return place_rows(m, t, row0, row_step, col0, src, rows, cols, cols); });
-}
-
-// heads x `per` rows, every head moved to a stride of `per_p` rows.
-void add_head_rows(agpu_ritevik *m, const std::string &name, Mat t, int heads, int per, int per_p, int64_t cols) {
-    add_mat(m, name, (int64_t)heads * per, cols, [=](const uint16_t *src) {
-        int32_t rc = AGPU_OK;
-        for (int h = 0; h < heads && rc == AGPU_OK; ++h) rc = place_rows(m, t, h * per_p, 1, 0, src + (size_t)h * per * cols, per, cols, cols);
-        return rc;
-    });
-}
-
-int32_t add_vec(agpu_ritevik *m, const std::string &name, float **dst, int64_t rows, int64_t cols, size_t alloc = 0, size_t off = 0) {
-    if (!*dst) {
-        int32_t rc = own(m, (void **)dst, (alloc ? alloc : (size_t)(rows * cols)) * sizeof(float), &m->weight_bytes);
-        if (rc != AGPU_OK) return rc;
-    }
-    Slot s;
-    s.name = name;
-    s.rows = rows;
-    s.cols = cols;
-    s.vec = true;
-    s.vec_dst = dst;
-    s.vec_off = off;
-    m->slots.push_back(std::move(s));
-    return AGPU_OK;
-}
-
-#define AGPU_TRY(expr)                    \
-    do {                                  \
-        const int32_t rc_ = (expr);       \
-        if (rc_ != AGPU_OK) return rc_;   \
-    } while (0)
 
 int32_t build_layer(agpu_ritevik *m, int i) {
     Layer &L = m->layers[i];
@@ -208,7 +91,7 @@ int32_t build_layer(agpu_ritevik *m, int i) {
     L.mix_w = c.heads * c.vdim;
     L.mix_wp = pad32(L.mix_w);
     L.ffp = pad32(c.ff);
-    AGPU_TRY(add_vec(m, p + "norm1", &L.norm1, 1, d));
+    AGPU_TRY(m->add_vec(p + "norm1", &L.norm1, 1, d));
     if (c.mixer == AGPU_MIXER_LATENT_ATTENTION) {
         if (c.kv_rank <= 0 || c.rot_dim < 0 || c.rot_dims < 0 || c.rot_dims > c.rot_dim || c.rot_dims % 2 != 0 || c.kv_rank > 1024 || c.dim > 1024)
             return agpu_fail(m->ctx, AGPU_ERR_SHAPE_MISMATCH, "ritevik: bad latent attention sizes of layer %d", i);
@@ -219,23 +102,26 @@ int32_t build_layer(agpu_ritevik *m, int i) {
         L.col_q = 0;
         L.col_k = pad32(nq);
         L.n_plain = L.col_k + pad32(nd);
-        AGPU_TRY(new_mat(m, L.in, L.n_plain + 2 * L.ffp, dp));
-        add_rows(m, p + "mix.q", L.in, L.col_q, 0, nq, d);
-        add_rows(m, p + "mix.dkv", L.in, L.col_k, 0, nd, d);
-        AGPU_TRY(add_vec(m, p + "mix.dkv.norm", &L.dkv_norm, 1, c.kv_rank));
-        AGPU_TRY(new_mat(m, L.uk, c.heads * s.dimp(), s.rankp()));
-        add_head_rows(m, p + "mix.uk", L.uk, c.heads, c.dim, s.dimp(), c.kv_rank);
-        AGPU_TRY(new_mat(m, L.uv, c.heads * s.vdimp(), s.rankp()));
-        add_head_rows(m, p + "mix.uv", L.uv, c.heads, c.vdim, s.vdimp(), c.kv_rank);
-        AGPU_TRY(add_vec(m, p + "mix.sink", &L.sink, 1, c.heads));
+        AGPU_TRY(m->new_mat(L.in, L.n_plain + 2 * L.ffp, dp));
+        m->add_rows(p + "mix.q", L.in, L.col_q, 0, nq, d);
+        m->add_rows(p + "mix.dkv", L.in, L.col_k, 0, nd, d);
+        AGPU_TRY(m->add_vec(p + "mix.dkv.norm", &L.dkv_norm, 1, c.kv_rank));
+        AGPU_TRY(m->new_mat(L.uk, c.heads * s.dimp(), s.rankp()));
+        m->add_head_rows(p + "mix.uk", L.uk, c.heads, c.dim, s.dimp(), c.kv_rank);
+        AGPU_TRY(m->new_mat(L.uv, c.heads * s.vdimp(), s.rankp()));
+        m->add_head_rows(p + "mix.uv", L.uv, c.heads, c.vdim, s.vdimp(), c.kv_rank);
+        AGPU_TRY(m->add_vec(p + "mix.sink", &L.sink, 1, c.heads));
         float2 *rope = nullptr;
         for (int j = 0; j < i; ++j) {  // layers that turn alike share a table
             const Layer &o = m->layers[j];
             if (o.c.mixer == c.mixer && o.c.rot_dims == c.rot_dims && o.c.rot_base == c.rot_base) rope = const_cast<float2 *>(o.lw.rope);
         }
         if (!rope && c.rot_dims > 0) {
-            AGPU_TRY(own(m, (void **)&rope, (size_t)m->P * (c.rot_dims / 2) * sizeof(float2), nullptr));
-            AGPU_TRY(rope_table_launch(m->ctx, rope, m->P, c.rot_dims, c.rot_base));
+            AGPU_TRY(m->own((void **)&rope, (size_t)m->P * (c.rot_dims / 2) * sizeof(float2), nullptr));
+            RopeSpec spec;
+            spec.dims = c.rot_dims;
+            spec.base = c.rot_base;
+            AGPU_TRY(rope_table_launch(m->ctx, rope, m->P, spec));
         }
         L.lw.norm = L.dkv_norm; L.lw.uk = L.uk.w; L.lw.uv = L.uv.w; L.lw.sink = L.sink; L.lw.rope = rope;
     } else if (c.mixer == AGPU_MIXER_CHANNEL_DELTA) {
@@ -251,41 +137,41 @@ int32_t build_layer(agpu_ritevik *m, int i) {
         L.col_a1 = L.col_b + pad32(c.heads);
         L.col_g1 = L.col_a1 + s.rank_ap();
         L.n_plain = L.col_g1 + s.rank_gp();
-        AGPU_TRY(new_mat(m, L.in, L.n_plain + 2 * L.ffp, dp));
-        add_rows(m, p + "mix.q", L.in, L.col_q, 0, nk, d);
-        add_rows(m, p + "mix.k", L.in, L.col_k, 0, nk, d);
-        add_rows(m, p + "mix.v", L.in, L.col_v, 0, nv, d);
-        add_rows(m, p + "mix.b", L.in, L.col_b, 0, c.heads, d);
-        add_rows(m, p + "mix.a1", L.in, L.col_a1, 0, c.decay_rank, d);
-        add_rows(m, p + "mix.g1", L.in, L.col_g1, 0, c.gate_rank, d);
+        AGPU_TRY(m->new_mat(L.in, L.n_plain + 2 * L.ffp, dp));
+        m->add_rows(p + "mix.q", L.in, L.col_q, 0, nk, d);
+        m->add_rows(p + "mix.k", L.in, L.col_k, 0, nk, d);
+        m->add_rows(p + "mix.v", L.in, L.col_v, 0, nv, d);
+        m->add_rows(p + "mix.b", L.in, L.col_b, 0, c.heads, d);
+        m->add_rows(p + "mix.a1", L.in, L.col_a1, 0, c.decay_rank, d);
+        m->add_rows(p + "mix.g1", L.in, L.col_g1, 0, c.gate_rank, d);
         const size_t conv = (size_t)s.channels() * c.conv;
-        AGPU_TRY(add_vec(m, p + "mix.q.conv", &L.conv, nk, c.conv, conv, 0));
-        AGPU_TRY(add_vec(m, p + "mix.k.conv", &L.conv, nk, c.conv, conv, (size_t)nk * c.conv));
-        AGPU_TRY(add_vec(m, p + "mix.v.conv", &L.conv, nv, c.conv, conv, (size_t)2 * nk * c.conv));
-        AGPU_TRY(add_vec(m, p + "mix.A_log", &L.a_log, 1, c.heads));
-        AGPU_TRY(add_vec(m, p + "mix.dt_bias", &L.dt_bias, 1, (int64_t)c.heads * c.dim));
-        AGPU_TRY(add_vec(m, p + "mix.norm", &L.mix_norm, 1, c.vdim));
-        AGPU_TRY(new_mat(m, L.a2, c.heads * s.state_row(), s.rank_ap()));
-        add_head_rows(m, p + "mix.a2", L.a2, c.heads, c.dim, s.state_row(), c.decay_rank);
-        AGPU_TRY(new_mat(m, L.g2, nv, s.rank_gp()));
-        add_rows(m, p + "mix.g2", L.g2, 0, 0, nv, c.gate_rank);
+        AGPU_TRY(m->add_vec(p + "mix.q.conv", &L.conv, nk, c.conv, conv, 0));
+        AGPU_TRY(m->add_vec(p + "mix.k.conv", &L.conv, nk, c.conv, conv, (size_t)nk * c.conv));
+        AGPU_TRY(m->add_vec(p + "mix.v.conv", &L.conv, nv, c.conv, conv, (size_t)2 * nk * c.conv));
+        AGPU_TRY(m->add_vec(p + "mix.A_log", &L.a_log, 1, c.heads));
+        AGPU_TRY(m->add_vec(p + "mix.dt_bias", &L.dt_bias, 1, (int64_t)c.heads * c.dim));
+        AGPU_TRY(m->add_vec(p + "mix.norm", &L.mix_norm, 1, c.vdim));
+        AGPU_TRY(m->new_mat(L.a2, c.heads * s.state_row(), s.rank_ap()));
+        m->add_head_rows(p + "mix.a2", L.a2, c.heads, c.dim, s.state_row(), c.decay_rank);
+        AGPU_TRY(m->new_mat(L.g2, nv, s.rank_gp()));
+        m->add_rows(p + "mix.g2", L.g2, 0, 0, nv, c.gate_rank);
         L.dw.conv = L.conv; L.dw.a_log = L.a_log; L.dw.dt_bias = L.dt_bias; L.dw.a2 = L.a2.w; L.dw.g2 = L.g2.w; L.dw.norm = L.mix_norm;
     } else {
         return agpu_fail(m->ctx, AGPU_ERR_UNSUPPORTED, "ritevik: unknown mixer %d of layer %d", c.mixer, i);
     }
-    AGPU_TRY(new_mat(m, L.out, dp, L.cat_k()));
-    add_rows(m, p + "mix.o", L.out, 0, 0, d, L.mix_w);
+    AGPU_TRY(m->new_mat(L.out, dp, L.cat_k()));
+    m->add_rows(p + "mix.o", L.out, 0, 0, d, L.mix_w);
     if (c.ff > 0) {
-        add_rows(m, p + "mlp.gate", L.in, L.n_plain, 0, c.ff, d, 2);
-        add_rows(m, p + "mlp.up", L.in, L.n_plain + 1, 0, c.ff, d, 2);
-        add_rows(m, p + "mlp.down", L.out, 0, L.mix_wp, d, c.ff);
+        m->add_rows(p + "mlp.gate", L.in, L.n_plain, 0, c.ff, d, 2);
+        m->add_rows(p + "mlp.up", L.in, L.n_plain + 1, 0, c.ff, d, 2);
+        m->add_rows(p + "mlp.down", L.out, 0, L.mix_wp, d, c.ff);
     }
     if (m->cfg.side_dim > 0) {
-        AGPU_TRY(new_mat(m, L.side_gate, m->side_p, dp));
-        add_rows(m, p + "side.gate", L.side_gate, 0, 0, m->cfg.side_dim, d);
-        AGPU_TRY(new_mat(m, L.side_proj, dp, m->side_p));
-        add_rows(m, p + "side.proj", L.side_proj, 0, 0, d, m->cfg.side_dim);
-        AGPU_TRY(add_vec(m, p + "side.norm", &L.side_norm, 1, d));
+        AGPU_TRY(m->new_mat(L.side_gate, m->side_p, dp));
+        m->add_rows(p + "side.gate", L.side_gate, 0, 0, m->cfg.side_dim, d);
+        AGPU_TRY(m->new_mat(L.side_proj, dp, m->side_p));
+        m->add_rows(p + "side.proj", L.side_proj, 0, 0, d, m->cfg.side_dim);
+        AGPU_TRY(m->add_vec(p + "side.norm", &L.side_norm, 1, d));
     }
     m->max_cat = std::max(m->max_cat, L.cat_k());
     m->max_in = std::max(m->max_in, L.n_plain);
@@ -298,39 +184,32 @@ int32_t build(agpu_ritevik *m) {
     Mat et;
     et.N = V;
     et.K = d;
-    AGPU_TRY(own(m, (void **)&m->embed, (size_t)V * d * 2, &m->weight_bytes));
+    AGPU_TRY(m->own((void **)&m->embed, (size_t)V * d * 2, &m->weight_bytes));
     et.w = m->embed;
-    add_rows(m, "embed", et, 0, 0, V, d);
-    AGPU_TRY(add_vec(m, "embed.norm", &m->embed_norm, 1, d));
+    m->add_rows("embed", et, 0, 0, V, d);
+    AGPU_TRY(m->add_vec("embed.norm", &m->embed_norm, 1, d));
     if (c.loop_times > 0) {
-        AGPU_TRY(new_mat(m, m->loop_in, dp, 2 * dp));
+        AGPU_TRY(m->new_mat(m->loop_in, dp, 2 * dp));
         const Mat t = m->loop_in;
-        add_mat(m, "loop.in", d, 2 * d, [=](const uint16_t *src) {
-            int32_t rc = place_rows(m, t, 0, 1, 0, src, d, d, 2 * d);
-            return rc == AGPU_OK ? place_rows(m, t, 0, 1, dp, src + d, d, d, 2 * d) : rc;
+        m->add_mat("loop.in", d, 2 * d, [=](const uint16_t *src) {
+            int32_t rc = place_rows(m->ctx, t, 0, 1, 0, src, d, d, 2 * d);
+            return rc == AGPU_OK ? place_rows(m->ctx, t, 0, 1, dp, src + d, d, d, 2 * d) : rc;
         });
         // rows of the step table have the padded stride of the residual stream
-        AGPU_TRY(own(m, (void **)&m->loop_step, (size_t)c.loop_times * dp * sizeof(float), &m->weight_bytes));
-        Slot s;
-        s.name = "loop.step";
-        s.rows = c.loop_times;
-        s.cols = d;
-        s.vec = true;
-        s.vec_dst = &m->loop_step;
-        m->slots.push_back(std::move(s));
+        AGPU_TRY(m->add_vec("loop.step", &m->loop_step, c.loop_times, d, (size_t)c.loop_times * dp, 0, d, dp));
     }
     if (c.side_dim > 0) {
         Mat st;
         st.N = V;
         st.K = c.n_layer * c.side_dim;
-        AGPU_TRY(own(m, (void **)&m->side_embed, (size_t)st.N * st.K * 2, &m->weight_bytes));
+        AGPU_TRY(m->own((void **)&m->side_embed, (size_t)st.N * st.K * 2, &m->weight_bytes));
         st.w = m->side_embed;
-        add_rows(m, "side.embed", st, 0, 0, V, st.K);
+        m->add_rows("side.embed", st, 0, 0, V, st.K);
     }
     for (int i = 0; i < c.n_layer; ++i) AGPU_TRY(build_layer(m, i));
-    AGPU_TRY(add_vec(m, "final.norm", &m->final_norm, 1, d));
-    AGPU_TRY(new_mat(m, m->head, pad32(V), dp));
-    add_rows(m, "head", m->head, 0, 0, V, d);
+    AGPU_TRY(m->add_vec("final.norm", &m->final_norm, 1, d));
+    AGPU_TRY(m->new_mat(m->head, pad32(V), dp));
+    m->add_rows("head", m->head, 0, 0, V, d);
 
     // the layer runs in order, each with a cache or state of its own
     auto push = [&](int layer, int step) {
@@ -354,15 +233,9 @@ int32_t build(agpu_ritevik *m) {
     for (int t = 0; t < c.loop_times; ++t)
         for (int i = lo; i < hi; ++i) push(i, i == lo ? t : -1);
     for (int i = hi; i < c.n_layer; ++i) push(i, -1);
-    if (m->latent_elems) AGPU_TRY(own(m, &m->latents, m->latent_elems * (m->f32 ? 4 : 2), &m->cache_bytes));
-    if (m->state_floats) AGPU_TRY(own(m, (void **)&m->state, m->state_floats * sizeof(float), &m->cache_bytes));
+    if (m->latent_elems) AGPU_TRY(m->own(&m->latents, m->latent_elems * (m->f32 ? 4 : 2), &m->cache_bytes));
+    if (m->state_floats) AGPU_TRY(m->own((void **)&m->state, m->state_floats * sizeof(float), &m->cache_bytes));
     return AGPU_OK;
-}
-
-// A Linear on rows that a matrix-core kernel reads: `a` is bf16 or fp32 as the model computes.
-int32_t gemm(agpu_ritevik *m, const void *a, int lda, const Mat &w, int M, const DenseOut &o) {
-    if (m->f32) return dense_gemm_f32_launch(m->ctx, (const float *)a, lda, w.w, w.K, M, w.N, w.K, o);
-    return dense_gemm_bf16_launch(m->ctx, (const uint16_t *)a, lda, w.w, w.K, M, w.N, w.K, o);
 }
 
 int32_t mixer(agpu_ritevik *m, const Run &r, int B, int new_len, int max_kv, void *cat, bool cat_bf16) {
@@ -439,9 +312,7 @@ int32_t agpu_ritevik::launch_forward(const uint32_t *tokens, int B, int new_len,
     const int R = B * new_len;
     const bool gemv = small(R), a16 = !f32 && !gemv;
     float *x = (float *)xa.p, *spare = (float *)xb.p;
-    hipLaunchKernelGGL(ritevik_embed_kernel, dim3((unsigned)R), dim3(256), 0, ctx->stream, tokens, embed, embed_norm, x, cfg.loop_times > 0 ? (float *)x0.p : nullptr,
-                       V, d, dp, cfg.norm_eps);
-    AGPU_TRY(AGPU_LAUNCH_CHECK(ctx, "ritevik_embed_kernel"));
+    AGPU_TRY(embed_rows_launch(ctx, tokens, embed, d, embed_norm, x, cfg.loop_times > 0 ? (float *)x0.p : nullptr, R, V, d, dp, cfg.norm_eps));
     const float *pending = nullptr;  // the side norm of a layer whose addend still waits in `y`
     auto rows_of = [&](const float *norm_w) {
         DenseRows in;
@@ -471,7 +342,7 @@ int32_t agpu_ritevik::launch_forward(const uint32_t *tokens, int B, int new_len,
                 AGPU_TRY(dense_gemv_launch(ctx, in, loop_in.w, R, loop_in.N, loop_in.K, o));
             } else {
                 AGPU_TRY(dense_rows_launch(ctx, in, R, h.p, 2 * dp, a16));
-                AGPU_TRY(gemm(this, h.p, 2 * dp, loop_in, R, o));
+                AGPU_TRY(gemm(h.p, 2 * dp, loop_in, R, o));
             }
             std::swap(x, spare);
             pending = nullptr;
@@ -490,7 +361,7 @@ int32_t agpu_ritevik::launch_forward(const uint32_t *tokens, int B, int new_len,
         } else {
             if (pending) in.x_out = x;
             AGPU_TRY(dense_rows_launch(ctx, in, R, h.p, dp, a16));
-            AGPU_TRY(gemm(this, h.p, dp, L.in, R, o));
+            AGPU_TRY(gemm(h.p, dp, L.in, R, o));
         }
         pending = nullptr;
         AGPU_TRY(mixer(this, r, B, new_len, max_kv, cat.p, a16));
@@ -504,7 +375,7 @@ int32_t agpu_ritevik::launch_forward(const uint32_t *tokens, int B, int new_len,
             ci.ldx = ci.d = ci.dp = L.cat_k();
             AGPU_TRY(dense_gemv_launch(ctx, ci, L.out.w, R, L.out.N, L.out.K, oo));
         } else {
-            AGPU_TRY(gemm(this, cat.p, L.cat_k(), L.out, R, oo));
+            AGPU_TRY(gemm(cat.p, L.cat_k(), L.out, R, oo));
         }
         if (cfg.side_dim > 0) {
             DenseOut og, op;
@@ -531,8 +402,8 @@ int32_t agpu_ritevik::launch_forward(const uint32_t *tokens, int B, int new_len,
                     AGPU_TRY(dense_rows_launch(ctx, rows_of(nullptr), R, h.p, dp, 1));
                     xin = h.p;
                 }
-                AGPU_TRY(gemm(this, xin, dp, L.side_gate, R, og));
-                AGPU_TRY(gemm(this, side.p, side_p, L.side_proj, R, op));
+                AGPU_TRY(gemm(xin, dp, L.side_gate, R, og));
+                AGPU_TRY(gemm(side.p, side_p, L.side_proj, R, op));
             }
             pending = L.side_norm;
         }
@@ -543,7 +414,7 @@ int32_t agpu_ritevik::launch_forward(const uint32_t *tokens, int B, int new_len,
                 AGPU_TRY(dense_rows_launch(ctx, fi, R, nullptr, 0, 0));
                 pending = nullptr;
             }
-            AGPU_TRY(agpu_hip(ctx, hipMemcpyAsync(tap + i * (size_t)R * dp, x, (size_t)R * dp * 4, hipMemcpyDeviceToDevice, ctx->stream), "hipMemcpyAsync"));
+            AGPU_TRY(save_tap(i, x, R));
         }
     }
     const int rows = all_rows_logits ? R : B;
@@ -554,7 +425,7 @@ int32_t agpu_ritevik::launch_forward(const uint32_t *tokens, int B, int new_len,
     o.out = (float *)logits.p;
     if (dense_gemv_supported(rows, dp)) return dense_gemv_launch(ctx, in, head.w, rows, head.N, head.K, o);
     AGPU_TRY(dense_rows_launch(ctx, in, rows, h.p, dp, !f32));
-    return gemm(this, h.p, dp, head, rows, o);
+    return gemm(h.p, dp, head, rows, o);
 }
 
 int32_t agpu_ritevik::ensure_buffers(int B, int new_len, bool all_rows_logits) {
@@ -596,12 +467,6 @@ int32_t agpu_ritevik::ensure_buffers(int B, int new_len, bool all_rows_logits) {
     return AGPU_OK;
 }
 
-int32_t agpu_ritevik::check_ready() {
-    for (const Slot &s : slots)
-        if (!s.set) return agpu_fail(ctx, AGPU_ERR_NULL_POINTER, "ritevik: tensor '%s' not set", s.name.c_str());
-    return AGPU_OK;
-}
-
 void agpu_ritevik::mix_addresses(AddrHash &hash, bool) const {
     for (void *p : owned) hash.mix(p);
     for (const DevBuf *b : {&xa, &xb, &x0, &y, &h, &proj, &cat, &side, &qlat, &partial}) hash.mix(b->p);
@@ -640,75 +505,19 @@ AGPU_EXPORT int32_t agpu_ritevik_create(agpu_ctx *ctx, const agpu_ritevik_config
 
 AGPU_EXPORT int32_t agpu_ritevik_destroy(agpu_ritevik *m) {
     if (!m) return AGPU_OK;
-    if (m->ctx) (void)hipStreamSynchronize(m->ctx->stream);
-    for (void *p : m->owned) (void)hipFree(p);
-    for (DevBuf *b : {&m->xa, &m->xb, &m->x0, &m->y, &m->h, &m->proj, &m->cat, &m->side, &m->qlat, &m->partial, &m->qb, &m->kx, &m->vx, &m->dqkg, &m->dv,
-                      &m->dstep, &m->dbkq, &m->dgate, &m->dout})
-        if (b->p) (void)hipFree(b->p);
-    lm_release(m);
+    layered_release(m, {&m->xa, &m->xb, &m->x0, &m->y, &m->h, &m->proj, &m->cat, &m->side, &m->qlat, &m->partial, &m->qb, &m->kx, &m->vx, &m->dqkg, &m->dv,
+                        &m->dstep, &m->dbkq, &m->dgate, &m->dout});
     delete m;
     return AGPU_OK;
 }
 
 AGPU_EXPORT int32_t agpu_ritevik_set_tensor(agpu_ritevik *m, const char *name, const void *data_host, int32_t dtype, int64_t rows, int64_t cols) {
-    if (!m) return AGPU_ERR_NULL_POINTER;
-    agpu_ctx *ctx = m->ctx;
-    AGPU_REQUIRE_CTX(ctx);
-    if (!name || !data_host) return agpu_fail(ctx, AGPU_ERR_NULL_POINTER, "ritevik_set_tensor: null pointer");
-    if (dtype != AGPU_DTYPE_BF16 && dtype != AGPU_DTYPE_F32) return agpu_fail(ctx, AGPU_ERR_UNSUPPORTED, "ritevik_set_tensor: unknown dtype %d", dtype);
-    Slot *s = nullptr;
-    for (Slot &t : m->slots)
-        if (t.name == name) s = &t;
-    if (!s) return agpu_fail(ctx, AGPU_ERR_KERNEL_NOT_FOUND, "ritevik_set_tensor: this configuration has no tensor '%s'", name);
-    if (rows != s->rows || cols != s->cols)
-        return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "ritevik_set_tensor: '%s' is [%lld, %lld], expected [%lld, %lld]", name, (long long)rows,
-                         (long long)cols, (long long)s->rows, (long long)s->cols);
-    const size_t n = (size_t)(rows * cols);
-    int32_t rc;
-    if (s->vec) {
-        std::vector<float> v(n);
-        if (dtype == AGPU_DTYPE_F32) {
-            std::memcpy(v.data(), data_host, n * sizeof(float));
-        } else {
-            for (size_t i = 0; i < n; ++i) {
-                const uint32_t u = (uint32_t)((const uint16_t *)data_host)[i] << 16;
-                std::memcpy(&v[i], &u, 4);
-            }
-        }
-        float *dst = *s->vec_dst + s->vec_off;
-        if (dst == m->loop_step) {
-            hipError_t e = hipMemcpy2DAsync(dst, (size_t)m->dp * 4, v.data(), (size_t)cols * 4, (size_t)cols * 4, (size_t)rows, hipMemcpyHostToDevice,
-                                            ctx->stream);
-            if (e == hipSuccess) e = hipStreamSynchronize(ctx->stream);
-            rc = agpu_hip(ctx, e, "hipMemcpy2DAsync(weights)");
-        } else {
-            rc = upload(ctx, dst, v.data(), n * sizeof(float), 0);
-        }
-    } else if (dtype == AGPU_DTYPE_BF16) {
-        rc = s->place((const uint16_t *)data_host);
-    } else {
-        std::vector<uint16_t> v(n);
-        for (size_t i = 0; i < n; ++i) {
-            uint32_t u;
-            std::memcpy(&u, (const float *)data_host + i, 4);
-            v[i] = (u & 0x7fffffffu) > 0x7f800000u ? (uint16_t)((u >> 16) | 0x40u) : (uint16_t)((u + 0x7fffu + ((u >> 16) & 1u)) >> 16);
-        }
-        rc = s->place(v.data());
-    }
-    if (rc == AGPU_OK) s->set = true;
-    return rc;
+    return m ? lm_set_tensor(m, name, data_host, dtype, rows, cols) : AGPU_ERR_NULL_POINTER;
 }
 
 AGPU_EXPORT int32_t agpu_ritevik_tensor_info(const agpu_ritevik *m, int32_t i, const char **name_out, int64_t *rows_out, int64_t *cols_out,
                                              int32_t *is_set_out) {
-    if (!m || !name_out || !rows_out || !cols_out || !is_set_out) return AGPU_ERR_NULL_POINTER;
-    if (i < 0 || (size_t)i >= m->slots.size()) return AGPU_ERR_DIM_OUT_OF_RANGE;
-    const Slot &s = m->slots[(size_t)i];
-    *name_out = s.name.c_str();
-    *rows_out = s.rows;
-    *cols_out = s.cols;
-    *is_set_out = s.set ? 1 : 0;
-    return AGPU_OK;
+    return m ? lm_tensor_info(m, i, name_out, rows_out, cols_out, is_set_out) : AGPU_ERR_NULL_POINTER;
 }
 
 AGPU_EXPORT int64_t agpu_ritevik_weight_bytes(const agpu_ritevik *m) { return m ? m->weight_bytes : 0; }
@@ -753,21 +562,5 @@ AGPU_EXPORT int32_t agpu_ritevik_last_logits(agpu_ritevik *m, int32_t batch, flo
 }
 
 AGPU_EXPORT int32_t agpu_ritevik_layer_streams(agpu_ritevik *m, const uint32_t *tokens, int32_t new_len, float *streams_out_host) {
-    if (!m) return AGPU_ERR_NULL_POINTER;
-    agpu_ctx *ctx = m->ctx;
-    AGPU_REQUIRE_CTX(ctx);
-    if (!streams_out_host || new_len <= 0) return agpu_fail(ctx, AGPU_ERR_NULL_POINTER, "ritevik_layer_streams: null pointer or no tokens");
-    const size_t rows = m->runs.size() * (size_t)new_len;
-    AGPU_TRY(dev_alloc(ctx, (void **)&m->tap, rows * m->dp * sizeof(float)));
-    int32_t rc = lm_forward_cached(m, tokens, 1, new_len, nullptr, 0);
-    if (rc == AGPU_OK) {
-        hipError_t e = hipMemcpy2DAsync(streams_out_host, (size_t)m->d * 4, m->tap, (size_t)m->dp * 4, (size_t)m->d * 4, rows, hipMemcpyDeviceToHost,
-                                        ctx->stream);
-        if (e == hipSuccess) e = hipStreamSynchronize(ctx->stream);
-        rc = agpu_hip(ctx, e, "ritevik_layer_streams");
-    }
-    (void)hipStreamSynchronize(ctx->stream);
-    (void)hipFree(m->tap);
-    m->tap = nullptr;
-    return rc;
+    return m ? lm_layer_streams(m, tokens, new_len, streams_out_host) : AGPU_ERR_NULL_POINTER;
 }

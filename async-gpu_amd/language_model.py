@@ -1,5 +1,5 @@
 """What every language model of the library shares on the Python side: the calls over the generation runtime that each
-model exports under its own prefix (agpu_gpt2_*, agpu_ritevik_*)."""
+model exports under its own prefix (agpu_gpt2_*, agpu_ritevik_*, agpu_piralix_*)."""
 import ctypes as C
 
 import numpy as np

@@ -8,9 +8,18 @@ import os
 from . import weights
 
 
-def _ritevik(path, dtype, n_positions, max_batch, ctx, device):
+def _layered(model_class, path, dtype, n_positions, max_batch, ctx, device):
+    return model_class.from_directory(path, ctx, device, dtype=dtype, n_positions=n_positions or 1024, max_batch=max_batch)
+
+
+def _ritevik(*args):
     from .ritevik import RitevikModel
-    return RitevikModel.from_directory(path, ctx, device, dtype=dtype, n_positions=n_positions or 1024, max_batch=max_batch)
+    return _layered(RitevikModel, *args)
+
+
+def _piralix(*args):
+    from .piralix import PiralixModel
+    return _layered(PiralixModel, *args)
 
 
 def _gpt2(path, dtype, n_positions, max_batch, ctx, device):
@@ -21,7 +30,7 @@ def _gpt2(path, dtype, n_positions, max_batch, ctx, device):
     return Int4Gpt2Model.from_file(path, ctx=ctx, device=device, max_batch=max_batch)
 
 
-ARCHITECTURES = {"Ritevik": _ritevik, "GPT2LMHeadModel": _gpt2}
+ARCHITECTURES = {"Ritevik": _ritevik, "Piralix": _piralix, "GPT2LMHeadModel": _gpt2}
 
 
 def architecture(path):

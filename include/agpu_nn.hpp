@@ -27,6 +27,7 @@
 
 #include "agpu.h"
 #include "agpu_gpt2.h"
+#include "agpu_piralix.h"
 #include "agpu_ritevik.h"
 
 namespace agpu {
@@ -771,24 +772,25 @@ private:
     agpu_gpt2 *h_ = nullptr;
 };
 
-// RitevikModel over include/agpu_ritevik.h (no counterpart in the reference; the calls follow Int4Gpt2Model).  The caller
-// fills the configuration structs and hands every tensor over by its name in the model file.
-class RitevikModel {
+// The models with bf16 weights (no counterpart in the reference; the calls follow Int4Gpt2Model).  The caller fills the
+// configuration structs and hands every tensor over by its name in the model file.  `Api` names a model's C entry points.
+template <class Api>
+class LayeredModel {
 public:
-    RitevikModel(const agpu_ritevik_config &config, const std::vector<agpu_ritevik_layer> &layers, const Registry &reg) : config_(config), reg_(reg) {
+    LayeredModel(const typename Api::Config &config, const std::vector<typename Api::Layer> &layers, const Registry &reg) : config_(config), reg_(reg) {
         if (layers.size() != (size_t)config.n_layer)
             throw NnError::shape_mismatch(std::to_string(config.n_layer) + " layers", std::to_string(layers.size()));
-        reg->check(agpu_ritevik_create(reg->device(), &config, layers.data(), &h_));
+        reg->check(Api::create(reg->device(), &config, layers.data(), &h_));
     }
-    RitevikModel(RitevikModel &&o) noexcept : config_(o.config_), reg_(std::move(o.reg_)), h_(o.h_) { o.h_ = nullptr; }
-    RitevikModel(const RitevikModel &) = delete;
-    ~RitevikModel() {
-        if (h_) agpu_ritevik_destroy(h_);
+    LayeredModel(LayeredModel &&o) noexcept : config_(o.config_), reg_(std::move(o.reg_)), h_(o.h_) { o.h_ = nullptr; }
+    LayeredModel(const LayeredModel &) = delete;
+    ~LayeredModel() {
+        if (h_) Api::destroy(h_);
     }
     // bf16 bits in the file's shape; a vector has rows = 1
     void set_tensor(const std::string &name, const std::vector<uint16_t> &bits, size_t rows, size_t cols) const {
         if (bits.size() != rows * cols) throw NnError::shape_mismatch(std::to_string(rows * cols) + " values", std::to_string(bits.size()));
-        reg_->check(agpu_ritevik_set_tensor(h_, name.c_str(), bits.data(), AGPU_DTYPE_BF16, (int64_t)rows, (int64_t)cols));
+        reg_->check(Api::set_tensor(h_, name.c_str(), bits.data(), AGPU_DTYPE_BF16, (int64_t)rows, (int64_t)cols));
     }
     // (name, rows, cols) of every tensor the configuration needs
     std::vector<std::tuple<std::string, size_t, size_t>> tensors() const {
@@ -796,20 +798,20 @@ public:
         const char *name = nullptr;
         int64_t rows = 0, cols = 0;
         int32_t set = 0;
-        for (int32_t i = 0; agpu_ritevik_tensor_info(h_, i, &name, &rows, &cols, &set) == AGPU_OK; ++i) out.emplace_back(name, (size_t)rows, (size_t)cols);
+        for (int32_t i = 0; Api::tensor_info(h_, i, &name, &rows, &cols, &set) == AGPU_OK; ++i) out.emplace_back(name, (size_t)rows, (size_t)cols);
         return out;
     }
-    size_t cache_len() const { return (size_t)agpu_ritevik_cache_len(h_); }
-    void reset_cache() const { reg_->check(agpu_ritevik_reset_cache(h_)); }
+    size_t cache_len() const { return (size_t)Api::cache_len(h_); }
+    void reset_cache() const { reg_->check(Api::reset_cache(h_)); }
     GpuTensor forward_cached(const GpuBufferU32 &token_ids, size_t new_len) const {
         GpuTensor logits = GpuTensor::zeros({new_len, (size_t)config_.vocab_size}, reg_);
-        reg_->check(agpu_ritevik_forward_cached(h_, token_ids.data(), 1, (int32_t)new_len, logits.data(), 1));
+        reg_->check(Api::forward_cached(h_, token_ids.data(), 1, (int32_t)new_len, logits.data(), 1));
         return logits;
     }
     std::vector<uint32_t> generate_cached(const std::vector<uint32_t> &prompt, size_t max_new_tokens, int eos = -1) const {
         std::vector<uint32_t> out(prompt.size() + max_new_tokens);
         int32_t len = 0;
-        reg_->check(agpu_ritevik_generate_cached(h_, prompt.data(), 1, (int32_t)prompt.size(), (int32_t)max_new_tokens, eos, out.data(), &len, nullptr));
+        reg_->check(Api::generate_cached(h_, prompt.data(), 1, (int32_t)prompt.size(), (int32_t)max_new_tokens, eos, out.data(), &len, nullptr));
         out.resize((size_t)len);
         return out;
     }
@@ -817,18 +819,49 @@ public:
                                                    SimpleRng &rng, int eos = -1) const {
         std::vector<uint32_t> out(prompt.size() + max_new_tokens);
         int32_t len = 0;
-        reg_->check(agpu_ritevik_generate_cached_sampling(h_, prompt.data(), (int32_t)prompt.size(), (int32_t)max_new_tokens, (int32_t)top_k, temperature,
+        reg_->check(Api::generate_cached_sampling(h_, prompt.data(), (int32_t)prompt.size(), (int32_t)max_new_tokens, (int32_t)top_k, temperature,
                                                           rng.state(), eos, out.data(), &len));
         out.resize((size_t)len);
         return out;
     }
-    const agpu_ritevik_config &config() const { return config_; }
+    const typename Api::Config &config() const { return config_; }
 
 private:
-    agpu_ritevik_config config_;
+    typename Api::Config config_;
     Registry reg_;
-    agpu_ritevik *h_ = nullptr;
+    typename Api::Model *h_ = nullptr;
 };
+
+struct RitevikApi {  // include/agpu_ritevik.h
+    using Model = agpu_ritevik;
+    using Config = agpu_ritevik_config;
+    using Layer = agpu_ritevik_layer;
+    static constexpr auto cache_len = agpu_ritevik_cache_len;
+    static constexpr auto create = agpu_ritevik_create;
+    static constexpr auto destroy = agpu_ritevik_destroy;
+    static constexpr auto forward_cached = agpu_ritevik_forward_cached;
+    static constexpr auto generate_cached = agpu_ritevik_generate_cached;
+    static constexpr auto generate_cached_sampling = agpu_ritevik_generate_cached_sampling;
+    static constexpr auto reset_cache = agpu_ritevik_reset_cache;
+    static constexpr auto set_tensor = agpu_ritevik_set_tensor;
+    static constexpr auto tensor_info = agpu_ritevik_tensor_info;
+};
+struct PiralixApi {  // include/agpu_piralix.h
+    using Model = agpu_piralix;
+    using Config = agpu_piralix_config;
+    using Layer = agpu_piralix_layer;
+    static constexpr auto cache_len = agpu_piralix_cache_len;
+    static constexpr auto create = agpu_piralix_create;
+    static constexpr auto destroy = agpu_piralix_destroy;
+    static constexpr auto forward_cached = agpu_piralix_forward_cached;
+    static constexpr auto generate_cached = agpu_piralix_generate_cached;
+    static constexpr auto generate_cached_sampling = agpu_piralix_generate_cached_sampling;
+    static constexpr auto reset_cache = agpu_piralix_reset_cache;
+    static constexpr auto set_tensor = agpu_piralix_set_tensor;
+    static constexpr auto tensor_info = agpu_piralix_tensor_info;
+};
+using RitevikModel = LayeredModel<RitevikApi>;
+using PiralixModel = LayeredModel<PiralixApi>;
 
 }  // namespace nn
 }  // namespace agpu

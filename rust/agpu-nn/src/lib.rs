@@ -12,13 +12,14 @@
 //! | `ops::*` | nn/ops/{gemm,norm,activation,reshape,attention,quantize}.rs |
 //! | `Int4Linear`, `LayerNorm`, `Embedding`, `Module` | nn/layers/*.rs |
 //! | `Gpt2Config`, `Int4Gpt2Model` | nn/models/gpt2.rs:20-93, 712-783, 1341-1580 |
-//! | `RitevikModel` | none |
+//! | `RitevikModel`, `PiralixModel` | none |
 pub mod error;
 pub mod gpt2;
 pub mod gpu_array;
 pub mod layers;
 pub mod ops;
 pub mod registry;
+pub mod piralix;
 pub mod ritevik;
 pub mod tensor;
 
@@ -27,5 +28,6 @@ pub use gpt2::{Gpt2Config, Int4Gpt2Model};
 pub use gpu_array::{GpuArray, Residency};
 pub use layers::{Embedding, Int4Linear, LayerNorm, Module};
 pub use registry::KernelRegistry;
+pub use piralix::PiralixModel;
 pub use ritevik::RitevikModel;
 pub use tensor::GpuTensor;

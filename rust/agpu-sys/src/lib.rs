@@ -1,6 +1,6 @@
 //! agpu-sys: the raw `extern "C"` surface of libagpu_hip.so, the MI355X (gfx950) implementation of async_gpu's
-//! quantized GPT-2 inference path.  One declaration per function of `include/agpu.h`, `agpu_gpt2.h` and `agpu_ritevik.h`,
-//! in header order; `build.rs` compiles the HIP sources with hipcc and links the shared library.
+//! quantized GPT-2 inference path.  One declaration per function of `include/agpu.h`, `agpu_gpt2.h`, `agpu_ritevik.h` and
+//! `agpu_piralix.h`, in header order; `build.rs` compiles the HIP sources with hipcc and links the shared library.
 //!
 //! What each function replaces in the reference is stated next to its C declaration.  The safe layer over these
 //! declarations, with the reference's own names (`KernelRegistry`, `GpuTensor`, `GpuArray`, `Int4Linear`,
@@ -140,6 +140,54 @@ pub struct agpu_ritevik_layer {
     pub gate_rank: i32,
 }
 
+/// Opaque Piralix model.
+#[repr(C)]
+pub struct agpu_piralix {
+    _private: [u8; 0],
+}
+
+/// `agpu_piralix_config` of include/agpu_piralix.h.
+#[repr(C)]
+#[derive(Clone, Copy, Debug, Default)]
+pub struct agpu_piralix_config {
+    pub n_layer: i32,
+    pub width: i32,
+    pub vocab_size: i32,
+    pub n_positions: i32,
+    pub max_batch: i32,
+    pub norm_eps: f32,
+    pub loop_start: i32,
+    pub loop_stop: i32,
+    pub loop_times: i32,
+    pub dtype: i32,
+    pub argmax_last: i32,
+}
+
+/// `agpu_piralix_layer` of include/agpu_piralix.h.
+#[repr(C)]
+#[derive(Clone, Copy, Debug, Default)]
+pub struct agpu_piralix_layer {
+    pub mixer: i32,
+    pub heads: i32,
+    pub dim: i32,
+    pub vdim: i32,
+    pub ff: i32,
+    pub ff_limit: f32,
+    pub gate_cap: f32,
+    pub scale: f32,
+    pub softcap: f32,
+    pub kv_heads: i32,
+    pub rot_dims: i32,
+    pub rot_base: f64,
+    pub rot_factor: f64,
+    pub rot_original: f64,
+    pub rot_fast: f64,
+    pub rot_slow: f64,
+    pub lru_width: i32,
+    pub blocks: i32,
+    pub conv: i32,
+}
+
 pub const AGPU_OK: i32 = 0;
 pub const AGPU_ERR_SHAPE_MISMATCH: i32 = -1;
 pub const AGPU_ERR_DIM_OUT_OF_RANGE: i32 = -2;
@@ -173,6 +221,9 @@ pub const AGPU_DTYPE_F32: i32 = 1;
 pub const AGPU_DENSE_GATED: u32 = 1;
 pub const AGPU_MIXER_LATENT_ATTENTION: i32 = 0;
 pub const AGPU_MIXER_CHANNEL_DELTA: i32 = 1;
+pub const AGPU_MIXER_MATRIX_MEMORY: i32 = 2;
+pub const AGPU_MIXER_GROUPED_ATTENTION: i32 = 3;
+pub const AGPU_MIXER_GATED_LRU: i32 = 4;
 
 extern "C" {
     // ---- include/agpu.h ----
@@ -280,4 +331,23 @@ extern "C" {
     pub fn agpu_ritevik_decode_steps(m: *mut agpu_ritevik, batch: i32, steps: i32, ms_total_out_host: *mut f32) -> i32;
     pub fn agpu_ritevik_last_logits(m: *mut agpu_ritevik, batch: i32, logits_out_host: *mut f32) -> i32;
     pub fn agpu_ritevik_layer_streams(m: *mut agpu_ritevik, tokens: *const u32, new_len: i32, streams_out_host: *mut f32) -> i32;
+
+    // ---- include/agpu_piralix.h ----
+    pub fn agpu_piralix_create(ctx: *mut agpu_ctx, cfg: *const agpu_piralix_config, layers: *const agpu_piralix_layer, out: *mut *mut agpu_piralix) -> i32;
+    pub fn agpu_piralix_destroy(m: *mut agpu_piralix) -> i32;
+    pub fn agpu_piralix_set_tensor(m: *mut agpu_piralix, name: *const c_char, data_host: *const c_void, dtype: i32, rows: i64, cols: i64) -> i32;
+    pub fn agpu_piralix_tensor_info(m: *const agpu_piralix, i: i32, name_out: *mut *const c_char, rows_out: *mut i64, cols_out: *mut i64, is_set_out: *mut i32) -> i32;
+    pub fn agpu_piralix_weight_bytes(m: *const agpu_piralix) -> i64;
+    pub fn agpu_piralix_cache_bytes(m: *const agpu_piralix) -> i64;
+    pub fn agpu_piralix_layer_runs(m: *const agpu_piralix) -> i32;
+    pub fn agpu_piralix_reset_cache(m: *mut agpu_piralix) -> i32;
+    pub fn agpu_piralix_cache_len(m: *const agpu_piralix) -> i32;
+    pub fn agpu_piralix_forward_cached(m: *mut agpu_piralix, tokens: *const u32, batch: i32, new_len: i32, logits: *mut f32, all_rows: i32) -> i32;
+    pub fn agpu_piralix_generate_cached(m: *mut agpu_piralix, prompt_host: *const u32, batch: i32, prompt_len: i32, max_new_tokens: i32, eos: i32, tokens_out_host: *mut u32, lengths_out_host: *mut i32, timing_ms_out_host: *mut f32) -> i32;
+    pub fn agpu_piralix_generate(m: *mut agpu_piralix, prompt_host: *const u32, prompt_len: i32, max_new_tokens: i32, eos: i32, tokens_out_host: *mut u32, length_out_host: *mut i32) -> i32;
+    pub fn agpu_piralix_generate_cached_sampling(m: *mut agpu_piralix, prompt_host: *const u32, prompt_len: i32, max_new_tokens: i32, top_k: i32, temperature: f32, rng_state: *mut u64, eos: i32, tokens_out_host: *mut u32, length_out_host: *mut i32) -> i32;
+    pub fn agpu_piralix_set_decode_mode(m: *mut agpu_piralix, mode: i32) -> i32;
+    pub fn agpu_piralix_decode_steps(m: *mut agpu_piralix, batch: i32, steps: i32, ms_total_out_host: *mut f32) -> i32;
+    pub fn agpu_piralix_last_logits(m: *mut agpu_piralix, batch: i32, logits_out_host: *mut f32) -> i32;
+    pub fn agpu_piralix_layer_streams(m: *mut agpu_piralix, tokens: *const u32, new_len: i32, streams_out_host: *mut f32) -> i32;
 }

@@ -71,7 +71,8 @@ def test_every_header_function_is_bound_with_the_same_signature():
 
 @pytest.mark.parametrize("header_name, struct", [("agpu_gpt2.h", "agpu_gpt2_config"), ("agpu.h", "agpu_latent_attention_desc"),
                                                  ("agpu.h", "agpu_channel_delta_desc"), ("agpu_ritevik.h", "agpu_ritevik_config"),
-                                                 ("agpu_ritevik.h", "agpu_ritevik_layer")])
+                                                 ("agpu_ritevik.h", "agpu_ritevik_layer"), ("agpu_piralix.h", "agpu_piralix_config"),
+                                                 ("agpu_piralix.h", "agpu_piralix_layer")])
 def test_config_struct_fields_match(header_name, struct):
     header = open(os.path.join(ROOT, "include", header_name)).read()
     body = re.search(r"typedef struct %s \{(.*?)\} %s;" % (struct, struct), header, flags=re.S).group(1)
@@ -93,11 +94,11 @@ def test_constants_match_the_headers():
     rust = open(os.path.join(ROOT, "rust", "agpu-sys", "src", "lib.rs")).read()
     consts = {m.group(1): int(m.group(2), 0) for m in re.finditer(r"pub const (AGPU_\w+): \w+ = (-?(?:0x)?[0-9a-fA-F]+);", rust)}
     assert len(consts) >= 25
-    for fn in ("agpu.h", "agpu_gpt2.h", "agpu_ritevik.h"):
+    for fn in ("agpu.h", "agpu_gpt2.h", "agpu_ritevik.h", "agpu_piralix.h"):
         text = open(os.path.join(ROOT, "include", fn)).read()
         for m in re.finditer(r"#define (AGPU_\w+) \(?(-?(?:0x)?[0-9a-fA-F]+)u?\)?", text):
             name, value = m.group(1), int(m.group(2), 0)
-            if name in ("AGPU_H", "AGPU_GPT2_H", "AGPU_RITEVIK_H"):
+            if name in ("AGPU_H", "AGPU_GPT2_H", "AGPU_RITEVIK_H", "AGPU_PIRALIX_H"):
                 continue
             assert name in consts, f"{name} of {fn} has no Rust constant"
             assert consts[name] == value, name
