@@ -147,22 +147,30 @@ RITEVIK_SMALL = ritevik_spec(768, 12, 64, 32, 256, 3072, 8, 50257, 64, loop=dict
 RITEVIK_LARGE = ritevik_spec(2048, 16, 128, 64, 512, 8192, 24, 50257, 128)
 
 
+class _Draw:
+    """Random bf16 weights by name.  Matrices are cut from one pool of N(0, 1) values scaled to 1 / sqrt(K), so a model of billions of
+    weights takes seconds."""
+
+    def __init__(self, seed):
+        self.rng = np.random.default_rng(seed)
+        self.pool = self.rng.standard_normal(1 << 22, dtype=np.float32)
+        self.out = {}
+
+    def mat(self, name, rows, cols, gain=1.0):
+        from .weights import f32_to_bf16
+        n, lo = rows * cols, int(self.rng.integers(0, self.pool.size))
+        base = f32_to_bf16(np.roll(self.pool, -lo)[: min(n, self.pool.size)] * np.float32(gain / np.sqrt(cols)))
+        self.out[name] = ("BF16", np.resize(base, (rows, cols)))
+
+    def vec(self, name, shape, centre=0.0, spread=0.1):
+        from .weights import f32_to_bf16
+        self.out[name] = ("BF16", f32_to_bf16((centre + spread * self.rng.standard_normal(shape)).astype(np.float32)))
+
+
 def ritevik_tensors(spec, seed, rank=None):
-    """{name: (dtype, array)} of random bf16 weights.  Matrices are cut from one pool of N(0, 1) values scaled to 1 / sqrt(K), so
-    a model of billions of weights takes seconds; `rank` is the low-rank size of the delta layers (default: head dim)."""
-    from .weights import f32_to_bf16
-    rng = np.random.default_rng(seed)
-    pool = rng.standard_normal(1 << 22, dtype=np.float32)
-    out = {}
-
-    def mat(name, rows, cols, gain=1.0):
-        n, lo = rows * cols, int(rng.integers(0, pool.size))
-        base = f32_to_bf16(np.roll(pool, -lo)[: min(n, pool.size)] * np.float32(gain / np.sqrt(cols)))
-        out[name] = ("BF16", np.resize(base, (rows, cols)))
-
-    def vec(name, shape, centre=0.0, spread=0.1):
-        out[name] = ("BF16", f32_to_bf16((centre + spread * rng.standard_normal(shape)).astype(np.float32)))
-
+    """{name: (dtype, array)} of random bf16 weights; `rank` is the low-rank size of the delta layers (default: head dim)."""
+    draw = _Draw(seed)
+    mat, vec, out = draw.mat, draw.vec, draw.out
     d, V, n_layer = spec["width"], spec["vocab"], len(spec["layers"])
     mat("embed", V, d, np.sqrt(d))
     vec("embed.norm", d)
@@ -209,4 +217,72 @@ def ritevik_tensors(spec, seed, rank=None):
             vec(p + "side.norm", d, 0.2)
     vec("final.norm", d)
     mat("head", V, d)
+    return out
+
+
+def piralix_spec(width, heads, kv_heads, head_dim, memory_heads, lru_blocks, ff, n_layer, vocab, loop=None):
+    """Two matrix memories, an attention and a gated recurrent layer in turn, each with a feed-forward; the memory's values take the
+    full width, its keys half of it."""
+    mlp = dict(kind="dense", ff=ff, limit=7.0)
+    vdim = width // memory_heads
+    memory = dict(type="mlstm", mlp=mlp, mixer=dict(heads=memory_heads, dim=vdim // 2, vdim=vdim, gate_cap=15.0))
+    attend = dict(type="attention", mlp=mlp, mixer=dict(heads=heads, kv_heads=kv_heads, dim=head_dim, vdim=head_dim, scale=head_dim ** -0.5, softcap=50.0,
+                                                        rot=dict(base=10000.0, dims=head_dim, scaling=dict(factor=8.0, fast=32.0, slow=1.0, original=4096))))
+    lru = dict(type="rglru", mlp=mlp, mixer=dict(width=width, blocks=lru_blocks, conv=4))
+    return dict(architecture="Piralix", width=width, vocab=vocab, norm=dict(eps=1e-6), loop=loop,
+                layers=[(memory, attend, memory, lru)[i % 4] for i in range(n_layer)])
+
+
+PIRALIX_SMALL = piralix_spec(768, 12, 4, 64, 6, 12, 3072, 8, 50257, loop=dict(start=2, stop=6, times=2))  # 12 layer runs
+PIRALIX_LARGE = piralix_spec(2048, 16, 4, 128, 8, 16, 8192, 24, 50257)
+
+
+def piralix_tensors(spec, seed):
+    """{name: (dtype, array)} of random bf16 weights."""
+    draw = _Draw(seed)
+    mat, vec, out = draw.mat, draw.vec, draw.out
+    d, V = spec["width"], spec["vocab"]
+    mat("embed", V, d, np.sqrt(d))
+    if spec.get("loop"):
+        vec("loop.step", (spec["loop"]["times"], d))
+    for i, e in enumerate(spec["layers"]):
+        p, m = f"l{i}.", e["mixer"]
+        q = p + "mix."
+        vec(p + "norm1", d, 1.0)
+        vec(p + "norm1b", d, 0.5)
+        if e["type"] == "mlstm":
+            H, nk, nv = m["heads"], m["heads"] * m["dim"], m["heads"] * m["vdim"]
+            for t, n in (("q", nk), ("k", nk), ("v", nv), ("g", nv), ("i", H), ("f", H)):
+                mat(q + t, n, d)
+            vec(q + "norm", nv, 1.0)
+            vec(q + "i.b", H)
+            vec(q + "f.b", H, 4.0, 1.0)
+            mat(q + "o", d, nv)
+        elif e["type"] == "attention":
+            H, G, D, DV = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+            for t, n in (("q", H * D), ("k", G * D), ("v", G * DV), ("g", H * DV)):
+                mat(q + t, n, d)
+            vec(q + "sink", H, 0.0, 1.0)
+            mat(q + "o", d, H * DV)
+        else:
+            W, B = m["width"], m["blocks"]
+            for t in "yx":
+                mat(q + t, W, d)
+                vec(q + t + ".b", W)
+            vec(q + "conv", (W, m["conv"]), 0.0, 0.6)
+            vec(q + "conv.b", W)
+            for t in ("ra", "ri"):
+                mat(q + t, W, W // B)
+                out[q + t] = ("BF16", out[q + t][1].reshape(B, W // B, W // B))
+                vec(q + t + ".b", (B, W // B))
+            vec(q + "lam", W, -4.0, 1.0)
+            mat(q + "o", d, W)
+        if e.get("mlp"):
+            ff = e["mlp"]["ff"]
+            vec(p + "norm2", d, 1.0)
+            vec(p + "norm2b", d, 0.5)
+            mat(p + "mlp.gate", ff, d)
+            mat(p + "mlp.up", ff, d)
+            mat(p + "mlp.down", d, ff)
+    vec("final.norm", d, 1.0)
     return out

@@ -112,6 +112,11 @@ def main():
                          "default both), one JSON line")
     ap.add_argument("--ritevik-trace", choices=("ritevik", "gpt2"), help="with --ritevik: a short run of that model alone, for kernel traces")
     ap.add_argument("--ritevik-context", type=int, default=1024, help="with --ritevik-trace: prompt length")
+    ap.add_argument("--piralix", nargs="*", choices=("small", "large"), metavar="SIZE",
+                    help="instead of the default workload: prefill and decode of Piralix beside Ritevik of the same size (small, large; default "
+                         "both), one JSON line")
+    ap.add_argument("--piralix-trace", choices=("piralix", "ritevik"), help="with --piralix: a short run of that model alone, for kernel traces")
+    ap.add_argument("--piralix-context", type=int, default=1024, help="with --piralix-trace: prompt length")
     args = ap.parse_args()
     if args.gpus != 1:
         sys.exit("bench.py: this build measures one GPU only (every GPU box here has one MI355X); run with --gpus 1")
@@ -121,6 +126,10 @@ def main():
     if not torch.cuda.is_available():
         sys.exit("bench.py: no GPU visible; the HIP path has no CPU fallback")
     pkg = entry.load_package()
+    if args.piralix is not None:
+        import bench_piralix
+        bench_piralix.run(args.piralix or ("small", "large"), args.piralix_trace, args.piralix_context)
+        return
     if args.ritevik is not None:
         import bench_ritevik
         bench_ritevik.run(args.ritevik or ("small", "large"), args.ritevik_trace, args.ritevik_context)
