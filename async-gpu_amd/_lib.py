@@ -102,6 +102,14 @@ SIGNATURES = {
     "agpu_latent_attention": (_i32, [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp]),
     "agpu_channel_delta_workspace_bytes": (_sz, [_vp, _vp]),
     "agpu_channel_delta": (_i32, [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp]),
+    "agpu_rope_table_stretched": (_i32, [_vp, _vp, _i32, _i32] + [C.c_double] * 5),
+    "agpu_grouped_kv_stride": (_i32, [_i32]),
+    "agpu_grouped_attention_workspace_bytes": (_sz, [_vp, _vp]),
+    "agpu_grouped_attention": (_i32, [_vp] * 12),
+    "agpu_matrix_memory_workspace_bytes": (_sz, [_vp, _vp]),
+    "agpu_matrix_memory": (_i32, [_vp] * 11),
+    "agpu_gated_lru_workspace_bytes": (_sz, [_vp, _vp]),
+    "agpu_gated_lru": (_i32, [_vp] * 12),
     # include/agpu_gpt2.h (first argument is the model handle, or the config / context)
     "agpu_gpt2_config_small": (_i32, [_vp]),
     "agpu_gpt2_config_xl": (_i32, [_vp]),
@@ -191,6 +199,22 @@ class ChannelDeltaDesc(C.Structure):
     """agpu_channel_delta_desc of include/agpu.h."""
     _fields_ = [(n, _i32) for n in ("heads", "kv_heads", "dim", "vdim", "taps", "decay_rank", "gate_rank")] + [("eps", _f)] + \
                [(n, _i32) for n in ("batch", "new_len", "cached", "ld", "ldo", "col_q", "col_k", "col_v", "col_b", "col_a1", "col_g1")]
+
+
+class GroupedAttentionDesc(C.Structure):
+    """agpu_grouped_attention_desc of include/agpu.h."""
+    _fields_ = [(n, _i32) for n in ("heads", "kv_heads", "dim", "vdim", "rot_dims")] + [("scale", _f), ("softcap", _f)] + \
+               [(n, _i32) for n in ("positions", "batch", "new_len", "cached", "ld", "ldo", "cache_dtype")]
+
+
+class MatrixMemoryDesc(C.Structure):
+    """agpu_matrix_memory_desc of include/agpu.h."""
+    _fields_ = [("heads", _i32), ("dim", _i32), ("vdim", _i32), ("gate_cap", _f)] + [(n, _i32) for n in ("batch", "new_len", "cached", "ld", "ldo")]
+
+
+class GatedLruDesc(C.Structure):
+    """agpu_gated_lru_desc of include/agpu.h."""
+    _fields_ = [(n, _i32) for n in ("width", "blocks", "taps", "batch", "new_len", "cached", "ld", "ldo", "col_y", "col_x")]
 
 
 class RitevikConfigStruct(C.Structure):

@@ -19,7 +19,7 @@ struct GroupedShape {
 // are zero.
 struct GroupedArgs {
     GroupedShape s;
-    const float2 *rope = nullptr;  // [positions][rot_dims / 2]: cos, sin
+    const float2 *rope = nullptr;  // [positions][rot_dims / 2]: cos, sin; never null
     const float *sink = nullptr;   // [heads] or null
     // rows [batch * new_len], stride ld: heads x dimp, kv_heads x dimp, kv_heads x vdimp, heads x vdimp (gate before its sigmoid, or null)
     const float *q = nullptr, *k = nullptr, *v = nullptr, *gate = nullptr;

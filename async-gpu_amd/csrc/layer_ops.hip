@@ -3,7 +3,10 @@
 
 #include "dense_linear.h"
 #include "gated_delta.h"
+#include "gated_lru.h"
+#include "grouped_attention.h"
 #include "latent_attention.h"
+#include "matrix_memory.h"
 
 namespace {
 
@@ -78,6 +81,63 @@ void delta_carve(const agpu_channel_delta_desc &d, Carver &c, DeltaArgs &a, int 
     a.o = c.take<float>(rows * s.heads * s.vdim);
 }
 
+bool rows_ok(int batch, int new_len, int cached) { return batch > 0 && new_len > 0 && cached >= 0 && (int64_t)batch * new_len <= 65535; }
+
+GroupedShape grouped_shape(const agpu_grouped_attention_desc &d) {
+    GroupedShape s;
+    s.heads = d.heads; s.kv_heads = d.kv_heads; s.dim = d.dim; s.vdim = d.vdim; s.rot_dims = d.rot_dims; s.scale = d.scale; s.softcap = d.softcap;
+    return s;
+}
+
+bool grouped_desc_ok(const agpu_grouped_attention_desc &d) {
+    return grouped_supported(grouped_shape(d)) && d.dim % 32 == 0 && d.vdim % 32 == 0 && rows_ok(d.batch, d.new_len, d.cached) && d.positions > 0 &&
+           d.cached <= d.positions - d.new_len && d.ld > 0 && d.ld % 4 == 0 && d.ldo % 4 == 0 && d.ldo >= d.heads * d.vdim &&
+           (d.cache_dtype == AGPU_DTYPE_BF16 || d.cache_dtype == AGPU_DTYPE_F32);
+}
+
+void grouped_carve(const agpu_ctx *ctx, const agpu_grouped_attention_desc &d, Carver &c, GroupedArgs &a, int **pos, float2 **no_turn) {
+    *pos = c.take<int>(1);
+    *no_turn = c.take<float2>(1);
+    a.partial = c.take<float>(grouped_partial_floats(ctx, grouped_shape(d), d.batch, d.new_len, d.cached + d.new_len));
+}
+
+MemoryShape memory_shape(const agpu_matrix_memory_desc &d) {
+    MemoryShape s;
+    s.heads = d.heads; s.dim = d.dim; s.vdim = d.vdim; s.cap = d.gate_cap;
+    return s;
+}
+
+bool memory_desc_ok(const agpu_matrix_memory_desc &d) {
+    return memory_supported(memory_shape(d)) && d.dim % 32 == 0 && d.vdim % 32 == 0 && rows_ok(d.batch, d.new_len, d.cached) && d.ld > 0 && d.ld % 4 == 0 &&
+           d.ldo % 4 == 0 && d.ldo >= d.heads * d.vdim;
+}
+
+void memory_carve(const agpu_matrix_memory_desc &d, Carver &c, MemoryArgs &a, int **pos) {
+    *pos = c.take<int>(1);
+    if (d.new_len > 1) a.scratch = c.take<char>(memory_scratch_bytes(memory_shape(d), d.batch, d.new_len));
+}
+
+LruShape lru_shape(const agpu_gated_lru_desc &d) {
+    LruShape s;
+    s.width = d.width; s.blocks = d.blocks; s.taps = d.taps;
+    return s;
+}
+
+bool lru_desc_ok(const agpu_gated_lru_desc &d) {
+    return lru_supported(lru_shape(d)) && d.width / d.blocks % 32 == 0 && rows_ok(d.batch, d.new_len, d.cached) && d.ld > 0 && d.ld % 4 == 0 &&
+           d.ldo >= d.width && d.col_y >= 0 && d.col_y % 4 == 0 && d.col_x >= 0 && d.col_x % 4 == 0;
+}
+
+void lru_carve(const agpu_gated_lru_desc &d, Carver &c, LruArgs &a, int **pos) {
+    const LruShape s = lru_shape(d);
+    const size_t rows = (size_t)d.batch * d.new_len;
+    *pos = c.take<int>(1);
+    if (d.new_len == 1) return;
+    a.u = c.take<float>(rows * s.widthp());
+    a.gates = c.take<float>(rows * 2 * s.widthp());
+    a.carries = c.take<float>(lru_carry_floats(s, d.batch, d.new_len));
+}
+
 int32_t set_position(agpu_ctx *ctx, int *pos, int value) {
     hipLaunchKernelGGL(set_position_kernel, dim3(1), dim3(1), 0, ctx->stream, pos, value);
     return AGPU_LAUNCH_CHECK(ctx, "set_position_kernel");
@@ -138,6 +198,17 @@ AGPU_EXPORT int32_t agpu_rope_table(agpu_ctx *ctx, float *table, int32_t positio
     RopeSpec spec;
     spec.dims = dims;
     spec.base = base;
+    return rope_table_launch(ctx, (float2 *)table, positions, spec);
+}
+
+AGPU_EXPORT int32_t agpu_rope_table_stretched(agpu_ctx *ctx, float *table, int32_t positions, int32_t dims, double base, double factor, double original,
+                                              double fast, double slow) {
+    AGPU_REQUIRE_CTX(ctx);
+    AGPU_REQUIRE_PTR(ctx, table);
+    if (positions <= 0 || dims <= 0 || dims % 2 != 0 || !(base > 1.0) || !(factor > 0.0) || !(original > 0.0) || !(fast > 0.0) || !(slow > 0.0))
+        return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "rope_table_stretched: positions %d, dims %d, base %g, factor %g", positions, dims, base, factor);
+    RopeSpec spec;
+    spec.dims = dims; spec.base = base; spec.factor = factor; spec.original = original; spec.fast = fast; spec.slow = slow;
     return rope_table_launch(ctx, (float2 *)table, positions, spec);
 }
 
@@ -213,4 +284,102 @@ AGPU_EXPORT int32_t agpu_channel_delta(agpu_ctx *ctx, const agpu_channel_delta_d
     const int32_t rc = set_position(ctx, pos, d.cached);
     if (rc != AGPU_OK) return rc;
     return d.new_len == 1 ? delta_step_launch(ctx, a) : delta_prefill_launch(ctx, a);
+}
+
+AGPU_EXPORT int32_t agpu_grouped_kv_stride(int32_t positions) { return grouped_kv_stride(positions); }
+
+AGPU_EXPORT size_t agpu_grouped_attention_workspace_bytes(const agpu_ctx *ctx, const agpu_grouped_attention_desc *desc) {
+    if (!ctx || !desc || !grouped_desc_ok(*desc)) return 0;
+    Carver c{nullptr};
+    GroupedArgs a;
+    int *pos;
+    float2 *no_turn;
+    grouped_carve(ctx, *desc, c, a, &pos, &no_turn);
+    return c.at;
+}
+
+AGPU_EXPORT int32_t agpu_grouped_attention(agpu_ctx *ctx, const agpu_grouped_attention_desc *desc, const float *q, const float *k, const float *v,
+                                           const float *gate, const float *sink, const float *rope, void *kcache, void *vcache, float *out,
+                                           void *workspace) {
+    AGPU_REQUIRE_CTX(ctx);
+    for (const void *p : {(const void *)desc, (const void *)q, (const void *)k, (const void *)v, (const void *)kcache, (const void *)vcache, (const void *)out,
+                          (const void *)workspace})
+        AGPU_REQUIRE_PTR(ctx, p);
+    if (!grouped_desc_ok(*desc)) return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "grouped_attention: sizes not supported");
+    if (desc->rot_dims > 0) AGPU_REQUIRE_PTR(ctx, rope);
+    const agpu_grouped_attention_desc &d = *desc;
+    GroupedArgs a;
+    a.s = grouped_shape(d);
+    a.q = q; a.k = k; a.v = v; a.gate = gate; a.sink = sink; a.ld = d.ld;
+    a.kcache = kcache; a.vcache = vcache; a.cache_bf16 = d.cache_dtype == AGPU_DTYPE_BF16; a.positions = d.positions;
+    a.batch = d.batch; a.new_len = d.new_len; a.kv_max = d.cached + d.new_len;
+    a.out = out; a.ldo = d.ldo;
+    Carver c{(char *)workspace};
+    int *pos = nullptr;
+    float2 *no_turn = nullptr;
+    grouped_carve(ctx, d, c, a, &pos, &no_turn);
+    a.pos_dev = pos;
+    a.rope = rope ? (const float2 *)rope : no_turn;
+    const int32_t rc = set_position(ctx, pos, d.cached);
+    return rc == AGPU_OK ? grouped_attention_launch(ctx, a) : rc;
+}
+
+AGPU_EXPORT size_t agpu_matrix_memory_workspace_bytes(const agpu_ctx *ctx, const agpu_matrix_memory_desc *desc) {
+    if (!ctx || !desc || !memory_desc_ok(*desc)) return 0;
+    Carver c{nullptr};
+    MemoryArgs a;
+    int *pos;
+    memory_carve(*desc, c, a, &pos);
+    return c.at;
+}
+
+AGPU_EXPORT int32_t agpu_matrix_memory(agpu_ctx *ctx, const agpu_matrix_memory_desc *desc, const float *q, const float *k, const float *v, const float *i,
+                                       const float *f, float *state, float *norm, float *out, void *workspace) {
+    AGPU_REQUIRE_CTX(ctx);
+    for (const void *p : {(const void *)desc, (const void *)q, (const void *)k, (const void *)v, (const void *)i, (const void *)f, (const void *)state,
+                          (const void *)norm, (const void *)out, (const void *)workspace})
+        AGPU_REQUIRE_PTR(ctx, p);
+    if (!memory_desc_ok(*desc)) return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "matrix_memory: sizes not supported");
+    const agpu_matrix_memory_desc &d = *desc;
+    MemoryArgs a;
+    a.s = memory_shape(d);
+    a.q = q; a.k = k; a.v = v; a.i = i; a.f = f; a.ld = d.ld;
+    a.state = state; a.norm = norm; a.batch = d.batch; a.new_len = d.new_len; a.out = out; a.ldo = d.ldo;
+    Carver c{(char *)workspace};
+    int *pos = nullptr;
+    memory_carve(d, c, a, &pos);
+    a.pos_dev = pos;
+    const int32_t rc = set_position(ctx, pos, d.cached);
+    return rc == AGPU_OK ? memory_launch(ctx, a) : rc;
+}
+
+AGPU_EXPORT size_t agpu_gated_lru_workspace_bytes(const agpu_ctx *ctx, const agpu_gated_lru_desc *desc) {
+    if (!ctx || !desc || !lru_desc_ok(*desc)) return 0;
+    Carver c{nullptr};
+    LruArgs a;
+    int *pos;
+    lru_carve(*desc, c, a, &pos);
+    return c.at;
+}
+
+AGPU_EXPORT int32_t agpu_gated_lru(agpu_ctx *ctx, const agpu_gated_lru_desc *desc, const float *proj, const float *conv, const float *conv_bias,
+                                   const uint16_t *gates, const float *gate_bias, const float *lam, float *state, float *ring, float *out,
+                                   void *workspace) {
+    AGPU_REQUIRE_CTX(ctx);
+    for (const void *p : {(const void *)desc, (const void *)proj, (const void *)conv, (const void *)conv_bias, (const void *)gates, (const void *)gate_bias,
+                          (const void *)lam, (const void *)state, (const void *)ring, (const void *)out, (const void *)workspace})
+        AGPU_REQUIRE_PTR(ctx, p);
+    if (!lru_desc_ok(*desc)) return agpu_fail(ctx, AGPU_ERR_SHAPE_MISMATCH, "gated_lru: sizes not supported");
+    const agpu_gated_lru_desc &d = *desc;
+    LruArgs a;
+    a.s = lru_shape(d);
+    a.w.conv = conv; a.w.conv_bias = conv_bias; a.w.gates = gates; a.w.gate_bias = gate_bias; a.w.lam = lam;
+    a.proj = proj; a.ld = d.ld; a.col_y = d.col_y; a.col_x = d.col_x;
+    a.state = state; a.ring = ring; a.batch = d.batch; a.new_len = d.new_len; a.out = out; a.ldo = d.ldo;
+    Carver c{(char *)workspace};
+    int *pos = nullptr;
+    lru_carve(d, c, a, &pos);
+    a.pos_dev = pos;
+    const int32_t rc = set_position(ctx, pos, d.cached);
+    return rc == AGPU_OK ? lru_launch(ctx, a) : rc;
 }

@@ -6,16 +6,15 @@
 // Many tokens, in chunks of 64.  With F the running sum of the log forget gates of a chunk and a_s = i_s - F_s, the weight of
 // token s in the state after token t is exp(a_s - M_t) with M_t = max(m, max_{s <= t} a_s), m the running maximum in front of
 // the chunk, and m_t = F_t + M_t.  All of it is at most 1, however strong the gates.  F, a and M are kept in double precision:
-// their differences are small where a weight matters, themselves they are not.  Three launches:
+// their differences are small where a weight matters, themselves they are not.  Four launches:
 //   scores  P[t][s] = (q_t . k_s) exp(a_s - A_t), A_t = max_{s <= t} a_s, its row sums, the weights exp(a_s - A_last)
-//   states  S and n in front of every chunk, chunk after chunk: S <- exp(m - M) S + exp(A - M) sum_s weight_s k_s v_s^T
+//   increments, scan  S and n in front of every chunk: S <- exp(m - M) S + exp(A - M) sum_s weight_s k_s v_s^T
 //   outputs o_t = (exp(m - M_t) S^T q_t + exp(A_t - M_t) P v) / (max(|n_t . q_t|, exp(-m_t)) + 1e-6)
-// The products run on the fp32 matrix cores (v_mfma_f32_32x32x2_f32, v_mfma_f32_16x16x4_f32).
+// The products run on the fp32 matrix cores (v_mfma_f32_32x32x2_f32).
 #include "matrix_memory.h"
 
 namespace {
 
-typedef float f32x4 __attribute__((ext_vector_type(4)));
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 
 constexpr int C = kMemoryChunk;
@@ -191,100 +190,109 @@ __global__ __launch_bounds__(256) void memory_scores_kernel(MemoryArgs a, int di
     for (int i = tid; i < C * C; i += 256) p[i] = tile[i / C][i % C];
 }
 
-// grid (tiles of 32 dimensions, tiles of 64 value dimensions, heads * batch), four waves of 16 value dimensions each; the
-// chunks one after the other.
-__global__ __launch_bounds__(256) void memory_states_kernel(MemoryArgs a, int dimp, int vdimp, int chunks) {
-    __shared__ __align__(16) float sk[2][C][48], sv[2][C][80];  // 32 and 64 used: rows of a k step on different banks
+// grid (tiles of 64 dimensions * chunks, tiles of 64 value dimensions, heads * batch), 2 x 2 waves: what the chunk adds to S and n,
+// sum_s weight_s v_s k_s^T and sum_s weight_s k_s.
+__global__ __launch_bounds__(256) void memory_increments_kernel(MemoryArgs a, int dimp, int vdimp, int chunks) {
+    __shared__ __align__(16) float sk[C][64], sv[C][64];
     const MemoryShape &s = a.s;
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lc = lane & 15, lg = lane >> 4;
-    const int d0 = blockIdx.x * 32, j0 = blockIdx.y * 64, h = blockIdx.z % s.heads, b = blockIdx.z / s.heads, T = a.new_len, pos = *a.pos_dev;
-    const size_t bh = (size_t)b * s.heads + h, row0 = (size_t)b * T;
-    const Scratch x = scratch_of(a.scratch, bh, chunks, dimp, vdimp);
-    float *norm = a.norm + bh * 2 * (dimp + 4);
-    const float *old = norm + (pos & 1) * (dimp + 4);
-    const bool keeps_norm = blockIdx.y == 0 && tid < 32;
-    float n = keeps_norm ? old[d0 + tid] : 0.0f;
-    double m = (double)old[dimp];
-    // register r of tile i: value dimension j0 + 16 wave + 4 lg + r, dimension d0 + 16 i + lc
-    const int j = j0 + 16 * wave + 4 * lg;
-    const bool on = j0 + 16 * wave < vdimp;
-    float *st = a.state + (bh * vdimp + min(j, vdimp - 4)) * dimp + d0 + lc;
-    f32x4 S[2];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, wm = wave >> 1, wn = wave & 1, lr = lane & 31, lh = lane >> 5;
+    const int d0 = blockIdx.x / chunks * 64, chunk = blockIdx.x % chunks, j0 = blockIdx.y * 64, h = blockIdx.z % s.heads, b = blockIdx.z / s.heads;
+    const int T = a.new_len, t0 = chunk * C, nt = min(C, T - t0);
+    const size_t row0 = (size_t)b * T + t0;
+    const Scratch x = scratch_of(a.scratch, (size_t)b * s.heads + h, chunks, dimp, vdimp);
+    const int e = (tid & 15) * 4;
+    float4 rk[4], rv[4];
+    float rw[4];
 #pragma unroll
-    for (int i = 0; i < 2; ++i)
+    for (int i = 0; i < 4; ++i) {
+        const int t = (tid >> 4) + 16 * i;
+        const float *row = a.k + (row0 + min(t, nt - 1)) * a.ld;
+        rk[i] = *(const float4 *)(row + h * dimp + min(d0 + e, dimp - 4));
+        rv[i] = *(const float4 *)(a.v + (row0 + min(t, nt - 1)) * a.ld + h * vdimp + min(j0 + e, vdimp - 4));
+        rw[i] = x.weight[(size_t)chunk * C + t];  // 0 behind the last token
+    }
 #pragma unroll
-        for (int r = 0; r < 4; ++r) S[i][r] = st[(size_t)r * dimp + 16 * i];
-    float4 rk[2], rv[4];
-    float rw[2];
-    auto request = [&](int chunk) {
-        const int t0 = chunk * C, nt = min(C, T - t0);
-#pragma unroll
-        for (int i = 0; i < 2; ++i) {
-            const int t = (tid >> 3) + 32 * i;
-            rk[i] = *(const float4 *)(a.k + (row0 + t0 + min(t, nt - 1)) * a.ld + h * dimp + d0 + (tid & 7) * 4);
-            rw[i] = x.weight[(size_t)chunk * C + t];  // 0 behind the last token
-        }
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int t = (tid >> 4) + 16 * i;
-            rv[i] = *(const float4 *)(a.v + (row0 + t0 + min(t, nt - 1)) * a.ld + h * vdimp + min(j0 + (tid & 15) * 4, vdimp - 4));
-        }
-    };
-    auto stage = [&](int buf) {
-#pragma unroll
-        for (int i = 0; i < 2; ++i)
-            *(float4 *)&sk[buf][(tid >> 3) + 32 * i][(tid & 7) * 4] = make_float4(rk[i].x * rw[i], rk[i].y * rw[i], rk[i].z * rw[i], rk[i].w * rw[i]);
-#pragma unroll
-        for (int i = 0; i < 4; ++i) *(float4 *)&sv[buf][(tid >> 4) + 16 * i][(tid & 15) * 4] = rv[i];
-    };
-    request(0);
-    stage(0);
+    for (int i = 0; i < 4; ++i) {
+        const int t = (tid >> 4) + 16 * i;
+        *(float4 *)&sk[t][e] = make_float4(rk[i].x * rw[i], rk[i].y * rw[i], rk[i].z * rw[i], rk[i].w * rw[i]);
+        *(float4 *)&sv[t][e] = rv[i];
+    }
     __syncthreads();
-    int buf = 0;
-    for (int chunk = 0; chunk < chunks; ++chunk, buf ^= 1) {
-        const bool more = chunk + 1 < chunks;
-        if (more) request(chunk + 1);
-        if (on) {
-            float *out = x.s + ((size_t)chunk * vdimp + j) * dimp + d0 + lc;
+    f32x16 acc;
 #pragma unroll
-            for (int i = 0; i < 2; ++i)
+    for (int r = 0; r < 16; ++r) acc[r] = 0.0f;
+#pragma unroll 8
+    for (int t = 0; t < C; t += 2) acc = __builtin_amdgcn_mfma_f32_32x32x2f32(sv[t + lh][32 * wm + lr], sk[t + lh][32 * wn + lr], acc, 0, 0, 0);
+    const int d = d0 + 32 * wn + lr;
+    if (d < dimp) {
+        float *out = x.s + (size_t)chunk * vdimp * dimp + d;
 #pragma unroll
-                for (int r = 0; r < 4; ++r) out[(size_t)r * dimp + 16 * i] = S[i][r];
+        for (int r = 0; r < 16; ++r) {
+            const int j = j0 + 32 * wm + 8 * (r >> 2) + 4 * lh + (r & 3);
+            if (j < vdimp) out[(size_t)j * dimp] = acc[r];
         }
-        if (keeps_norm) x.n[(size_t)chunk * dimp + d0 + tid] = n;
-        if (blockIdx.x == 0 && blockIdx.y == 0 && tid == 0) x.m[chunk] = m;
-        const double F = x.total[2 * chunk], A = x.total[2 * chunk + 1], M = fmax(m, A);
-        const float keep = expf((float)(m - M)), take = expf((float)(A - M));
-        m = F + M;
-        f32x4 u[2] = {{0.0f, 0.0f, 0.0f, 0.0f}, {0.0f, 0.0f, 0.0f, 0.0f}};
-#pragma unroll
-        for (int t = 0; t < C; t += 4) {
-            const float v = sv[buf][t + lg][16 * wave + lc];
-#pragma unroll
-            for (int i = 0; i < 2; ++i) u[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(v, sk[buf][t + lg][16 * i + lc], u[i], 0, 0, 0);
-        }
-#pragma unroll
-        for (int i = 0; i < 2; ++i)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) S[i][r] = fmaf(take, u[i][r], keep * S[i][r]);
-        if (keeps_norm) {
-            float v = 0.0f;
+    }
+    if (blockIdx.y == 0 && tid < 64 && d0 + tid < dimp) {
+        float v = 0.0f;
 #pragma unroll 16
-            for (int t = 0; t < C; ++t) v += sk[buf][t][tid];
-            n = fmaf(take, v, keep * n);
+        for (int t = 0; t < C; ++t) v += sk[t][tid];
+        x.n[(size_t)chunk * dimp + d0 + tid] = v;
+    }
+}
+
+// grid (groups of 1024 values of S and then n, heads * batch): the chunks one after the other; every increment gives way to the
+// state in front of its chunk.
+__global__ __launch_bounds__(256) void memory_scan_kernel(MemoryArgs a, int dimp, int vdimp, int chunks) {
+    extern __shared__ double sm[];  // [chunks + 1] running maximum in front of every chunk, [chunks][2] totals; [chunks] float2 factors
+    double *st = sm + chunks + 1;
+    float2 *sf = (float2 *)(st + 2 * chunks);
+    const int tid = threadIdx.x, pos = *a.pos_dev;
+    const size_t bh = blockIdx.y;  // sequence * heads + head
+    const Scratch x = scratch_of(a.scratch, bh, chunks, dimp, vdimp);
+    const float *old = a.norm + (bh * 2 + (pos & 1)) * (dimp + 4);
+    const int values = vdimp * dimp, at = (blockIdx.x * 256 + tid) * 4;
+    const bool on = at < values + dimp, is_n = at >= values;
+    float *buf = is_n ? x.n + min(at - values, dimp - 4) : x.s + at;
+    const size_t step = is_n ? dimp : values;
+    float4 S = *(const float4 *)(is_n ? old + min(at - values, dimp - 4) : a.state + bh * values + at);
+    for (int i = tid; i < 2 * chunks; i += 256) st[i] = x.total[i];
+    __syncthreads();
+    if (tid == 0) {
+        double m = (double)old[dimp];
+        for (int c = 0; c < chunks; ++c) {
+            sm[c] = m;
+            m = st[2 * c] + fmax(m, st[2 * c + 1]);
         }
-        if (more) stage(buf ^ 1);
-        __syncthreads();
+        sm[chunks] = m;
     }
-    if (on) {
-#pragma unroll
-        for (int i = 0; i < 2; ++i)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) st[(size_t)r * dimp + 16 * i] = S[i][r];
+    __syncthreads();
+    for (int c = tid; c < chunks; c += 256) {
+        const double M = fmax(sm[c], st[2 * c + 1]);
+        sf[c] = make_float2(expf((float)(sm[c] - M)), expf((float)(st[2 * c + 1] - M)));
     }
-    // The other workgroups may still read the slot that n and m go to: the next launch moves them.
-    if (keeps_norm) x.n[(size_t)chunks * dimp + d0 + tid] = n;
-    if (blockIdx.x == 0 && blockIdx.y == 0 && tid == 0) x.m[chunks] = m;
+    if (blockIdx.x == 0)
+        for (int c = tid; c <= chunks; c += 256) x.m[c] = sm[c];
+    __syncthreads();
+    if (!on) return;
+    constexpr int U = 8;
+#pragma unroll 1
+    for (int c0 = 0; c0 < chunks; c0 += U) {
+        float4 u[U];
+#pragma unroll
+        for (int i = 0; i < U; ++i) u[i] = *(const float4 *)(buf + (size_t)min(c0 + i, chunks - 1) * step);
+#pragma unroll
+        for (int i = 0; i < U; ++i) {
+            if (c0 + i >= chunks) break;
+            const float2 f = sf[c0 + i];
+            *(float4 *)(buf + (size_t)(c0 + i) * step) = S;
+            S.x = fmaf(f.y, u[i].x, f.x * S.x);
+            S.y = fmaf(f.y, u[i].y, f.x * S.y);
+            S.z = fmaf(f.y, u[i].z, f.x * S.z);
+            S.w = fmaf(f.y, u[i].w, f.x * S.w);
+        }
+    }
+    // the other workgroups may still read the slot that n and m go to: the next launch moves them
+    *(float4 *)(is_n ? buf + (size_t)chunks * step : a.state + bh * values + at) = S;
 }
 
 // grid (tiles of 64 value dimensions, chunks, heads * batch): 64 tokens x 64 value dimensions on 2 x 2 waves.
@@ -296,7 +304,7 @@ __global__ __launch_bounds__(256) void memory_outputs_kernel(MemoryArgs a, int d
     const int j0 = blockIdx.x * 64, chunk = blockIdx.y, h = blockIdx.z % s.heads, b = blockIdx.z / s.heads, T = a.new_len, t0 = chunk * C, nt = min(C, T - t0);
     const size_t bh = (size_t)b * s.heads + h, row0 = (size_t)b * T + t0;
     const Scratch x = scratch_of(a.scratch, bh, chunks, dimp, vdimp);
-    if (blockIdx.x == 0 && chunk == 0) {  // what the states kernel left for the next call
+    if (blockIdx.x == 0 && chunk == 0) {  // what the scan left for the next call
         float *norm = a.norm + (bh * 2 + ((*a.pos_dev + T) & 1)) * (dimp + 4);
         for (int d = tid; d < dimp; d += 256) norm[d] = x.n[(size_t)chunks * dimp + d];
         if (tid == 0) norm[dimp] = (float)x.m[chunks];
@@ -387,9 +395,12 @@ int32_t memory_launch(agpu_ctx *ctx, const MemoryArgs &a) {
     int32_t rc;
     hipLaunchKernelGGL(memory_scores_kernel, dim3((unsigned)chunks, (unsigned)s.heads, (unsigned)a.batch), dim3(256), 0, ctx->stream, a, dimp, vdimp);
     if ((rc = AGPU_LAUNCH_CHECK(ctx, "memory_scores_kernel")) != AGPU_OK) return rc;
-    hipLaunchKernelGGL(memory_states_kernel, dim3((unsigned)(dimp / 32), (unsigned)ceil_div(vdimp, 64), (unsigned)(s.heads * a.batch)), dim3(256), 0, ctx->stream,
-                       a, dimp, vdimp, chunks);
-    if ((rc = AGPU_LAUNCH_CHECK(ctx, "memory_states_kernel")) != AGPU_OK) return rc;
+    hipLaunchKernelGGL(memory_increments_kernel, dim3((unsigned)(ceil_div(dimp, 64) * chunks), (unsigned)ceil_div(vdimp, 64), (unsigned)(s.heads * a.batch)), dim3(256),
+                       0, ctx->stream, a, dimp, vdimp, chunks);
+    if ((rc = AGPU_LAUNCH_CHECK(ctx, "memory_increments_kernel")) != AGPU_OK) return rc;
+    hipLaunchKernelGGL(memory_scan_kernel, dim3((unsigned)ceil_div((vdimp + 1) * dimp, 1024), (unsigned)(s.heads * a.batch)), dim3(256),
+                       (size_t)(chunks + 1) * 4 * sizeof(double), ctx->stream, a, dimp, vdimp, chunks);
+    if ((rc = AGPU_LAUNCH_CHECK(ctx, "memory_scan_kernel")) != AGPU_OK) return rc;
     hipLaunchKernelGGL(memory_outputs_kernel, dim3((unsigned)ceil_div(vdimp, 64), (unsigned)chunks, (unsigned)(s.heads * a.batch)), dim3(256), 0, ctx->stream, a,
                        dimp, vdimp, chunks);
     return AGPU_LAUNCH_CHECK(ctx, "memory_outputs_kernel");

@@ -7,7 +7,7 @@
 //   up    act(norm2(x) W)                                                                one Linear, the activation in its epilogue
 //   down  y = W_down act                                                                 one Linear
 // The norm behind a sublayer and its addition are left to whatever reads x next (DenseRows::y), as are the additions in front
-// of a loop's pass; the matrix memory's head norm and gate are left to its out Linear (DenseRows::gate).  Up to four rows run
+// of a loop's pass; the matrix memory's head norm and gate are left to its out Linear (DenseRows::gate).  One or two rows run
 // as GEMVs that do all this in their prologue; more rows go through dense_rows_launch and the matrix cores.
 //
 // Heads and blocks are padded to multiples of 32 columns everywhere (projections, cache, state, mixer output, columns of W_o),
@@ -70,7 +70,8 @@ struct agpu_piralix final : LayeredModel {
     int max_in = 0, max_mix = 0, max_ff = 0;
     DevBuf xa, xb, x0, y, h, proj, raw, mix, act, partial, memory, lru_u, lru_gates, lru_carries;
 
-    bool small(int rows) const { return dense_gemv_supported(rows, std::max({dp, max_mix, max_ff})); }
+    // more rows than these pay more for a prologue per workgroup than for row launches and the matrix cores
+    bool small(int rows) const { return rows <= 2 && dense_gemv_supported(rows, std::max({dp, max_mix, max_ff})); }
 };
 
 namespace {

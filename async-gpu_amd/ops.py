@@ -324,9 +324,13 @@ def dense_linear(x, w, bias=None, residual=None, dtype=_lib.DTYPE_BF16, gated=Fa
     return y
 
 
-def rope_table(positions, dims, base, device=0):
+def rope_table(positions, dims, base, device=0, stretch=None):
+    """cos and sin [positions, dims / 2, 2]; stretch: (factor, original, fast, slow) of a stretched context."""
     t = torch.empty((positions, dims // 2, 2), dtype=torch.float32, device=f"cuda:{device}")
-    context(device).call("agpu_rope_table", t, positions, dims, float(base))
+    if stretch:
+        context(device).call("agpu_rope_table_stretched", t, positions, dims, float(base), *(float(x) for x in stretch))
+    else:
+        context(device).call("agpu_rope_table", t, positions, dims, float(base))
     return t
 
 
@@ -358,3 +362,29 @@ def channel_delta(desc, proj, conv, a_log, dt_bias, a2, g2, norm, state, ring):
     ws = _workspace(c, "agpu_channel_delta_workspace_bytes", desc, proj.device)
     c.call("agpu_channel_delta", C.addressof(desc), proj, conv, a_log, dt_bias, a2, g2, norm, state, ring, out, ws)
     return out
+
+
+def _mixer(name, desc, first, args, columns):
+    """A mixer operator on a filled descriptor: workspace and output rows [batch * new_len, columns]."""
+    import ctypes as C
+    c = context(first.device.index or 0)
+    desc.ldo = columns
+    out = torch.empty((desc.batch * desc.new_len, columns), dtype=torch.float32, device=first.device)
+    ws = _workspace(c, name + "_workspace_bytes", desc, first.device)
+    c.call(name, C.addressof(desc), first, *args, out, ws)
+    return out
+
+
+def grouped_attention(desc, q, k, v, gate, sink, rope, kcache, vcache):
+    """agpu_grouped_attention on a filled _lib.GroupedAttentionDesc; appends to the caches."""
+    return _mixer("agpu_grouped_attention", desc, q, (k, v, gate, sink, rope, kcache, vcache), desc.heads * desc.vdim)
+
+
+def matrix_memory(desc, q, k, v, i, f, state, norm):
+    """agpu_matrix_memory on a filled _lib.MatrixMemoryDesc; advances `state` and `norm`."""
+    return _mixer("agpu_matrix_memory", desc, q, (k, v, i, f, state, norm), desc.heads * desc.vdim)
+
+
+def gated_lru(desc, proj, conv, conv_bias, gates, gate_bias, lam, state, ring):
+    """agpu_gated_lru on a filled _lib.GatedLruDesc; advances `state` and `ring`."""
+    return _mixer("agpu_gated_lru", desc, proj, (conv, conv_bias, gates, gate_bias, lam, state, ring), desc.width)

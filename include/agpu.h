@@ -419,6 +419,69 @@ int32_t agpu_channel_delta(agpu_ctx *ctx, const agpu_channel_delta_desc *desc, c
                            const float *dt_bias, const uint16_t *a2, const uint16_t *g2, const float *norm, float *state, float *ring,
                            float *out, void *workspace);
 
+/* The rotation table of a stretched context (YaRN), same layout as agpu_rope_table: with pair(t) = dims ln(original / (2 pi t)) /
+ * (2 ln base), pair i turns base^(-2 i / dims) per position below pair(fast), `factor` times slower above pair(slow), and a
+ * linear ramp lies between; cos and sin are multiplied by 0.1 ln(factor) + 1. */
+int32_t agpu_rope_table_stretched(agpu_ctx *ctx, float *table, int32_t positions, int32_t dims, double base, double factor, double original,
+                                  double fast, double slow);
+
+/*
+ * Causal attention of grouped heads, `new_len` tokens of each of `batch` sequences behind `cached` ones: query head h uses key and
+ * value head h / (heads / kv_heads).
+ *   q, k, v, gate: rows [batch * new_len], row stride ld, of heads x dim, kv_heads x dim, kv_heads x vdim, heads x vdim values
+ *   q and k turn: dimension 2 i with 2 i + 1 for 2 i < rot_dims, by the angles of `rope` [positions][rot_dims / 2] (cos, sin)
+ *   score = q . k * scale, then softcap tanh(score / softcap) if softcap > 0; softmax over the cached and new tokens up to the
+ *   query's own, with exp(sink[h]) in the denominator if sink is not null
+ *   out rows [.., ldo] = the weighted values, times sigmoid(gate) if gate is not null
+ * kcache [batch][kv_heads][positions][dim], vcache [batch][kv_heads][vdim][agpu_grouped_kv_stride(positions)], AGPU_DTYPE_BF16 or
+ * _F32; appended to.  Sizes: dim, vdim % 32 == 0 and <= 256 (the model driver pads; this operator does not), rot_dims even,
+ * ld, ldo % 4 == 0, all rows 16-byte aligned.  rope may be null if rot_dims is 0.
+ */
+typedef struct agpu_grouped_attention_desc {
+    int32_t heads, kv_heads, dim, vdim, rot_dims;
+    float scale, softcap;
+    int32_t positions, batch, new_len, cached, ld, ldo, cache_dtype;
+} agpu_grouped_attention_desc;
+int32_t agpu_grouped_kv_stride(int32_t positions);
+size_t agpu_grouped_attention_workspace_bytes(const agpu_ctx *ctx, const agpu_grouped_attention_desc *desc);
+int32_t agpu_grouped_attention(agpu_ctx *ctx, const agpu_grouped_attention_desc *desc, const float *q, const float *k, const float *v,
+                               const float *gate, const float *sink, const float *rope, void *kcache, void *vcache, float *out, void *workspace);
+
+/*
+ * Matrix memory with exponential gates (mLSTM), `new_len` tokens of each of `batch` sequences behind `cached` ones.
+ *   q, k, v, i, f: rows [batch * new_len], row stride ld, of heads x dim, heads x dim, heads x vdim, heads, heads values
+ *   per head: log gates i <- cap tanh(i / cap), f <- log sigmoid(cap tanh(f / cap)); m' = max(f + m, i);
+ *   S <- exp(f + m - m') S + exp(i - m') k v^T, n likewise with k alone, m <- m'
+ *   out rows [.., ldo] = S^T q dim^-1/2 / (max(|n . q| dim^-1/2, exp(-m)) + 1e-6)
+ * state: fp32 [batch][heads][vdim][dim]; norm: fp32 [batch][heads][2][dim + 4], n and m of the last token in the slot of
+ * (tokens so far) mod 2; both start as zeros.  Sizes: dim, vdim % 32 == 0, dim <= 256, ld, ldo % 4 == 0, all rows 16-byte aligned.
+ */
+typedef struct agpu_matrix_memory_desc {
+    int32_t heads, dim, vdim;
+    float gate_cap;
+    int32_t batch, new_len, cached, ld, ldo;
+} agpu_matrix_memory_desc;
+size_t agpu_matrix_memory_workspace_bytes(const agpu_ctx *ctx, const agpu_matrix_memory_desc *desc);
+int32_t agpu_matrix_memory(agpu_ctx *ctx, const agpu_matrix_memory_desc *desc, const float *q, const float *k, const float *v, const float *i,
+                           const float *f, float *state, float *norm, float *out, void *workspace);
+
+/*
+ * Real-gated linear recurrent unit, `new_len` tokens of each of `batch` sequences behind `cached` ones.
+ *   proj rows [batch * new_len, ld] hold y and x (width channels each) at columns col_y and col_x
+ *   u = causal convolution of x with `taps` taps per channel (conv [width][taps], last column the current token) + conv_bias;
+ *   r = sigmoid(R u + b_r), i = sigmoid(I u + b_i), block by block of width / blocks channels: gates [blocks][R, I][out][in],
+ *   gate_bias [blocks][2][out]; log a = -8 r softplus(lam); S <- a S + sqrt(1 - a^2) i u
+ *   out rows [.., ldo] = S * gelu_tanh(y)
+ * state: fp32 [batch][width], ring [batch][taps][width]: the convolution inputs of the last tokens (slot: position % taps); both
+ * start as zeros.  Sizes: width / blocks % 32 == 0, columns and ld % 4 == 0.
+ */
+typedef struct agpu_gated_lru_desc {
+    int32_t width, blocks, taps, batch, new_len, cached, ld, ldo, col_y, col_x;
+} agpu_gated_lru_desc;
+size_t agpu_gated_lru_workspace_bytes(const agpu_ctx *ctx, const agpu_gated_lru_desc *desc);
+int32_t agpu_gated_lru(agpu_ctx *ctx, const agpu_gated_lru_desc *desc, const float *proj, const float *conv, const float *conv_bias,
+                       const uint16_t *gates, const float *gate_bias, const float *lam, float *state, float *ring, float *out, void *workspace);
+
 #ifdef __cplusplus
 }
 #endif

@@ -96,6 +96,57 @@ pub struct agpu_channel_delta_desc {
     pub col_g1: i32,
 }
 
+/// `agpu_grouped_attention_desc` of include/agpu.h.
+#[repr(C)]
+#[derive(Clone, Copy, Debug, Default)]
+pub struct agpu_grouped_attention_desc {
+    pub heads: i32,
+    pub kv_heads: i32,
+    pub dim: i32,
+    pub vdim: i32,
+    pub rot_dims: i32,
+    pub scale: f32,
+    pub softcap: f32,
+    pub positions: i32,
+    pub batch: i32,
+    pub new_len: i32,
+    pub cached: i32,
+    pub ld: i32,
+    pub ldo: i32,
+    pub cache_dtype: i32,
+}
+
+/// `agpu_matrix_memory_desc` of include/agpu.h.
+#[repr(C)]
+#[derive(Clone, Copy, Debug, Default)]
+pub struct agpu_matrix_memory_desc {
+    pub heads: i32,
+    pub dim: i32,
+    pub vdim: i32,
+    pub gate_cap: f32,
+    pub batch: i32,
+    pub new_len: i32,
+    pub cached: i32,
+    pub ld: i32,
+    pub ldo: i32,
+}
+
+/// `agpu_gated_lru_desc` of include/agpu.h.
+#[repr(C)]
+#[derive(Clone, Copy, Debug, Default)]
+pub struct agpu_gated_lru_desc {
+    pub width: i32,
+    pub blocks: i32,
+    pub taps: i32,
+    pub batch: i32,
+    pub new_len: i32,
+    pub cached: i32,
+    pub ld: i32,
+    pub ldo: i32,
+    pub col_y: i32,
+    pub col_x: i32,
+}
+
 /// Opaque Ritevik model.
 #[repr(C)]
 pub struct agpu_ritevik {
@@ -286,6 +337,14 @@ extern "C" {
     pub fn agpu_latent_attention(ctx: *mut agpu_ctx, desc: *const agpu_latent_attention_desc, q: *const f32, down: *const f32, norm: *const f32, uk: *const u16, uv: *const u16, sink: *const f32, rope: *const f32, cache: *mut c_void, out: *mut f32, workspace: *mut c_void) -> i32;
     pub fn agpu_channel_delta_workspace_bytes(ctx: *const agpu_ctx, desc: *const agpu_channel_delta_desc) -> usize;
     pub fn agpu_channel_delta(ctx: *mut agpu_ctx, desc: *const agpu_channel_delta_desc, proj: *const f32, conv: *const f32, a_log: *const f32, dt_bias: *const f32, a2: *const u16, g2: *const u16, norm: *const f32, state: *mut f32, ring: *mut f32, out: *mut f32, workspace: *mut c_void) -> i32;
+    pub fn agpu_rope_table_stretched(ctx: *mut agpu_ctx, table: *mut f32, positions: i32, dims: i32, base: f64, factor: f64, original: f64, fast: f64, slow: f64) -> i32;
+    pub fn agpu_grouped_kv_stride(positions: i32) -> i32;
+    pub fn agpu_grouped_attention_workspace_bytes(ctx: *const agpu_ctx, desc: *const agpu_grouped_attention_desc) -> usize;
+    pub fn agpu_grouped_attention(ctx: *mut agpu_ctx, desc: *const agpu_grouped_attention_desc, q: *const f32, k: *const f32, v: *const f32, gate: *const f32, sink: *const f32, rope: *const f32, kcache: *mut c_void, vcache: *mut c_void, out: *mut f32, workspace: *mut c_void) -> i32;
+    pub fn agpu_matrix_memory_workspace_bytes(ctx: *const agpu_ctx, desc: *const agpu_matrix_memory_desc) -> usize;
+    pub fn agpu_matrix_memory(ctx: *mut agpu_ctx, desc: *const agpu_matrix_memory_desc, q: *const f32, k: *const f32, v: *const f32, i: *const f32, f: *const f32, state: *mut f32, norm: *mut f32, out: *mut f32, workspace: *mut c_void) -> i32;
+    pub fn agpu_gated_lru_workspace_bytes(ctx: *const agpu_ctx, desc: *const agpu_gated_lru_desc) -> usize;
+    pub fn agpu_gated_lru(ctx: *mut agpu_ctx, desc: *const agpu_gated_lru_desc, proj: *const f32, conv: *const f32, conv_bias: *const f32, gates: *const u16, gate_bias: *const f32, lam: *const f32, state: *mut f32, ring: *mut f32, out: *mut f32, workspace: *mut c_void) -> i32;
     // ---- include/agpu_gpt2.h ----
     pub fn agpu_gpt2_config_small(out: *mut agpu_gpt2_config) -> i32;
     pub fn agpu_gpt2_config_xl(out: *mut agpu_gpt2_config) -> i32;

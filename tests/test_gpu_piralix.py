@@ -73,6 +73,105 @@ def test_each_mechanism_alone(what, dtype):
     check_rows(feed(m, t, [70, 1]), want, dtype, what)
 
 
+def to_device(dev, a):
+    return torch.from_numpy(np.ascontiguousarray(a.view(np.int16) if a.dtype == np.uint16 else a)).to(dev)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_attention_operator(dev, dtype):
+    """The attention operator on its own, without sink and gate and with them: portions of 33, 1, 5 and 1 tokens over one cache."""
+    from async_gpu_amd import _lib, ops
+    H, G, D, DV, B, P, T, scale, cap = 6, 2, 32, 64, 2, 96, 40, 0.4, 7.0
+    rng = np.random.default_rng(5)
+    rot = dict(dims=24, base=300.0, scaling=dict(factor=3.0, original=32, fast=4.0, slow=1.0))
+    cols = dict(q=H * D, k=G * D, v=G * DV, g=H * DV)
+    x = rng.standard_normal((B, T, sum(cols.values()))).astype(np.float32)
+    sink = rng.standard_normal(H).astype(np.float32)
+    rope = ops.rope_table(P, 24, 300.0, stretch=(3.0, 32, 4.0, 1.0))
+    f, grow = plain.frequencies(rot)
+    table = np.stack([np.cos(np.outer(np.arange(P), f)), np.sin(np.outer(np.arange(P), f))], -1) * grow
+    assert np.abs(rope.cpu().numpy() - table).max() <= 1e-6
+    for with_gate in (False, True):
+        want = []
+        for b in range(B):  # the plain layer with identity projections in and out; a large gate is open
+            w, at = {}, 0
+            for n, c in cols.items():
+                w[n] = np.eye(x.shape[2])[at:at + c]
+                at += c
+            h = x[b].astype(np.float64)
+            if not with_gate:
+                h = np.concatenate([h[:, :-H * DV], np.full((T, H * DV), 1e3)], 1)
+            w.update(sink=sink.astype(np.float64) if with_gate else np.full(H, -1e30), o=np.eye(H * DV))
+            want.append(plain.attention(h, w, dict(heads=H, kv_heads=G, dim=D, vdim=DV, scale=scale, softcap=cap, rot=rot), 0.0))
+        want, bf16 = np.stack(want), dtype == "bfloat16"
+        ct = torch.int16 if bf16 else torch.float32
+        kc = torch.zeros((B, G, P, D), dtype=ct, device=dev)
+        vc = torch.zeros((B, G, DV, _lib.cdll().agpu_grouped_kv_stride(P)), dtype=ct, device=dev)
+        at = 0
+        for n in (33, 1, 5, 1):
+            r = to_device(dev, x[:, at:at + n].reshape(B * n, -1).copy())
+            d = _lib.GroupedAttentionDesc(H, G, D, DV, 24, scale, cap, P, B, n, at, x.shape[2], 0, _lib.DTYPE_BF16 if bf16 else _lib.DTYPE_F32)
+            c = np.cumsum([0] + list(cols.values()))
+            out = ops.grouped_attention(d, r, r[:, c[1]:], r[:, c[2]:], r[:, c[3]:] if with_gate else None, to_device(dev, sink) if with_gate else None, rope, kc, vc)
+            e = np.abs(out.cpu().numpy().reshape(B, n, -1) - want[:, at:at + n]).max() / np.abs(want).max()
+            assert e <= (2e-2 if bf16 else 1e-5), (with_gate, at, n, e)
+            at += n
+
+
+def test_memory_operator(dev):
+    """The matrix memory on its own: portions of 70, 1, 64, 2, 1 and 5 tokens over one state, against the recurrence."""
+    from async_gpu_amd import _lib, ops
+    H, D, DV, B, cap, T = 3, 32, 96, 2, 5.0, 143
+    rng = np.random.default_rng(6)
+    cols = dict(q=H * D, k=H * D, v=H * DV, i=4, f=4)  # columns padded to fours
+    x = rng.standard_normal((B, T, sum(cols.values()))).astype(np.float32)
+    c = dict(zip(cols, np.cumsum([0] + list(cols.values()))))
+    x[:, :, c["f"]:] += 3.0
+    x[:, :, c["i"]:c["f"]] *= 4.0
+    want = []
+    for b in range(B):
+        h = x[b].astype(np.float64)
+        part = lambda n, e: h[:, c[n]:c[n] + H * e].reshape(T, H, e)  # noqa: E731
+        want.append(plain.matrix_memory_recurrence(part("q", D) / np.sqrt(D), part("k", D), part("v", DV), plain.soft_cap(part("i", 1)[..., 0], cap),
+                                                   plain.log_sigmoid(plain.soft_cap(part("f", 1)[..., 0], cap))).reshape(T, -1))
+    want = np.stack(want)
+    state, norm = torch.zeros((B, H, DV, D), device=dev), torch.zeros((B, H, 2, D + 4), device=dev)
+    at = 0
+    for n in (70, 1, 64, 2, 1, 5):
+        r = to_device(dev, x[:, at:at + n].reshape(B * n, -1).copy())
+        d = _lib.MatrixMemoryDesc(H, D, DV, cap, B, n, at, x.shape[2], 0)
+        out = ops.matrix_memory(d, r, *(r[:, c[t]:] for t in "kvif"), state, norm).cpu().numpy().reshape(B, n, -1)
+        # a read-out whose denominator is small magnifies rounding: each against its own size
+        e = np.abs(out - want[:, at:at + n]) / (np.abs(want[:, at:at + n]).max(-1, keepdims=True) + 1e-3)
+        assert np.quantile(e, 0.99) <= 2e-5 and e.max() <= 1e-3, (at, n, e.max())
+        at += n
+
+
+def test_recurrent_unit_operator(dev):
+    """The gated recurrent unit on its own: portions of 40, 2, 1 and 5 tokens over one state, batch of two."""
+    from async_gpu_amd import _lib, ops
+    W, blocks, N, B, T = 192, 3, 4, 2, 48
+    bs = W // blocks
+    rng = np.random.default_rng(7)
+    x = rng.standard_normal((B, T, 2 * W)).astype(np.float32)
+    f32 = lambda *s: rng.standard_normal(s).astype(np.float32)  # noqa: E731
+    conv, cb, gb, lam = 0.6 * f32(W, N), f32(W), f32(blocks, 2, bs), f32(W) - 2.0
+    gates = bf16_bits(rng.standard_normal((blocks, 2, bs, bs)) / 8)
+    g = bf16_values(gates)
+    w = {"y": np.eye(2 * W)[:W], "x": np.eye(2 * W)[W:], "y.b": 0.0, "x.b": 0.0, "conv": conv.astype(np.float64), "conv.b": cb.astype(np.float64), "ra": g[:, 0],
+         "ri": g[:, 1], "ra.b": gb[:, 0].astype(np.float64), "ri.b": gb[:, 1].astype(np.float64), "lam": lam.astype(np.float64), "o": np.eye(W)}
+    want = np.stack([plain.rglru(x[b].astype(np.float64), w, None, None) for b in range(B)])
+    state, ring = torch.zeros((B, W), device=dev), torch.zeros((B, N, W), device=dev)
+    at = 0
+    for n in (40, 2, 1, 5):
+        d = _lib.GatedLruDesc(W, blocks, N, B, n, at, 2 * W, 0, 0, W)
+        out = ops.gated_lru(d, to_device(dev, x[:, at:at + n].reshape(B * n, -1).copy()), to_device(dev, conv), to_device(dev, cb), to_device(dev, gates),
+                            to_device(dev, gb), to_device(dev, lam), state, ring)
+        e = np.abs(out.cpu().numpy().reshape(B, n, -1) - want[:, at:at + n]).max() / np.abs(want).max()
+        assert e <= 2e-5, (at, n, e)
+        at += n
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("name", sorted(SPECS))
 def test_prompt_against_token_by_token(name, dtype):

@@ -70,7 +70,8 @@ def test_every_header_function_is_bound_with_the_same_signature():
 
 
 @pytest.mark.parametrize("header_name, struct", [("agpu_gpt2.h", "agpu_gpt2_config"), ("agpu.h", "agpu_latent_attention_desc"),
-                                                 ("agpu.h", "agpu_channel_delta_desc"), ("agpu_ritevik.h", "agpu_ritevik_config"),
+                                                 ("agpu.h", "agpu_channel_delta_desc"), ("agpu.h", "agpu_grouped_attention_desc"),
+                                                 ("agpu.h", "agpu_matrix_memory_desc"), ("agpu.h", "agpu_gated_lru_desc"), ("agpu_ritevik.h", "agpu_ritevik_config"),
                                                  ("agpu_ritevik.h", "agpu_ritevik_layer"), ("agpu_piralix.h", "agpu_piralix_config"),
                                                  ("agpu_piralix.h", "agpu_piralix_layer")])
 def test_config_struct_fields_match(header_name, struct):
