@@ -226,8 +226,8 @@ def piralix_spec(width, heads, kv_heads, head_dim, memory_heads, lru_blocks, ff,
     mlp = dict(kind="dense", ff=ff, limit=7.0)
     vdim = width // memory_heads
     memory = dict(type="mlstm", mlp=mlp, mixer=dict(heads=memory_heads, dim=vdim // 2, vdim=vdim, gate_cap=15.0))
-    attend = dict(type="attention", mlp=mlp, mixer=dict(heads=heads, kv_heads=kv_heads, dim=head_dim, vdim=head_dim, scale=head_dim ** -0.5, softcap=50.0,
-                                                        rot=dict(base=10000.0, dims=head_dim, scaling=dict(factor=8.0, fast=32.0, slow=1.0, original=4096))))
+    attend = dict(type="attention", mlp=mlp, mixer=dict(heads=heads, kv_heads=kv_heads, dim=head_dim, vdim=head_dim, scale=head_dim ** -0.5, softcap=30.0,
+                                                        rot=dict(base=500000.0, dims=head_dim, scaling=dict(factor=4.0, fast=16.0, slow=2.0, original=8192))))
     lru = dict(type="rglru", mlp=mlp, mixer=dict(width=width, blocks=lru_blocks, conv=4))
     return dict(architecture="Piralix", width=width, vocab=vocab, norm=dict(eps=1e-6), loop=loop,
                 layers=[(memory, attend, memory, lru)[i % 4] for i in range(n_layer)])

@@ -20,13 +20,15 @@ def test_rotation_turns_neighbours_and_keeps_the_rest():
 
 def test_stretched_frequencies():
     """Fast pairs keep their frequency, slow ones are divided by the factor, the ramp lies between; a ramp of no width is a step."""
-    rot = dict(dims=64, base=10000.0, scaling=dict(factor=8.0, fast=32.0, slow=1.0, original=4096))
+    rot = dict(dims=48, base=20000.0, scaling=dict(factor=6.0, fast=20.0, slow=2.0, original=3000))
     f, grow = plain.frequencies(rot)
-    f0, one = plain.frequencies(dict(dims=64, base=10000.0))
-    assert one == 1.0 and np.isclose(grow, 0.1 * np.log(8.0) + 1.0)
-    assert np.allclose(f[:5], f0[:5]) and np.allclose(f[-3:], f0[-3:] / 8.0) and (np.diff(f0 / f) >= 0).all() and ((f0 / f)[8:18] > 1.0).any()
-    narrow, _ = plain.frequencies(dict(dims=64, base=10000.0, scaling=dict(factor=8.0, fast=1e9, slow=1e9, original=64)))
-    assert np.allclose(f0[1:] / narrow[1:], 8.0) and np.isclose(f0[0], narrow[0])
+    f0, one = plain.frequencies(dict(dims=48, base=20000.0))
+    assert one == 1.0 and np.isclose(grow, 0.1 * np.log(6.0) + 1.0)
+    assert np.allclose(f[:5], f0[:5]) and np.allclose(f[-3:], f0[-3:] / 6.0) and (np.diff(f0 / f) >= 0).all()
+    turns = 3000 * f0 / (2 * np.pi)  # over the original positions
+    assert np.allclose(f[turns > 40], f0[turns > 40]) and np.allclose(f[turns < 1], f0[turns < 1] / 6.0) and ((f0 / f > 1.01) & (f0 / f < 5.99)).any()
+    narrow, _ = plain.frequencies(dict(dims=48, base=20000.0, scaling=dict(factor=6.0, fast=1e9, slow=1e9, original=64)))
+    assert np.allclose(f0[1:] / narrow[1:], 6.0) and np.isclose(f0[0], narrow[0])
 
 
 def test_memory_reads_back_what_was_written():
